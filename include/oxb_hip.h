@@ -298,6 +298,42 @@ int  oxb_hip_sample_logits(const float* logits, uint32_t vocab, uint32_t batch, 
 int  oxb_hip_prefill_tokens(uint64_t model, uint64_t embedding, uint32_t seq, const uint32_t* ids, uint32_t n_tokens,
                             uint32_t pos_start, float* logits_or_null, uint32_t* token_out_or_null);
 
+/* ---- model designs described by a config.json (layer programs), and one loader for every kind of checkpoint.
+ * A checkpoint is a GGUF file (as above) or a folder with config.json and model.safetensors; config.json's "architecture"
+ * names the design in the library's registry (Fulirax: latent attention with sinks, dynamic-tanh norms, dense tanh-GELU
+ * feed-forwards, a loop over a range of layers).  The model behind the handle is driven by the same calls as any other:
+ * oxb_hip_decode, oxb_hip_prefill[_tokens], oxb_hip_decode_tokens[_sampled], oxb_hip_forward_tokens, the paged-cache calls
+ * and oxb_hip_model_reset / _destroy.  Its cache holds latent rows in the compute type: kv_dtype and window options, read_kv,
+ * set_rope_rows, set_lm_head and decode_hidden do not apply and answer InvalidArgument. */
+enum { OXB_COMPUTE_BF16 = 0, OXB_COMPUTE_F32 = 1 };   /* F32: every product in 32 bits */
+typedef struct {
+    char architecture[32];
+    uint32_t n_layers, n_runs;      /* layers with weights; layer runs of a forward (a repeated layer counts each time) */
+    uint32_t h, vocab;
+    uint32_t context_length;        /* 0: the checkpoint names none */
+    uint32_t is_gguf;
+} oxb_checkpoint_info;
+int  oxb_hip_checkpoint_info(const char* path, oxb_checkpoint_info* info);   /* no GPU needed */
+/* max_seq 0: the file's context length (GGUF only).  compute_type applies to configured designs. */
+int  oxb_hip_load_checkpoint(const char* path, int compute_type, uint32_t max_seq, uint32_t batch, uint64_t* model, uint64_t* embedding,
+                             oxb_checkpoint_info* info_or_null);
+/* The same from memory: config.json's text and the tensors (GGUF type ids: 0 F32, 1 F16, 30 BF16; row-major). */
+typedef struct {
+    const char* name;
+    int type;
+    uint32_t n_dims;
+    uint64_t shape[4];
+    const void* data;
+    uint64_t n_bytes;
+} oxb_tensor;
+int  oxb_hip_model_from_tensors(const char* config_json, const oxb_tensor* tensors, uint32_t n_tensors, int compute_type, uint32_t max_seq,
+                                uint32_t batch, uint64_t* model, uint64_t* embedding);
+/* A portion of one sequence: n_tokens ids at positions pos_start .. , continuing from the cache, with the logits of any of
+ * its tokens: logits[n_want][vocab] for portion indices want[n_want] (n_want 0: cache rows only).  A single token of a
+ * batch-1 model is a decode step (the captured graph); everything else a prefill. */
+int  oxb_hip_forward_tokens(uint64_t model, uint64_t embedding, uint32_t seq, const uint32_t* ids, uint32_t n_tokens,
+                            uint32_t pos_start, const uint32_t* want, uint32_t n_want, float* logits);
+
 /* ---- host-only helpers (no GPU needed): the upload-time repack, exposed so it can be checked on any machine.
  * reformat_q1_aos_to_soa / reformat_tq2_blocks_to_soa (KG/cuda_graph/cudagraph_reformat_*_group.rs). */
 int  oxb_hip_repack_sizes(int fmt, uint32_t n_rows, uint32_t k, size_t* codes_bytes, size_t* scales_bytes);

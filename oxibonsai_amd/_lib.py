@@ -82,6 +82,10 @@ _SIGNATURES = {
     "oxb_hip_sum_in_order": ([f32p, C.c_uint32, f32p], C.c_int),
     "oxb_hip_set_gemv_packed_min_batch": ([C.c_uint32], C.c_int),
     "oxb_hip_prefill_tokens": ([C.c_uint64, C.c_uint64, C.c_uint32, u32p, C.c_uint32, C.c_uint32, f32p, u32p], C.c_int),
+    "oxb_hip_checkpoint_info": ([C.c_char_p, C.c_void_p], C.c_int),
+    "oxb_hip_load_checkpoint": ([C.c_char_p, C.c_int, C.c_uint32, C.c_uint32, u64p, u64p, C.c_void_p], C.c_int),
+    "oxb_hip_model_from_tensors": ([C.c_char_p, C.c_void_p, C.c_uint32, C.c_int, C.c_uint32, C.c_uint32, u64p, u64p], C.c_int),
+    "oxb_hip_forward_tokens": ([C.c_uint64, C.c_uint64, C.c_uint32, u32p, C.c_uint32, C.c_uint32, u32p, C.c_uint32, f32p], C.c_int),
     "oxb_hip_repack_sizes": ([C.c_int, C.c_uint32, C.c_uint32, szp, szp], C.c_int),
     "oxb_hip_repack": ([C.c_int, u8p, C.c_size_t, C.c_uint32, C.c_uint32, u8p, C.c_size_t, u8p, C.c_size_t], C.c_int),
     "oxb_hip_unpack": ([C.c_int, u8p, C.c_size_t, u8p, C.c_size_t, C.c_uint32, C.c_uint32, u8p, C.c_size_t], C.c_int),

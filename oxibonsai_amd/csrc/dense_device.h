@@ -1,0 +1,143 @@
+// dense_device.h — matrix-core operands of 32 k-values in bf16 or fp32, and the scalar functions of the dense designs.
+//
+// One unit of work is a 16 x 16 x 32 product.  bf16: one v_mfma_f32_16x16x32_bf16, lane 16 g + r holding row r,
+// k = 8 g + e.  fp32: eight v_mfma_f32_16x16x4_f32 (full 32-bit multiply and add), step e taking element e of every lane,
+// so the four k-values of a step are 8 g + e, g = 0..3: the order of k inside a unit is free as long as both operands use
+// the same one, and kernels are written once for both types.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+#include "dense_kernels.h"
+#include "device_utils.h"
+
+typedef __bf16 v8b __attribute__((ext_vector_type(8)));
+typedef __bf16 v4b __attribute__((ext_vector_type(4)));
+typedef float v8f __attribute__((ext_vector_type(8)));
+
+template <typename T> struct Dt;
+template <> struct Dt<__bf16> {
+    typedef v8b frag;
+    typedef v4b quad;
+    static constexpr bool is_f32 = false;
+    static constexpr uint32_t unit_bytes = 1024, sub = 1;  // 1 KiB pieces per unit
+};
+template <> struct Dt<float> {
+    typedef v8f frag;
+    typedef v4f quad;
+    static constexpr bool is_f32 = true;
+    static constexpr uint32_t unit_bytes = 2048, sub = 2;
+};
+
+__device__ __forceinline__ v4f mfma32(v8b a, v8b b, v4f c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+__device__ __forceinline__ v4f mfma32(v8f a, v8f b, v4f c) {
+#pragma unroll
+    for (int e = 0; e < 8; e++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], b[e], c, 0, 0, 0);
+    return c;
+}
+
+// The lane's eight elements of a unit in operand order (global or LDS memory).
+__device__ __forceinline__ v8b load_unit(const __bf16* unit, uint32_t lane) { return *reinterpret_cast<const v8b*>(unit + lane * 8); }
+__device__ __forceinline__ v8f load_unit(const float* unit, uint32_t lane) {
+    const v4f a = *reinterpret_cast<const v4f*>(unit + lane * 4), b = *reinterpret_cast<const v4f*>(unit + 256 + lane * 4);
+    return (v8f){a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
+__device__ __forceinline__ void store_unit(__bf16* unit, uint32_t lane, v8b v) { *reinterpret_cast<v8b*>(unit + lane * 8) = v; }
+__device__ __forceinline__ void store_unit(float* unit, uint32_t lane, v8f v) {
+    *reinterpret_cast<v4f*>(unit + lane * 4) = (v4f){v[0], v[1], v[2], v[3]};
+    *reinterpret_cast<v4f*>(unit + 256 + lane * 4) = (v4f){v[4], v[5], v[6], v[7]};
+}
+// Eight consecutive elements of a row.
+__device__ __forceinline__ v8b load_row8(const __bf16* p) { return *reinterpret_cast<const v8b*>(p); }
+__device__ __forceinline__ v8f load_row8(const float* p) {
+    const v4f a = *reinterpret_cast<const v4f*>(p), b = *reinterpret_cast<const v4f*>(p + 4);
+    return (v8f){a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
+__device__ __forceinline__ v8b zero_frag(const __bf16*) { return (v8b)(__bf16)0.f; }
+__device__ __forceinline__ v8f zero_frag(const float*) { return (v8f)0.f; }
+
+// Memory -> LDS without a trip through registers, 16 bytes per lane: lane l's 16 bytes land at base + 16 l (base is
+// wave-uniform).  `src` is the lane's own address.
+typedef __attribute__((address_space(3))) void* lds_dst_t;
+typedef const __attribute__((address_space(1))) void* global_src_t;
+__device__ __forceinline__ void copy16_to_lds(const void* src, void* lds_base) {
+    __builtin_amdgcn_global_load_lds((global_src_t)src, (lds_dst_t)lds_base, 16, 0, 0);
+}
+// The lane's eight consecutive elements at `row8` into its place of the unit at `unit` (LDS).
+__device__ __forceinline__ void copy_row8_to_unit(const __bf16* row8, __bf16* unit) { copy16_to_lds(row8, unit); }
+__device__ __forceinline__ void copy_row8_to_unit(const float* row8, float* unit) {
+    copy16_to_lds(row8, unit);
+    copy16_to_lds(row8 + 4, unit + 256);
+}
+__device__ __forceinline__ void wait_lds_copies() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+
+// tanh in fp32: the library's for the fp32 kernels; for bf16 results 1 - 2 / (e^(2|z|) + 1) on the hardware exponential
+// (absolute error around 1e-7), with the odd series near zero where that form cancels.
+template <typename T> __device__ __forceinline__ float tanh_of(float z) {
+    if constexpr (Dt<T>::is_f32) return tanhf(z);
+    const float a = fabsf(z);
+    const float e = __builtin_amdgcn_exp2f(a * 2.8853900817779268f);
+    const float big = 1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f);
+    const float s = a * a;
+    const float small = a * (1.0f + s * (-0.33333333333f + s * (0.13333333333f - 0.053968253968f * s)));
+    return copysignf(a < 0.125f ? small : big, z);
+}
+template <typename T> __device__ __forceinline__ float gelu_tanh_of(float z) {
+    return 0.5f * z * (1.0f + tanh_of<T>(0.79788456080286536f * (z + 0.044715f * z * z * z)));
+}
+template <typename T> __device__ __forceinline__ float exp_of(float z) {  // e^z, z <= 0 in every use
+    if constexpr (Dt<T>::is_f32) return expf(z);
+    return __builtin_amdgcn_exp2f(z * 1.4426950408889634f);
+}
+
+// Four consecutive outputs y[m][n0 .. n0 + 3] through the epilogue.
+template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogue& e, uint32_t m, uint32_t n0, v4f y) {
+    const uint32_t lim = e.n > e.fill ? e.n : e.fill;
+    if (n0 >= lim) return;
+    y *= e.scale;
+    if (n0 + 4 <= e.n && (e.ld32 & 3u) == 0) {
+        if (e.add) y += *reinterpret_cast<const v4f*>(e.add + n0);
+        if (e.act == OXB_ACT_GELU_TANH) {
+#pragma unroll
+            for (int i = 0; i < 4; i++) y[i] = gelu_tanh_of<T>(y[i]);
+        }
+        const size_t o = (size_t)m * e.ld32 + n0;
+        if (e.resid) y += *reinterpret_cast<const v4f*>(e.resid + o);
+        if (e.out32) *reinterpret_cast<v4f*>(e.out32 + o) = y;
+        if (!e.out_t) return;
+        if (e.norm == OXB_NORM_DYT) {
+            const v4f w = *reinterpret_cast<const v4f*>(e.nw + n0), b = *reinterpret_cast<const v4f*>(e.nb + n0);
+#pragma unroll
+            for (int i = 0; i < 4; i++) y[i] = tanh_of<T>(e.alpha * y[i]) * w[i] + b[i];
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const uint32_t n = n0 + i;
+            if (n >= e.n) {
+                y[i] = 0.f;
+                continue;
+            }
+            float v = y[i];
+            if (e.add) v += e.add[n];
+            if (e.act == OXB_ACT_GELU_TANH) v = gelu_tanh_of<T>(v);
+            const size_t o = (size_t)m * e.ld32 + n;
+            if (e.resid) v += e.resid[o];
+            if (e.out32) e.out32[o] = v;
+            if (e.norm == OXB_NORM_DYT) v = tanh_of<T>(e.alpha * v) * e.nw[n] + e.nb[n];
+            y[i] = v;
+        }
+        if (!e.out_t) return;
+    }
+    T* t = reinterpret_cast<T*>(e.out_t) + (size_t)m * e.ld_t + n0;
+    if (n0 + 4 <= e.fill && (((uintptr_t)t) & (sizeof(T) * 4 - 1)) == 0) {
+        typename Dt<T>::quad q;
+#pragma unroll
+        for (int i = 0; i < 4; i++) q[i] = (T)y[i];
+        *reinterpret_cast<typename Dt<T>::quad*>(t) = q;
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (n0 + i < e.fill) t[i] = (T)y[i];
+    }
+}

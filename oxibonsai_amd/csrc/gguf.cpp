@@ -114,7 +114,7 @@ bool read_value(Cursor& c, uint32_t type, GgufValue* v, int depth) {
 uint64_t gguf_tensor_bytes(uint32_t type, uint64_t elements) {
     switch (type) {
         case GGUF_F32: return elements * 4;
-        case GGUF_F16: return elements * 2;
+        case GGUF_F16: case GGUF_BF16: return elements * 2;
         case GGUF_Q1_0_G128: return (elements + 127) / 128 * 18;
         case GGUF_TQ2_0_G128: return (elements + 127) / 128 * 34;
         default: return 0;

@@ -18,6 +18,8 @@ namespace oxb {
 enum GgufTensorType : uint32_t {  // crates/oxibonsai-core/src/gguf/types.rs:17-44 (the ids this tier consumes)
     GGUF_F32 = 0,
     GGUF_F16 = 1,
+    GGUF_I32 = 26,
+    GGUF_BF16 = 30,
     GGUF_Q1_0_G128 = 41,
     GGUF_TQ2_0_G128 = 42,
 };

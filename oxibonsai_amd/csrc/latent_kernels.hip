@@ -1,0 +1,578 @@
+// latent_kernels.hip — latent attention on the matrix cores (see latent_kernels.h for the two forms).
+//
+// Precision: scores, softmax and sums are fp32.  Probabilities meet bf16 values as a bf16 hi + lo pair (two products), so
+// a weight keeps 16 bits; the fp32 kernels use fp32 operands throughout.
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+#include "dense_device.h"
+#include "latent_kernels.h"
+
+__device__ __forceinline__ uint32_t row_pos(const OxbRows& r, uint32_t m) { return r.pos ? r.pos[m] : r.pos0 + m; }
+__device__ __forceinline__ uint32_t row_seq(const OxbRows& r, uint32_t m) { return r.seq0 + m * r.seq_step; }
+
+// Element i of a rotated part v (rot elements, the first rot_dims of them in pairs (i, i + rot_dims / 2)).
+__device__ __forceinline__ float rotated(const float* v, uint32_t i, uint32_t rot_dims, const float* cs, const float* sn) {
+    const uint32_t half = rot_dims >> 1;
+    if (i < half) return v[i] * cs[i] - v[i + half] * sn[i];
+    if (i < rot_dims) return v[i] * cs[i - half] + v[i - half] * sn[i - half];
+    return v[i];
+}
+
+// ---------------------------------------------------------------------------
+// New tokens: blocks [0, n_abs) of a grid row absorb queries (4 waves, one 16-row tile of (head, latent) each), the 16
+// blocks behind them take one token row each: RMS norm of the latent and rotation of the key part into the cache, rotation
+// of the query parts into q_abs.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, uint32_t n_abs, uint32_t tiles_per_head) {
+    typedef typename Dt<T>::frag frag;
+    const OxbLatentDims& d = p.d;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, m0 = blockIdx.y * 16;
+    const uint32_t kl = d.rank_p + d.rot_p, qh = d.dim_p + d.rot_p;
+    T* q_abs = reinterpret_cast<T*>(p.q_abs);
+    if (blockIdx.x < n_abs) {
+        const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+        const uint32_t tile = blockIdx.x * 4 + wave, c = lane & 15u, g = lane >> 4;
+        if (tile >= d.heads * tiles_per_head) return;
+        const uint32_t head = tile / tiles_per_head, rt = tile % tiles_per_head, nu = p.k_uk / 32;
+        const T* w = reinterpret_cast<const T*>(p.w_uk_t) + (size_t)tile * nu * 512;
+        const bool have = m0 + c < p.rows.m;
+        const float* q = p.qkv + (size_t)(have ? m0 + c : 0) * p.ld_qkv + head * qh + 8 * g;
+        v4f acc = {0.f, 0.f, 0.f, 0.f};
+        for (uint32_t u = 0; u < nu; u++) {
+            frag b = zero_frag((const T*)nullptr);
+            if (have && 32 * u < d.dim_p) {
+                const v4f lo = *reinterpret_cast<const v4f*>(q + 32 * u), hi = *reinterpret_cast<const v4f*>(q + 32 * u + 4);
+#pragma unroll
+                for (int e = 0; e < 4; e++) b[e] = (T)lo[e], b[4 + e] = (T)hi[e];
+            }
+            acc = mfma32(load_unit(w + (size_t)u * 512, lane), b, acc);
+        }
+        if (have) {
+            typename Dt<T>::quad o;
+#pragma unroll
+            for (int i = 0; i < 4; i++) o[i] = (T)acc[i];
+            *reinterpret_cast<typename Dt<T>::quad*>(q_abs + ((size_t)(m0 + c) * d.heads + head) * kl + rt * 16 + 4 * g) = o;
+        }
+        return;
+    }
+    const uint32_t m = m0 + blockIdx.x - n_abs;
+    if (m >= p.rows.m) return;
+    const uint32_t pos = row_pos(p.rows, m), half = d.rot_dims >> 1;
+    const float* cs = p.cos_t + (size_t)pos * half;
+    const float* sn = p.sin_t + (size_t)pos * half;
+    const float* row = p.qkv + (size_t)m * p.ld_qkv;
+    const float* lat = row + d.heads * qh;
+    __shared__ float red[4];
+    float ss = 0.f;
+    for (uint32_t i = tid; i < d.rank; i += 256) ss = fmaf(lat[i], lat[i], ss);
+    ss = wave_sum_f32(ss);
+    if (lane == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)d.rank + d.eps);
+    T* dst = reinterpret_cast<T*>(p.cache) + kv_row(p.kv, row_seq(p.rows, m), 0, 0, pos) * p.ld;
+    for (uint32_t i = tid; i < kl; i += 256) {
+        float v = 0.f;
+        if (i < d.rank) v = lat[i] * inv * p.c_norm[i];
+        else if (i >= d.rank_p && i - d.rank_p < d.rot) v = rotated(lat + d.rank_p, i - d.rank_p, d.rot_dims, cs, sn);
+        dst[i] = (T)v;
+    }
+    if (q_abs)
+        for (uint32_t i = tid; i < d.heads * d.rot_p; i += 256) {
+            const uint32_t head = i / d.rot_p, j = i % d.rot_p;
+            q_abs[((size_t)m * d.heads + head) * kl + d.rank_p + j] =
+                (T)(j < d.rot ? rotated(row + head * qh + d.dim_p, j, d.rot_dims, cs, sn) : 0.f);
+        }
+}
+
+// ---------------------------------------------------------------------------
+// Absorbed attention.  Grid (split, head tile, token row); the 16 heads of a tile are the columns of the products, so a
+// latent row is read once for all of them and serves as key and as value:
+//   S^T[key][head] = K[key] . q_abs[head]          K rows of 32 keys from LDS in operand order, q_abs resident in registers
+//   O^T[r][head]  += c[key][r] P[head][key]        the same LDS rows through the transposing read
+// Wave w of a workgroup takes keys [32 w, 32 w + 32) of a chunk with a softmax of its own and LDS of its own (memory -> LDS
+// copies, no barrier in the walk); the waves meet once at the end.  NT: accumulator tiles of 16 latent elements, KS: k
+// units of q_abs held in registers.
+// ---------------------------------------------------------------------------
+template <typename T>
+__device__ __forceinline__ typename Dt<T>::frag value_frag(const T* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g);
+template <>
+__device__ __forceinline__ v8b value_frag<__bf16>(const __bf16* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g) {
+    // keys 4 g .. 4 g + 3 of either key tile, latent element 16 sl + qi: two transposing reads
+    const uint32_t s = sl >> 1, r = 4 * g + (qi >> 2), slot = ((sl & 1u) * 2 + ((qi & 3u) >> 1)) * 16 + r;
+    const _Float16* a = reinterpret_cast<const _Float16*>(lds) + (size_t)s * 512 + slot * 8 + (qi & 1u) * 4;
+    const v4b t0 = __builtin_bit_cast(v4b, lds_read_tr16(a)), t1 = __builtin_bit_cast(v4b, lds_read_tr16(a + (size_t)ks * 512));
+    return (v8b){t0[0], t0[1], t0[2], t0[3], t1[0], t1[1], t1[2], t1[3]};
+}
+template <>
+__device__ __forceinline__ v8f value_frag<float>(const float* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g) {
+    const uint32_t d = 16 * sl + qi, e = d & 7u;
+    const float* a = lds + (size_t)(d >> 5) * 512 + (e >> 2) * 256 + (((d & 31u) >> 3) * 16 + 4 * g) * 4 + (e & 3u);
+    const float* b = a + (size_t)ks * 512;
+    return (v8f){a[0], a[4], a[8], a[12], b[0], b[4], b[8], b[12]};
+}
+
+template <typename T, int NT, int KS>
+__global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p) {
+    typedef typename Dt<T>::frag frag;
+    extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+    __shared__ float wave_ml[4][16][2];
+    const OxbLatentDims& d = p.d;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4, nw = blockDim.x >> 6;
+    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+    const uint32_t split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
+    const uint32_t pos = row_pos(p.rows, m), seq = row_seq(p.rows, m), chunk = 32 * nw, n_chunks = pos / chunk + 1;
+    if (split >= min(p.n_splits, n_chunks)) return;
+    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16;
+    T* lds = reinterpret_cast<T*>(smem) + (size_t)wave * 2 * ks * 512;
+    const T* cache = reinterpret_cast<const T*>(p.cache);
+
+    frag q[KS];
+    {
+        const uint32_t head = ht * 16 + qi;
+        const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(head, d.heads - 1)) * p.ld + 8 * g;
+#pragma unroll
+        for (int s = 0; s < KS; s++)
+            if ((uint32_t)s < ks) q[s] = load_row8(src + 32 * s);
+    }
+    v4f O[NT];
+#pragma unroll
+    for (int i = 0; i < NT; i++) O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;
+
+    for (uint32_t ch = split; ch < n_chunks; ch += p.n_splits) {
+        const uint32_t key0 = ch * chunk + wave * 32;
+        if (key0 > pos) break;  // (only the last chunk can end before this wave's keys)
+        // rows past the newest position repeat it; their scores are masked
+        const T* r0 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + qi, pos)) * p.ld + 8 * g;
+        const T* r1 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + 16 + qi, pos)) * p.ld + 8 * g;
+        for (uint32_t s = 0; s < ks; s++) {
+            copy_row8_to_unit(r0 + 32 * s, lds + (size_t)s * 512);
+            copy_row8_to_unit(r1 + 32 * s, lds + (size_t)(ks + s) * 512);
+        }
+        wait_lds_copies();
+        v4f s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < KS; s++)
+            if ((uint32_t)s < ks) {
+                s0 = mfma32(load_unit(lds + (size_t)s * 512, lane), q[s], s0);
+                s1 = mfma32(load_unit(lds + (size_t)(ks + s) * 512, lane), q[s], s1);
+            }
+        float sv[8], mx = -INFINITY;
+#pragma unroll
+        for (int v = 0; v < 4; v++) {
+            const uint32_t k = key0 + 4 * g + v;
+            sv[v] = k <= pos ? s0[v] * d.scale : -INFINITY;
+            sv[4 + v] = k + 16 <= pos ? s1[v] * d.scale : -INFINITY;
+            mx = fmaxf(mx, fmaxf(sv[v], sv[4 + v]));
+        }
+        mx = max_rows4(mx);  // finite: key0 <= pos
+        const float m_new = fmaxf(m_run, mx), alpha = exp_of<T>(m_run - m_new);
+        float sum = 0.f;
+        frag hi, lo;
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const float pe = exp_of<T>(sv[e] - m_new);
+            sum += pe;
+            hi[e] = (T)pe;
+            if constexpr (!Dt<T>::is_f32) lo[e] = (T)(pe - (float)hi[e]);
+        }
+        l_run = l_run * alpha + sum_rows4(sum);
+        const bool moved = __any(m_new != m_run);
+        m_run = m_new;
+#pragma unroll
+        for (int i = 0; i < NT; i++)
+            if ((uint32_t)i < nt) {
+                const frag a = value_frag<T>(lds, ks, i, qi, g);
+                if (moved) O[i] *= alpha;
+                O[i] = mfma32(a, hi, O[i]);
+                if constexpr (!Dt<T>::is_f32) O[i] = mfma32(a, lo, O[i]);
+            }
+        // the LDS reads above are complete (their results are in use) before the next copies overwrite the rows
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    }
+
+    // the waves' results: common maximum, sums in wave order
+    if (g == 0) wave_ml[wave][qi][0] = m_run, wave_ml[wave][qi][1] = l_run;
+    __syncthreads();
+    float M = -INFINITY;
+    for (uint32_t w = 0; w < nw; w++) M = fmaxf(M, wave_ml[w][qi][0]);
+    const float f = m_run == -INFINITY ? 0.f : exp_of<T>(m_run - M);
+    float* mine = reinterpret_cast<float*>(smem) + (size_t)wave * 16 * d.rank_p;   // (every wave is done with its rows)
+#pragma unroll
+    for (int i = 0; i < NT; i++)
+        if ((uint32_t)i < nt) *reinterpret_cast<v4f*>(mine + qi * d.rank_p + 16 * i + 4 * g) = O[i] * f;
+    __syncthreads();
+    const size_t slot = ((size_t)m * gridDim.y + ht) * p.n_splits + split;
+    float* po = p.part_o + slot * 16 * d.rank_p;
+    const float* all = reinterpret_cast<const float*>(smem);
+    for (uint32_t i = tid * 4; i < 16 * d.rank_p; i += blockDim.x * 4) {
+        v4f y = *reinterpret_cast<const v4f*>(all + i);
+        for (uint32_t w = 1; w < nw; w++) y += *reinterpret_cast<const v4f*>(all + (size_t)w * 16 * d.rank_p + i);
+        *reinterpret_cast<v4f*>(po + i) = y;
+    }
+    if (tid < 16) {
+        float l = 0.f;
+        for (uint32_t w = 0; w < nw; w++) {
+            const float mw = wave_ml[w][tid][0];
+            if (mw != -INFINITY) l += wave_ml[w][tid][1] * exp_of<T>(mw - M);
+        }
+        p.part_ml[slot * 32 + tid * 2] = M;
+        p.part_ml[slot * 32 + tid * 2 + 1] = l;
+    }
+}
+
+// ---------------------------------------------------------------------------
+// Merge of one head's splits - the sink joins the denominator here, once - and the value product W_uv (sum p c).
+// Grid (head, token row), 4 waves.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void latent_merge_kernel(OxbLatentParams p, uint32_t chunk) {
+    typedef typename Dt<T>::frag frag;
+    extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+    __shared__ float wgt[OXB_LATENT_MAX_SPLITS];
+    const OxbLatentDims& d = p.d;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, c = lane & 15u, g = lane >> 4;
+    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+    const uint32_t head = blockIdx.x, m = blockIdx.y, ht = head / 16, col = head % 16, n_ht = (d.heads + 15) / 16;
+    const uint32_t used = min(p.n_splits, row_pos(p.rows, m) / chunk + 1);
+    const size_t slot0 = ((size_t)m * n_ht + ht) * p.n_splits;
+    const float sink = p.sink[head];
+    T* lat = reinterpret_cast<T*>(smem);  // [k_uv]
+    {
+        // every wave forms the weights (at most two splits per lane); wave 0 leaves them in LDS
+        float ms[2], ls[2], M = sink;
+#pragma unroll
+        for (int i = 0; i < 2; i++) {
+            const uint32_t s = lane + 64 * i;
+            ms[i] = s < used ? p.part_ml[(slot0 + s) * 32 + col * 2] : -INFINITY;
+            ls[i] = s < used ? p.part_ml[(slot0 + s) * 32 + col * 2 + 1] : 0.f;
+            M = fmaxf(M, ms[i]);
+        }
+        M = wave_max_f32(M);
+        float w[2], L = 0.f;
+#pragma unroll
+        for (int i = 0; i < 2; i++) {
+            w[i] = ms[i] == -INFINITY ? 0.f : exp_of<T>(ms[i] - M);
+            L += w[i] * ls[i];
+        }
+        L = wave_sum_f32(L) + exp_of<T>(sink - M);
+        if (wave == 0) {
+#pragma unroll
+            for (int i = 0; i < 2; i++)
+                if (lane + 64 * i < used) wgt[lane + 64 * i] = w[i] / L;
+        }
+    }
+    __syncthreads();
+    const float* po = p.part_o + (slot0 * 16 + col) * d.rank_p;
+    for (uint32_t i = tid; i < p.k_uv; i += 256) {
+        float y = 0.f;
+        if (i < d.rank_p)
+            for (uint32_t s = 0; s < used; s++) y = fmaf(wgt[s], po[(size_t)s * 16 * d.rank_p + i], y);
+        lat[i] = (T)y;
+    }
+    __syncthreads();
+    const uint32_t nu = p.k_uv / 32, tiles = d.vdim_p / 16;
+    T* out = reinterpret_cast<T*>(p.out) + (size_t)m * p.ld_out;
+    for (uint32_t t = wave; t < tiles; t += 4) {
+        const T* w = reinterpret_cast<const T*>(p.w_uv) + (size_t)(head * tiles + t) * nu * 512;
+        v4f acc = {0.f, 0.f, 0.f, 0.f};
+        for (uint32_t u = 0; u < nu; u++) {
+            const frag b = c == 0 ? load_row8(lat + 32 * u + 8 * g) : zero_frag((const T*)nullptr);
+            acc = mfma32(load_unit(w + (size_t)u * 512, lane), b, acc);
+        }
+        if (c == 0) {
+            typename Dt<T>::quad o;
+#pragma unroll
+            for (int i = 0; i < 4; i++) o[i] = (T)acc[i];
+            *reinterpret_cast<typename Dt<T>::quad*>(out + head * d.vdim_p + t * 16 + 4 * g) = o;
+        }
+    }
+    if (head == d.heads - 1)
+        for (uint32_t i = d.heads * d.vdim_p + tid; i < p.ld_out; i += 256) out[i] = (T)0.f;
+}
+
+// ---------------------------------------------------------------------------
+// Expanded attention: a wave owns 16 QT queries of one head, the four waves of a workgroup take consecutive query tiles
+// and share the keys and values of each 32-key block through LDS (two buffers if they fit; memory -> LDS copies of block
+// i + 1 run under block i).  Keys enter the score product in the order that leaves lane (query, g) with keys
+// 8 g .. 8 g + 7 of the block - row 4 a + v of key tile t is key 8 a + 4 t + v - which is exactly the k order in which
+// the transposed values are read, 16 bytes per lane.
+// ---------------------------------------------------------------------------
+template <typename T, int QT, int KS, int VT>
+__global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, uint32_t n_buf) {
+    typedef typename Dt<T>::frag frag;
+    extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+    const OxbLatentDims& d = p.d;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4;
+    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+    const uint32_t n_qb = (p.rows.m + 64 * QT - 1) / (64 * QT);
+    const uint32_t qb = n_qb - 1 - blockIdx.x / d.heads, head = blockIdx.x % d.heads;   // long (late) query blocks first
+    const uint32_t kd = d.dim_p / 32, kr = d.rot_p / 32, ks = kd + kr, vt = d.vdim_p / 16;
+    const uint32_t kl = d.rank_p + d.rot_p, qh = d.dim_p + d.rot_p, half = d.rot_dims >> 1;
+    const uint32_t units = 2 * ks + vt;
+    T* lds = reinterpret_cast<T*>(smem);
+    const T* cache = reinterpret_cast<const T*>(p.cache);
+    const uint32_t q_last = min((qb + 1) * 64 * QT, p.rows.m) - 1;
+    const uint32_t kv_len = p.rows.pos0 + q_last + 1;   // keys the workgroup's last query sees
+
+    // queries of this wave, rotated, in operand order; rows past the end repeat the last one and are not stored
+    frag q[QT][KS];
+    uint32_t qpos[QT];
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        const uint32_t row = min(qb * 64 * QT + (wave * QT + t) * 16 + qi, p.rows.m - 1);
+        qpos[t] = p.rows.pos0 + row;
+        const float* src = p.qkv + (size_t)row * p.ld_qkv + head * qh;
+        const float* cs = p.cos_t + (size_t)qpos[t] * half;
+        const float* sn = p.sin_t + (size_t)qpos[t] * half;
+#pragma unroll
+        for (int s = 0; s < KS; s++) {
+            if ((uint32_t)s >= ks) continue;
+            if ((uint32_t)s < kd) {
+                const v8f x = load_row8(src + 32 * s + 8 * g);
+#pragma unroll
+                for (int e = 0; e < 8; e++) q[t][s][e] = (T)x[e];
+            } else {
+                const float* rp = src + d.dim_p;
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const uint32_t i = 32 * (s - kd) + 8 * g + e;
+                    q[t][s][e] = (T)(i < d.rot ? rotated(rp, i, d.rot_dims, cs, sn) : 0.f);
+                }
+            }
+        }
+    }
+    v4f O[QT][VT];
+    float m_run[QT], l_run[QT];
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        m_run[t] = -INFINITY, l_run[t] = 0.f;
+#pragma unroll
+        for (int i = 0; i < VT; i++) O[t][i] = (v4f){0.f, 0.f, 0.f, 0.f};
+    }
+
+    // unit un of a block: key tile un / ks, k unit un % ks for the first 2 ks; value tile un - 2 ks behind them
+    auto stage = [&](uint32_t key0, uint32_t buf) {
+        T* base = lds + (size_t)buf * units * 512;
+        for (uint32_t un = wave; un < units; un += 4) {
+            const T* src;
+            if (un < 2 * ks) {
+                const uint32_t t = un >= ks ? 1u : 0u, s = un - t * ks;
+                const uint32_t key = min(key0 + 8 * (qi >> 2) + 4 * t + (qi & 3u), kv_len - 1);
+                src = s < kd ? reinterpret_cast<const T*>(p.k_exp) + (size_t)key * p.ld_k + head * d.dim_p + 32 * s + 8 * g
+                             : cache + kv_row(p.kv, p.rows.seq0, 0, 0, key) * kl + d.rank_p + 32 * (s - kd) + 8 * g;
+            } else {
+                src = reinterpret_cast<const T*>(p.v_exp_t) + (size_t)(head * d.vdim_p + (un - 2 * ks) * 16 + qi) * p.ld_v + key0 + 8 * g;
+            }
+            copy_row8_to_unit(src, base + (size_t)un * 512);
+        }
+    };
+    stage(0, 0);
+    uint32_t buf = 0;
+    for (uint32_t key0 = 0; key0 < kv_len; key0 += 32) {
+        wait_lds_copies();
+        __syncthreads();
+        if (n_buf > 1 && key0 + 32 < kv_len) stage(key0 + 32, buf ^ 1u);
+        const T* kb = lds + (size_t)buf * units * 512;
+        const T* vb = kb + (size_t)2 * ks * 512;
+        v4f s0[QT], s1[QT];
+#pragma unroll
+        for (int t = 0; t < QT; t++) s0[t] = s1[t] = (v4f){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < KS; s++)
+            if ((uint32_t)s < ks) {
+                const frag k0 = load_unit(kb + (size_t)s * 512, lane), k1 = load_unit(kb + (size_t)(ks + s) * 512, lane);
+#pragma unroll
+                for (int t = 0; t < QT; t++) {
+                    s0[t] = mfma32(k0, q[t][s], s0[t]);
+                    s1[t] = mfma32(k1, q[t][s], s1[t]);
+                }
+            }
+        frag hi[QT], lo[QT];
+        bool moved = false;
+        float alpha[QT];
+#pragma unroll
+        for (int t = 0; t < QT; t++) {
+            float sv[8], mx = -INFINITY;
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const float x = e < 4 ? s0[t][e & 3] : s1[t][e & 3];
+                sv[e] = key0 + 8 * g + e <= qpos[t] ? x * d.scale : -INFINITY;
+                mx = fmaxf(mx, sv[e]);
+            }
+            mx = max_rows4(mx);
+            const float m_new = fmaxf(m_run[t], mx);   // finite from the first block on: key 0 is visible to every query
+            alpha[t] = exp_of<T>(m_run[t] - m_new);
+            float sum = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const float pe = exp_of<T>(sv[e] - m_new);
+                sum += pe;
+                hi[t][e] = (T)pe;
+                if constexpr (!Dt<T>::is_f32) lo[t][e] = (T)(pe - (float)hi[t][e]);
+            }
+            l_run[t] = l_run[t] * alpha[t] + sum_rows4(sum);
+            moved |= m_new != m_run[t];
+            m_run[t] = m_new;
+        }
+        if (__any(moved)) {
+#pragma unroll
+            for (int t = 0; t < QT; t++)
+#pragma unroll
+                for (int i = 0; i < VT; i++) O[t][i] *= alpha[t];
+        }
+#pragma unroll
+        for (int i = 0; i < VT; i++)
+            if ((uint32_t)i < vt) {
+                const frag a = load_unit(vb + (size_t)i * 512, lane);
+#pragma unroll
+                for (int t = 0; t < QT; t++) {
+                    O[t][i] = mfma32(a, hi[t], O[t][i]);
+                    if constexpr (!Dt<T>::is_f32) O[t][i] = mfma32(a, lo[t], O[t][i]);
+                }
+            }
+        if (n_buf > 1) {
+            buf ^= 1u;
+        } else if (key0 + 32 < kv_len) {
+            __syncthreads();
+            stage(key0 + 32, 0);
+        }
+    }
+    const float sink = p.sink[head];
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+        const uint32_t row = qb * 64 * QT + (wave * QT + t) * 16 + qi;
+        if (row >= p.rows.m) continue;
+        const float M = fmaxf(m_run[t], sink), f = exp_of<T>(m_run[t] - M);
+        const float inv = f / (l_run[t] * f + exp_of<T>(sink - M));
+        T* o = reinterpret_cast<T*>(p.out) + (size_t)row * p.ld_out + head * d.vdim_p + 4 * g;
+#pragma unroll
+        for (int i = 0; i < VT; i++)
+            if ((uint32_t)i < vt) {
+                typename Dt<T>::quad w;
+#pragma unroll
+                for (int v = 0; v < 4; v++) w[v] = (T)(O[t][i][v] * inv);
+                *reinterpret_cast<typename Dt<T>::quad*>(o + 16 * i) = w;
+            }
+        if (head == d.heads - 1)
+            for (uint32_t i = d.heads * d.vdim_p + g; i < p.ld_out; i += 4) reinterpret_cast<T*>(p.out)[(size_t)row * p.ld_out + i] = (T)0.f;
+    }
+}
+
+// ---------------------------------------------------------------------------
+static constexpr uint32_t kLdsMax = 160u << 10, kLdsStatic = 1024;   // (decode keeps 512 B of statics beside the dynamic part)
+
+static uint32_t decode_waves(const OxbLatentDims& d, int dt) {
+    for (uint32_t nw = 4; nw; nw >>= 1)
+        if (nw * 32 * (d.rank_p + d.rot_p) * oxb_dt_bytes(dt) <= kLdsMax - kLdsStatic) return nw;
+    return 0;
+}
+static uint32_t prefill_block_bytes(const OxbLatentDims& d, int dt) {
+    return (2 * (d.dim_p + d.rot_p) / 32 + d.vdim_p / 16) * 512 * oxb_dt_bytes(dt);
+}
+uint32_t oxb_latent_chunk(const OxbLatentDims& d, int dt) { return 32 * decode_waves(d, dt); }
+
+const char* oxb_latent_check(const OxbLatentDims& d, int dt) {
+    if (!d.heads || !d.dim || !d.rot || !d.rank || !d.vdim) return "a latent attention size is 0";
+    if (d.rot_dims > d.rot || d.rot_dims % 2) return "rotated dimensions must be even and within the rotated part";
+    if (d.rank > 1024 || d.rot > 128) return "latent size beyond 1024 or rotated part beyond 128";
+    if (d.dim_p + d.rot_p > 512 || d.vdim > 512) return "head size beyond 512";
+    if (!decode_waves(d, dt)) return "a block of latent rows exceeds the LDS";
+    if (prefill_block_bytes(d, dt) > kLdsMax) return "a block of keys and values exceeds the LDS";
+    return nullptr;
+}
+
+static bool rows_ok(const OxbLatentParams& p) {
+    const OxbLatentDims& d = p.d;
+    return p.rows.m && p.cache && p.qkv && p.cos_t && p.sin_t && p.c_norm && p.sink && p.ld == d.rank_p + d.rot_p &&
+           p.ld_qkv >= d.heads * (d.dim_p + d.rot_p) + d.rank_p + d.rot_p && p.kv.n_layers == 1 && p.kv.nkv == 1 &&
+           (!p.kv.page_table || (p.kv.page_shift >= 4 && p.kv.page_shift <= 7));
+}
+
+hipError_t oxb_launch_latent_store(const OxbLatentParams& p, bool absorb, int dt, hipStream_t st) {
+    if (!rows_ok(p) || (absorb && (!p.q_abs || !p.w_uk_t || p.k_uk < p.d.dim_p || p.k_uk % 32))) return hipErrorInvalidValue;
+    OxbLatentParams q = p;
+    if (!absorb) q.q_abs = nullptr;
+    const uint32_t tph = p.d.rank_p / 16, n_abs = absorb ? (p.d.heads * tph + 3) / 4 : 0;
+    const dim3 grid(n_abs + 16, (p.rows.m + 15) / 16);
+    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_store_kernel<__bf16>), grid, dim3(256), 0, st, q, n_abs, tph);
+    else hipLaunchKernelGGL((latent_store_kernel<float>), grid, dim3(256), 0, st, q, n_abs, tph);
+    return hipGetLastError();
+}
+
+template <typename T, int NT, int KS>
+static hipError_t launch_decode(const OxbLatentParams& p, uint32_t nw, hipStream_t st) {
+    const uint32_t lds = nw * 32 * p.ld * sizeof(T);
+    hipLaunchKernelGGL((latent_decode_kernel<T, NT, KS>), dim3(p.n_splits, (p.d.heads + 15) / 16, p.rows.m), dim3(64 * nw), lds, st, p);
+    return hipGetLastError();
+}
+
+template <typename T>
+static hipError_t pick_decode(const OxbLatentParams& p, uint32_t nw, hipStream_t st) {
+    const uint32_t nt = p.d.rank_p / 16, ks = p.ld / 32;   // ks - nt / 2 = rot_p / 32 <= 4
+    if (nt <= 8 && ks <= 6) return launch_decode<T, 8, 6>(p, nw, st);
+    if (nt <= 16 && ks <= 12) return launch_decode<T, 16, 12>(p, nw, st);
+    if (nt <= 32 && ks <= 20) return launch_decode<T, 32, 20>(p, nw, st);
+    return launch_decode<T, 64, 36>(p, nw, st);
+}
+
+hipError_t oxb_launch_latent_decode(const OxbLatentParams& p, int dt, hipStream_t st) {
+    const uint32_t nw = decode_waves(p.d, dt);
+    if (!rows_ok(p) || oxb_latent_check(p.d, dt) || !p.q_abs || !p.part_o || !p.part_ml || !p.n_splits || p.n_splits > OXB_LATENT_MAX_SPLITS)
+        return hipErrorInvalidValue;
+    return dt == OXB_DT_BF16 ? pick_decode<__bf16>(p, nw, st) : pick_decode<float>(p, nw, st);
+}
+
+hipError_t oxb_launch_latent_merge(const OxbLatentParams& p, int dt, hipStream_t st) {
+    if (!rows_ok(p) || !p.part_o || !p.part_ml || !p.out || !p.w_uv || p.k_uv < p.d.rank_p || p.k_uv % 32 || p.ld_out < p.d.heads * p.d.vdim_p ||
+        !p.n_splits || p.n_splits > OXB_LATENT_MAX_SPLITS)
+        return hipErrorInvalidValue;
+    const dim3 grid(p.d.heads, p.rows.m);
+    const uint32_t lds = p.k_uv * oxb_dt_bytes(dt), chunk = oxb_latent_chunk(p.d, dt);
+    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_merge_kernel<__bf16>), grid, dim3(256), lds, st, p, chunk);
+    else hipLaunchKernelGGL((latent_merge_kernel<float>), grid, dim3(256), lds, st, p, chunk);
+    return hipGetLastError();
+}
+
+template <typename T, int QT, int KS, int VT>
+static hipError_t launch_prefill(const OxbLatentParams& p, uint32_t block_bytes, hipStream_t st) {
+    const uint32_t n_buf = 2 * block_bytes <= kLdsMax ? 2u : 1u, n_qb = (p.rows.m + 64 * QT - 1) / (64 * QT);
+    hipLaunchKernelGGL((latent_prefill_kernel<T, QT, KS, VT>), dim3(n_qb * p.d.heads), dim3(256), n_buf * block_bytes, st, p, n_buf);
+    return hipGetLastError();
+}
+
+template <typename T>
+static hipError_t pick_prefill(const OxbLatentParams& p, uint32_t bytes, hipStream_t st) {
+    const uint32_t ks = (p.d.dim_p + p.d.rot_p) / 32, vt = p.d.vdim_p / 16;
+    if (ks <= 4 && vt <= 8) return launch_prefill<T, 2, 4, 8>(p, bytes, st);
+    if (ks <= 6 && vt <= 8) return launch_prefill<T, 2, 6, 8>(p, bytes, st);
+    if (ks <= 8 && vt <= 16) return launch_prefill<T, 1, 8, 16>(p, bytes, st);
+    return launch_prefill<T, 1, 16, 32>(p, bytes, st);
+}
+
+// Dynamic LDS beyond 64 KB has to be asked for, per kernel; done ahead of any launch so that none has to do it inside a
+// stream capture.
+template <typename T>
+static hipError_t raise_lds() {
+    const void* decode[] = {(const void*)&latent_decode_kernel<T, 8, 6>, (const void*)&latent_decode_kernel<T, 16, 12>,
+                            (const void*)&latent_decode_kernel<T, 32, 20>, (const void*)&latent_decode_kernel<T, 64, 36>};
+    const void* prefill[] = {(const void*)&latent_prefill_kernel<T, 2, 4, 8>, (const void*)&latent_prefill_kernel<T, 2, 6, 8>,
+                             (const void*)&latent_prefill_kernel<T, 1, 8, 16>, (const void*)&latent_prefill_kernel<T, 1, 16, 32>};
+    hipError_t e = hipSuccess;
+    for (int i = 0; i < 4 && e == hipSuccess; i++) {
+        e = hipFuncSetAttribute(decode[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kLdsStatic));
+        if (e == hipSuccess) e = hipFuncSetAttribute(prefill[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLdsMax);
+    }
+    return e;
+}
+hipError_t oxb_latent_prepare(int dt) { return dt == OXB_DT_BF16 ? raise_lds<__bf16>() : raise_lds<float>(); }
+
+hipError_t oxb_launch_latent_prefill(const OxbLatentParams& p, int dt, hipStream_t st) {
+    if (!rows_ok(p) || oxb_latent_check(p.d, dt) || p.rows.pos || p.rows.seq_step || !p.k_exp || !p.v_exp_t || !p.out ||
+        p.ld_k < p.d.heads * p.d.dim_p || p.ld_v % 32 || p.ld_v < p.rows.pos0 + p.rows.m || p.ld_out < p.d.heads * p.d.vdim_p)
+        return hipErrorInvalidValue;
+    const uint32_t bytes = prefill_block_bytes(p.d, dt);
+    return dt == OXB_DT_BF16 ? pick_prefill<__bf16>(p, bytes, st) : pick_prefill<float>(p, bytes, st);
+}

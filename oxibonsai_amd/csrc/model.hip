@@ -13,6 +13,8 @@
 #include <hip/hip_runtime.h>
 #include <hip/hip_fp16.h>
 
+#include <sys/stat.h>
+
 #include <cmath>
 #include <cstdlib>
 #include <cstring>
@@ -26,73 +28,26 @@
 #include "gemv_kernels.h"
 #include "kv_quant_device.h"
 #include "layer_kernels.h"
+#include "model_internal.h"
 #include "prefill_kernels.h"
+#include "program.h"
 #include "runtime_internal.h"
 #include "token_kernels.h"
 
 namespace oxb {
 
-struct Model {
-    oxb_model_desc d;
-    std::vector<oxb_layer_ids> layers;
-    // activations
-    float *hidden = nullptr, *qkv = nullptr, *attn_part = nullptr, *attn_out = nullptr,
-          *gu = nullptr, *act = nullptr, *logits = nullptr;  // gu: [batch][2 inter] gate || up sums, act: [batch][inter] SwiGLU output
-    uint32_t *tokens = nullptr, *pos = nullptr;
-    // pinned host staging of a decode call's small transfers (embedding rows and positions in, tokens out): copies from
-    // and to pageable memory go through the runtime's own staging and cost about 10 us per call more
-    float* h_hidden = nullptr;
-    uint32_t *h_pos = nullptr, *h_tokens = nullptr;
-    uint32_t* attn_done = nullptr;  // [batch][nkv] arrival counters of the attention workgroups, 0 between launches
-    void* argmax_ws = nullptr;
-    // KV cache: rows of hd fp16 values or one-byte codes, a quantised cache also one f32 scale per row.  Contiguous:
-    // [batch][n_layers][nkv][row_stride] rows; paged: a pool [n_pages][n_layers][nkv][2^page_shift] rows and, per
-    // sequence, a table of page numbers (kv_quant_device.h: OxbKvLayout)
-    void *k_cache = nullptr, *v_cache = nullptr;
-    float *k_scale = nullptr, *v_scale = nullptr;
-    uint32_t kv_mode = OXB_KV_F16, row_stride = 0, window = 0, sinks = 0;
-    uint32_t page_shift = 0, n_pages = 0, table_stride = 0;   // n_pages 0: contiguous
-    std::vector<uint32_t> free_pages;                          // stack of free physical pages
-    std::vector<std::vector<uint32_t>> seq_pages;              // pages of each sequence slot, in position order
-    std::vector<uint32_t> h_table;                             // [batch][table_stride], mirrored in d_table
-    uint32_t* d_table = nullptr;
-    bool table_dirty = false;
-    float *cos_t = nullptr, *sin_t = nullptr;
-    uint32_t chunk = 0, n_splits = 0;
-    // graph
-    hipGraphExec_t graph_exec = nullptr;
-    uint64_t checked_gen = 0;  // g_rt.weights_gen when every handle was last looked up
-    uint64_t graph_gen = 0;  // g_rt.weights_gen at capture: the graph holds the weights' device pointers of that moment
-    bool graph_failed = false;
-    bool want_logits_in_graph = true;
-    size_t logits_cap = 0;  // floats m.logits holds
-    std::vector<void*> allocs;
-    // prefill activations for up to pf_cap token rows (allocated on first use)
-    uint32_t pf_cap = 0;
-    float *pf_hidden = nullptr, *pf_qkv = nullptr, *pf_attn = nullptr, *pf_gu = nullptr;
-    std::vector<void*> pf_allocs;
-    GemmWorkspace gws;  // GEMM scratch of the captured large-batch decode step: sized at creation, never moved
-    DevBuf gpack;       // quantised activation vectors of the captured GEMV-based step (batches of two to eight): likewise
-    DevBuf gpack_o;     // the O projection's quantised input where the attention kernel writes it itself; starts as zeros (= zero vectors) and
-                        // nothing else writes it, so the slots of a last vector group's absent vectors stay zero vectors
-    // a model loaded from a file owns the weights it uploaded
-    std::vector<uint64_t> owned_mats, owned_vecs;
-    DevBuf tok_hist, tok_ids;  // token history of the on-device generation loop; prompt ids of a token prefill
-    DevBuf sample_ws, rng;     // sampler scratch and per-sequence xorshift64 states
-};
-
-struct Embedding {  // token embedding table in its stored form
-    void* d = nullptr;
-    int type = 0;   // GGUF tensor type id: 0 F32, 1 F16, 41 Q1_0_g128, 42 TQ2_0_g128
-    uint32_t vocab = 0, h = 0;
-    size_t bytes = 0;
-};
 static std::unordered_map<uint64_t, Embedding> g_embeddings;
 
 static std::unordered_map<uint64_t, std::unique_ptr<Model>> g_models;
 static uint64_t g_next_model = 1;
 
-static int dev_alloc(Model& m, void** p, size_t bytes) {
+uint64_t add_model(std::unique_ptr<Model> m) {
+    const uint64_t id = g_next_model++;
+    g_models[id] = std::move(m);
+    return id;
+}
+
+int dev_alloc(Model& m, void** p, size_t bytes) {
     hipError_t e = hipMalloc(p, bytes ? bytes : 16);
     if (e != hipSuccess)
         return fail(OXB_HIP_OUT_OF_MEMORY, "out of device memory: requested %zu bytes on device %d", bytes, g_rt.device);
@@ -114,7 +69,7 @@ static void free_kv_cache(Model& m) {
     m.table_dirty = false;
 }
 
-static void free_model(Model& m) {
+void free_model(Model& m) {
     if (m.graph_exec) (void)hipGraphExecDestroy(m.graph_exec);
     m.graph_exec = nullptr;
     if (m.h_hidden) (void)hipHostFree(m.h_hidden);
@@ -134,6 +89,8 @@ static void free_model(Model& m) {
     m.tok_ids.release();
     m.sample_ws.release();
     m.rng.release();
+    m.want_rows.release();
+    if (m.prog) program_release(*m.prog);
 }
 
 void shutdown_models() {
@@ -143,7 +100,7 @@ void shutdown_models() {
     g_embeddings.clear();
 }
 
-static const float* vec_ptr(uint64_t id, uint32_t n, const char* what, int* rc) {
+const float* vec_ptr(uint64_t id, uint32_t n, const char* what, int* rc) {
     auto it = g_rt.vectors.find(id);
     if (it == g_rt.vectors.end()) {
         *rc = fail(OXB_HIP_WEIGHT_NOT_FOUND, "weight handle %llu (%s) not found", (unsigned long long)id, what);
@@ -172,17 +129,6 @@ static const Weight* mat_ptr(uint64_t id, int fmt, uint32_t n_rows, uint32_t k, 
     }
     return w;
 }
-
-#define OXB_TRY_HIP(expr, what)                               \
-    do {                                                      \
-        hipError_t e_ = (expr);                               \
-        if (e_ != hipSuccess) return hip_fail(e_, what);      \
-    } while (0)
-#define OXB_TRY(expr)            \
-    do {                         \
-        int rc_ = (expr);        \
-        if (rc_) return rc_;     \
-    } while (0)
 
 // nb activation vectors through one projection.  From gemv_packed_min_batch(K) vectors on they are quantised by a launch
 // of their own into `pack` (sized by the caller: this runs inside stream captures) and up to eight share the pass.
@@ -228,6 +174,11 @@ static uint32_t decode_chunk(uint32_t batch) { return batch <= OXB_GEMV_PACKED_M
 // without one).  Run at creation and again whenever a weight or vector was replaced or freed since, before a decode
 // step is captured: inside the capture nothing may allocate.
 static int check_model_handles(Model& m) {
+    if (m.prog) {
+        OXB_TRY(program_check_handles(m));
+        m.checked_gen = g_rt.weights_gen;
+        return OXB_HIP_OK;
+    }
     const oxb_model_desc& d = m.d;
     const uint32_t qd = d.nq * d.hd, kd = d.nkv * d.hd, qkv_rows = qd + 2 * kd;
     int rc = OXB_HIP_OK;
@@ -291,7 +242,7 @@ static int size_gemm_workspaces(Model& m) {
     return OXB_HIP_OK;
 }
 
-static OxbKvLayout kv_layout(const Model& m) {
+OxbKvLayout kv_layout(const Model& m) {
     OxbKvLayout L;
     L.page_table = m.n_pages ? m.d_table : nullptr;
     L.page_shift = m.page_shift;
@@ -418,6 +369,7 @@ static int encode_decode_step_gemm(Model& m) {
 
 // Every kernel of one decode step, for all sequences of the batch (no host synchronisation).
 static int encode_decode_step(Model& m, bool with_lm_head) {
+    if (m.prog) return program_decode_step(m);
     if (m.d.batch >= OXB_DECODE_GEMM_MIN_BATCH && with_lm_head) return encode_decode_step_gemm(m);
     const oxb_model_desc& d = m.d;
     hipStream_t st = g_rt.stream;
@@ -469,7 +421,8 @@ static int encode_decode_step(Model& m, bool with_lm_head) {
 }
 
 // Prefill buffers for `rows` token rows.
-static int ensure_prefill_buffers(Model& m, uint32_t rows) {
+static int ensure_prefill_buffers(Model& m, uint32_t rows, uint32_t pos_start) {
+    if (m.prog) return program_prefill_buffers(m, rows, pos_start);
     if (rows <= m.pf_cap) return OXB_HIP_OK;
     (void)hipStreamSynchronize(g_rt.stream);
     for (void* p : m.pf_allocs) (void)hipFree(p);
@@ -493,8 +446,24 @@ static int ensure_prefill_buffers(Model& m, uint32_t rows) {
 
 // All layers for M token rows of sequence `seq` at positions pos_start .. pos_start + M - 1: batched
 // projections on the matrix cores (RMSNorm and SwiGLU fused into the fp16 packer of the GEMM that consumes them), one causal attention launch per layer, KV written to the cache; then the
-// LM head and the greedy token for the last row.
-static int encode_prefill(Model& m, uint32_t seq, uint32_t M, uint32_t pos_start) {
+// LM head and the greedy token for the last row; with `want` instead the logits of those rows of the portion, each copied
+// to the host behind its product.
+static int encode_prefill(Model& m, uint32_t seq, uint32_t M, uint32_t pos_start, const uint32_t* want = nullptr, uint32_t n_want = 1,
+                          float* want_logits = nullptr) {
+    if (m.prog) {
+        float* dst = m.logits + (size_t)seq * m.d.vocab;
+        if (want) {
+            OXB_TRY(m.sample_ws.ensure((size_t)n_want * m.d.vocab * 4));
+            dst = (float*)m.sample_ws.ptr;
+        }
+        OXB_TRY(program_prefill(m, seq, M, pos_start, want, n_want, dst));
+        if (want) {
+            if (n_want) OXB_TRY_HIP(hipMemcpyAsync(want_logits, dst, (size_t)n_want * m.d.vocab * 4, hipMemcpyDeviceToHost, g_rt.stream), "logits download");
+            return OXB_HIP_OK;
+        }
+        OXB_TRY_HIP(oxb_launch_argmax(dst, m.d.vocab, 1, m.tokens + seq, m.argmax_ws, g_rt.stream), "kernel launch failed: argmax");
+        return OXB_HIP_OK;
+    }
     const oxb_model_desc& d = m.d;
     hipStream_t st = g_rt.stream;
     const uint32_t qd = d.nq * d.hd, kd = d.nkv * d.hd, qkv_rows = qd + 2 * kd;
@@ -573,6 +542,16 @@ static int encode_prefill(Model& m, uint32_t seq, uint32_t M, uint32_t pos_start
     const Weight* lm = mat_ptr(d.lm_head, d.fmt, d.vocab, d.h, "lm_head", &rc);
     if (rc) return rc;
     float* last = m.hidden + (size_t)seq * d.h;
+    if (want) {
+        for (uint32_t i = 0; i < n_want; i++) {
+            OXB_TRY_HIP(hipMemcpyAsync(last, m.pf_hidden + (size_t)want[i] * d.h, (size_t)d.h * 4, hipMemcpyDeviceToDevice, st), "row copy");
+            OXB_TRY(gemv_launch(*lm, last, d.h, 1, m.logits + (size_t)seq * d.vocab, d.vocab, OXB_GEMV_PRO_RMSNORM, final_norm, d.eps,
+                                OXB_GEMV_STORE, nullptr));
+            OXB_TRY_HIP(hipMemcpyAsync(want_logits + (size_t)i * d.vocab, m.logits + (size_t)seq * d.vocab, (size_t)d.vocab * 4, hipMemcpyDeviceToHost, st),
+                        "logits download");
+        }
+        return OXB_HIP_OK;
+    }
     OXB_TRY_HIP(hipMemcpyAsync(last, m.pf_hidden + (size_t)(M - 1) * d.h, (size_t)d.h * 4, hipMemcpyDeviceToDevice, st), "last row copy");
     OXB_TRY(gemv_launch(*lm, last, d.h, 1, m.logits + (size_t)seq * d.vocab, d.vocab, OXB_GEMV_PRO_RMSNORM, final_norm, d.eps,
                         OXB_GEMV_STORE, nullptr));
@@ -660,15 +639,18 @@ static int alloc_kv_cache(Model& m, uint32_t kv_mode, uint32_t page_size, uint32
     const oxb_model_desc& d = m.d;
     free_kv_cache(m);
     m.row_stride = (d.max_seq + OXB_ATTN_CHUNK_POSITIONS - 1) / OXB_ATTN_CHUNK_POSITIONS * OXB_ATTN_CHUNK_POSITIONS;
-    const size_t rows = n_pages ? (size_t)n_pages * d.n_layers * d.nkv * page_size : (size_t)d.batch * d.n_layers * d.nkv * m.row_stride;
-    const size_t bytes = rows * d.hd * (kv_mode == OXB_KV_F16 ? 2 : 1);
+    // a layer program keeps latent rows, one region per layer run (program.hip), in k_cache alone
+    const size_t rows = m.prog ? (n_pages ? (size_t)n_pages * page_size : (size_t)d.batch * m.row_stride)
+                               : (n_pages ? (size_t)n_pages * d.n_layers * d.nkv * page_size : (size_t)d.batch * d.n_layers * d.nkv * m.row_stride);
+    const size_t bytes = m.prog ? rows * program_cache_row_bytes(*m.prog) : rows * d.hd * (kv_mode == OXB_KV_F16 ? 2 : 1);
     auto grab = [&](void** p, size_t n) -> int {
         if (hipMalloc(p, n ? n : 16) == hipSuccess) return OXB_HIP_OK;
         *p = nullptr;
         return fail(OXB_HIP_OUT_OF_MEMORY, "out of device memory: requested %zu bytes of KV cache on device %d", n, g_rt.device);
     };
     OXB_TRY(grab(&m.k_cache, bytes));
-    OXB_TRY(grab(&m.v_cache, bytes));
+    if (m.prog) OXB_TRY_HIP(hipMemset(m.k_cache, 0, bytes), "cache clear");   // rows are written whole; nothing unwritten may be a NaN
+    else OXB_TRY(grab(&m.v_cache, bytes));
     if (kv_mode != OXB_KV_F16) {
         const size_t sb = rows * sizeof(float);
         OXB_TRY(grab((void**)&m.k_scale, sb));
@@ -692,6 +674,12 @@ static int alloc_kv_cache(Model& m, uint32_t kv_mode, uint32_t page_size, uint32
     m.kv_mode = kv_mode;
     return OXB_HIP_OK;
 }
+
+}  // extern "C"
+
+int oxb::model_alloc_cache(Model& m, uint32_t page_size, uint32_t n_pages) { return alloc_kv_cache(m, OXB_KV_F16, page_size, n_pages); }
+
+extern "C" {
 
 int oxb_hip_model_create(const oxb_model_desc* desc, uint64_t* model) {
     OXB_API_BEGIN
@@ -776,8 +764,7 @@ int oxb_hip_model_create(const oxb_model_desc* desc, uint64_t* model) {
     m.logits_cap = B * (d.lm_head ? d.vocab : 1);
     const char* no_graph = getenv("OXB_HIP_DISABLE_GRAPH");
     m.graph_failed = no_graph && no_graph[0] == '1';
-    *model = g_next_model++;
-    g_models[*model] = std::move(mp);
+    *model = add_model(std::move(mp));
     return OXB_HIP_OK;
     OXB_API_END
 }
@@ -805,6 +792,8 @@ int oxb_hip_model_set_attention(uint64_t model, const oxb_attention_options* opt
     if (!opt) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null pointer");
     if (opt->kv_dtype != OXB_KV_DTYPE_F16 && opt->kv_dtype != OXB_KV_DTYPE_I8 && opt->kv_dtype != OXB_KV_DTYPE_FP8_E4M3)
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: unknown KV cache type %d", opt->kv_dtype);
+    if (m->prog && (opt->kv_dtype != OXB_KV_DTYPE_F16 || opt->window_size))
+        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: a latent cache keeps its rows in the model's own type and has no window (paging is available)");
     OXB_TRY_HIP(hipStreamSynchronize(g_rt.stream), "synchronize");
     // the captured decode step holds the cache pointers and the options: it is captured again on the next step
     if (m->graph_exec) (void)hipGraphExecDestroy(m->graph_exec);
@@ -821,7 +810,7 @@ int oxb_hip_model_set_attention(uint64_t model, const oxb_attention_options* opt
             return rc;
         }
     }
-    m->n_splits = attn_slots(*m, m->kv_mode);
+    if (!m->prog) m->n_splits = attn_slots(*m, m->kv_mode);
     m->window = opt->window_size;
     m->sinks = opt->sink_tokens;
     return OXB_HIP_OK;
@@ -850,6 +839,7 @@ int oxb_hip_model_read_kv(uint64_t model, uint32_t seq, uint32_t layer, uint32_t
     Model* m = find_model(model);
     if (!m) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: unknown model %llu", (unsigned long long)model);
     const oxb_model_desc& d = m->d;
+    if (m->prog) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the rows of a latent cache are not key / value rows");
     if (seq >= d.batch || layer >= d.n_layers || kv_head >= d.nkv || (uint64_t)pos + n_pos > d.max_seq)
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: cache rows (sequence %u, layer %u, head %u, positions %u..%llu) out of range",
                     seq, layer, kv_head, pos, (unsigned long long)pos + n_pos);
@@ -1094,6 +1084,7 @@ int oxb_hip_model_set_lm_head(uint64_t model, uint64_t final_norm, uint64_t lm_h
     Model* mp = find_model(model);
     if (!mp) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: unknown model %llu", (unsigned long long)model);
     Model& m = *mp;
+    if (m.prog) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the head of a configured design is part of it");
     if (lm_head && (!final_norm || !vocab))
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: an LM head needs the final norm vector and a vocabulary size");
     int rc = OXB_HIP_OK;
@@ -1136,6 +1127,7 @@ int oxb_hip_decode_hidden(uint64_t model, const float* hidden, const uint32_t* p
     for (uint32_t b = 0; b < d.batch; b++)
         if (pos[b] >= d.max_seq)
             return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: position %u exceeds the context of %u", pos[b], d.max_seq);
+    if (m.prog) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: a configured design ends in its own head (oxb_hip_decode returns its logits)");
     // the normed rows go through the gate || up buffer (free once the last layer is done): 2 * inter values per
     // sequence.  Checked, like every argument, before the step touches the cache.
     if ((size_t)2 * d.inter < d.h) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: hidden %u exceeds 2 x intermediate %u", d.h, d.inter);
@@ -1166,6 +1158,7 @@ int oxb_hip_model_set_rope_rows(uint64_t model, uint32_t pos_start, uint32_t n_p
     Model* mp = find_model(model);
     if (!mp) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: unknown model %llu", (unsigned long long)model);
     Model& m = *mp;
+    if (m.prog) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: a configured design forms its own rotation tables");
     if (!cos_rows || !sin_rows || n_pos == 0) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null table or no positions");
     if ((uint64_t)pos_start + n_pos > m.d.max_seq)
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: positions %u..%llu exceed the context of %u", pos_start,
@@ -1199,7 +1192,7 @@ int oxb_hip_prefill(uint64_t model, uint32_t seq, const float* hidden, uint32_t 
                     (unsigned long long)pos_start + n_tokens - 1, d.max_seq);
     OXB_TRY(kv_reserve(m, seq, (uint64_t)pos_start + n_tokens));
     OXB_TRY(kv_sync_table(m));
-    OXB_TRY(ensure_prefill_buffers(m, n_tokens));
+    OXB_TRY(ensure_prefill_buffers(m, n_tokens, pos_start));
     hipStream_t st = g_rt.stream;
     OXB_TRY_HIP(hipMemcpyAsync(m.pf_hidden, hidden, (size_t)n_tokens * d.h * 4, hipMemcpyHostToDevice, st), "hidden upload");
     OXB_TRY(encode_prefill(m, seq, n_tokens, pos_start));
@@ -1290,8 +1283,8 @@ int oxb_hip_upload_embedding(uint64_t* id, const void* table, size_t n_bytes, in
     OXB_API_BEGIN
     std::lock_guard<std::recursive_mutex> lk(g_mu);
     if (!id || !table) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null id or table");
-    if (gguf_type != GGUF_F32 && gguf_type != GGUF_F16 && gguf_type != GGUF_Q1_0_G128 && gguf_type != GGUF_TQ2_0_G128)
-        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: embedding tensor type %d (supported: 0 F32, 1 F16, 41, 42)", gguf_type);
+    if (gguf_type != GGUF_F32 && gguf_type != GGUF_F16 && gguf_type != GGUF_BF16 && gguf_type != GGUF_Q1_0_G128 && gguf_type != GGUF_TQ2_0_G128)
+        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: embedding tensor type %d (supported: 0 F32, 1 F16, 30 BF16, 41, 42)", gguf_type);
     if (vocab == 0 || h == 0 || (gguf_type >= 41 && h % 128))
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: embedding of %u rows x %u values", vocab, h);
     const size_t need = (size_t)gguf_tensor_bytes((uint32_t)gguf_type, (uint64_t)vocab * h);
@@ -1506,7 +1499,7 @@ int oxb_hip_prefill_tokens(uint64_t model, uint64_t embedding, uint32_t seq, con
     OXB_TRY(check_ids(*e, ids, n_tokens));
     OXB_TRY(kv_reserve(m, seq, (uint64_t)pos_start + n_tokens));
     OXB_TRY(kv_sync_table(m));
-    OXB_TRY(ensure_prefill_buffers(m, n_tokens));
+    OXB_TRY(ensure_prefill_buffers(m, n_tokens, pos_start));
     OXB_TRY(m.tok_ids.ensure((size_t)n_tokens * 4));
     hipStream_t st = g_rt.stream;
     OXB_TRY_HIP(hipMemcpyAsync(m.tok_ids.ptr, ids, (size_t)n_tokens * 4, hipMemcpyHostToDevice, st), "token id upload");
@@ -1768,6 +1761,146 @@ int oxb_hip_load_gguf(const char* path, uint32_t max_seq, uint32_t batch, uint64
     *model = mid;
     *embedding = emb_id;
     return OXB_HIP_OK;
+    OXB_API_END
+}
+
+int oxb_hip_forward_tokens(uint64_t model, uint64_t embedding, uint32_t seq, const uint32_t* ids, uint32_t n_tokens,
+                           uint32_t pos_start, const uint32_t* want, uint32_t n_want, float* logits) {
+    OXB_API_BEGIN
+    std::lock_guard<std::recursive_mutex> lk(g_mu);
+    Model* mp;
+    Embedding* e;
+    OXB_TRY(model_and_embedding(model, embedding, &mp, &e));
+    Model& m = *mp;
+    const oxb_model_desc& d = m.d;
+    if (!ids || n_tokens == 0) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null ids or no tokens");
+    if (n_want && (!want || !logits)) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null rows or logits");
+    if (!d.lm_head) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the model has no LM head");
+    for (uint32_t i = 0; i < n_want; i++)
+        if (want[i] >= n_tokens) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: logits of token %u of a portion of %u", want[i], n_tokens);
+    if (seq >= d.batch) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: sequence %u of a batch of %u", seq, d.batch);
+    if ((uint64_t)pos_start + n_tokens > d.max_seq)
+        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: positions %u..%llu exceed the context of %u", pos_start,
+                    (unsigned long long)pos_start + n_tokens - 1, d.max_seq);
+    if (m.checked_gen != g_rt.weights_gen) OXB_TRY(check_model_handles(m));
+    OXB_TRY(check_ids(*e, ids, n_tokens));
+    OXB_TRY(kv_reserve(m, seq, (uint64_t)pos_start + n_tokens));
+    OXB_TRY(kv_sync_table(m));
+    hipStream_t st = g_rt.stream;
+    if (n_tokens == 1 && d.batch == 1) {   // a decode step, the one the token loops replay
+        OXB_TRY_HIP(hipMemcpyAsync(m.tokens, ids, 4, hipMemcpyHostToDevice, st), "token upload");
+        OXB_TRY_HIP(hipMemcpyAsync(m.pos, &pos_start, 4, hipMemcpyHostToDevice, st), "position upload");
+        OXB_TRY_HIP(oxb_launch_embedding_gather(e->d, e->type, e->vocab, d.h, m.tokens, 1, m.hidden, st), "kernel launch failed: embedding_gather");
+        OXB_TRY(run_decode_step(m));
+        for (uint32_t i = 0; i < n_want; i++)
+            OXB_TRY_HIP(hipMemcpyAsync(logits + (size_t)i * d.vocab, m.logits, (size_t)d.vocab * 4, hipMemcpyDeviceToHost, st), "logits download");
+    } else {
+        OXB_TRY(ensure_prefill_buffers(m, n_tokens, pos_start));
+        OXB_TRY(m.tok_ids.ensure((size_t)n_tokens * 4));
+        OXB_TRY_HIP(hipMemcpyAsync(m.tok_ids.ptr, ids, (size_t)n_tokens * 4, hipMemcpyHostToDevice, st), "token id upload");
+        OXB_TRY_HIP(oxb_launch_embedding_gather(e->d, e->type, e->vocab, d.h, (const uint32_t*)m.tok_ids.ptr, n_tokens, m.pf_hidden, st),
+                    "kernel launch failed: embedding_gather");
+        static const uint32_t none = 0;
+        OXB_TRY(encode_prefill(m, seq, n_tokens, pos_start, want ? want : &none, n_want, logits));
+    }
+    hipError_t he = hipStreamSynchronize(st);
+    if (he != hipSuccess) return fail(OXB_HIP_SYNC_FAILED, "device synchronization failed: forward_tokens: %s", hipGetErrorString(he));
+    return OXB_HIP_OK;
+    OXB_API_END
+}
+
+// --- checkpoints of any kind this tier reads: a GGUF file, or a folder with config.json and model.safetensors ---------
+static bool is_dir(const char* path) {
+    struct stat sb;
+    return stat(path, &sb) == 0 && S_ISDIR(sb.st_mode);
+}
+
+static int read_design_dir(const std::string& dir, DesignConfig* c) {
+    std::string text, err;
+    if (!read_text_file(dir + "/config.json", &text, &err) || !read_design(text, c, &err))
+        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: %s", err.c_str());
+    return OXB_HIP_OK;
+}
+
+static void describe_design(const DesignConfig& c, oxb_checkpoint_info* info) {
+    memset(info, 0, sizeof *info);
+    snprintf(info->architecture, sizeof info->architecture, "%s", c.architecture.c_str());
+    info->n_layers = (uint32_t)c.layers.size();
+    info->n_runs = (uint32_t)layer_runs(c).size();
+    info->h = c.width;
+    info->vocab = c.vocab;
+}
+
+static void describe_gguf(const oxb_gguf_info& g, oxb_checkpoint_info* info) {
+    memset(info, 0, sizeof *info);
+    snprintf(info->architecture, sizeof info->architecture, "%s", g.architecture);
+    info->n_layers = info->n_runs = g.n_layers;
+    info->h = g.h;
+    info->vocab = g.vocab;
+    info->context_length = g.context_length;
+    info->is_gguf = 1;
+}
+
+int oxb_hip_checkpoint_info(const char* path, oxb_checkpoint_info* info) {
+    OXB_API_BEGIN
+    if (!path || !info) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null path or info");
+    if (is_dir(path)) {
+        DesignConfig c;
+        OXB_TRY(read_design_dir(path, &c));
+        describe_design(c, info);
+        return OXB_HIP_OK;
+    }
+    oxb_gguf_info g;
+    OXB_TRY(oxb_hip_gguf_info(path, &g));
+    describe_gguf(g, info);
+    return OXB_HIP_OK;
+    OXB_API_END
+}
+
+int oxb_hip_load_checkpoint(const char* path, int compute_type, uint32_t max_seq, uint32_t batch, uint64_t* model, uint64_t* embedding,
+                            oxb_checkpoint_info* info_or_null) {
+    OXB_API_BEGIN
+    std::lock_guard<std::recursive_mutex> lk(g_mu);
+    if (!path || !model || !embedding) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null path, model or embedding pointer");
+    if (!is_dir(path)) {
+        oxb_gguf_info g;
+        if (compute_type != OXB_COMPUTE_BF16)
+            return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: a GGUF checkpoint runs in its own format (compute type %d)", compute_type);
+        OXB_TRY(oxb_hip_load_gguf(path, max_seq, batch, model, embedding, &g));
+        if (info_or_null) describe_gguf(g, info_or_null);
+        return OXB_HIP_OK;
+    }
+    DesignConfig c;
+    OXB_TRY(read_design_dir(path, &c));
+    SafetensorsFile f;
+    std::string err;
+    if (!f.open((std::string(path) + "/model.safetensors").c_str(), &err)) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: safetensors: %s", err.c_str());
+    OXB_TRY(program_create(c, f.tensors, compute_type, max_seq, batch, model, embedding));
+    if (info_or_null) describe_design(c, info_or_null);
+    return OXB_HIP_OK;
+    OXB_API_END
+}
+
+int oxb_hip_model_from_tensors(const char* config_json, const oxb_tensor* tensors, uint32_t n_tensors, int compute_type, uint32_t max_seq,
+                               uint32_t batch, uint64_t* model, uint64_t* embedding) {
+    OXB_API_BEGIN
+    std::lock_guard<std::recursive_mutex> lk(g_mu);
+    if (!config_json || (n_tensors && !tensors) || !model || !embedding) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: null pointer");
+    DesignConfig c;
+    std::string err;
+    if (!read_design(config_json, &c, &err)) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: %s", err.c_str());
+    TensorMap map;
+    for (uint32_t i = 0; i < n_tensors; i++) {
+        const oxb_tensor& t = tensors[i];
+        if (!t.name || !t.data || t.n_dims > 4) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: tensor %u has no name or data, or too many dimensions", i);
+        TensorView v;
+        v.type = t.type;
+        v.shape.assign(t.shape, t.shape + t.n_dims);
+        v.data = static_cast<const uint8_t*>(t.data);
+        v.bytes = t.n_bytes;
+        map[t.name] = std::move(v);
+    }
+    return program_create(c, map, compute_type, max_seq, batch, model, embedding);
     OXB_API_END
 }
 

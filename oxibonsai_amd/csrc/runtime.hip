@@ -404,6 +404,8 @@ void oxb_hip_shutdown(void) {
     g_rt.weights.clear();
     for (auto& kv : g_rt.vectors) (void)hipFree(kv.second.d);
     g_rt.vectors.clear();
+    for (auto& kv : g_rt.dense) (void)hipFree(kv.second.d);
+    g_rt.dense.clear();
     g_rt.ws_x.release();
     g_rt.ws_y.release();
     g_rt.ws_aux.release();
@@ -481,6 +483,14 @@ int oxb_hip_upload_tq2_raw(uint64_t* id, const uint8_t* aos, size_t n_bytes) {
 int oxb_hip_free_weight(uint64_t id) {
     OXB_API_BEGIN
     std::lock_guard<std::recursive_mutex> lk(g_mu);
+    auto dense = g_rt.dense.find(id);
+    if (dense != g_rt.dense.end()) {
+        if (g_rt.ready) (void)hipStreamSynchronize(g_rt.stream);
+        (void)hipFree(dense->second.d);
+        g_rt.dense.erase(dense);
+        g_rt.weights_gen++;
+        return OXB_HIP_OK;
+    }
     Weight* w = find_weight(id);
     if (!w) return fail(OXB_HIP_WEIGHT_NOT_FOUND, "weight handle %llu not found", (unsigned long long)id);
     if (g_rt.ready) (void)hipStreamSynchronize(g_rt.stream);

@@ -46,6 +46,13 @@ struct Vector {  // a resident fp32 vector (norm weights)
     float absmax = 0.f;  // max |value|, the RMSNorm kernel's bound for its output range
 };
 
+// One resident matrix of a configured design: dense bf16 or fp32 weights in operand units (dense_kernels.h).
+struct DenseWeight {
+    int dt = 0;              // OXB_DT_*
+    uint32_t n_pad = 0, k_pad = 0;
+    void* d = nullptr;
+};
+
 struct Runtime {
     bool ready = false;
     int device = -1;
@@ -54,6 +61,7 @@ struct Runtime {
     hipStream_t own_stream = nullptr, stream = nullptr;
     std::unordered_map<uint64_t, Weight> weights;
     std::unordered_map<uint64_t, Vector> vectors;
+    std::unordered_map<uint64_t, DenseWeight> dense;
     uint64_t next_id = 1ull << 40;  // library-allocated handles stay clear of caller-chosen ids
     // Counts every free or replacement of a resident matrix or vector.  A captured decode graph holds their device
     // pointers; a model compares the count it captured under with this one and captures again when they differ.

@@ -4,7 +4,7 @@
 #include <stdint.h>
 
 // Token embedding lookup: out[i][0..h) = row ids[i] of the table kept in its stored form (gguf_type 0 F32, 1 F16,
-// 41 Q1_0_g128 blocks, 42 TQ2_0_g128 blocks), widened / dequantised as the reference's loader does.  ids are device
+// 30 BF16, 41 Q1_0_g128 blocks, 42 TQ2_0_g128 blocks), widened / dequantised as the reference's loader does.  ids are device
 // memory; an id >= vocab yields a row of NaN (host-supplied ids are validated before the launch).
 hipError_t oxb_launch_embedding_gather(const void* d_table, int gguf_type, uint32_t vocab, uint32_t h, const uint32_t* d_ids,
                                        uint32_t n, float* d_out, hipStream_t st);

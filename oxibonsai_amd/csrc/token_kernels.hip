@@ -30,6 +30,9 @@ __global__ __launch_bounds__(256) void embedding_gather_kernel(const uint8_t* __
     } else if (type == 1) {
         const __half* src = reinterpret_cast<const __half*>(table) + (size_t)id * h;
         for (uint32_t i = threadIdx.x; i < h; i += 256) o[i] = __half2float(src[i]);
+    } else if (type == 30) {
+        const uint16_t* src = reinterpret_cast<const uint16_t*>(table) + (size_t)id * h;
+        for (uint32_t i = threadIdx.x; i < h; i += 256) o[i] = __uint_as_float((uint32_t)src[i] << 16);
     } else {
         const uint32_t bb = type == 41 ? 18u : 34u;
         const uint8_t* src = table + (size_t)id * (h / 128u) * bb;
@@ -626,7 +629,7 @@ __global__ __launch_bounds__(256) void full_pick_kernel(const float* __restrict_
 hipError_t oxb_launch_embedding_gather(const void* d_table, int gguf_type, uint32_t vocab, uint32_t h, const uint32_t* d_ids,
                                        uint32_t n, float* d_out, hipStream_t st) {
     if (n == 0) return hipSuccess;
-    if ((gguf_type != 0 && gguf_type != 1 && gguf_type != 41 && gguf_type != 42) || (gguf_type >= 41 && h % 128u)) return hipErrorInvalidValue;
+    if ((gguf_type != 0 && gguf_type != 1 && gguf_type != 30 && gguf_type != 41 && gguf_type != 42) || (gguf_type >= 41 && h % 128u)) return hipErrorInvalidValue;
     hipLaunchKernelGGL(embedding_gather_kernel, dim3(n), dim3(256), 0, st, static_cast<const uint8_t*>(d_table), gguf_type, vocab, h,
                        d_ids, d_out);
     return hipGetLastError();

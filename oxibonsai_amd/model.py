@@ -8,6 +8,8 @@ call of ``oxb_hip_decode`` = ``try_cuda_full_forward_with_gpu_lm_head``."""
 from __future__ import annotations
 
 import ctypes as C
+import json
+import os
 
 import numpy as np
 
@@ -63,6 +65,33 @@ def gguf_tensor(path: str, name: str) -> dict:
     _check(_lib.lib().oxb_hip_gguf_tensor(str(path).encode(), name.encode(), C.byref(t), C.byref(nd), sh, C.byref(off), C.byref(nb)))
     return {"type": t.value, "shape": [int(sh[i]) for i in range(min(nd.value, 4))], "n_dims": nd.value,
             "file_offset": off.value, "bytes": nb.value}
+
+
+class CheckpointInfo(C.Structure):
+    """oxb_checkpoint_info: what a checkpoint of any kind (GGUF file, or folder with config.json) tells about its model."""
+    _fields_ = [("architecture", C.c_char * 32)] + \
+               [(n, C.c_uint32) for n in ("n_layers", "n_runs", "h", "vocab", "context_length", "is_gguf")]
+
+    def as_dict(self) -> dict:
+        d = {n: getattr(self, n) for n, _ in self._fields_}
+        d["architecture"] = self.architecture.decode()
+        return d
+
+
+class Tensor(C.Structure):
+    """oxb_tensor: one named row-major tensor in host memory (GGUF type ids: 0 F32, 1 F16, 30 BF16)."""
+    _fields_ = [("name", C.c_char_p), ("type", C.c_int), ("n_dims", C.c_uint32), ("shape", C.c_uint64 * 4),
+                ("data", C.c_void_p), ("n_bytes", C.c_uint64)]
+
+
+COMPUTE = {"bfloat16": 0, "float32": 1}   # OXB_COMPUTE_*
+
+
+def checkpoint_info(path: str) -> dict:
+    """Architecture and sizes of a checkpoint; needs no GPU."""
+    info = CheckpointInfo()
+    _check(_lib.lib().oxb_hip_checkpoint_info(str(path).encode(), C.byref(info)))
+    return info.as_dict()
 
 
 class Sampling(C.Structure):
@@ -205,6 +234,57 @@ class HipModel:
                         vocab=d["lm_head_rows"], max_seq=max_seq or d["context_length"], eps=d["eps"], rope_theta=d["rope_theta"])
         self.id = mid.value
         return self, Embedding(None, d["embedding_type"], d["vocab"], d["h"], _id=eid.value), d
+
+    @classmethod
+    def from_checkpoint(cls, backend: NativeHipBackend, path: str, dtype: str = "bfloat16", max_seq: int = 0, batch: int = 1):
+        """Any checkpoint the library reads, chosen by what it is: a GGUF file, or a folder whose config.json names a design
+        of the registry -> (model, embedding, info dict).  The model owns the weights it uploaded."""
+        if not os.path.isdir(path) and dtype == "bfloat16":
+            return cls.from_gguf(backend, path, max_seq, batch)
+        info, mid, eid = CheckpointInfo(), C.c_uint64(0), C.c_uint64(0)
+        _check(_lib.lib().oxb_hip_load_checkpoint(str(path).encode(), COMPUTE[dtype], max_seq, batch, C.byref(mid), C.byref(eid),
+                                                  C.byref(info)))
+        d = info.as_dict()
+        self = cls._adopt(backend, mid.value, batch, d["h"], d["vocab"], max_seq)
+        return self, Embedding(None, 30, d["vocab"], d["h"], _id=eid.value), d
+
+    @classmethod
+    def from_tensors(cls, backend: NativeHipBackend, config: dict, tensors: dict, dtype: str = "bfloat16", max_seq: int = 4096,
+                     batch: int = 1):
+        """A configured design from memory: config as in config.json, tensors name -> array (float32, float16, or uint16 for
+        bfloat16 bit patterns) -> (model, embedding)."""
+        arr = (Tensor * len(tensors))()
+        keep = []
+        for i, (name, value) in enumerate(tensors.items()):
+            shape = np.shape(value)
+            a = np.ascontiguousarray(value)   # (makes a scalar one-dimensional: the shape is taken before)
+            t = {"float32": 0, "float16": 1, "uint16": 30}[a.dtype.name]
+            keep.append(a)
+            arr[i] = Tensor(name.encode(), t, len(shape), (C.c_uint64 * 4)(*shape), a.ctypes.data, a.nbytes)
+        mid, eid = C.c_uint64(0), C.c_uint64(0)
+        _check(_lib.lib().oxb_hip_model_from_tensors(json.dumps(config).encode(), arr, len(tensors), COMPUTE[dtype], max_seq, batch,
+                                                     C.byref(mid), C.byref(eid)))
+        self = cls._adopt(backend, mid.value, batch, config["width"], config["vocab"], max_seq)
+        return self, Embedding(None, 30, config["vocab"], config["width"], _id=eid.value)
+
+    @classmethod
+    def _adopt(cls, backend, mid: int, batch: int, h: int, vocab: int, max_seq: int):
+        self = cls.__new__(cls)
+        self.be, self.batch, self._lib = backend, batch, _lib.lib()
+        self._mats, self._vecs, self._shaped, self._has_lm = [], [], True, True
+        self.cfg = dict(h=h, vocab=vocab, max_seq=max_seq)
+        self.id = mid
+        return self
+
+    def forward_tokens(self, embedding: Embedding, ids, pos_start: int = 0, seq: int = 0, want=None) -> np.ndarray:
+        """A portion of one sequence, continuing from the cache: ids at positions pos_start .. -> logits of the tokens named
+        by `want` (indices into the portion; default: the last one), [len(want), vocab]."""
+        iv = np.ascontiguousarray(ids, dtype=np.uint32).reshape(-1)
+        wv = np.ascontiguousarray([iv.size - 1] if want is None else want, dtype=np.uint32).reshape(-1)
+        logits = np.empty((wv.size, self.cfg["vocab"]), dtype=np.float32)
+        _check(self._lib.oxb_hip_forward_tokens(self.id, embedding.id, seq, iv.ctypes.data_as(_lib.u32p), iv.size, pos_start,
+                                                wv.ctypes.data_as(_lib.u32p), wv.size, logits.ctypes.data_as(_lib.f32p)))
+        return logits
 
     def _mat(self, blocks, n_rows, k):
         fmt = self.cfg["fmt"]

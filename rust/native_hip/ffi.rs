@@ -78,6 +78,27 @@ pub struct OxbKvPoolInfo {
 }
 
 #[repr(C)]
+pub struct OxbCheckpointInfo {
+    pub architecture: [c_char; 32],
+    pub n_layers: u32,
+    pub n_runs: u32,
+    pub h: u32,
+    pub vocab: u32,
+    pub context_length: u32,
+    pub is_gguf: u32,
+}
+
+#[repr(C)]
+pub struct OxbTensor {
+    pub name: *const c_char,
+    pub type_: c_int,
+    pub n_dims: u32,
+    pub shape: [u64; 4],
+    pub data: *const c_void,
+    pub n_bytes: u64,
+}
+
+#[repr(C)]
 pub struct OxbSampling {
     pub temperature: f32,
     pub top_k: u32,
@@ -182,6 +203,14 @@ extern "C" {
                                  tokens_out: *mut u32) -> c_int;
     pub fn oxb_hip_prefill_tokens(model: u64, embedding: u64, seq: u32, ids: *const u32, n_tokens: u32, pos_start: u32,
                                   logits_or_null: *mut f32, token_out_or_null: *mut u32) -> c_int;
+    // configured designs, checkpoints of any kind, portions with logits of chosen tokens
+    pub fn oxb_hip_checkpoint_info(path: *const c_char, info: *mut OxbCheckpointInfo) -> c_int;
+    pub fn oxb_hip_load_checkpoint(path: *const c_char, compute_type: c_int, max_seq: u32, batch: u32, model: *mut u64,
+                                   embedding: *mut u64, info_or_null: *mut OxbCheckpointInfo) -> c_int;
+    pub fn oxb_hip_model_from_tensors(config_json: *const c_char, tensors: *const OxbTensor, n_tensors: u32, compute_type: c_int,
+                                      max_seq: u32, batch: u32, model: *mut u64, embedding: *mut u64) -> c_int;
+    pub fn oxb_hip_forward_tokens(model: u64, embedding: u64, seq: u32, ids: *const u32, n_tokens: u32, pos_start: u32,
+                                  want: *const u32, n_want: u32, logits: *mut f32) -> c_int;
     // host-only repack helpers
     pub fn oxb_hip_repack_sizes(fmt: c_int, n_rows: u32, k: u32, codes_bytes: *mut usize, scales_bytes: *mut usize) -> c_int;
     pub fn oxb_hip_repack(fmt: c_int, aos: *const u8, n_bytes: usize, n_rows: u32, k: u32, codes: *mut u8, codes_cap: usize,

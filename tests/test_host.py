@@ -202,7 +202,8 @@ def test_ctypes_structs_match_the_header_layout(tmp_path):
     import subprocess
     from oxibonsai_amd import model as M
     mirrors = {"oxb_layer_ids": M._LayerIds, "oxb_model_desc": M._ModelDesc, "oxb_gguf_info": M.GgufInfo,
-               "oxb_sampling": M.Sampling, "oxb_attention_options": M.AttentionOptions, "oxb_kv_pool_info": M.KvPoolInfo}
+               "oxb_sampling": M.Sampling, "oxb_attention_options": M.AttentionOptions, "oxb_kv_pool_info": M.KvPoolInfo,
+               "oxb_checkpoint_info": M.CheckpointInfo, "oxb_tensor": M.Tensor}
     cc = shutil.which("gcc") or shutil.which("cc")
     if not cc:
         pytest.skip("no C compiler")
