@@ -883,18 +883,22 @@ __global__ __launch_bounds__(64) void argmax_final_kernel(const float* __restric
 
 // Pinned host staging -> device: the hidden rows and positions of a decode call, in one launch ahead of the step's
 // graph (two small asynchronous copies cost more than the step's first kernel).
-__global__ __launch_bounds__(256) void stage_in_kernel(const float4* __restrict__ h_hidden, uint32_t n4, const uint32_t* __restrict__ h_pos,
+__global__ __launch_bounds__(256) void stage_in_kernel(const float4* __restrict__ h_hidden, uint32_t n_floats, const uint32_t* __restrict__ h_pos,
                                                         uint32_t n_pos, float4* __restrict__ hidden, uint32_t* __restrict__ pos) {
-    const uint32_t i = blockIdx.x * 256 + threadIdx.x;
+    const uint32_t i = blockIdx.x * 256 + threadIdx.x, n4 = n_floats / 4;
     if (i < n4) hidden[i] = h_hidden[i];
+    else if (i < n4 + (n_floats & 3u)) {  // up to three single values behind the last group of four
+        const uint32_t j = n4 * 4 + (i - n4);
+        reinterpret_cast<float*>(hidden)[j] = reinterpret_cast<const float*>(h_hidden)[j];
+    }
     if (i < n_pos) pos[i] = h_pos[i];
 }
 
 hipError_t oxb_launch_stage_in(const float* h_hidden, uint32_t n_floats, const uint32_t* h_pos, uint32_t n_pos, float* d_hidden,
                                uint32_t* d_pos, hipStream_t st) {
-    if ((n_floats & 3u) || n_floats == 0) return hipErrorInvalidValue;
-    const uint32_t n4 = n_floats / 4, n = n4 > n_pos ? n4 : n_pos;
-    hipLaunchKernelGGL(stage_in_kernel, dim3((n + 255) / 256), dim3(256), 0, st, reinterpret_cast<const float4*>(h_hidden), n4, h_pos, n_pos,
+    if (n_floats == 0) return hipErrorInvalidValue;
+    const uint32_t n4 = n_floats / 4 + (n_floats & 3u), n = n4 > n_pos ? n4 : n_pos;
+    hipLaunchKernelGGL(stage_in_kernel, dim3((n + 255) / 256), dim3(256), 0, st, reinterpret_cast<const float4*>(h_hidden), n_floats, h_pos, n_pos,
                        reinterpret_cast<float4*>(d_hidden), d_pos);
     return hipGetLastError();
 }

@@ -478,7 +478,9 @@ struct Loader {
         const TensorView* t;
         OXB_TRY(vector(name, n, &out->w));
         OXB_TRY(vector(name + ".b", n, &out->b));
-        OXB_TRY(get(name + ".alpha", {}, &t));
+        auto a = tensors.find(name + ".alpha");   // a scalar; a vector of one value will do
+        const bool one = a != tensors.end() && a->second.shape.size() == 1;
+        OXB_TRY(get(name + ".alpha", one ? std::vector<uint64_t>{1} : std::vector<uint64_t>{}, &t));
         out->alpha = element(*t, 0);
         return OXB_HIP_OK;
     }
