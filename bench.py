@@ -371,6 +371,125 @@ def decode_ternary_leg(be, prompt_len: int, n_tokens: int) -> dict:
             "tok_per_s": round(n_tokens / spent, 2), "ms_per_token": round(spent / n_tokens * 1e3, 4)}
 
 
+# Fulirax at sizes that resemble a real model's layers, next to the Q1 Qwen3 model of the same width, heads, feed-forward
+# width, vocabulary and layer count.
+FULIRAX_SHAPES = [dict(width=2048, heads=16, ff=6144), dict(width=4096, heads=32, ff=12288)]
+FULIRAX_LATENT = dict(dim=128, rot_dim=64, vdim=128, kv_rank=512)
+
+
+def fulirax_model(be, shape: dict, layers: int, vocab: int, max_seq: int, batch: int):
+    """Random weights: every matrix is a window of one random buffer (bf16 bit patterns), scaled by its fan-in."""
+    from oxibonsai_amd.model import HipModel
+    w, ff, m = shape["width"], shape["ff"], dict(heads=shape["heads"], **FULIRAX_LATENT)
+    base = np.random.default_rng(0xF01).standard_normal(1 << 22, dtype=np.float32)
+
+    def tensor(*dims, std):
+        n = int(np.prod(dims))
+        return np.resize((base * std).view(np.uint32) >> 16, n).astype(np.uint16).reshape(dims)
+
+    def norm(out, name):
+        out[name], out[name + ".b"] = np.full(w, 0x3F80, np.uint16), np.zeros(w, np.uint16)
+        out[name + ".alpha"] = np.uint16(0x3F00)
+
+    t = {"embed": tensor(vocab, w, std=1.0), "loop.in": tensor(w, 2 * w, std=(2 * w) ** -0.5), "loop.step": tensor(1, w, std=0.1)}
+    kinds = {"q": (m["heads"] * (m["dim"] + m["rot_dim"]), w), "dkv": (m["kv_rank"] + m["rot_dim"], w), "uk": (m["heads"] * m["dim"], m["kv_rank"]),
+             "uv": (m["heads"] * m["vdim"], m["kv_rank"]), "o": (w, m["heads"] * m["vdim"]), "up": (ff, w), "down": (w, ff)}
+    shared = {k: tensor(*d, std=d[1] ** -0.5) for k, d in kinds.items()}
+    for i in range(layers):
+        p = f"l{i}."
+        norm(t, p + "norm1")
+        norm(t, p + "norm2")
+        t[p + "mix.dkv.norm"], t[p + "mix.sink"] = np.full(m["kv_rank"], 0x3F80, np.uint16), np.zeros(m["heads"], np.uint16)
+        for k in ("q", "dkv", "uk", "uv", "o"):
+            t[p + "mix." + k] = shared[k]
+        t[p + "mlp.up"], t[p + "mlp.down"] = shared["up"], shared["down"]
+    norm(t, "final.norm")
+    layer = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff},
+             "mixer": dict(m, rot={"base": 10000.0, "dims": m["rot_dim"]}, scale=(m["dim"] + m["rot_dim"]) ** -0.5)}
+    cfg = {"architecture": "Fulirax", "width": w, "vocab": vocab, "layers": [layer] * layers, "loop": {"start": 0, "stop": 1, "times": 1},
+           "norm": {"eps": 1e-6}, "logit_scale": 1.0}
+    model, emb = HipModel.from_tensors(be, cfg, t, max_seq=max_seq, batch=batch)
+    macs = sum(a * b for a, b in kinds.values())
+    return model, emb, macs
+
+
+def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, long_context: int, only: str = "") -> list:
+    """Prefill and decode of both models from token ids, the token loops on the device; host-timed around whole calls."""
+    from oxibonsai_amd import synth
+    from oxibonsai_amd.model import Embedding, HipModel
+    ids = (synth.splitmix64(0xF0120F, max(prompt, long_context)) % np.uint64(vocab)).astype(np.int64)
+    chunk = 2048
+
+    def fill(m, e, n, seq):
+        for at in range(0, n, chunk):
+            m.prefill_tokens(e, ids[at:min(n, at + chunk)], at, seq, want_logits=False)
+
+    def measure(build) -> dict:
+        r = {}
+        m, e = build(prompt + 2 * steps, 1)
+        fill(m, e, prompt, 0)
+        samples = []
+        for _ in range(5):
+            t0 = time.perf_counter()
+            m.prefill_tokens(e, ids[:prompt], 0, 0, want_logits=False)
+            samples.append(time.perf_counter() - t0)
+        t = sorted(samples)[2]
+        r["prefill_ms"], r["prefill_tok_per_s"] = round(t * 1e3, 3), round(prompt / t, 1)
+
+        def decode(m, e, n, batch):
+            pos = np.full(batch, n)
+            m.generate(e, np.arange(batch), pos, 2)
+            t0 = time.perf_counter()
+            m.generate(e, np.arange(batch), pos, steps)
+            return (time.perf_counter() - t0) / steps
+
+        t = decode(m, e, prompt, 1)
+        r["decode_batch1"] = {"ms_per_step": round(t * 1e3, 4), "tok_per_s": round(1 / t, 1)}
+        m.close()
+        for b in batches:
+            m2, e2 = build(prompt + 2 * steps, b)
+            for q in range(b):
+                fill(m2, e2, prompt, q)
+            t = decode(m2, e2, prompt, b)
+            r[f"decode_batch{b}"] = {"ms_per_step": round(t * 1e3, 4), "tok_per_s": round(b / t, 1)}
+            m2.close()
+            e2.close()
+        if long_context:
+            m3, e3 = build(long_context + 2 * steps, 1)
+            fill(m3, e3, long_context, 0)
+            t0 = time.perf_counter()
+            m3.prefill_tokens(e3, ids[long_context - chunk:long_context], long_context - chunk, 0, want_logits=False)
+            tp = time.perf_counter() - t0
+            t = decode(m3, e3, long_context, 1)
+            r[f"context_{long_context}"] = {"last_2048_prefill_ms": round(tp * 1e3, 3), "decode_ms_per_step": round(t * 1e3, 4)}
+            m3.close()
+            e3.close()
+        e.close()
+        return r
+
+    out = []
+    for shape in FULIRAX_SHAPES:
+        cfg = dict(fmt=FMT_Q1, n_layers=layers, h=shape["width"], inter=shape["ff"], nq=shape["heads"], nkv=8, hd=128, vocab=vocab,
+                   max_seq=0, eps=1e-6, rope_theta=1e6)
+        row = {"shape": dict(shape, layers=layers, vocab=vocab, **FULIRAX_LATENT)}
+        if only != "qwen3":
+            macs = fulirax_model(be, shape, 1, 64, 64, 1)
+            macs[0].close()
+            macs[1].close()
+            row["fulirax"] = measure(lambda n, b: fulirax_model(be, shape, layers, vocab, n, b)[:2])
+            flop = 2.0 * prompt * layers * macs[2] + 2.0 * layers * shape["heads"] * (192 + 128) * prompt * (prompt + 1) / 2
+            row["fulirax"]["prefill_TFLOPs"] = round(flop / row["fulirax"]["prefill_ms"] / 1e9, 1)
+            row["fulirax"]["weight_bytes_per_token"] = 2 * (layers * macs[2] + vocab * shape["width"] + 2 * shape["width"] ** 2)
+            row["fulirax"]["cache_bytes_per_position"] = 2 * layers * (FULIRAX_LATENT["kv_rank"] + FULIRAX_LATENT["rot_dim"])
+        if only != "fulirax":
+            weights = synth.make_model(dict(cfg, max_seq=prompt), 0xF012)
+            table = synth.make_q1_blocks(0xF0E, vocab * (shape["width"] // 128), 0.01, 0.1)
+            row["qwen3_q1"] = measure(lambda n, b: (HipModel(be, dict(cfg, max_seq=n), weights, batch=b), Embedding(table, 41, vocab, shape["width"])))
+        out.append(row)
+        print(json.dumps(row), file=sys.stderr, flush=True)
+    return out
+
+
 PREFILL_SHAPES = [("qkv", 5120, 2560), ("gate_up", 19456, 2560), ("down", 2560, 9728)]   # BASELINE.json configs[2]
 MFMA_F16_PEAK_TFLOPS = 2500.0
 
@@ -460,6 +579,10 @@ def main() -> int:
     ap.add_argument("--long-context-batches", type=str, default="8,32",
                     help="batch sizes decoded with every sequence at the long context (fp16 cache; 32 sequences hold 151 GB of cache)")
     ap.add_argument("--no-ternary", action="store_true", help="skip the ternary 1.7B-shape decode leg")
+    ap.add_argument("--fulirax", action="store_true",
+                    help="instead of the default workload: prefill and decode of Fulirax at real layer sizes, next to the Q1 Qwen3 model of equal size")
+    ap.add_argument("--fulirax-layers", type=int, default=8)
+    ap.add_argument("--fulirax-only", choices=["", "fulirax", "qwen3"], default="", help="one of the two models alone (profiling)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build targets one GPU; run with --gpus 1 (multi-GPU sharding is design-only)",
@@ -476,6 +599,12 @@ def main() -> int:
         return 1
     torch.cuda.set_device(0)
     be = ox.NativeHipBackend(0)
+    if args.fulirax:
+        rows = fulirax_leg(be, args.fulirax_layers, 32768, args.decode_context, args.decode_tokens,
+                           tuple(int(b) for b in args.decode_batches.split(",") if b), args.long_context, args.fulirax_only)
+        print(json.dumps({"metric": "Fulirax prefill and decode", "n_gpus": 1, "dtype": "bf16", "data": "synthetic, random weights",
+                          "prompt": args.decode_context, "steps": args.decode_tokens, "shapes": rows}), flush=True)
+        return 0
     L = _lib.lib()
     stream = torch.cuda.Stream()          # a real stream: handle 0 would mean "the library's own"
     torch.cuda.set_stream(stream)

@@ -57,18 +57,30 @@ __device__ __forceinline__ v8b zero_frag(const __bf16*) { return (v8b)(__bf16)0.
 __device__ __forceinline__ v8f zero_frag(const float*) { return (v8f)0.f; }
 
 // Memory -> LDS without a trip through registers, 16 bytes per lane: lane l's 16 bytes land at base + 16 l (base is
-// wave-uniform).  `src` is the lane's own address.
-typedef __attribute__((address_space(3))) void* lds_dst_t;
-typedef const __attribute__((address_space(1))) void* global_src_t;
+// wave-uniform).  `src` is the lane's own address.  Written as an instruction, not through the compiler's builtin: the
+// builtin makes the compiler wait for every outstanding copy in front of any LDS read that it cannot tell apart from the
+// copies' target, and the kernels here read one buffer while the next one fills.  They place the waits themselves
+// (wait_lds_copies, or a counted wait), always together with a barrier or before the wave's own reads; those waits carry the
+// memory clobber that keeps LDS accesses on their side.
 __device__ __forceinline__ void copy16_to_lds(const void* src, void* lds_base) {
-    __builtin_amdgcn_global_load_lds((global_src_t)src, (lds_dst_t)lds_base, 16, 0, 0);
+    const uint32_t at = (uint32_t)__builtin_amdgcn_readfirstlane((int)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)lds_base);
+    asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(at), "v"(src) : "m0");
 }
-// The lane's eight consecutive elements at `row8` into its place of the unit at `unit` (LDS).
-__device__ __forceinline__ void copy_row8_to_unit(const __bf16* row8, __bf16* unit) { copy16_to_lds(row8, unit); }
-__device__ __forceinline__ void copy_row8_to_unit(const float* row8, float* unit) {
+// Staged units: 16 rows x 32 columns in LDS, filled by such copies from row-major memory.  Lane l brings columns
+// 8 stage_col(l) .. + 7 of row stage_row(l), so four lanes in turn read one row's 64 (128) contiguous bytes, and its 16 bytes
+// land in slot l: row r, column group g sits in slot 4 r + (g ^ (r >> 2)).  The exclusive-or keeps the operand reads of the
+// matrix cores (16 rows, one column group) on distinct banks.  fp32: the first halves of all groups, then the second.
+__device__ __forceinline__ uint32_t stage_row(uint32_t lane) { return lane >> 2; }
+__device__ __forceinline__ uint32_t stage_col(uint32_t lane) { return (lane & 3u) ^ (lane >> 4); }
+__device__ __forceinline__ uint32_t staged_slot(uint32_t r, uint32_t g) { return r * 4 + (g ^ (r >> 2)); }
+__device__ __forceinline__ void stage_unit(const __bf16* row8, __bf16* unit) { copy16_to_lds(row8, unit); }
+__device__ __forceinline__ void stage_unit(const float* row8, float* unit) {
     copy16_to_lds(row8, unit);
     copy16_to_lds(row8 + 4, unit + 256);
 }
+// Operand of lane 16 g + r: `slot` = staged_slot(r, g).
+__device__ __forceinline__ v8b load_staged(const __bf16* unit, uint32_t slot) { return *reinterpret_cast<const v8b*>(unit + slot * 8); }
+__device__ __forceinline__ v8f load_staged(const float* unit, uint32_t slot) { return load_unit(unit, slot); }
 __device__ __forceinline__ void wait_lds_copies() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
 
 // tanh in fp32: the library's for the fp32 kernels; for bf16 results 1 - 2 / (e^(2|z|) + 1) on the hardware exponential
@@ -90,19 +102,26 @@ template <typename T> __device__ __forceinline__ float exp_of(float z) {  // e^z
     return __builtin_amdgcn_exp2f(z * 1.4426950408889634f);
 }
 
-// Four consecutive outputs y[m][n0 .. n0 + 3] through the epilogue.
-template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogue& e, uint32_t m, uint32_t n0, v4f y) {
+// The residual's four values for outputs y[m][n0 .. n0 + 3], requested ahead of the arithmetic (zeros where epilogue4 fetches
+// them itself).
+__device__ __forceinline__ bool epilogue_whole(const OxbEpilogue& e, uint32_t n0) { return n0 + 4 <= e.n && (e.ld32 & 3u) == 0; }
+__device__ __forceinline__ v4f epilogue_resid(const OxbEpilogue& e, uint32_t m, uint32_t n0) {
+    if (!e.resid || !epilogue_whole(e, n0)) return (v4f){0.f, 0.f, 0.f, 0.f};
+    return *reinterpret_cast<const v4f*>(e.resid + (size_t)m * e.ld32 + n0);
+}
+// Four consecutive outputs through the epilogue; resid = epilogue_resid(e, m, n0).
+template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogue& e, uint32_t m, uint32_t n0, v4f y, v4f resid) {
     const uint32_t lim = e.n > e.fill ? e.n : e.fill;
     if (n0 >= lim) return;
     y *= e.scale;
-    if (n0 + 4 <= e.n && (e.ld32 & 3u) == 0) {
+    if (epilogue_whole(e, n0)) {
         if (e.add) y += *reinterpret_cast<const v4f*>(e.add + n0);
         if (e.act == OXB_ACT_GELU_TANH) {
 #pragma unroll
             for (int i = 0; i < 4; i++) y[i] = gelu_tanh_of<T>(y[i]);
         }
         const size_t o = (size_t)m * e.ld32 + n0;
-        if (e.resid) y += *reinterpret_cast<const v4f*>(e.resid + o);
+        y += resid;
         if (e.out32) *reinterpret_cast<v4f*>(e.out32 + o) = y;
         if (!e.out_t) return;
         if (e.norm == OXB_NORM_DYT) {

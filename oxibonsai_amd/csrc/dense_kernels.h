@@ -3,7 +3,8 @@
 // Resident layout, "operand units": the matrix W [n][k] (y = W x) is cut into units of 16 rows x 32 columns, row tiles
 // outermost, and a unit holds its 512 elements in the order a wave64 feeds them to the matrix cores: lane
 // l = 16 g + r keeps row r, columns 8 g .. 8 g + 7.  bf16: the lane's eight elements are its 16 bytes at 16 l (1 KiB per
-// unit).  fp32: its first four are 16 bytes at 16 l, its last four 16 bytes at 1024 + 16 l (2 KiB per unit), so both
+// unit).  Row tiles lie 256 bytes further apart than their units need, so that workgroups walking different tiles in step
+// do not all draw on the same memory channels.  fp32: its first four are 16 bytes at 16 l, its last four 16 bytes at 1024 + 16 l (2 KiB per unit), so both
 // types load a unit with fully coalesced 16-byte lane loads.  Rows and columns pad with zeros to multiples of 64.
 //
 // Activations are row-major [token][ld], bf16 or fp32 like the weights, ld a multiple of 64.  Whoever writes an
@@ -18,6 +19,14 @@ static inline uint32_t oxb_dt_bytes(int dt) { return dt == OXB_DT_BF16 ? 2u : 4u
 
 #define OXB_DENSE_PAD 64u
 static inline uint32_t oxb_dense_pad(uint32_t n) { return (n + OXB_DENSE_PAD - 1) / OXB_DENSE_PAD * OXB_DENSE_PAD; }
+// Elements from one row tile of a packed matrix to the next.
+#if defined(__HIPCC__)
+__host__ __device__
+#endif
+static inline size_t oxb_tile_stride(uint32_t k_pad, uint32_t elem_bytes) { return (size_t)(k_pad / 32u) * 512u + 256u / elem_bytes; }
+// Row stride of an activation matrix of n columns: padded columns, and 128 elements more where rows would otherwise start a
+// multiple of 1 KiB apart (the 16 rows of an operand would all come out of one or two L2 channels).
+static inline uint32_t oxb_act_ld(uint32_t n) { const uint32_t p = oxb_dense_pad(n); return p % 512u ? p : p + 128u; }
 #define OXB_DENSE_GEMV_MAX_ROWS 16u   // token rows the few-row kernel takes per pass over the weights (one MFMA column tile)
 
 // What happens to y[m][n] behind the product, in this order:

@@ -25,7 +25,7 @@ __global__ __launch_bounds__(512) void dense_pack_kernel(const void* __restrict_
         else if (type == 1) v = __half2float(static_cast<const __half*>(src)[i]);
         else v = __uint_as_float((uint32_t)static_cast<const uint16_t*>(src)[i] << 16);
     }
-    T* unit = dst + (size_t)blockIdx.x * 512;
+    T* unit = dst + tile * oxb_tile_stride(n_units_k * 32, sizeof(T)) + (size_t)u * 512;
     if constexpr (Dt<T>::is_f32) unit[(e >> 2) * 256 + lane * 4 + (e & 3u)] = v;
     else unit[lane * 8 + e] = (T)v;
 }
@@ -64,7 +64,7 @@ __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
     const uint32_t nu = p.k_pad / 32, n_tiles = p.n_pad / 16, m0 = blockIdx.y * 16, mc = min(p.m - m0, 16u);
     const T* w[RT];
 #pragma unroll
-    for (int r = 0; r < RT; r++) w[r] = reinterpret_cast<const T*>(p.w) + (size_t)min(blockIdx.x * RT + r, n_tiles - 1) * nu * 512;
+    for (int r = 0; r < RT; r++) w[r] = reinterpret_cast<const T*>(p.w) + (size_t)min(blockIdx.x * RT + r, n_tiles - 1) * oxb_tile_stride(p.k_pad, sizeof(T));
     const bool have = c < mc;
     const T* x = reinterpret_cast<const T*>(p.x) + (have ? x_row(p, m0 + c) : 0) * p.ldx + 8 * g;
     v4f acc[RT];
@@ -75,7 +75,7 @@ __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
 #pragma unroll
         for (int i = 0; i < UN; i++) {
             const uint32_t u = u0 + 8 * i;
-            b[i] = have && u < nu && 32 * u + 8 * g + 8 <= p.ldx ? load_row8(x + 32 * u) : zero_frag((const T*)nullptr);
+            b[i] = have && u < nu ? load_row8(x + 32 * u) : zero_frag((const T*)nullptr);
         }
 #pragma unroll
         for (int i = 0; i < UN; i++) {
@@ -88,59 +88,62 @@ __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
 #pragma unroll
             for (int r = 0; r < RT; r++) acc[r] = mfma32(a[i][r], b[i], acc[r]);
     }
+    const uint32_t fr = tid >> 6, fq = tid & 3u, ft = (tid & 63u) >> 2, fn = (blockIdx.x * RT + fr) * 16 + 4 * fq;   // what a finishing thread owns
+    v4f resid = {0.f, 0.f, 0.f, 0.f};
+    if (fr < RT && ft < mc) resid = epilogue_resid(p.e, m0 + ft, fn);
 #pragma unroll
     for (int r = 0; r < RT; r++) *reinterpret_cast<v4f*>(&red[wave][r][c][4 * g]) = acc[r];
     __syncthreads();
     if (tid < 64 * RT) {
-        const uint32_t r = tid >> 6, q = tid & 3u, t = (tid & 63u) >> 2;
-        v4f y = *reinterpret_cast<const v4f*>(&red[0][r][t][4 * q]);
+        v4f y = *reinterpret_cast<const v4f*>(&red[0][fr][ft][4 * fq]);
 #pragma unroll
-        for (int i = 1; i < 8; i++) y += *reinterpret_cast<const v4f*>(&red[i][r][t][4 * q]);
-        if (t < mc && blockIdx.x * RT + r < n_tiles) epilogue4<T>(p.e, m0 + t, (blockIdx.x * RT + r) * 16 + 4 * q, y);
+        for (int i = 1; i < 8; i++) y += *reinterpret_cast<const v4f*>(&red[i][fr][ft][4 * fq]);
+        if (ft < mc && blockIdx.x * RT + fr < n_tiles) epilogue4<T>(p.e, m0 + ft, fn, y, resid);
     }
 }
 
 // ---------------------------------------------------------------------------
 // Tiled GEMM: a workgroup of 4 waves owns 64 RT rows x 16 CT tokens.  The weights come from memory already in operand
-// order, so each wave loads its own RT tiles straight into registers, one stage ahead; the token tile is shared by the
-// waves and goes memory -> LDS without registers, also in operand order (every LDS access is linear in the lane), two
-// stages.  A stage is UK units of k (64 values bf16, 32 fp32).  SWAP exchanges the operands' roles: the lane then holds
-// four consecutive tokens of one output row, which is the transposed store of the value rows of attention.
+// order, so each wave loads its own RT tiles straight into registers; the token tile is shared by the waves and goes
+// memory -> LDS without registers, as staged units (dense_device.h).  A stage is two units of k; tokens run
+// three stages ahead (four LDS buffers; fp32: one, two buffers), weights two (two register sets).  The one barrier of a stage
+// sits between its two units: it hands back the buffer of the stage before and admits reads of the next stage, which run
+// under the second unit's products.  It waits for the requests of earlier regions alone; what was requested since the last
+// barrier stays in flight.  The last stages request their own data again so that the count of requests in flight never
+// changes.  SWAP exchanges the operands' roles: the lane then holds four consecutive tokens of one
+// output row, which is the transposed store of the value rows of attention.
 // ---------------------------------------------------------------------------
 template <typename T, int RT, int CT, bool SWAP>
-__global__ __launch_bounds__(256, 2) void dense_gemm_kernel(OxbDenseParams p, uint32_t n_tm, uint32_t n_tn) {
+__global__ __launch_bounds__(256, RT == 4 && Dt<T>::is_f32 ? 1 : 2) void dense_gemm_kernel(OxbDenseParams p, uint32_t n_tm, uint32_t n_tn) {
     typedef typename Dt<T>::frag frag;
-    constexpr int UK = Dt<T>::is_f32 ? 1 : 2;
+    constexpr int UK = 2, SUB = Dt<T>::sub;
     constexpr int UNITS = CT * UK;          // LDS units of a stage
-    __shared__ __attribute__((aligned(16))) T xs[2][UNITS * 512];
+    __shared__ __attribute__((aligned(16))) T xs[Dt<T>::is_f32 ? 2 : 4][UNITS * 512];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, c = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
     // consecutive workgroups go to different XCDs: give each XCD a contiguous run of tiles with the token tiles innermost,
     // so that the workgroups sharing a row tile's weights share an L2
     const uint32_t total = n_tm * n_tn, per = (total + 7) / 8, id = (blockIdx.x & 7u) * per + (blockIdx.x >> 3);
     if (id >= total || (blockIdx.x >> 3) >= per) return;
-    const uint32_t tm = id % n_tm, tn = id / n_tm;
+    const uint32_t tm = id % n_tm, tn = id / n_tm, slot = staged_slot(c, g);
     const uint32_t nu = p.k_pad / 32, n_tiles = p.n_pad / 16, n_stages = nu / UK;  // (k_pad is a multiple of 64)
     const T* w[RT];
 #pragma unroll
-    for (int r = 0; r < RT; r++) w[r] = reinterpret_cast<const T*>(p.w) + (size_t)min((tn * 4 + wave) * RT + r, n_tiles - 1) * nu * 512;
+    for (int r = 0; r < RT; r++) w[r] = reinterpret_cast<const T*>(p.w) + min((tn * 4 + wave) * RT + r, n_tiles - 1) * oxb_tile_stride(p.k_pad, sizeof(T));
     // the units of the token tile this wave brings in: unit i -> token tile i / UK, k unit i % UK
-    constexpr int MINE = (UNITS + 3) / 4;
+    constexpr int MINE = UNITS / 4;
+    static_assert(UNITS % 4 == 0, "the waves bring in equal shares");
     const T* xr[MINE];
 #pragma unroll
     for (int i = 0; i < MINE; i++) {
         const uint32_t un = wave + 4 * i;
-        xr[i] = reinterpret_cast<const T*>(p.x) + x_row(p, min(tm * (16 * CT) + (un / UK) * 16 + c, p.m - 1)) * p.ldx;
+        xr[i] = reinterpret_cast<const T*>(p.x) + x_row(p, min(tm * (16 * CT) + (un / UK) * 16 + stage_row(lane), p.m - 1)) * p.ldx + (un % UK) * 32 + 8 * stage_col(lane);
     }
-    auto stage_x = [&](uint32_t st, int buf) {
+    auto stage_x = [&](uint32_t st, uint32_t buf) {
 #pragma unroll
         for (int i = 0; i < MINE; i++) {
             const uint32_t un = wave + 4 * i;
-            if (UNITS % 4 == 0 || un < (uint32_t)UNITS) {
-                // (columns past the row's end meet zero weights; any finite value will do)
-                const uint32_t k = min((st * UK + un % UK) * 32 + 8 * g, p.ldx - 8);
-                copy_row8_to_unit(xr[i] + k, &xs[buf][un * 512]);
-            }
+            stage_unit(xr[i] + st * (32 * UK), &xs[buf][un * 512]);
         }
     };
     v4f acc[RT][CT];
@@ -148,52 +151,115 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(OxbDenseParams p, ui
     for (int r = 0; r < RT; r++)
 #pragma unroll
         for (int t = 0; t < CT; t++) acc[r][t] = (v4f){0.f, 0.f, 0.f, 0.f};
-    frag a[UK][RT];
-    stage_x(0, 0);
+    frag a[2][UK][RT], b[CT];
+    auto load_w = [&](uint32_t st, int set, int k) {
 #pragma unroll
-    for (int k = 0; k < UK; k++)
-#pragma unroll
-        for (int r = 0; r < RT; r++) a[k][r] = load_unit(w[r] + (size_t)min((uint32_t)k, nu - 1) * 512, lane);
-    for (uint32_t st = 0; st < n_stages; st++) {
-        wait_lds_copies();
-        __syncthreads();
-        const int buf = st & 1u;
-        if (st + 1 < n_stages) stage_x(st + 1, buf ^ 1);
-#pragma unroll
-        for (int k = 0; k < UK; k++) {
-#pragma unroll
-            for (int t = 0; t < CT; t++) {
-                const frag b = load_unit(&xs[buf][(t * UK + k) * 512], lane);
-#pragma unroll
-                for (int r = 0; r < RT; r++) acc[r][t] = SWAP ? mfma32(b, a[k][r], acc[r][t]) : mfma32(a[k][r], b, acc[r][t]);
-            }
-            const uint32_t un = min((st + 1) * UK + k, nu - 1);
-#pragma unroll
-            for (int r = 0; r < RT; r++) a[k][r] = load_unit(w[r] + (size_t)un * 512, lane);
-        }
-    }
-#pragma unroll
-    for (int r = 0; r < RT; r++) {
-        const uint32_t tile = (tn * 4 + wave) * RT + r;
-        if (tile >= n_tiles) continue;
+        for (int r = 0; r < RT; r++) a[set][k][r] = load_unit(w[r] + (size_t)(st * UK + k) * 512, lane);
+    };
+    auto read_x = [&](uint32_t buf, int k, int t) { b[t] = load_staged(&xs[buf][(t * UK + k) * 512], slot); };
+    // One half of a stage: the products of unit k; each token operand is replaced by that of the unit behind it (in the
+    // second half: the next stage's first) right after its last use.
+    auto half = [&](int set, int k, uint32_t next_buf) {
 #pragma unroll
         for (int t = 0; t < CT; t++) {
-            if constexpr (SWAP) {
+#pragma unroll
+            for (int r = 0; r < RT; r++) acc[r][t] = SWAP ? mfma32(b[t], a[set][k][r], acc[r][t]) : mfma32(a[set][k][r], b[t], acc[r][t]);
+            read_x(next_buf, k ^ 1, t);
+        }
+#pragma unroll
+        for (int t = 0; t < CT; t++) {
+            __builtin_amdgcn_sched_group_barrier(0x008, RT * (Dt<T>::is_f32 ? 8 : 1), 0);   // matrix core
+            __builtin_amdgcn_sched_group_barrier(0x100, SUB, 0);                            // LDS read
+        }
+    };
+    auto clamp_st = [&](uint32_t st) { return min(st, n_stages - 1); };
+    constexpr uint32_t NB = Dt<T>::is_f32 ? 2 : 4;   // LDS buffers
+    constexpr int AHEAD = NB - 1, REGION = (MINE + UK * RT) * SUB;   // stages the tokens run ahead; requests between two barriers
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) stage_x(clamp_st(i), i);
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int k = 0; k < UK; k++) load_w(clamp_st(i), i, k);
+    asm volatile("s_waitcnt vmcnt(0)\n\ts_barrier" ::: "memory");
+#pragma unroll
+    for (int t = 0; t < CT; t++) read_x(0, 0, t);
+    auto stage = [&](uint32_t st, int set) {
+        const uint32_t nxt = clamp_st(st + 2);
+        if constexpr (AHEAD == 1) stage_x(clamp_st(st + 1), (st + 1) % NB);   // (everyone is through with the stage before)
+        half(set, 0, st % NB);
+        load_w(nxt, set, 0);
+        __builtin_amdgcn_sched_barrier(0);
+        // the next stage's tokens have arrived, and every wave is through with the stage before this one: its buffer can be
+        // filled again
+        if constexpr (AHEAD == 1) asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        else asm volatile("s_waitcnt vmcnt(%0)\n\ts_barrier" ::"n"((AHEAD - 2) * REGION) : "memory");
+        if constexpr (AHEAD > 1) stage_x(clamp_st(st + AHEAD), (st + AHEAD) % NB);
+        __builtin_amdgcn_sched_barrier(0);
+        half(set, 1, (st + 1) % NB);
+        load_w(nxt, set, 1);
+        __builtin_amdgcn_sched_barrier(0);
+    };
+    uint32_t st = 0;
+    for (; st + 1 < n_stages; st += 2) {
+        stage(st, 0);
+        stage(st + 1, 1);
+    }
+    if (st < n_stages) stage(st, 0);
+    wait_lds_copies();
+    if constexpr (SWAP) {
+#pragma unroll
+        for (int r = 0; r < RT; r++) {
+            const uint32_t n = ((tn * 4 + wave) * RT + r) * 16 + c;
+#pragma unroll
+            for (int t = 0; t < CT; t++) {
                 typename Dt<T>::quad q;
 #pragma unroll
                 for (int i = 0; i < 4; i++) q[i] = (T)(acc[r][t][i] * p.e.scale);
-                const uint32_t n = tile * 16 + c, m = (tm * CT + t) * 16 + 4 * g;
+                const uint32_t m = (tm * CT + t) * 16 + 4 * g;
                 if (n < p.e.n && m < p.e.ld_t) *reinterpret_cast<typename Dt<T>::quad*>(reinterpret_cast<T*>(p.e.out_t) + (size_t)n * p.e.ld_t + m) = q;
-            } else {
-                const uint32_t m = (tm * CT + t) * 16 + c;
-                if (m < p.m) epilogue4<T>(p.e, m, tile * 16 + 4 * g, acc[r][t]);
+            }
+        }
+    } else {
+        // Through LDS, PT token tiles at a time: a wave then finishes whole runs of one token's outputs, and the epilogue is a
+        // short loop instead of RT x CT inlined copies.  Quad q of token t sits at q ^ t (distinct banks).
+        constexpr int PT = CT / RT > 0 ? CT / RT : 1, QUADS = 16 * RT, UN = 4;
+        float* ys = reinterpret_cast<float*>(&xs[0][0]);
+        static_assert(PT * 16 * QUADS * 16 <= (int)NB * UNITS * (int)Dt<T>::unit_bytes && (PT * 16 * QUADS) % (256 * UN) == 0, "the stages' LDS holds a pass");
+#pragma unroll 1
+        for (int t0 = 0; t0 < CT; t0 += PT) {
+            __syncthreads();
+#pragma unroll
+            for (int s = 0; s < CT; s += PT)
+                if (s == t0) {
+#pragma unroll
+                    for (int r = 0; r < RT; r++)
+#pragma unroll
+                        for (int t = 0; t < PT; t++)
+                            *reinterpret_cast<v4f*>(ys + ((t * 16 + c) * QUADS + (((wave * RT + r) * 4 + g) ^ c)) * 4) = acc[r][s + t];
+                }
+            __syncthreads();
+#pragma unroll 1
+            for (uint32_t i0 = tid; i0 < PT * 16 * QUADS; i0 += 256 * UN) {
+                v4f resid[UN];
+#pragma unroll
+                for (int k = 0; k < UN; k++) {
+                    const uint32_t i = i0 + 256 * k, m = (tm * CT + t0) * 16 + i / QUADS;
+                    resid[k] = m < p.m ? epilogue_resid(p.e, m, tn * 64 * RT + i % QUADS * 4) : (v4f){0.f, 0.f, 0.f, 0.f};
+                }
+#pragma unroll
+                for (int k = 0; k < UN; k++) {
+                    const uint32_t i = i0 + 256 * k, t = i / QUADS, q = i % QUADS, m = (tm * CT + t0) * 16 + t;
+                    if (m < p.m)
+                        epilogue4<T>(p.e, m, tn * 64 * RT + q * 4, *reinterpret_cast<const v4f*>(ys + (t * QUADS + (q ^ (t & 15u))) * 4), resid[k]);
+                }
             }
         }
     }
 }
 
 static hipError_t check(const OxbDenseParams& p, int dt) {
-    if (!p.w || !p.x || !p.m || !p.n_pad || !p.k_pad || p.n_pad % OXB_DENSE_PAD || p.k_pad % OXB_DENSE_PAD || p.ldx < 32 || p.ldx % 8 ||
+    if (!p.w || !p.x || !p.m || !p.n_pad || !p.k_pad || p.n_pad % OXB_DENSE_PAD || p.k_pad % OXB_DENSE_PAD || p.ldx < p.k_pad || p.ldx % 8 ||
         (dt != OXB_DT_BF16 && dt != OXB_DT_F32) || p.e.n > p.n_pad || p.e.fill > p.n_pad || (p.row_table && (p.row_shift < 4 || p.row_shift > 7)))
         return hipErrorInvalidValue;
     return hipSuccess;
@@ -211,22 +277,23 @@ static hipError_t launch_gemm(const OxbDenseParams& p, hipStream_t st) {
 template <typename T, bool SWAP>
 static hipError_t pick_gemm(const OxbDenseParams& p, uint32_t n_cus, hipStream_t st) {
     struct { int rt, ct; double mac_cost; } const opt[] = {{4, 8, 1.0}, {2, 8, 1.15}, {4, 4, 1.2}, {2, 4, 1.4}, {1, 8, 1.5}, {1, 4, 1.8}};
-    int best = 0;
+    int best = -1;
     double best_cost = 0;
     for (int i = 0; i < 6; i++) {
         const double wgs = (double)((p.m + 16 * opt[i].ct - 1) / (16 * opt[i].ct)) * ((p.n_pad + 64 * opt[i].rt - 1) / (64 * opt[i].rt));
         const double slots = n_cus, rounds = wgs <= slots ? 1.0 : (double)(uint64_t)((wgs + slots - 1) / slots);
         const double cost = rounds * opt[i].rt * opt[i].ct * opt[i].mac_cost;
-        if (i == 0 || cost < best_cost) best = i, best_cost = cost;
+        if (Dt<T>::is_f32 && opt[i].ct == 8) continue;   // (fp32 stages are twice as large)
+        if (best < 0 || cost < best_cost) best = i, best_cost = cost;
     }
-    switch (best) {
-        case 0: return launch_gemm<T, 4, 8, SWAP>(p, st);
-        case 1: return launch_gemm<T, 2, 8, SWAP>(p, st);
-        case 2: return launch_gemm<T, 4, 4, SWAP>(p, st);
-        case 3: return launch_gemm<T, 2, 4, SWAP>(p, st);
-        case 4: return launch_gemm<T, 1, 8, SWAP>(p, st);
-        default: return launch_gemm<T, 1, 4, SWAP>(p, st);
+    if constexpr (!Dt<T>::is_f32) {
+        if (best == 0) return launch_gemm<T, 4, 8, SWAP>(p, st);
+        if (best == 1) return launch_gemm<T, 2, 8, SWAP>(p, st);
+        if (best == 4) return launch_gemm<T, 1, 8, SWAP>(p, st);
     }
+    if (best == 2) return launch_gemm<T, 4, 4, SWAP>(p, st);
+    if (best == 3) return launch_gemm<T, 2, 4, SWAP>(p, st);
+    return launch_gemm<T, 1, 4, SWAP>(p, st);
 }
 
 template <typename T>
@@ -259,30 +326,34 @@ hipError_t oxb_launch_dense_gemm_t(const OxbDenseParams& p, int dt, uint32_t n_c
     return dt == OXB_DT_BF16 ? pick_gemm<__bf16, true>(p, n_cus, st) : pick_gemm<float, true>(p, n_cus, st);
 }
 
+// Grid (1024 columns, token row), four columns per thread.
 template <typename T>
 __global__ __launch_bounds__(256) void stream_enter_kernel(const float* __restrict__ x, uint32_t width, T* __restrict__ x0, uint32_t ld_x0,
                                                            uint32_t x0_col, uint32_t x0_fill, OxbEpilogue e) {
-    const uint32_t m = blockIdx.x;
+    const uint32_t m = blockIdx.y, n0 = (blockIdx.x * 256 + threadIdx.x) * 4;
     const float* row = x + (size_t)m * width;
-    if (x0)
-        for (uint32_t i = threadIdx.x; x0_col + i < x0_fill; i += 256) x0[(size_t)m * ld_x0 + x0_col + i] = (T)(i < width ? row[i] : 0.f);
-    const uint32_t lim = e.n > e.fill ? e.n : e.fill;
-    for (uint32_t n0 = threadIdx.x * 4; n0 < lim; n0 += 1024) {
-        v4f y = {0.f, 0.f, 0.f, 0.f};
+    v4f y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+        if (n0 + i < width) y[i] = row[n0 + i];
+    if (x0) {
 #pragma unroll
         for (int i = 0; i < 4; i++)
-            if (n0 + i < width) y[i] = row[n0 + i];
-        epilogue4<T>(e, m, n0, y);
+            if (x0_col + n0 + i < x0_fill) x0[(size_t)m * ld_x0 + x0_col + n0 + i] = (T)y[i];
     }
+    epilogue4<T>(e, m, n0, y, epilogue_resid(e, m, n0));
 }
 
 hipError_t oxb_launch_stream_enter(const float* x, uint32_t width, uint32_t m, void* x0_out, uint32_t ld_x0, uint32_t x0_col,
                                    uint32_t x0_fill, const OxbEpilogue& e, int dt, hipStream_t st) {
     if (!x || !width || !m || (x0_out && (x0_fill > ld_x0 || x0_col + width > x0_fill)) || !e.out_t || e.n != width) return hipErrorInvalidValue;
+    uint32_t cols = e.n > e.fill ? e.n : e.fill;
+    if (x0_out && x0_fill - x0_col > cols) cols = x0_fill - x0_col;
+    const dim3 grid((cols + 1023) / 1024, m);
     if (dt == OXB_DT_BF16)
-        hipLaunchKernelGGL((stream_enter_kernel<__bf16>), dim3(m), dim3(256), 0, st, x, width, (__bf16*)x0_out, ld_x0, x0_col, x0_fill, e);
+        hipLaunchKernelGGL((stream_enter_kernel<__bf16>), grid, dim3(256), 0, st, x, width, (__bf16*)x0_out, ld_x0, x0_col, x0_fill, e);
     else
-        hipLaunchKernelGGL((stream_enter_kernel<float>), dim3(m), dim3(256), 0, st, x, width, (float*)x0_out, ld_x0, x0_col, x0_fill, e);
+        hipLaunchKernelGGL((stream_enter_kernel<float>), grid, dim3(256), 0, st, x, width, (float*)x0_out, ld_x0, x0_col, x0_fill, e);
     return hipGetLastError();
 }
 

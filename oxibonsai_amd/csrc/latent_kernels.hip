@@ -20,34 +20,39 @@ __device__ __forceinline__ float rotated(const float* v, uint32_t i, uint32_t ro
 }
 
 // ---------------------------------------------------------------------------
-// New tokens: blocks [0, n_abs) of a grid row absorb queries (4 waves, one 16-row tile of (head, latent) each), the 16
-// blocks behind them take one token row each: RMS norm of the latent and rotation of the key part into the cache, rotation
-// of the query parts into q_abs.
+// New tokens.  The first n_abs blocks of a grid row absorb queries (4 waves, one 16-row tile of (head, latent) each); the
+// blocks behind them belong to the 16 token rows in turn: block 0 of a row brings the RMS-normed latent and the rotated key
+// part into the cache, the others rotate 1024 elements of the row's query parts into q_abs.
 // ---------------------------------------------------------------------------
 template <typename T>
-__global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, uint32_t n_abs, uint32_t tiles_per_head) {
+__global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, uint32_t n_abs, uint32_t tiles_per_head, uint32_t per_row) {
     typedef typename Dt<T>::frag frag;
     const OxbLatentDims& d = p.d;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, m0 = blockIdx.y * 16;
     const uint32_t kl = d.rank_p + d.rot_p, qh = d.dim_p + d.rot_p;
     T* q_abs = reinterpret_cast<T*>(p.q_abs);
     if (blockIdx.x < n_abs) {
+        constexpr int UN = 4;
         const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
         const uint32_t tile = blockIdx.x * 4 + wave, c = lane & 15u, g = lane >> 4;
         if (tile >= d.heads * tiles_per_head) return;
-        const uint32_t head = tile / tiles_per_head, rt = tile % tiles_per_head, nu = p.k_uk / 32;
-        const T* w = reinterpret_cast<const T*>(p.w_uk_t) + (size_t)tile * nu * 512;
+        const uint32_t head = tile / tiles_per_head, rt = tile % tiles_per_head, nu = d.dim_p / 32;
+        const T* w = reinterpret_cast<const T*>(p.w_uk_t) + tile * oxb_tile_stride(p.k_uk, sizeof(T));
         const bool have = m0 + c < p.rows.m;
         const float* q = p.qkv + (size_t)(have ? m0 + c : 0) * p.ld_qkv + head * qh + 8 * g;
         v4f acc = {0.f, 0.f, 0.f, 0.f};
-        for (uint32_t u = 0; u < nu; u++) {
-            frag b = zero_frag((const T*)nullptr);
-            if (have && 32 * u < d.dim_p) {
-                const v4f lo = *reinterpret_cast<const v4f*>(q + 32 * u), hi = *reinterpret_cast<const v4f*>(q + 32 * u + 4);
+        for (uint32_t u0 = 0; u0 < nu; u0 += UN) {
+            frag a[UN], b[UN];
 #pragma unroll
-                for (int e = 0; e < 4; e++) b[e] = (T)lo[e], b[4 + e] = (T)hi[e];
+            for (int i = 0; i < UN; i++) {
+                const uint32_t u = min(u0 + i, nu - 1);
+                a[i] = load_unit(w + (size_t)u * 512, lane);
+                const v8f x = load_row8(q + 32 * u);
+#pragma unroll
+                for (int e = 0; e < 8; e++) b[i][e] = have && u0 + i < nu ? (T)x[e] : (T)0.f;
             }
-            acc = mfma32(load_unit(w + (size_t)u * 512, lane), b, acc);
+#pragma unroll
+            for (int i = 0; i < UN; i++) acc = mfma32(a[i], b[i], acc);
         }
         if (have) {
             typename Dt<T>::quad o;
@@ -57,12 +62,23 @@ __global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, ui
         }
         return;
     }
-    const uint32_t m = m0 + blockIdx.x - n_abs;
+    const uint32_t m = m0 + (blockIdx.x - n_abs) / per_row, part = (blockIdx.x - n_abs) % per_row;
     if (m >= p.rows.m) return;
     const uint32_t pos = row_pos(p.rows, m), half = d.rot_dims >> 1;
     const float* cs = p.cos_t + (size_t)pos * half;
     const float* sn = p.sin_t + (size_t)pos * half;
     const float* row = p.qkv + (size_t)m * p.ld_qkv;
+    if (part) {
+#pragma unroll
+        for (int k = 0; k < 4; k++) {
+            const uint32_t i = (part - 1) * 1024 + k * 256 + tid;
+            if (i >= d.heads * d.rot_p) break;
+            const uint32_t head = i / d.rot_p, j = i % d.rot_p;
+            q_abs[((size_t)m * d.heads + head) * kl + d.rank_p + j] =
+                (T)(j < d.rot ? rotated(row + head * qh + d.dim_p, j, d.rot_dims, cs, sn) : 0.f);
+        }
+        return;
+    }
     const float* lat = row + d.heads * qh;
     __shared__ float red[4];
     float ss = 0.f;
@@ -78,12 +94,6 @@ __global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, ui
         else if (i >= d.rank_p && i - d.rank_p < d.rot) v = rotated(lat + d.rank_p, i - d.rank_p, d.rot_dims, cs, sn);
         dst[i] = (T)v;
     }
-    if (q_abs)
-        for (uint32_t i = tid; i < d.heads * d.rot_p; i += 256) {
-            const uint32_t head = i / d.rot_p, j = i % d.rot_p;
-            q_abs[((size_t)m * d.heads + head) * kl + d.rank_p + j] =
-                (T)(j < d.rot ? rotated(row + head * qh + d.dim_p, j, d.rot_dims, cs, sn) : 0.f);
-        }
 }
 
 // ---------------------------------------------------------------------------
@@ -100,7 +110,7 @@ __device__ __forceinline__ typename Dt<T>::frag value_frag(const T* lds, uint32_
 template <>
 __device__ __forceinline__ v8b value_frag<__bf16>(const __bf16* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g) {
     // keys 4 g .. 4 g + 3 of either key tile, latent element 16 sl + qi: two transposing reads
-    const uint32_t s = sl >> 1, r = 4 * g + (qi >> 2), slot = ((sl & 1u) * 2 + ((qi & 3u) >> 1)) * 16 + r;
+    const uint32_t s = sl >> 1, r = 4 * g + (qi >> 2), slot = staged_slot(r, (sl & 1u) * 2 + ((qi & 3u) >> 1));
     const _Float16* a = reinterpret_cast<const _Float16*>(lds) + (size_t)s * 512 + slot * 8 + (qi & 1u) * 4;
     const v4b t0 = __builtin_bit_cast(v4b, lds_read_tr16(a)), t1 = __builtin_bit_cast(v4b, lds_read_tr16(a + (size_t)ks * 512));
     return (v8b){t0[0], t0[1], t0[2], t0[3], t1[0], t1[1], t1[2], t1[3]};
@@ -108,9 +118,10 @@ __device__ __forceinline__ v8b value_frag<__bf16>(const __bf16* lds, uint32_t ks
 template <>
 __device__ __forceinline__ v8f value_frag<float>(const float* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g) {
     const uint32_t d = 16 * sl + qi, e = d & 7u;
-    const float* a = lds + (size_t)(d >> 5) * 512 + (e >> 2) * 256 + (((d & 31u) >> 3) * 16 + 4 * g) * 4 + (e & 3u);
+    // (the slots of rows 4 g .. 4 g + 3 lie four apart: they share r >> 2)
+    const float* a = lds + (size_t)(d >> 5) * 512 + (e >> 2) * 256 + staged_slot(4 * g, (d & 31u) >> 3) * 4 + (e & 3u);
     const float* b = a + (size_t)ks * 512;
-    return (v8f){a[0], a[4], a[8], a[12], b[0], b[4], b[8], b[12]};
+    return (v8f){a[0], a[16], a[32], a[48], b[0], b[16], b[32], b[48]};
 }
 
 template <typename T, int NT, int KS>
@@ -124,7 +135,7 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
     const uint32_t split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
     const uint32_t pos = row_pos(p.rows, m), seq = row_seq(p.rows, m), chunk = 32 * nw, n_chunks = pos / chunk + 1;
     if (split >= min(p.n_splits, n_chunks)) return;
-    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16;
+    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, slot = staged_slot(qi, g);
     T* lds = reinterpret_cast<T*>(smem) + (size_t)wave * 2 * ks * 512;
     const T* cache = reinterpret_cast<const T*>(p.cache);
 
@@ -145,19 +156,19 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
         const uint32_t key0 = ch * chunk + wave * 32;
         if (key0 > pos) break;  // (only the last chunk can end before this wave's keys)
         // rows past the newest position repeat it; their scores are masked
-        const T* r0 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + qi, pos)) * p.ld + 8 * g;
-        const T* r1 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + 16 + qi, pos)) * p.ld + 8 * g;
+        const T* r0 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + stage_row(lane), pos)) * p.ld + 8 * stage_col(lane);
+        const T* r1 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + 16 + stage_row(lane), pos)) * p.ld + 8 * stage_col(lane);
         for (uint32_t s = 0; s < ks; s++) {
-            copy_row8_to_unit(r0 + 32 * s, lds + (size_t)s * 512);
-            copy_row8_to_unit(r1 + 32 * s, lds + (size_t)(ks + s) * 512);
+            stage_unit(r0 + 32 * s, lds + (size_t)s * 512);
+            stage_unit(r1 + 32 * s, lds + (size_t)(ks + s) * 512);
         }
         wait_lds_copies();
         v4f s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < KS; s++)
             if ((uint32_t)s < ks) {
-                s0 = mfma32(load_unit(lds + (size_t)s * 512, lane), q[s], s0);
-                s1 = mfma32(load_unit(lds + (size_t)(ks + s) * 512, lane), q[s], s1);
+                s0 = mfma32(load_staged(lds + (size_t)s * 512, slot), q[s], s0);
+                s1 = mfma32(load_staged(lds + (size_t)(ks + s) * 512, slot), q[s], s1);
             }
         float sv[8], mx = -INFINITY;
 #pragma unroll
@@ -204,8 +215,8 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
     for (int i = 0; i < NT; i++)
         if ((uint32_t)i < nt) *reinterpret_cast<v4f*>(mine + qi * d.rank_p + 16 * i + 4 * g) = O[i] * f;
     __syncthreads();
-    const size_t slot = ((size_t)m * gridDim.y + ht) * p.n_splits + split;
-    float* po = p.part_o + slot * 16 * d.rank_p;
+    const size_t part = ((size_t)m * gridDim.y + ht) * p.n_splits + split;
+    float* po = p.part_o + part * 16 * d.rank_p;
     const float* all = reinterpret_cast<const float*>(smem);
     for (uint32_t i = tid * 4; i < 16 * d.rank_p; i += blockDim.x * 4) {
         v4f y = *reinterpret_cast<const v4f*>(all + i);
@@ -218,18 +229,19 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
             const float mw = wave_ml[w][tid][0];
             if (mw != -INFINITY) l += wave_ml[w][tid][1] * exp_of<T>(mw - M);
         }
-        p.part_ml[slot * 32 + tid * 2] = M;
-        p.part_ml[slot * 32 + tid * 2 + 1] = l;
+        p.part_ml[part * 32 + tid * 2] = M;
+        p.part_ml[part * 32 + tid * 2 + 1] = l;
     }
 }
 
 // ---------------------------------------------------------------------------
 // Merge of one head's splits - the sink joins the denominator here, once - and the value product W_uv (sum p c).
-// Grid (head, token row), 4 waves.
+// Grid (head, token row), 8 waves, a tile of 16 value rows each; UN units of the product's weights are in flight per wave.
 // ---------------------------------------------------------------------------
 template <typename T>
-__global__ __launch_bounds__(256) void latent_merge_kernel(OxbLatentParams p, uint32_t chunk) {
+__global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, uint32_t chunk) {
     typedef typename Dt<T>::frag frag;
+    constexpr int UN = 8;
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
     __shared__ float wgt[OXB_LATENT_MAX_SPLITS];
     const OxbLatentDims& d = p.d;
@@ -239,6 +251,12 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(OxbLatentParams p, ui
     const uint32_t used = min(p.n_splits, row_pos(p.rows, m) / chunk + 1);
     const size_t slot0 = ((size_t)m * n_ht + ht) * p.n_splits;
     const float sink = p.sink[head];
+    const uint32_t nu = p.k_uv / 32, tiles = d.vdim_p / 16;
+    const size_t ts = oxb_tile_stride(p.k_uv, sizeof(T));
+    const T* w_head = reinterpret_cast<const T*>(p.w_uv) + head * tiles * ts;
+    frag a0[UN];   // the wave's first weights travel while the splits are merged
+#pragma unroll
+    for (int i = 0; i < UN; i++) a0[i] = load_unit(w_head + min(wave, tiles - 1) * ts + (size_t)min((uint32_t)i, nu - 1) * 512, lane);
     T* lat = reinterpret_cast<T*>(smem);  // [k_uv]
     {
         // every wave forms the weights (at most two splits per lane); wave 0 leaves them in LDS
@@ -266,21 +284,34 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(OxbLatentParams p, ui
     }
     __syncthreads();
     const float* po = p.part_o + (slot0 * 16 + col) * d.rank_p;
-    for (uint32_t i = tid; i < p.k_uv; i += 256) {
+    for (uint32_t i = tid; i < p.k_uv; i += 512) {
         float y = 0.f;
-        if (i < d.rank_p)
-            for (uint32_t s = 0; s < used; s++) y = fmaf(wgt[s], po[(size_t)s * 16 * d.rank_p + i], y);
+        if (i < d.rank_p) {
+            for (uint32_t s0 = 0; s0 < used; s0 += 8) {
+                float v[8];
+#pragma unroll
+                for (int k = 0; k < 8; k++) v[k] = po[(size_t)min(s0 + k, used - 1) * 16 * d.rank_p + i];
+#pragma unroll
+                for (int k = 0; k < 8; k++) y = fmaf(s0 + k < used ? wgt[s0 + k] : 0.f, v[k], y);
+            }
+        }
         lat[i] = (T)y;
     }
     __syncthreads();
-    const uint32_t nu = p.k_uv / 32, tiles = d.vdim_p / 16;
     T* out = reinterpret_cast<T*>(p.out) + (size_t)m * p.ld_out;
-    for (uint32_t t = wave; t < tiles; t += 4) {
-        const T* w = reinterpret_cast<const T*>(p.w_uv) + (size_t)(head * tiles + t) * nu * 512;
+    for (uint32_t t = wave; t < tiles; t += 8) {
+        const T* w = w_head + t * ts;
         v4f acc = {0.f, 0.f, 0.f, 0.f};
-        for (uint32_t u = 0; u < nu; u++) {
-            const frag b = c == 0 ? load_row8(lat + 32 * u + 8 * g) : zero_frag((const T*)nullptr);
-            acc = mfma32(load_unit(w + (size_t)u * 512, lane), b, acc);
+        for (uint32_t u0 = 0; u0 < nu; u0 += UN) {
+            if (u0 || t != wave) {
+#pragma unroll
+                for (int i = 0; i < UN; i++) a0[i] = load_unit(w + (size_t)min(u0 + i, nu - 1) * 512, lane);
+            }
+#pragma unroll
+            for (int i = 0; i < UN; i++) {
+                const frag b = c == 0 && u0 + i < nu ? load_row8(lat + 32 * min(u0 + i, nu - 1) + 8 * g) : zero_frag((const T*)nullptr);
+                acc = mfma32(a0[i], b, acc);
+            }
         }
         if (c == 0) {
             typename Dt<T>::quad o;
@@ -290,7 +321,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(OxbLatentParams p, ui
         }
     }
     if (head == d.heads - 1)
-        for (uint32_t i = d.heads * d.vdim_p + tid; i < p.ld_out; i += 256) out[i] = (T)0.f;
+        for (uint32_t i = d.heads * d.vdim_p + tid; i < p.ld_out; i += 512) out[i] = (T)0.f;
 }
 
 // ---------------------------------------------------------------------------
@@ -311,7 +342,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
     const uint32_t qb = n_qb - 1 - blockIdx.x / d.heads, head = blockIdx.x % d.heads;   // long (late) query blocks first
     const uint32_t kd = d.dim_p / 32, kr = d.rot_p / 32, ks = kd + kr, vt = d.vdim_p / 16;
     const uint32_t kl = d.rank_p + d.rot_p, qh = d.dim_p + d.rot_p, half = d.rot_dims >> 1;
-    const uint32_t units = 2 * ks + vt;
+    const uint32_t units = 2 * ks + vt, slot = staged_slot(qi, g), sr = stage_row(lane), sc = 8 * stage_col(lane);
     T* lds = reinterpret_cast<T*>(smem);
     const T* cache = reinterpret_cast<const T*>(p.cache);
     const uint32_t q_last = min((qb + 1) * 64 * QT, p.rows.m) - 1;
@@ -360,13 +391,13 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
             const T* src;
             if (un < 2 * ks) {
                 const uint32_t t = un >= ks ? 1u : 0u, s = un - t * ks;
-                const uint32_t key = min(key0 + 8 * (qi >> 2) + 4 * t + (qi & 3u), kv_len - 1);
-                src = s < kd ? reinterpret_cast<const T*>(p.k_exp) + (size_t)key * p.ld_k + head * d.dim_p + 32 * s + 8 * g
-                             : cache + kv_row(p.kv, p.rows.seq0, 0, 0, key) * kl + d.rank_p + 32 * (s - kd) + 8 * g;
+                const uint32_t key = min(key0 + 8 * (sr >> 2) + 4 * t + (sr & 3u), kv_len - 1);
+                src = s < kd ? reinterpret_cast<const T*>(p.k_exp) + (size_t)key * p.ld_k + head * d.dim_p + 32 * s + sc
+                             : cache + kv_row(p.kv, p.rows.seq0, 0, 0, key) * kl + d.rank_p + 32 * (s - kd) + sc;
             } else {
-                src = reinterpret_cast<const T*>(p.v_exp_t) + (size_t)(head * d.vdim_p + (un - 2 * ks) * 16 + qi) * p.ld_v + key0 + 8 * g;
+                src = reinterpret_cast<const T*>(p.v_exp_t) + (size_t)(head * d.vdim_p + (un - 2 * ks) * 16 + sr) * p.ld_v + key0 + sc;
             }
-            copy_row8_to_unit(src, base + (size_t)un * 512);
+            stage_unit(src, base + (size_t)un * 512);
         }
     };
     stage(0, 0);
@@ -383,7 +414,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
 #pragma unroll
         for (int s = 0; s < KS; s++)
             if ((uint32_t)s < ks) {
-                const frag k0 = load_unit(kb + (size_t)s * 512, lane), k1 = load_unit(kb + (size_t)(ks + s) * 512, lane);
+                const frag k0 = load_staged(kb + (size_t)s * 512, slot), k1 = load_staged(kb + (size_t)(ks + s) * 512, slot);
 #pragma unroll
                 for (int t = 0; t < QT; t++) {
                     s0[t] = mfma32(k0, q[t][s], s0[t]);
@@ -426,7 +457,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
 #pragma unroll
         for (int i = 0; i < VT; i++)
             if ((uint32_t)i < vt) {
-                const frag a = load_unit(vb + (size_t)i * 512, lane);
+                const frag a = load_staged(vb + (size_t)i * 512, slot);
 #pragma unroll
                 for (int t = 0; t < QT; t++) {
                     O[t][i] = mfma32(a, hi[t], O[t][i]);
@@ -496,9 +527,10 @@ hipError_t oxb_launch_latent_store(const OxbLatentParams& p, bool absorb, int dt
     OxbLatentParams q = p;
     if (!absorb) q.q_abs = nullptr;
     const uint32_t tph = p.d.rank_p / 16, n_abs = absorb ? (p.d.heads * tph + 3) / 4 : 0;
-    const dim3 grid(n_abs + 16, (p.rows.m + 15) / 16);
-    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_store_kernel<__bf16>), grid, dim3(256), 0, st, q, n_abs, tph);
-    else hipLaunchKernelGGL((latent_store_kernel<float>), grid, dim3(256), 0, st, q, n_abs, tph);
+    const uint32_t per_row = absorb ? 1 + (p.d.heads * p.d.rot_p + 1023) / 1024 : 1;
+    const dim3 grid(n_abs + per_row * (p.rows.m < 16 ? p.rows.m : 16), (p.rows.m + 15) / 16);
+    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_store_kernel<__bf16>), grid, dim3(256), 0, st, q, n_abs, tph, per_row);
+    else hipLaunchKernelGGL((latent_store_kernel<float>), grid, dim3(256), 0, st, q, n_abs, tph, per_row);
     return hipGetLastError();
 }
 
@@ -531,8 +563,8 @@ hipError_t oxb_launch_latent_merge(const OxbLatentParams& p, int dt, hipStream_t
         return hipErrorInvalidValue;
     const dim3 grid(p.d.heads, p.rows.m);
     const uint32_t lds = p.k_uv * oxb_dt_bytes(dt), chunk = oxb_latent_chunk(p.d, dt);
-    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_merge_kernel<__bf16>), grid, dim3(256), lds, st, p, chunk);
-    else hipLaunchKernelGGL((latent_merge_kernel<float>), grid, dim3(256), lds, st, p, chunk);
+    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_merge_kernel<__bf16>), grid, dim3(512), lds, st, p, chunk);
+    else hipLaunchKernelGGL((latent_merge_kernel<float>), grid, dim3(512), lds, st, p, chunk);
     return hipGetLastError();
 }
 

@@ -159,7 +159,7 @@ static int feed_next(const Program& p, int i, const ActBuf& a, OxbEpilogue* e) {
     const ProgramNorm& n = next < p.runs.size() ? p.layers[p.runs[next].r.layer].norm1 : p.final_norm;
     e->out_t = a.act;
     e->ld_t = p.ld_act;
-    e->fill = p.ld_act;
+    e->fill = oxb_dense_pad(w);
     e->norm = OXB_NORM_DYT;
     e->nw = vec_ptr(n.w, w, "norm", &rc);
     if (!rc) e->nb = vec_ptr(n.b, w, "norm", &rc);
@@ -206,16 +206,17 @@ static int expand(Model& m, const ProgramLayer& l, OxbLatentParams& lp, uint32_t
     q.k_pad = uk->k_pad;
     q.e = epilogue(l.d.heads * l.d.dim_p);
     q.e.out_t = p.k_exp.ptr;
-    q.e.ld_t = q.e.fill = uk->n_pad;
+    q.e.ld_t = oxb_act_ld(uk->n_pad);
+    q.e.fill = uk->n_pad;
     OXB_TRY_HIP(oxb_launch_dense(q, p.dt, g_rt.n_cus, g_rt.stream), "kernel launch failed: key product");
     lp.k_exp = p.k_exp.ptr;
-    lp.ld_k = uk->n_pad;
+    lp.ld_k = q.e.ld_t;
     q.w = uv->d;
     q.n_pad = uv->n_pad;
     q.k_pad = uv->k_pad;
     q.e = epilogue(l.d.heads * l.d.vdim_p);
     q.e.out_t = p.v_exp.ptr;
-    q.e.ld_t = (kv_len + 127u) / 128u * 128u;
+    q.e.ld_t = oxb_act_ld((kv_len + 127u) / 128u * 128u);
     OXB_TRY_HIP(oxb_launch_dense_gemm_t(q, p.dt, g_rt.n_cus, g_rt.stream), "kernel launch failed: value product");
     lp.v_exp_t = p.v_exp.ptr;
     lp.ld_v = q.e.ld_t;
@@ -232,7 +233,7 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
     {
         OxbEpilogue e = epilogue(w);
         OXB_TRY(feed_next(p, -1, a, &e));
-        OXB_TRY_HIP(oxb_launch_stream_enter(x, w, M, p.loop_in ? a.cat : nullptr, p.ld_cat, w, p.ld_cat, e, p.dt, st), "kernel launch failed: stream_enter");
+        OXB_TRY_HIP(oxb_launch_stream_enter(x, w, M, p.loop_in ? a.cat : nullptr, p.ld_cat, w, oxb_dense_pad(2 * w), e, p.dt, st), "kernel launch failed: stream_enter");
     }
     for (size_t i = 0; i < p.runs.size(); i++) {
         const ProgramRun& run = p.runs[i];
@@ -246,7 +247,8 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
             e.out32 = x;
             e.ld32 = w;
             e.out_t = a.act;
-            e.ld_t = e.fill = p.ld_act;
+            e.ld_t = p.ld_act;
+            e.fill = oxb_dense_pad(w);
             e.norm = OXB_NORM_DYT;
             e.alpha = l.norm1.alpha;
             OXB_TRY(product(p, p.loop_in, a.cat, p.ld_cat, M, e, "kernel launch failed: loop input product"));
@@ -283,7 +285,7 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
         lp.part_ml = p.part_ml;
         lp.n_splits = decode_splits(m, l.d, p.dt, M);
         lp.out = a.attn;
-        lp.ld_out = oxb_dense_pad(l.d.heads * l.d.vdim_p);
+        lp.ld_out = oxb_act_ld(l.d.heads * l.d.vdim_p);
         OXB_TRY_HIP(oxb_launch_latent_store(lp, absorbed, p.dt, st), "kernel launch failed: latent_store");
         if (absorbed) {
             OXB_TRY_HIP(oxb_launch_latent_decode(lp, p.dt, st), "kernel launch failed: latent_decode");
@@ -297,7 +299,8 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
         e.ld32 = w;
         if (l.has_mlp) {
             e.out_t = a.act;
-            e.ld_t = e.fill = p.ld_act;
+            e.ld_t = p.ld_act;
+            e.fill = oxb_dense_pad(w);
             e.norm = OXB_NORM_DYT;
             e.nw = vec_ptr(l.norm2.w, w, "norm2", &rc);
             e.nb = rc ? nullptr : vec_ptr(l.norm2.b, w, "norm2", &rc);
@@ -311,7 +314,8 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
         OxbEpilogue eu = epilogue(l.ff);
         eu.act = OXB_ACT_GELU_TANH;
         eu.out_t = a.mid;
-        eu.ld_t = eu.fill = oxb_dense_pad(l.ff);
+        eu.ld_t = oxb_act_ld(l.ff);
+        eu.fill = oxb_dense_pad(l.ff);
         OXB_TRY(product(p, l.up, a.act, p.ld_act, M, eu, "kernel launch failed: up product"));
         OxbEpilogue ed = epilogue(w);
         ed.resid = ed.out32 = x;
@@ -411,13 +415,13 @@ int program_prefill_buffers(Model& m, uint32_t rows, uint32_t pos_start) {
     const size_t keys = ((size_t)pos_start + rows + 127) / 128 * 128, es = oxb_dt_bytes(p.dt);
     size_t k = 0, v = 0;
     for (const ProgramLayer& l : p.layers) {
-        const size_t nk = oxb_dense_pad(l.d.heads * l.d.dim_p), nv = (size_t)l.d.heads * l.d.vdim_p;
+        const size_t nk = oxb_act_ld(l.d.heads * l.d.dim_p), nv = (size_t)l.d.heads * l.d.vdim_p;
         if (nk > k) k = nk;
         if (nv > v) v = nv;
     }
     OXB_TRY_HIP(hipStreamSynchronize(g_rt.stream), "synchronize");
     OXB_TRY(p.k_exp.ensure(keys * k * es));
-    OXB_TRY(p.v_exp.ensure(keys * v * es));
+    OXB_TRY(p.v_exp.ensure((size_t)oxb_act_ld((uint32_t)keys) * v * es));
     return OXB_HIP_OK;
 }
 
@@ -511,7 +515,7 @@ struct Loader {
             int64_t* d_ro = (int64_t*)off.ptr;
             if (e == hipSuccess) e = hipMemcpy(d_ro, ro.data(), (size_t)n_pad * 8, hipMemcpyHostToDevice);
             if (e == hipSuccess) e = hipMemcpy(d_ro + n_pad, co.data(), (size_t)k_pad * 8, hipMemcpyHostToDevice);
-            if (e == hipSuccess && hipMalloc(&w.d, (size_t)n_pad * k_pad * oxb_dt_bytes(dt)) != hipSuccess)
+            if (e == hipSuccess && hipMalloc(&w.d, (n_pad / 16) * oxb_tile_stride(k_pad, oxb_dt_bytes(dt)) * oxb_dt_bytes(dt)) != hipSuccess)
                 rc = fail(OXB_HIP_OUT_OF_MEMORY, "out of device memory: a %u x %u matrix on device %d", n_pad, k_pad, g_rt.device);
             if (!rc && e == hipSuccess) e = oxb_launch_dense_pack(raw.ptr, src[0]->type, d_ro, d_ro + n_pad, n_pad, k_pad, dt, w.d, g_rt.stream);
             if (e == hipSuccess) e = hipStreamSynchronize(g_rt.stream);
@@ -650,17 +654,17 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
         OXB_TRY(load_layer(ld, p, c.layers[i], "l" + std::to_string(i) + ".", &p.layers[i]));
         OXB_TRY(rope_table(m, p, c.layers[i].mixer.rot_base, c.layers[i].mixer.rot_dims, &p.layers[i].rope));
     }
-    p.ld_act = oxb_dense_pad(w);
-    p.ld_cat = oxb_dense_pad(2 * w);
+    p.ld_act = oxb_act_ld(w);
+    p.ld_cat = oxb_act_ld(2 * w);
     const size_t R = m.d.batch > OXB_PROGRAM_SHORT ? m.d.batch : OXB_PROGRAM_SHORT;
     size_t part = 0, ml = 0;
     for (const ProgramLayer& l : p.layers) {
         const OxbLatentDims& d = l.d;
         auto grow = [](uint32_t* v, uint32_t n) { if (n > *v) *v = n; };
         grow(&p.ld_qkv, oxb_dense_pad(l.n_qkv));
-        grow(&p.ld_attn, oxb_dense_pad(d.heads * d.vdim_p));
+        grow(&p.ld_attn, oxb_act_ld(d.heads * d.vdim_p));
         grow(&p.n_q_abs, d.heads * (d.rank_p + d.rot_p));
-        if (l.has_mlp) grow(&p.ld_mid, oxb_dense_pad(l.ff));
+        if (l.has_mlp) grow(&p.ld_mid, oxb_act_ld(l.ff));
         const size_t tiles = (d.heads + 15) / 16;
         for (uint32_t r = 1; r <= R; r++) {
             const size_t slots = (size_t)r * tiles * decode_splits(m, d, dt, r);

@@ -18,25 +18,25 @@
 __global__ __launch_bounds__(256) void embedding_gather_kernel(const uint8_t* __restrict__ table, int type, uint32_t vocab,
                                                                 uint32_t h, const uint32_t* __restrict__ ids,
                                                                 float* __restrict__ out) {
-    const uint32_t row = blockIdx.x, id = ids[row];
+    const uint32_t row = blockIdx.x, id = ids[row], i0 = blockIdx.y * 1024 + threadIdx.x, i1 = min(h, (blockIdx.y + 1) * 1024);
     float* o = out + (size_t)row * h;
     if (id >= vocab) {
-        for (uint32_t i = threadIdx.x; i < h; i += 256) o[i] = __int_as_float(0x7FC00000);
+        for (uint32_t i = i0; i < i1; i += 256) o[i] = __int_as_float(0x7FC00000);
         return;
     }
     if (type == 0) {
         const float* src = reinterpret_cast<const float*>(table) + (size_t)id * h;
-        for (uint32_t i = threadIdx.x; i < h; i += 256) o[i] = src[i];
+        for (uint32_t i = i0; i < i1; i += 256) o[i] = src[i];
     } else if (type == 1) {
         const __half* src = reinterpret_cast<const __half*>(table) + (size_t)id * h;
-        for (uint32_t i = threadIdx.x; i < h; i += 256) o[i] = __half2float(src[i]);
+        for (uint32_t i = i0; i < i1; i += 256) o[i] = __half2float(src[i]);
     } else if (type == 30) {
         const uint16_t* src = reinterpret_cast<const uint16_t*>(table) + (size_t)id * h;
-        for (uint32_t i = threadIdx.x; i < h; i += 256) o[i] = __uint_as_float((uint32_t)src[i] << 16);
+        for (uint32_t i = i0; i < i1; i += 256) o[i] = __uint_as_float((uint32_t)src[i] << 16);
     } else {
         const uint32_t bb = type == 41 ? 18u : 34u;
         const uint8_t* src = table + (size_t)id * (h / 128u) * bb;
-        for (uint32_t i = threadIdx.x; i < h; i += 256) {
+        for (uint32_t i = i0; i < i1; i += 256) {
             const uint8_t* blk = src + (size_t)(i >> 7) * bb;
             const uint32_t j = i & 127u;
             float v;
@@ -630,7 +630,7 @@ hipError_t oxb_launch_embedding_gather(const void* d_table, int gguf_type, uint3
                                        uint32_t n, float* d_out, hipStream_t st) {
     if (n == 0) return hipSuccess;
     if ((gguf_type != 0 && gguf_type != 1 && gguf_type != 30 && gguf_type != 41 && gguf_type != 42) || (gguf_type >= 41 && h % 128u)) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(embedding_gather_kernel, dim3(n), dim3(256), 0, st, static_cast<const uint8_t*>(d_table), gguf_type, vocab, h,
+    hipLaunchKernelGGL(embedding_gather_kernel, dim3(n, (h + 1023) / 1024), dim3(256), 0, st, static_cast<const uint8_t*>(d_table), gguf_type, vocab, h,
                        d_ids, d_out);
     return hipGetLastError();
 }
