@@ -97,9 +97,28 @@ template <typename T> __device__ __forceinline__ float tanh_of(float z) {
 template <typename T> __device__ __forceinline__ float gelu_tanh_of(float z) {
     return 0.5f * z * (1.0f + tanh_of<T>(0.79788456080286536f * (z + 0.044715f * z * z * z)));
 }
-template <typename T> __device__ __forceinline__ float exp_of(float z) {  // e^z, z <= 0 in every use
-    if constexpr (Dt<T>::is_f32) return expf(z);
-    return __builtin_amdgcn_exp2f(z * 1.4426950408889634f);
+// 2^z, z <= 0 or little above in every use.
+template <typename T> __device__ __forceinline__ float exp2_of(float z) {
+    if constexpr (Dt<T>::is_f32) return exp2f(z);
+    return __builtin_amdgcn_exp2f(z);
+}
+// Eight fp32 weights as a matrix-core operand.  bf16: v = hi + lo, hi the upper half of v's bits (exact), lo the rounded
+// rest: 16 bits of the weight in two operands.
+__device__ __forceinline__ void split_hi_lo(const float (&v)[8], v8b& hi, v8b& lo) {
+    typedef uint32_t v4w __attribute__((ext_vector_type(4)));
+    v4w h;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const uint32_t a = __float_as_uint(v[2 * i]), b = __float_as_uint(v[2 * i + 1]);
+        h[i] = __builtin_amdgcn_perm(b, a, 0x07060302u);
+        lo[2 * i] = (__bf16)(v[2 * i] - __uint_as_float(a & 0xFFFF0000u));
+        lo[2 * i + 1] = (__bf16)(v[2 * i + 1] - __uint_as_float(b & 0xFFFF0000u));
+    }
+    hi = __builtin_bit_cast(v8b, h);
+}
+__device__ __forceinline__ void split_hi_lo(const float (&v)[8], v8f& hi, v8f& lo) {
+    hi = (v8f){v[0], v[1], v[2], v[3], v[4], v[5], v[6], v[7]};
+    lo = hi;   // (not used)
 }
 
 // The residual's four values for outputs y[m][n0 .. n0 + 3], requested ahead of the arithmetic (zeros where epilogue4 fetches

@@ -272,18 +272,16 @@ static hipError_t launch_gemm(const OxbDenseParams& p, hipStream_t st) {
     return hipGetLastError();
 }
 
-// Rounds of workgroups over the CUs (two resident per CU) x what one costs: the smallest estimate wins, larger tiles first
-// among equals.
+// Tile choice by measured cost (us for K = 4096): of a workgroup alone on its CU, and per workgroup where a CU gets several.
 template <typename T, bool SWAP>
 static hipError_t pick_gemm(const OxbDenseParams& p, uint32_t n_cus, hipStream_t st) {
-    struct { int rt, ct; double mac_cost; } const opt[] = {{4, 8, 1.0}, {2, 8, 1.15}, {4, 4, 1.2}, {2, 4, 1.4}, {1, 8, 1.5}, {1, 4, 1.8}};
+    struct { uint32_t rt, ct; double alone, each; } const opt[] = {{4, 8, 60, 64}, {2, 8, 42, 37.5}, {4, 4, 38, 38}, {2, 4, 28, 23.5}, {1, 8, 41, 28}, {1, 4, 24, 19}};
     int best = -1;
     double best_cost = 0;
     for (int i = 0; i < 6; i++) {
-        const double wgs = (double)((p.m + 16 * opt[i].ct - 1) / (16 * opt[i].ct)) * ((p.n_pad + 64 * opt[i].rt - 1) / (64 * opt[i].rt));
-        const double slots = n_cus, rounds = wgs <= slots ? 1.0 : (double)(uint64_t)((wgs + slots - 1) / slots);
-        const double cost = rounds * opt[i].rt * opt[i].ct * opt[i].mac_cost;
         if (Dt<T>::is_f32 && opt[i].ct == 8) continue;   // (fp32 stages are twice as large)
+        const uint64_t wgs = (uint64_t)((p.m + 16 * opt[i].ct - 1) / (16 * opt[i].ct)) * ((p.n_pad + 64 * opt[i].rt - 1) / (64 * opt[i].rt));
+        const double busy = (double)((wgs + n_cus - 1) / n_cus) * opt[i].each, cost = busy > opt[i].alone ? busy : opt[i].alone;
         if (best < 0 || cost < best_cost) best = i, best_cost = cost;
     }
     if constexpr (!Dt<T>::is_f32) {

@@ -127,6 +127,7 @@ __device__ __forceinline__ v8f value_frag<float>(const float* lds, uint32_t ks, 
 template <typename T, int NT, int KS>
 __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p) {
     typedef typename Dt<T>::frag frag;
+    constexpr int G = 4;   // k units / accumulator tiles per step: sizes round up to whole steps (zero queries, unused tiles)
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
     __shared__ float wave_ml[4][16][2];
     const OxbLatentDims& d = p.d;
@@ -138,23 +139,8 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
     const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, slot = staged_slot(qi, g);
     T* lds = reinterpret_cast<T*>(smem) + (size_t)wave * 2 * ks * 512;
     const T* cache = reinterpret_cast<const T*>(p.cache);
-
-    frag q[KS];
-    {
-        const uint32_t head = ht * 16 + qi;
-        const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(head, d.heads - 1)) * p.ld + 8 * g;
-#pragma unroll
-        for (int s = 0; s < KS; s++)
-            if ((uint32_t)s < ks) q[s] = load_row8(src + 32 * s);
-    }
-    v4f O[NT];
-#pragma unroll
-    for (int i = 0; i < NT; i++) O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
-    float m_run = -INFINITY, l_run = 0.f;
-
-    for (uint32_t ch = split; ch < n_chunks; ch += p.n_splits) {
-        const uint32_t key0 = ch * chunk + wave * 32;
-        if (key0 > pos) break;  // (only the last chunk can end before this wave's keys)
+    const float c2 = d.scale * 1.4426950408889634f;   // scores in units of log2(e): a probability is one exponential of one fma
+    auto request = [&](uint32_t key0) {
         // rows past the newest position repeat it; their scores are masked
         const T* r0 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + stage_row(lane), pos)) * p.ld + 8 * stage_col(lane);
         const T* r1 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + 16 + stage_row(lane), pos)) * p.ld + 8 * stage_col(lane);
@@ -162,54 +148,88 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
             stage_unit(r0 + 32 * s, lds + (size_t)s * 512);
             stage_unit(r1 + 32 * s, lds + (size_t)(ks + s) * 512);
         }
+    };
+    const uint32_t first = split * chunk + wave * 32;
+    if (first <= pos) request(first);
+
+    frag q[KS];
+    {
+        const uint32_t head = ht * 16 + qi;
+        const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(head, d.heads - 1)) * p.ld + 8 * g;
+#pragma unroll
+        for (int s = 0; s < KS; s++) {
+            q[s] = load_row8(src + 32 * min((uint32_t)s, ks - 1));
+            if ((uint32_t)s >= ks) q[s] = zero_frag((const T*)nullptr);
+        }
+    }
+    v4f O[NT];
+#pragma unroll
+    for (int i = 0; i < NT; i++) O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;   // maximum (times c2) and this lane's share of the sum
+
+    for (uint32_t ch = split; ch < n_chunks; ch += p.n_splits) {
+        const uint32_t key0 = ch * chunk + wave * 32;
+        if (key0 > pos) break;  // (only the last chunk can end before this wave's keys)
+        if (ch != split) request(key0);
         wait_lds_copies();
         v4f s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < KS; s++)
-            if ((uint32_t)s < ks) {
-                s0 = mfma32(load_staged(lds + (size_t)s * 512, slot), q[s], s0);
-                s1 = mfma32(load_staged(lds + (size_t)(ks + s) * 512, slot), q[s], s1);
+        for (int s4 = 0; s4 < KS; s4 += G)
+            if ((uint32_t)s4 < ks) {
+#pragma unroll
+                for (int j = 0; j < G; j++)
+                    if (s4 + j < KS) {
+                        const uint32_t s = min((uint32_t)(s4 + j), ks - 1);
+                        s0 = mfma32(load_staged(lds + (size_t)s * 512, slot), q[s4 + j], s0);
+                        s1 = mfma32(load_staged(lds + (size_t)(ks + s) * 512, slot), q[s4 + j], s1);
+                    }
             }
         float sv[8], mx = -INFINITY;
 #pragma unroll
         for (int v = 0; v < 4; v++) {
             const uint32_t k = key0 + 4 * g + v;
-            sv[v] = k <= pos ? s0[v] * d.scale : -INFINITY;
-            sv[4 + v] = k + 16 <= pos ? s1[v] * d.scale : -INFINITY;
+            sv[v] = k <= pos ? s0[v] * c2 : -INFINITY;
+            sv[4 + v] = k + 16 <= pos ? s1[v] * c2 : -INFINITY;
             mx = fmaxf(mx, fmaxf(sv[v], sv[4 + v]));
         }
         mx = max_rows4(mx);  // finite: key0 <= pos
-        const float m_new = fmaxf(m_run, mx), alpha = exp_of<T>(m_run - m_new);
-        float sum = 0.f;
+        const float m_new = fmaxf(m_run, mx), alpha = exp2_of<T>(m_run - m_new);
+        l_run *= alpha;
         frag hi, lo;
+        float pe[8];
 #pragma unroll
         for (int e = 0; e < 8; e++) {
-            const float pe = exp_of<T>(sv[e] - m_new);
-            sum += pe;
-            hi[e] = (T)pe;
-            if constexpr (!Dt<T>::is_f32) lo[e] = (T)(pe - (float)hi[e]);
+            pe[e] = exp2_of<T>(sv[e] - m_new);
+            l_run += pe[e];
         }
-        l_run = l_run * alpha + sum_rows4(sum);
+        split_hi_lo(pe, hi, lo);
         const bool moved = __any(m_new != m_run);
         m_run = m_new;
+        if (moved) {
 #pragma unroll
-        for (int i = 0; i < NT; i++)
-            if ((uint32_t)i < nt) {
-                const frag a = value_frag<T>(lds, ks, i, qi, g);
-                if (moved) O[i] *= alpha;
-                O[i] = mfma32(a, hi, O[i]);
-                if constexpr (!Dt<T>::is_f32) O[i] = mfma32(a, lo, O[i]);
+            for (int i = 0; i < NT; i++) O[i] *= alpha;
+        }
+#pragma unroll
+        for (int i4 = 0; i4 < NT; i4 += G)
+            if ((uint32_t)i4 < nt) {   // (nt is even: at most two tiles too many, and they read the first rotated unit)
+#pragma unroll
+                for (int j = 0; j < G; j++) {
+                    const frag a = value_frag<T>(lds, ks, i4 + j, qi, g);
+                    O[i4 + j] = mfma32(a, hi, O[i4 + j]);
+                    if constexpr (!Dt<T>::is_f32) O[i4 + j] = mfma32(a, lo, O[i4 + j]);
+                }
             }
-        // the LDS reads above are complete (their results are in use) before the next copies overwrite the rows
+        // the LDS reads above are complete before the next copies overwrite the rows
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     }
+    l_run = sum_rows4(l_run);
 
     // the waves' results: common maximum, sums in wave order
     if (g == 0) wave_ml[wave][qi][0] = m_run, wave_ml[wave][qi][1] = l_run;
     __syncthreads();
     float M = -INFINITY;
     for (uint32_t w = 0; w < nw; w++) M = fmaxf(M, wave_ml[w][qi][0]);
-    const float f = m_run == -INFINITY ? 0.f : exp_of<T>(m_run - M);
+    const float f = m_run == -INFINITY ? 0.f : exp2_of<T>(m_run - M);
     float* mine = reinterpret_cast<float*>(smem) + (size_t)wave * 16 * d.rank_p;   // (every wave is done with its rows)
 #pragma unroll
     for (int i = 0; i < NT; i++)
@@ -227,7 +247,7 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
         float l = 0.f;
         for (uint32_t w = 0; w < nw; w++) {
             const float mw = wave_ml[w][tid][0];
-            if (mw != -INFINITY) l += wave_ml[w][tid][1] * exp_of<T>(mw - M);
+            if (mw != -INFINITY) l += wave_ml[w][tid][1] * exp2_of<T>(mw - M);
         }
         p.part_ml[part * 32 + tid * 2] = M;
         p.part_ml[part * 32 + tid * 2 + 1] = l;
@@ -250,7 +270,7 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, ui
     const uint32_t head = blockIdx.x, m = blockIdx.y, ht = head / 16, col = head % 16, n_ht = (d.heads + 15) / 16;
     const uint32_t used = min(p.n_splits, row_pos(p.rows, m) / chunk + 1);
     const size_t slot0 = ((size_t)m * n_ht + ht) * p.n_splits;
-    const float sink = p.sink[head];
+    const float sink = p.sink[head] * 1.4426950408889634f;   // (maxima are in units of log2(e))
     const uint32_t nu = p.k_uv / 32, tiles = d.vdim_p / 16;
     const size_t ts = oxb_tile_stride(p.k_uv, sizeof(T));
     const T* w_head = reinterpret_cast<const T*>(p.w_uv) + head * tiles * ts;
@@ -272,10 +292,10 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, ui
         float w[2], L = 0.f;
 #pragma unroll
         for (int i = 0; i < 2; i++) {
-            w[i] = ms[i] == -INFINITY ? 0.f : exp_of<T>(ms[i] - M);
+            w[i] = ms[i] == -INFINITY ? 0.f : exp2_of<T>(ms[i] - M);
             L += w[i] * ls[i];
         }
-        L = wave_sum_f32(L) + exp_of<T>(sink - M);
+        L = wave_sum_f32(L) + exp2_of<T>(sink - M);
         if (wave == 0) {
 #pragma unroll
             for (int i = 0; i < 2; i++)
@@ -332,8 +352,10 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, ui
 // the transposed values are read, 16 bytes per lane.
 // ---------------------------------------------------------------------------
 template <typename T, int QT, int KS, int VT>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, uint32_t n_buf) {
+__global__ __launch_bounds__(256, QT == 2 && !Dt<T>::is_f32 ? 2 : 1) void latent_prefill_kernel(OxbLatentParams p, uint32_t n_buf) {
     typedef typename Dt<T>::frag frag;
+    constexpr int NU = (2 * KS + VT + 3) / 4;   // units a wave brings in per block, at most
+    constexpr float kLazy = 8.0f;               // the running maximum follows once it is 2^8 behind
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
     const OxbLatentDims& d = p.d;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4;
@@ -347,6 +369,47 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
     const T* cache = reinterpret_cast<const T*>(p.cache);
     const uint32_t q_last = min((qb + 1) * 64 * QT, p.rows.m) - 1;
     const uint32_t kv_len = p.rows.pos0 + q_last + 1;   // keys the workgroup's last query sees
+    const float c2 = d.scale * 1.4426950408889634f;
+
+    // Unit un of a block: key tile un / ks, k unit un % ks for the first 2 ks; value tile un - 2 ks behind them.  A wave
+    // keeps one running address per unit it brings in.  (Keys past the last one are whatever lies behind it in its buffer or
+    // page, inside the allocation: their scores are masked.)
+    const T* src[NU];
+    uint32_t step[NU], rot_key[NU];             // rot_key: the unit comes out of a paged cache, by key
+    const bool paged = p.kv.page_table != nullptr;
+#pragma unroll
+    for (int i = 0; i < NU; i++) {
+        const uint32_t un = wave + 4 * i;
+        src[i] = nullptr;
+        step[i] = rot_key[i] = 0;
+        if (un >= units) continue;
+        if (un < 2 * ks) {
+            const uint32_t t = un >= ks ? 1u : 0u, s = un - t * ks, key = 8 * (sr >> 2) + 4 * t + (sr & 3u);
+            if (s < kd) {
+                src[i] = reinterpret_cast<const T*>(p.k_exp) + (size_t)key * p.ld_k + head * d.dim_p + 32 * s + sc;
+                step[i] = 32 * p.ld_k;
+            } else {
+                src[i] = cache + d.rank_p + 32 * (s - kd) + sc;
+                if (paged) rot_key[i] = key + 1;
+                else src[i] += kv_row(p.kv, p.rows.seq0, 0, 0, key) * kl, step[i] = 32 * kl;
+            }
+        } else {
+            src[i] = reinterpret_cast<const T*>(p.v_exp_t) + (size_t)(head * d.vdim_p + (un - 2 * ks) * 16 + sr) * p.ld_v + sc;
+            step[i] = 32;
+        }
+    }
+    auto stage = [&](uint32_t key0, uint32_t buf) {
+        T* base = lds + ((size_t)buf * units + wave) * 512;
+#pragma unroll
+        for (int i = 0; i < NU; i++) {
+            if (wave + 4 * i >= units) break;
+            const T* a = src[i];
+            if (paged && rot_key[i]) a += kv_row(p.kv, p.rows.seq0, 0, 0, key0 + rot_key[i] - 1) * kl;
+            stage_unit(a, base + (size_t)i * 2048);
+            src[i] += step[i];
+        }
+    };
+    stage(0, 0);
 
     // queries of this wave, rotated, in operand order; rows past the end repeat the last one and are not stored
     frag q[QT][KS];
@@ -355,18 +418,19 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
     for (int t = 0; t < QT; t++) {
         const uint32_t row = min(qb * 64 * QT + (wave * QT + t) * 16 + qi, p.rows.m - 1);
         qpos[t] = p.rows.pos0 + row;
-        const float* src = p.qkv + (size_t)row * p.ld_qkv + head * qh;
+        const float* qs = p.qkv + (size_t)row * p.ld_qkv + head * qh;
         const float* cs = p.cos_t + (size_t)qpos[t] * half;
         const float* sn = p.sin_t + (size_t)qpos[t] * half;
 #pragma unroll
         for (int s = 0; s < KS; s++) {
+            q[t][s] = zero_frag((const T*)nullptr);
             if ((uint32_t)s >= ks) continue;
             if ((uint32_t)s < kd) {
-                const v8f x = load_row8(src + 32 * s + 8 * g);
+                const v8f x = load_row8(qs + 32 * s + 8 * g);
 #pragma unroll
                 for (int e = 0; e < 8; e++) q[t][s][e] = (T)x[e];
             } else {
-                const float* rp = src + d.dim_p;
+                const float* rp = qs + d.dim_p;
 #pragma unroll
                 for (int e = 0; e < 8; e++) {
                     const uint32_t i = 32 * (s - kd) + 8 * g + e;
@@ -375,32 +439,15 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
             }
         }
     }
+    const uint32_t q_first = p.rows.pos0 + min(qb * 64 * QT + wave * QT * 16, p.rows.m - 1);   // blocks up to here are wholly visible to the wave
     v4f O[QT][VT];
-    float m_run[QT], l_run[QT];
+    float m_run[QT], l_run[QT];   // maximum (times c2) and this lane's share of the sum
 #pragma unroll
     for (int t = 0; t < QT; t++) {
         m_run[t] = -INFINITY, l_run[t] = 0.f;
 #pragma unroll
         for (int i = 0; i < VT; i++) O[t][i] = (v4f){0.f, 0.f, 0.f, 0.f};
     }
-
-    // unit un of a block: key tile un / ks, k unit un % ks for the first 2 ks; value tile un - 2 ks behind them
-    auto stage = [&](uint32_t key0, uint32_t buf) {
-        T* base = lds + (size_t)buf * units * 512;
-        for (uint32_t un = wave; un < units; un += 4) {
-            const T* src;
-            if (un < 2 * ks) {
-                const uint32_t t = un >= ks ? 1u : 0u, s = un - t * ks;
-                const uint32_t key = min(key0 + 8 * (sr >> 2) + 4 * t + (sr & 3u), kv_len - 1);
-                src = s < kd ? reinterpret_cast<const T*>(p.k_exp) + (size_t)key * p.ld_k + head * d.dim_p + 32 * s + sc
-                             : cache + kv_row(p.kv, p.rows.seq0, 0, 0, key) * kl + d.rank_p + 32 * (s - kd) + sc;
-            } else {
-                src = reinterpret_cast<const T*>(p.v_exp_t) + (size_t)(head * d.vdim_p + (un - 2 * ks) * 16 + sr) * p.ld_v + key0 + sc;
-            }
-            stage_unit(src, base + (size_t)un * 512);
-        }
-    };
-    stage(0, 0);
     uint32_t buf = 0;
     for (uint32_t key0 = 0; key0 < kv_len; key0 += 32) {
         wait_lds_copies();
@@ -412,56 +459,66 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
 #pragma unroll
         for (int t = 0; t < QT; t++) s0[t] = s1[t] = (v4f){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < KS; s++)
-            if ((uint32_t)s < ks) {
-                const frag k0 = load_staged(kb + (size_t)s * 512, slot), k1 = load_staged(kb + (size_t)(ks + s) * 512, slot);
+        for (int s2 = 0; s2 < KS; s2 += 2)
+            if ((uint32_t)s2 < ks) {
 #pragma unroll
-                for (int t = 0; t < QT; t++) {
-                    s0[t] = mfma32(k0, q[t][s], s0[t]);
-                    s1[t] = mfma32(k1, q[t][s], s1[t]);
+                for (int j = 0; j < 2; j++) {
+                    const uint32_t s = min((uint32_t)(s2 + j), ks - 1);   // (past the end: against zero queries)
+                    const frag k0 = load_staged(kb + (size_t)s * 512, slot), k1 = load_staged(kb + (size_t)(ks + s) * 512, slot);
+#pragma unroll
+                    for (int t = 0; t < QT; t++) {
+                        s0[t] = mfma32(k0, q[t][s2 + j], s0[t]);
+                        s1[t] = mfma32(k1, q[t][s2 + j], s1[t]);
+                    }
                 }
             }
-        frag hi[QT], lo[QT];
-        bool moved = false;
-        float alpha[QT];
+        const bool whole = key0 + 31 <= q_first;
+        float sv[QT][8];
+        bool behind = false;
 #pragma unroll
         for (int t = 0; t < QT; t++) {
-            float sv[8], mx = -INFINITY;
+            float mx = -INFINITY;
 #pragma unroll
             for (int e = 0; e < 8; e++) {
-                const float x = e < 4 ? s0[t][e & 3] : s1[t][e & 3];
-                sv[e] = key0 + 8 * g + e <= qpos[t] ? x * d.scale : -INFINITY;
-                mx = fmaxf(mx, sv[e]);
+                sv[t][e] = (e < 4 ? s0[t][e & 3] : s1[t][e & 3]) * c2;
+                if (!whole && key0 + 8 * g + e > qpos[t]) sv[t][e] = -INFINITY;
+                mx = fmaxf(mx, sv[t][e]);
             }
-            mx = max_rows4(mx);
-            const float m_new = fmaxf(m_run[t], mx);   // finite from the first block on: key 0 is visible to every query
-            alpha[t] = exp_of<T>(m_run[t] - m_new);
-            float sum = 0.f;
+            s0[t][0] = mx = max_rows4(mx);
+            behind |= mx > m_run[t] + kLazy;   // (the first block: key 0 is visible to every query, -inf is behind)
+        }
+        if (__any(behind)) {
+#pragma unroll
+            for (int t = 0; t < QT; t++) {
+                const float m_new = fmaxf(m_run[t], s0[t][0]), alpha = exp2_of<T>(m_run[t] - m_new);
+                m_run[t] = m_new;
+                l_run[t] *= alpha;
+#pragma unroll
+                for (int i = 0; i < VT; i++) O[t][i] *= alpha;
+            }
+        }
+        frag hi[QT], lo[QT];
+#pragma unroll
+        for (int t = 0; t < QT; t++) {
+            float pe[8];
 #pragma unroll
             for (int e = 0; e < 8; e++) {
-                const float pe = exp_of<T>(sv[e] - m_new);
-                sum += pe;
-                hi[t][e] = (T)pe;
-                if constexpr (!Dt<T>::is_f32) lo[t][e] = (T)(pe - (float)hi[t][e]);
+                pe[e] = exp2_of<T>(sv[t][e] - m_run[t]);
+                l_run[t] += pe[e];
             }
-            l_run[t] = l_run[t] * alpha[t] + sum_rows4(sum);
-            moved |= m_new != m_run[t];
-            m_run[t] = m_new;
-        }
-        if (__any(moved)) {
-#pragma unroll
-            for (int t = 0; t < QT; t++)
-#pragma unroll
-                for (int i = 0; i < VT; i++) O[t][i] *= alpha[t];
+            split_hi_lo(pe, hi[t], lo[t]);
         }
 #pragma unroll
-        for (int i = 0; i < VT; i++)
-            if ((uint32_t)i < vt) {
-                const frag a = load_staged(vb + (size_t)i * 512, slot);
+        for (int i2 = 0; i2 < VT; i2 += 2)
+            if ((uint32_t)i2 < vt) {   // (vt is even)
 #pragma unroll
-                for (int t = 0; t < QT; t++) {
-                    O[t][i] = mfma32(a, hi[t], O[t][i]);
-                    if constexpr (!Dt<T>::is_f32) O[t][i] = mfma32(a, lo[t], O[t][i]);
+                for (int j = 0; j < 2; j++) {
+                    const frag a = load_staged(vb + (size_t)(i2 + j) * 512, slot);
+#pragma unroll
+                    for (int t = 0; t < QT; t++) {
+                        O[t][i2 + j] = mfma32(a, hi[t], O[t][i2 + j]);
+                        if constexpr (!Dt<T>::is_f32) O[t][i2 + j] = mfma32(a, lo[t], O[t][i2 + j]);
+                    }
                 }
             }
         if (n_buf > 1) {
@@ -471,13 +528,14 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(OxbLatentParams p, 
             stage(key0 + 32, 0);
         }
     }
-    const float sink = p.sink[head];
+    const float sink = p.sink[head] * 1.4426950408889634f;
 #pragma unroll
     for (int t = 0; t < QT; t++) {
         const uint32_t row = qb * 64 * QT + (wave * QT + t) * 16 + qi;
+        const float l = sum_rows4(l_run[t]);
         if (row >= p.rows.m) continue;
-        const float M = fmaxf(m_run[t], sink), f = exp_of<T>(m_run[t] - M);
-        const float inv = f / (l_run[t] * f + exp_of<T>(sink - M));
+        const float M = fmaxf(m_run[t], sink), f = exp2_of<T>(m_run[t] - M);
+        const float inv = f / (l * f + exp2_of<T>(sink - M));
         T* o = reinterpret_cast<T*>(p.out) + (size_t)row * p.ld_out + head * d.vdim_p + 4 * g;
 #pragma unroll
         for (int i = 0; i < VT; i++)
