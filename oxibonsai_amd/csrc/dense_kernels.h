@@ -27,7 +27,7 @@ static inline size_t oxb_tile_stride(uint32_t k_pad, uint32_t elem_bytes) { retu
 // Row stride of an activation matrix of n columns: padded columns, and 128 elements more where rows would otherwise start a
 // multiple of 1 KiB apart (the 16 rows of an operand would all come out of one or two L2 channels).
 static inline uint32_t oxb_act_ld(uint32_t n) { const uint32_t p = oxb_dense_pad(n); return p % 512u ? p : p + 128u; }
-#define OXB_DENSE_GEMV_MAX_ROWS 16u   // token rows the few-row kernel takes per pass over the weights (one MFMA column tile)
+#define OXB_DENSE_GEMV_MAX_ROWS 64u   // token rows up to which the few-row kernel is used (four column tiles)
 
 // What happens to y[m][n] behind the product, in this order:
 //   y = product * scale (+ add[n]) ; act(y) ; (+ resid[m][n]) -> out32[m][n] ; norm(y)[m][n] -> out_t (weights' type)
@@ -66,7 +66,7 @@ struct OxbDenseParams {
 // matrix is src[row_off[n] + col_off[k]], or zero where either offset is negative.  row_off [n_pad], col_off [k_pad].
 hipError_t oxb_launch_dense_pack(const void* src, int src_type, const int64_t* row_off, const int64_t* col_off, uint32_t n_pad,
                                  uint32_t k_pad, int dt, void* dst, hipStream_t st);
-// y = W x for up to any m: m <= 16 through the few-row kernel (weights streamed once, K split over the waves of a
+// y = W x for any m: up to OXB_DENSE_GEMV_MAX_ROWS through the few-row kernel (weights streamed once, K split over the waves of a
 // workgroup), more through the tiled GEMM.
 hipError_t oxb_launch_dense(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st);
 hipError_t oxb_launch_dense_gemm_t(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st);

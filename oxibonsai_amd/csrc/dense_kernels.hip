@@ -50,32 +50,36 @@ __device__ __forceinline__ size_t x_row(const OxbDenseParams& p, uint32_t t) {
 }
 
 // ---------------------------------------------------------------------------
-// Few rows (m <= 16 per grid row): a workgroup of 8 waves owns RT row tiles and splits K over its waves; wave w takes the
-// units w, w + 8, ... so that the workgroup walks its tile's bytes in order.  The token rows are the columns of the
-// product: lane 16 g + c loads eight activations of token c, lanes of absent tokens supply zeros.  UN units are in flight
-// per wave.  The waves' sums meet in LDS and are added in wave order.
+// Few token rows: a workgroup of 8 waves owns RT row tiles and splits K over its waves; wave w takes the units w, w + 8, ...
+// so that the workgroup walks its tiles' bytes in order.  The token rows are the columns of the product, CT tiles of 16:
+// lane 16 g + c loads eight activations of token c, lanes of absent tokens supply zeros.  UN units are in flight per wave.
+// The waves' sums meet in LDS and are added in wave order.
 // ---------------------------------------------------------------------------
-template <typename T, int RT, int UN>
+template <typename T, int RT, int CT, int UN>
 __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
     typedef typename Dt<T>::frag frag;
-    __shared__ __attribute__((aligned(16))) float red[8][RT][16][20];
+    __shared__ __attribute__((aligned(16))) float red[8][RT * CT][16][20];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, c = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
-    const uint32_t nu = p.k_pad / 32, n_tiles = p.n_pad / 16, m0 = blockIdx.y * 16, mc = min(p.m - m0, 16u);
+    const uint32_t nu = p.k_pad / 32, n_tiles = p.n_pad / 16;
     const T* w[RT];
 #pragma unroll
-    for (int r = 0; r < RT; r++) w[r] = reinterpret_cast<const T*>(p.w) + (size_t)min(blockIdx.x * RT + r, n_tiles - 1) * oxb_tile_stride(p.k_pad, sizeof(T));
-    const bool have = c < mc;
-    const T* x = reinterpret_cast<const T*>(p.x) + (have ? x_row(p, m0 + c) : 0) * p.ldx + 8 * g;
-    v4f acc[RT];
+    for (int r = 0; r < RT; r++) w[r] = reinterpret_cast<const T*>(p.w) + min(blockIdx.x * RT + r, n_tiles - 1) * oxb_tile_stride(p.k_pad, sizeof(T));
+    const T* x[CT];
 #pragma unroll
-    for (int r = 0; r < RT; r++) acc[r] = (v4f){0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < CT; t++) x[t] = reinterpret_cast<const T*>(p.x) + x_row(p, min(16u * t + c, p.m - 1)) * p.ldx + 8 * g;
+    v4f acc[RT][CT];
+#pragma unroll
+    for (int r = 0; r < RT; r++)
+#pragma unroll
+        for (int t = 0; t < CT; t++) acc[r][t] = (v4f){0.f, 0.f, 0.f, 0.f};
     for (uint32_t u0 = wave; u0 < nu; u0 += 8 * UN) {
-        frag b[UN], a[UN][RT];
+        frag b[UN][CT], a[UN][RT];
 #pragma unroll
         for (int i = 0; i < UN; i++) {
             const uint32_t u = u0 + 8 * i;
-            b[i] = have && u < nu ? load_row8(x + 32 * u) : zero_frag((const T*)nullptr);
+#pragma unroll
+            for (int t = 0; t < CT; t++) b[i][t] = u < nu && 16u * t + c < p.m ? load_row8(x[t] + 32 * u) : zero_frag((const T*)nullptr);
         }
 #pragma unroll
         for (int i = 0; i < UN; i++) {
@@ -86,19 +90,24 @@ __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
 #pragma unroll
         for (int i = 0; i < UN; i++)
 #pragma unroll
-            for (int r = 0; r < RT; r++) acc[r] = mfma32(a[i][r], b[i], acc[r]);
+            for (int r = 0; r < RT; r++)
+#pragma unroll
+                for (int t = 0; t < CT; t++) acc[r][t] = mfma32(a[i][r], b[i][t], acc[r][t]);
     }
-    const uint32_t fr = tid >> 6, fq = tid & 3u, ft = (tid & 63u) >> 2, fn = (blockIdx.x * RT + fr) * 16 + 4 * fq;   // what a finishing thread owns
-    v4f resid = {0.f, 0.f, 0.f, 0.f};
-    if (fr < RT && ft < mc) resid = epilogue_resid(p.e, m0 + ft, fn);
+    // what a finishing thread owns: a quad of outputs of one token
+    const uint32_t f = tid >> 6, fq = tid & 3u, ft = (f % CT) * 16 + ((tid & 63u) >> 2), fn = (blockIdx.x * RT + f / CT) * 16 + 4 * fq;
+    const bool finish = f < RT * CT && ft < p.m && blockIdx.x * RT + f / CT < n_tiles;
+    const v4f resid = finish ? epilogue_resid(p.e, ft, fn) : (v4f){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int r = 0; r < RT; r++) *reinterpret_cast<v4f*>(&red[wave][r][c][4 * g]) = acc[r];
+    for (int r = 0; r < RT; r++)
+#pragma unroll
+        for (int t = 0; t < CT; t++) *reinterpret_cast<v4f*>(&red[wave][r * CT + t][c][4 * g]) = acc[r][t];
     __syncthreads();
-    if (tid < 64 * RT) {
-        v4f y = *reinterpret_cast<const v4f*>(&red[0][fr][ft][4 * fq]);
+    if (finish) {
+        v4f y = *reinterpret_cast<const v4f*>(&red[0][f][ft & 15u][4 * fq]);
 #pragma unroll
-        for (int i = 1; i < 8; i++) y += *reinterpret_cast<const v4f*>(&red[i][fr][ft][4 * fq]);
-        if (ft < mc && blockIdx.x * RT + fr < n_tiles) epilogue4<T>(p.e, m0 + ft, fn, y, resid);
+        for (int i = 1; i < 8; i++) y += *reinterpret_cast<const v4f*>(&red[i][f][ft & 15u][4 * fq]);
+        epilogue4<T>(p.e, ft, fn, y, resid);
     }
 }
 
@@ -294,26 +303,31 @@ static hipError_t pick_gemm(const OxbDenseParams& p, uint32_t n_cus, hipStream_t
     return launch_gemm<T, 1, 4, SWAP>(p, st);
 }
 
-template <typename T>
-static hipError_t launch_gemv(const OxbDenseParams& p, uint32_t n_cus, hipStream_t st) {
-    const uint32_t tiles = p.n_pad / 16, my = (p.m + 15) / 16;
-    // units per wave and pass: as many as the wave has, up to what keeps the registers within two workgroups per CU
-    const uint32_t per_wave = (p.k_pad / 32 + 7) / 8;
-    constexpr int BIG = Dt<T>::is_f32 ? 4 : 8;
-    if (tiles >= 4 * n_cus) {
-        hipLaunchKernelGGL((dense_gemv_kernel<T, 2, BIG / 2>), dim3((tiles + 1) / 2, my), dim3(512), 0, st, p);
-    } else if (per_wave > 2) {
-        hipLaunchKernelGGL((dense_gemv_kernel<T, 1, BIG>), dim3(tiles, my), dim3(512), 0, st, p);
-    } else {
-        hipLaunchKernelGGL((dense_gemv_kernel<T, 1, 2>), dim3(tiles, my), dim3(512), 0, st, p);
-    }
+template <typename T, int RT, int CT, int UN>
+static hipError_t launch_gemv(const OxbDenseParams& p, hipStream_t st) {
+    hipLaunchKernelGGL((dense_gemv_kernel<T, RT, CT, UN>), dim3((p.n_pad / 16 + RT - 1) / RT), dim3(512), 0, st, p);
     return hipGetLastError();
+}
+
+// Two row tiles per workgroup where the matrix has tiles enough for every CU to get several workgroups all the same; units
+// in flight per wave within what the registers of two workgroups per CU allow.
+template <typename T>
+static hipError_t pick_gemv(const OxbDenseParams& p, uint32_t n_cus, hipStream_t st) {
+    const bool many = p.n_pad / 16 >= 4 * n_cus;
+    const uint32_t per_wave = (p.k_pad / 32 + 7) / 8;
+    constexpr int S = Dt<T>::is_f32 ? 2 : 1;
+    if (p.m <= 16) {
+        if (many) return launch_gemv<T, 2, 1, 4 / S>(p, st);
+        return per_wave > 2 ? launch_gemv<T, 1, 1, 8 / S>(p, st) : launch_gemv<T, 1, 1, 2>(p, st);
+    }
+    if (p.m <= 32) return many ? launch_gemv<T, 2, 2, 4 / S>(p, st) : launch_gemv<T, 1, 2, 4 / S>(p, st);
+    return launch_gemv<T, 1, 4, 2>(p, st);
 }
 
 hipError_t oxb_launch_dense(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st) {
     const hipError_t e = check(p, dt);
     if (e != hipSuccess) return e;
-    if (p.m <= OXB_DENSE_GEMV_MAX_ROWS) return dt == OXB_DT_BF16 ? launch_gemv<__bf16>(p, n_cus, st) : launch_gemv<float>(p, n_cus, st);
+    if (p.m <= OXB_DENSE_GEMV_MAX_ROWS) return dt == OXB_DT_BF16 ? pick_gemv<__bf16>(p, n_cus, st) : pick_gemv<float>(p, n_cus, st);
     return dt == OXB_DT_BF16 ? pick_gemm<__bf16, false>(p, n_cus, st) : pick_gemm<float, false>(p, n_cus, st);
 }
 

@@ -68,6 +68,6 @@ hipError_t oxb_launch_latent_prefill(const OxbLatentParams& p, int dt, hipStream
 hipError_t oxb_latent_prepare(int dt);
 // Whether the kernels can take these sizes, and why not.
 const char* oxb_latent_check(const OxbLatentDims& d, int dt);
-// Keys one workgroup of the absorbed form takes per step of its walk (a split walks chunks s, s + splits, ...).
-uint32_t oxb_latent_chunk(const OxbLatentDims& d, int dt);
+// Splits of the absorbed form a context of max_seq positions can keep busy.
+uint32_t oxb_latent_max_splits(uint32_t max_seq);
 #define OXB_LATENT_MAX_SPLITS 128u

@@ -97,160 +97,166 @@ __global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, ui
 }
 
 // ---------------------------------------------------------------------------
-// Absorbed attention.  Grid (split, head tile, token row); the 16 heads of a tile are the columns of the products, so a
-// latent row is read once for all of them and serves as key and as value:
-//   S^T[key][head] = K[key] . q_abs[head]          K rows of 32 keys from LDS in operand order, q_abs resident in registers
+// Absorbed attention.  Grid (split, head tile, token row), 8 waves; the 16 heads of a tile are the columns of the products,
+// so a latent row is read once for all of them and serves as key and as value:
+//   S^T[key][head] = K[key] . q_abs[head]          operand reads of the staged rows
 //   O^T[r][head]  += c[key][r] P[head][key]        the same LDS rows through the transposing read
-// Wave w of a workgroup takes keys [32 w, 32 w + 32) of a chunk with a softmax of its own and LDS of its own (memory -> LDS
-// copies, no barrier in the walk); the waves meet once at the end.  NT: accumulator tiles of 16 latent elements, KS: k
-// units of q_abs held in registers.
+// A split walks chunks of 32 keys through a ring of LDS buffers (memory -> LDS copies).  Wave w brings in and multiplies the
+// k units w / 2, w / 2 + 4, ... of key tile w % 2, so it starts on its own copies without a barrier; the partial scores of
+// the four k quarters meet in LDS behind the chunk's one barrier, every wave forms the same probabilities from them, and
+// takes its own eighth of the latent elements of O.  KSQ: k units per wave, NTW: accumulator tiles per wave.
 // ---------------------------------------------------------------------------
-template <typename T>
-__device__ __forceinline__ typename Dt<T>::frag value_frag(const T* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g);
-template <>
-__device__ __forceinline__ v8b value_frag<__bf16>(const __bf16* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g) {
-    // keys 4 g .. 4 g + 3 of either key tile, latent element 16 sl + qi: two transposing reads
-    const uint32_t s = sl >> 1, r = 4 * g + (qi >> 2), slot = staged_slot(r, (sl & 1u) * 2 + ((qi & 3u) >> 1));
-    const _Float16* a = reinterpret_cast<const _Float16*>(lds) + (size_t)s * 512 + slot * 8 + (qi & 1u) * 4;
-    const v4b t0 = __builtin_bit_cast(v4b, lds_read_tr16(a)), t1 = __builtin_bit_cast(v4b, lds_read_tr16(a + (size_t)ks * 512));
+static constexpr uint32_t kChunk = 32;
+// Splits in use at a position: two chunks each at least.
+__host__ __device__ static inline uint32_t latent_used_splits(uint32_t pos, uint32_t n_splits) {
+    const uint32_t pairs = (pos / kChunk + 2) / 2;
+    return pairs < n_splits ? pairs : n_splits;
+}
+
+// Value operand: keys 4 g .. 4 g + 3 of both key tiles, one latent element per lane.  `at` = value_at(..) of the tile.
+template <typename T> __device__ __forceinline__ uint32_t value_at(uint32_t sl, uint32_t qi, uint32_t g);
+template <> __device__ __forceinline__ uint32_t value_at<__bf16>(uint32_t sl, uint32_t qi, uint32_t g) {
+    // four consecutive halves per lane for the transposing read: row 4 g + qi / 4, columns 16 sl + 4 (qi % 4) ..
+    return (sl >> 1) * 512 + staged_slot(4 * g + (qi >> 2), (sl & 1u) * 2 + ((qi & 3u) >> 1)) * 8 + (qi & 1u) * 4;
+}
+template <> __device__ __forceinline__ uint32_t value_at<float>(uint32_t sl, uint32_t qi, uint32_t g) {
+    const uint32_t d = 16 * sl + qi, e = d & 7u;   // (the slots of rows 4 g .. 4 g + 3 lie four apart: they share r >> 2)
+    return (d >> 5) * 512 + (e >> 2) * 256 + staged_slot(4 * g, (d & 31u) >> 3) * 4 + (e & 3u);
+}
+__device__ __forceinline__ v8b value_frag(const __bf16* tile0, const __bf16* tile1) {
+    const v4b t0 = __builtin_bit_cast(v4b, lds_read_tr16(reinterpret_cast<const _Float16*>(tile0)));
+    const v4b t1 = __builtin_bit_cast(v4b, lds_read_tr16(reinterpret_cast<const _Float16*>(tile1)));
     return (v8b){t0[0], t0[1], t0[2], t0[3], t1[0], t1[1], t1[2], t1[3]};
 }
-template <>
-__device__ __forceinline__ v8f value_frag<float>(const float* lds, uint32_t ks, uint32_t sl, uint32_t qi, uint32_t g) {
-    const uint32_t d = 16 * sl + qi, e = d & 7u;
-    // (the slots of rows 4 g .. 4 g + 3 lie four apart: they share r >> 2)
-    const float* a = lds + (size_t)(d >> 5) * 512 + (e >> 2) * 256 + staged_slot(4 * g, (d & 31u) >> 3) * 4 + (e & 3u);
-    const float* b = a + (size_t)ks * 512;
-    return (v8f){a[0], a[16], a[32], a[48], b[0], b[16], b[32], b[48]};
-}
+__device__ __forceinline__ v8f value_frag(const float* a, const float* b) { return (v8f){a[0], a[16], a[32], a[48], b[0], b[16], b[32], b[48]}; }
 
-template <typename T, int NT, int KS>
-__global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p) {
+template <typename T, int KSQ, int NTW>
+__global__ __launch_bounds__(512) void latent_decode_kernel(OxbLatentParams p, uint32_t n_buf) {
     typedef typename Dt<T>::frag frag;
-    constexpr int G = 4;   // k units / accumulator tiles per step: sizes round up to whole steps (zero queries, unused tiles)
+    constexpr float kLazy = 8.0f;   // the running maximum follows once it is 2^8 behind
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
-    __shared__ float wave_ml[4][16][2];
+    __shared__ __attribute__((aligned(16))) float part_s[2][4][16][kChunk + 4];   // two chunks' worth: one barrier per chunk
     const OxbLatentDims& d = p.d;
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4, nw = blockDim.x >> 6;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
     const uint32_t split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
-    const uint32_t pos = row_pos(p.rows, m), seq = row_seq(p.rows, m), chunk = 32 * nw, n_chunks = pos / chunk + 1;
-    if (split >= min(p.n_splits, n_chunks)) return;
-    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, slot = staged_slot(qi, g);
-    T* lds = reinterpret_cast<T*>(smem) + (size_t)wave * 2 * ks * 512;
-    const T* cache = reinterpret_cast<const T*>(p.cache);
-    const float c2 = d.scale * 1.4426950408889634f;   // scores in units of log2(e): a probability is one exponential of one fma
-    auto request = [&](uint32_t key0) {
+    const uint32_t pos = row_pos(p.rows, m), seq = row_seq(p.rows, m), used = latent_used_splits(pos, p.n_splits);
+    if (split >= used) return;
+    const uint32_t n_mine = (pos / kChunk - split) / used + 1;   // chunks split, split + used, ...
+    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, kt = wave & 1u, kq = wave >> 1, slot = staged_slot(qi, g);
+    const uint32_t mine = kq < ks ? (ks - kq + 3) / 4 : 0;       // this wave's k units (kq + 4 j)
+    T* lds = reinterpret_cast<T*>(smem);
+    const uint32_t buf_elems = 2 * ks * 512;
+    const T* cache = reinterpret_cast<const T*>(p.cache) + 8 * stage_col(lane);
+    const float c2 = d.scale * 1.4426950408889634f;   // scores in units of log2(e)
+    auto unit_of = [&](int j) { return kq + 4 * min((uint32_t)j, mine - 1); };   // (past the end: the last one again)
+    auto request = [&](uint32_t i) {
         // rows past the newest position repeat it; their scores are masked
-        const T* r0 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + stage_row(lane), pos)) * p.ld + 8 * stage_col(lane);
-        const T* r1 = cache + kv_row(p.kv, seq, 0, 0, min(key0 + 16 + stage_row(lane), pos)) * p.ld + 8 * stage_col(lane);
-        for (uint32_t s = 0; s < ks; s++) {
-            stage_unit(r0 + 32 * s, lds + (size_t)s * 512);
-            stage_unit(r1 + 32 * s, lds + (size_t)(ks + s) * 512);
-        }
-    };
-    const uint32_t first = split * chunk + wave * 32;
-    if (first <= pos) request(first);
-
-    frag q[KS];
-    {
-        const uint32_t head = ht * 16 + qi;
-        const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(head, d.heads - 1)) * p.ld + 8 * g;
+        const uint32_t key = (split + i * used) * kChunk + kt * 16 + stage_row(lane);
+        const T* row = cache + kv_row(p.kv, seq, 0, 0, min(key, pos)) * p.ld;
+        T* base = lds + (i % n_buf) * buf_elems + (size_t)kt * ks * 512;
+        if (mine)
 #pragma unroll
-        for (int s = 0; s < KS; s++) {
-            q[s] = load_row8(src + 32 * min((uint32_t)s, ks - 1));
-            if ((uint32_t)s >= ks) q[s] = zero_frag((const T*)nullptr);
+            for (int j = 0; j < KSQ; j++) stage_unit(row + 32 * unit_of(j), base + (size_t)unit_of(j) * 512);
+    };
+    const uint32_t ahead = n_buf > 1 ? n_buf - 1 : 1;
+    for (uint32_t i = 0; i < ahead && i < n_mine; i++) request(i);
+
+    frag q[KSQ];
+    {
+        const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(ht * 16 + qi, d.heads - 1)) * p.ld + 8 * g;
+#pragma unroll
+        for (int j = 0; j < KSQ; j++) {
+            q[j] = zero_frag((const T*)nullptr);
+            if ((uint32_t)j < mine) q[j] = load_row8(src + 32 * (kq + 4 * j));
         }
     }
-    v4f O[NT];
+    const uint32_t ntw = (nt + 7) / 8;
+    uint32_t v_at[NTW];
+    v4f O[NTW];
 #pragma unroll
-    for (int i = 0; i < NT; i++) O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
-    float m_run = -INFINITY, l_run = 0.f;   // maximum (times c2) and this lane's share of the sum
+    for (int i = 0; i < NTW; i++) {
+        v_at[i] = value_at<T>(min(wave * ntw + i, nt - 1), qi, g);
+        O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
+    }
+    float m_run = -INFINITY, l_run = 0.f;   // maximum (times c2) and this lane's share of the sum; the same in every wave
 
-    for (uint32_t ch = split; ch < n_chunks; ch += p.n_splits) {
-        const uint32_t key0 = ch * chunk + wave * 32;
-        if (key0 > pos) break;  // (only the last chunk can end before this wave's keys)
-        if (ch != split) request(key0);
-        wait_lds_copies();
-        v4f s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+    for (uint32_t i = 0; i < n_mine; i++) {
+        const uint32_t key0 = (split + i * used) * kChunk;
+        const T* kb = lds + (i % n_buf) * buf_elems;
+        const T* tile = kb + (size_t)kt * ks * 512;
+        // this chunk's copies have arrived; those of later chunks may stay in flight
+        if (n_buf == 3 && i + 1 < n_mine) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KSQ * Dt<T>::sub) : "memory");
+        else wait_lds_copies();
+        v4f s = {0.f, 0.f, 0.f, 0.f};
+        if (mine) {
+            frag k[KSQ];
 #pragma unroll
-        for (int s4 = 0; s4 < KS; s4 += G)
-            if ((uint32_t)s4 < ks) {
+            for (int j = 0; j < KSQ; j++) k[j] = load_staged(tile + (size_t)unit_of(j) * 512, slot);
 #pragma unroll
-                for (int j = 0; j < G; j++)
-                    if (s4 + j < KS) {
-                        const uint32_t s = min((uint32_t)(s4 + j), ks - 1);
-                        s0 = mfma32(load_staged(lds + (size_t)s * 512, slot), q[s4 + j], s0);
-                        s1 = mfma32(load_staged(lds + (size_t)(ks + s) * 512, slot), q[s4 + j], s1);
-                    }
-            }
-        float sv[8], mx = -INFINITY;
-#pragma unroll
-        for (int v = 0; v < 4; v++) {
-            const uint32_t k = key0 + 4 * g + v;
-            sv[v] = k <= pos ? s0[v] * c2 : -INFINITY;
-            sv[4 + v] = k + 16 <= pos ? s1[v] * c2 : -INFINITY;
-            mx = fmaxf(mx, fmaxf(sv[v], sv[4 + v]));
+            for (int j = 0; j < KSQ; j++) s = mfma32(k[j], q[j], s);
         }
+        *reinterpret_cast<v4f*>(&part_s[i & 1u][kq][qi][kt * 16 + 4 * g]) = s;
+        lds_barrier();   // scores and rows of the whole chunk are in LDS, and every wave is through with the chunk before
+        if (n_buf > 1 && i + ahead < n_mine) request(i + ahead);
+        float sv[8], mx = -INFINITY;
+        {
+            v4f a = *reinterpret_cast<const v4f*>(&part_s[i & 1u][0][qi][4 * g]), b = *reinterpret_cast<const v4f*>(&part_s[i & 1u][0][qi][16 + 4 * g]);
+#pragma unroll
+            for (int k = 1; k < 4; k++) {
+                a += *reinterpret_cast<const v4f*>(&part_s[i & 1u][k][qi][4 * g]);
+                b += *reinterpret_cast<const v4f*>(&part_s[i & 1u][k][qi][16 + 4 * g]);
+            }
+#pragma unroll
+            for (int v = 0; v < 4; v++) sv[v] = a[v] * c2, sv[4 + v] = b[v] * c2;
+        }
+        if (key0 + kChunk - 1 > pos) {
+#pragma unroll
+            for (int v = 0; v < 4; v++) {
+                if (key0 + 4 * g + v > pos) sv[v] = -INFINITY;
+                if (key0 + 16 + 4 * g + v > pos) sv[4 + v] = -INFINITY;
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 8; e++) mx = fmaxf(mx, sv[e]);
         mx = max_rows4(mx);  // finite: key0 <= pos
-        const float m_new = fmaxf(m_run, mx), alpha = exp2_of<T>(m_run - m_new);
-        l_run *= alpha;
-        frag hi, lo;
+        if (__any(mx > m_run + kLazy)) {
+            const float m_new = fmaxf(m_run, mx), alpha = exp2_of<T>(m_run - m_new);
+            m_run = m_new;
+            l_run *= alpha;
+#pragma unroll
+            for (int t = 0; t < NTW; t++) O[t] *= alpha;
+        }
         float pe[8];
 #pragma unroll
         for (int e = 0; e < 8; e++) {
-            pe[e] = exp2_of<T>(sv[e] - m_new);
+            pe[e] = exp2_of<T>(sv[e] - m_run);
             l_run += pe[e];
         }
+        frag hi, lo;
         split_hi_lo(pe, hi, lo);
-        const bool moved = __any(m_new != m_run);
-        m_run = m_new;
-        if (moved) {
 #pragma unroll
-            for (int i = 0; i < NT; i++) O[i] *= alpha;
+        for (int t = 0; t < NTW; t++) {
+            const frag a = value_frag(kb + v_at[t], kb + v_at[t] + (size_t)ks * 512);
+            O[t] = mfma32(a, hi, O[t]);
+            if constexpr (!Dt<T>::is_f32) O[t] = mfma32(a, lo, O[t]);
         }
-#pragma unroll
-        for (int i4 = 0; i4 < NT; i4 += G)
-            if ((uint32_t)i4 < nt) {   // (nt is even: at most two tiles too many, and they read the first rotated unit)
-#pragma unroll
-                for (int j = 0; j < G; j++) {
-                    const frag a = value_frag<T>(lds, ks, i4 + j, qi, g);
-                    O[i4 + j] = mfma32(a, hi, O[i4 + j]);
-                    if constexpr (!Dt<T>::is_f32) O[i4 + j] = mfma32(a, lo, O[i4 + j]);
-                }
+        if (i + 1 < n_mine) {
+            if (n_buf == 1) {
+                lds_barrier();   // every wave is through with the buffer
+                request(i + 1);
             }
-        // the LDS reads above are complete before the next copies overwrite the rows
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    }
-    l_run = sum_rows4(l_run);
-
-    // the waves' results: common maximum, sums in wave order
-    if (g == 0) wave_ml[wave][qi][0] = m_run, wave_ml[wave][qi][1] = l_run;
-    __syncthreads();
-    float M = -INFINITY;
-    for (uint32_t w = 0; w < nw; w++) M = fmaxf(M, wave_ml[w][qi][0]);
-    const float f = m_run == -INFINITY ? 0.f : exp2_of<T>(m_run - M);
-    float* mine = reinterpret_cast<float*>(smem) + (size_t)wave * 16 * d.rank_p;   // (every wave is done with its rows)
-#pragma unroll
-    for (int i = 0; i < NT; i++)
-        if ((uint32_t)i < nt) *reinterpret_cast<v4f*>(mine + qi * d.rank_p + 16 * i + 4 * g) = O[i] * f;
-    __syncthreads();
-    const size_t part = ((size_t)m * gridDim.y + ht) * p.n_splits + split;
-    float* po = p.part_o + part * 16 * d.rank_p;
-    const float* all = reinterpret_cast<const float*>(smem);
-    for (uint32_t i = tid * 4; i < 16 * d.rank_p; i += blockDim.x * 4) {
-        v4f y = *reinterpret_cast<const v4f*>(all + i);
-        for (uint32_t w = 1; w < nw; w++) y += *reinterpret_cast<const v4f*>(all + (size_t)w * 16 * d.rank_p + i);
-        *reinterpret_cast<v4f*>(po + i) = y;
-    }
-    if (tid < 16) {
-        float l = 0.f;
-        for (uint32_t w = 0; w < nw; w++) {
-            const float mw = wave_ml[w][tid][0];
-            if (mw != -INFINITY) l += wave_ml[w][tid][1] * exp2_of<T>(mw - M);
         }
-        p.part_ml[part * 32 + tid * 2] = M;
-        p.part_ml[part * 32 + tid * 2 + 1] = l;
+    }
+    const size_t part = ((size_t)m * gridDim.y + ht) * p.n_splits + split;
+    float* po = p.part_o + part * 16 * d.rank_p + (size_t)qi * d.rank_p + 4 * g;
+#pragma unroll
+    for (int t = 0; t < NTW; t++)
+        if ((uint32_t)t < ntw && wave * ntw + t < nt) *reinterpret_cast<v4f*>(po + 16 * (wave * ntw + t)) = O[t];
+    l_run = sum_rows4(l_run);
+    if (wave == 0 && g == 0) {
+        p.part_ml[part * 32 + qi * 2] = m_run;
+        p.part_ml[part * 32 + qi * 2 + 1] = l_run;
     }
 }
 
@@ -259,7 +265,7 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(OxbLatentParams p
 // Grid (head, token row), 8 waves, a tile of 16 value rows each; UN units of the product's weights are in flight per wave.
 // ---------------------------------------------------------------------------
 template <typename T>
-__global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, uint32_t chunk) {
+__global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p) {
     typedef typename Dt<T>::frag frag;
     constexpr int UN = 8;
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
@@ -268,7 +274,7 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, ui
     const uint32_t tid = threadIdx.x, lane = tid & 63u, c = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
     const uint32_t head = blockIdx.x, m = blockIdx.y, ht = head / 16, col = head % 16, n_ht = (d.heads + 15) / 16;
-    const uint32_t used = min(p.n_splits, row_pos(p.rows, m) / chunk + 1);
+    const uint32_t used = latent_used_splits(row_pos(p.rows, m), p.n_splits);
     const size_t slot0 = ((size_t)m * n_ht + ht) * p.n_splits;
     const float sink = p.sink[head] * 1.4426950408889634f;   // (maxima are in units of log2(e))
     const uint32_t nu = p.k_uv / 32, tiles = d.vdim_p / 16;
@@ -303,19 +309,33 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p, ui
         }
     }
     __syncthreads();
-    const float* po = p.part_o + (slot0 * 16 + col) * d.rank_p;
-    for (uint32_t i = tid; i < p.k_uv; i += 512) {
-        float y = 0.f;
-        if (i < d.rank_p) {
-            for (uint32_t s0 = 0; s0 < used; s0 += 8) {
-                float v[8];
+    // four consecutive latent elements per thread; the threads beyond rank_p / 4 take further shares of the splits
+    {
+        const float* po = p.part_o + (slot0 * 16 + col) * d.rank_p;
+        const uint32_t cols = d.rank_p / 4, shares = 512 / cols > 8 ? 8 : (512 / cols ? 512 / cols : 1), share = tid / cols;
+        float* sums = reinterpret_cast<float*>(smem + p.k_uv * sizeof(T));   // [shares][rank_p]
+        for (uint32_t c0 = 0; c0 < cols; c0 += 512) {
+            const uint32_t i = shares > 1 ? tid % cols : c0 + tid;
+            if (i < cols && share < shares) {
+                v4f y = {0.f, 0.f, 0.f, 0.f};
+                for (uint32_t s0 = shares > 1 ? share : 0; s0 < used; s0 += 8 * shares) {
+                    v4f v[8];
 #pragma unroll
-                for (int k = 0; k < 8; k++) v[k] = po[(size_t)min(s0 + k, used - 1) * 16 * d.rank_p + i];
+                    for (int k = 0; k < 8; k++) v[k] = *reinterpret_cast<const v4f*>(po + (size_t)min(s0 + k * shares, used - 1) * 16 * d.rank_p + 4 * i);
 #pragma unroll
-                for (int k = 0; k < 8; k++) y = fmaf(s0 + k < used ? wgt[s0 + k] : 0.f, v[k], y);
+                    for (int k = 0; k < 8; k++)
+                        if (s0 + k * shares < used) y += v[k] * wgt[s0 + k * shares];
+                }
+                *reinterpret_cast<v4f*>(sums + (shares > 1 ? share : 0) * d.rank_p + 4 * i) = y;
             }
         }
-        lat[i] = (T)y;
+        __syncthreads();
+        for (uint32_t i = tid; i < p.k_uv; i += 512) {
+            float y = 0.f;
+            if (i < d.rank_p)
+                for (uint32_t k = 0; k < shares; k++) y += sums[k * d.rank_p + i];
+            lat[i] = (T)y;
+        }
     }
     __syncthreads();
     T* out = reinterpret_cast<T*>(p.out) + (size_t)m * p.ld_out;
@@ -551,24 +571,26 @@ __global__ __launch_bounds__(256, QT == 2 && !Dt<T>::is_f32 ? 2 : 1) void latent
 }
 
 // ---------------------------------------------------------------------------
-static constexpr uint32_t kLdsMax = 160u << 10, kLdsStatic = 1024;   // (decode keeps 512 B of statics beside the dynamic part)
+static constexpr uint32_t kLdsMax = 160u << 10, kDecodeStatic = 2 * 4 * 16 * (kChunk + 4) * 4;   // (decode's partial scores)
 
-static uint32_t decode_waves(const OxbLatentDims& d, int dt) {
-    for (uint32_t nw = 4; nw; nw >>= 1)
-        if (nw * 32 * (d.rank_p + d.rot_p) * oxb_dt_bytes(dt) <= kLdsMax - kLdsStatic) return nw;
-    return 0;
+static uint32_t decode_buffers(const OxbLatentDims& d, int dt) {
+    const uint32_t n = (kLdsMax - kDecodeStatic) / (kChunk * (d.rank_p + d.rot_p) * oxb_dt_bytes(dt));
+    return n > 3 ? 3 : n;
 }
 static uint32_t prefill_block_bytes(const OxbLatentDims& d, int dt) {
     return (2 * (d.dim_p + d.rot_p) / 32 + d.vdim_p / 16) * 512 * oxb_dt_bytes(dt);
 }
-uint32_t oxb_latent_chunk(const OxbLatentDims& d, int dt) { return 32 * decode_waves(d, dt); }
+uint32_t oxb_latent_max_splits(uint32_t max_seq) {
+    const uint32_t n = latent_used_splits(max_seq - 1, OXB_LATENT_MAX_SPLITS);
+    return n;
+}
 
 const char* oxb_latent_check(const OxbLatentDims& d, int dt) {
     if (!d.heads || !d.dim || !d.rot || !d.rank || !d.vdim) return "a latent attention size is 0";
     if (d.rot_dims > d.rot || d.rot_dims % 2) return "rotated dimensions must be even and within the rotated part";
     if (d.rank > 1024 || d.rot > 128) return "latent size beyond 1024 or rotated part beyond 128";
     if (d.dim_p + d.rot_p > 512 || d.vdim > 512) return "head size beyond 512";
-    if (!decode_waves(d, dt)) return "a block of latent rows exceeds the LDS";
+    if (!decode_buffers(d, dt)) return "a block of latent rows exceeds the LDS";
     if (prefill_block_bytes(d, dt) > kLdsMax) return "a block of keys and values exceeds the LDS";
     return nullptr;
 }
@@ -592,27 +614,27 @@ hipError_t oxb_launch_latent_store(const OxbLatentParams& p, bool absorb, int dt
     return hipGetLastError();
 }
 
-template <typename T, int NT, int KS>
-static hipError_t launch_decode(const OxbLatentParams& p, uint32_t nw, hipStream_t st) {
-    const uint32_t lds = nw * 32 * p.ld * sizeof(T);
-    hipLaunchKernelGGL((latent_decode_kernel<T, NT, KS>), dim3(p.n_splits, (p.d.heads + 15) / 16, p.rows.m), dim3(64 * nw), lds, st, p);
+template <typename T, int KSQ, int NTW>
+static hipError_t launch_decode(const OxbLatentParams& p, uint32_t n_buf, hipStream_t st) {
+    hipLaunchKernelGGL((latent_decode_kernel<T, KSQ, NTW>), dim3(p.n_splits, (p.d.heads + 15) / 16, p.rows.m), dim3(512),
+                       n_buf * kChunk * p.ld * (uint32_t)sizeof(T), st, p, n_buf);
     return hipGetLastError();
 }
 
 template <typename T>
-static hipError_t pick_decode(const OxbLatentParams& p, uint32_t nw, hipStream_t st) {
+static hipError_t pick_decode(const OxbLatentParams& p, uint32_t n_buf, hipStream_t st) {
     const uint32_t nt = p.d.rank_p / 16, ks = p.ld / 32;   // ks - nt / 2 = rot_p / 32 <= 4
-    if (nt <= 8 && ks <= 6) return launch_decode<T, 8, 6>(p, nw, st);
-    if (nt <= 16 && ks <= 12) return launch_decode<T, 16, 12>(p, nw, st);
-    if (nt <= 32 && ks <= 20) return launch_decode<T, 32, 20>(p, nw, st);
-    return launch_decode<T, 64, 36>(p, nw, st);
+    if (nt <= 8) return launch_decode<T, 2, 1>(p, n_buf, st);
+    if (nt <= 16) return launch_decode<T, 3, 2>(p, n_buf, st);
+    if (nt <= 32 && ks <= 20) return launch_decode<T, 5, 4>(p, n_buf, st);
+    return launch_decode<T, 9, 8>(p, n_buf, st);
 }
 
 hipError_t oxb_launch_latent_decode(const OxbLatentParams& p, int dt, hipStream_t st) {
-    const uint32_t nw = decode_waves(p.d, dt);
     if (!rows_ok(p) || oxb_latent_check(p.d, dt) || !p.q_abs || !p.part_o || !p.part_ml || !p.n_splits || p.n_splits > OXB_LATENT_MAX_SPLITS)
         return hipErrorInvalidValue;
-    return dt == OXB_DT_BF16 ? pick_decode<__bf16>(p, nw, st) : pick_decode<float>(p, nw, st);
+    const uint32_t n_buf = decode_buffers(p.d, dt);
+    return dt == OXB_DT_BF16 ? pick_decode<__bf16>(p, n_buf, st) : pick_decode<float>(p, n_buf, st);
 }
 
 hipError_t oxb_launch_latent_merge(const OxbLatentParams& p, int dt, hipStream_t st) {
@@ -620,9 +642,10 @@ hipError_t oxb_launch_latent_merge(const OxbLatentParams& p, int dt, hipStream_t
         !p.n_splits || p.n_splits > OXB_LATENT_MAX_SPLITS)
         return hipErrorInvalidValue;
     const dim3 grid(p.d.heads, p.rows.m);
-    const uint32_t lds = p.k_uv * oxb_dt_bytes(dt), chunk = oxb_latent_chunk(p.d, dt);
-    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_merge_kernel<__bf16>), grid, dim3(512), lds, st, p, chunk);
-    else hipLaunchKernelGGL((latent_merge_kernel<float>), grid, dim3(512), lds, st, p, chunk);
+    const uint32_t cols = p.d.rank_p / 4, shares = 512 / cols > 8 ? 8 : 512 / cols ? 512 / cols : 1;
+    const uint32_t lds = p.k_uv * oxb_dt_bytes(dt) + shares * p.d.rank_p * 4;
+    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((latent_merge_kernel<__bf16>), grid, dim3(512), lds, st, p);
+    else hipLaunchKernelGGL((latent_merge_kernel<float>), grid, dim3(512), lds, st, p);
     return hipGetLastError();
 }
 
@@ -646,13 +669,13 @@ static hipError_t pick_prefill(const OxbLatentParams& p, uint32_t bytes, hipStre
 // stream capture.
 template <typename T>
 static hipError_t raise_lds() {
-    const void* decode[] = {(const void*)&latent_decode_kernel<T, 8, 6>, (const void*)&latent_decode_kernel<T, 16, 12>,
-                            (const void*)&latent_decode_kernel<T, 32, 20>, (const void*)&latent_decode_kernel<T, 64, 36>};
+    const void* decode[] = {(const void*)&latent_decode_kernel<T, 2, 1>, (const void*)&latent_decode_kernel<T, 3, 2>,
+                            (const void*)&latent_decode_kernel<T, 5, 4>, (const void*)&latent_decode_kernel<T, 9, 8>};
     const void* prefill[] = {(const void*)&latent_prefill_kernel<T, 2, 4, 8>, (const void*)&latent_prefill_kernel<T, 2, 6, 8>,
                              (const void*)&latent_prefill_kernel<T, 1, 8, 16>, (const void*)&latent_prefill_kernel<T, 1, 16, 32>};
     hipError_t e = hipSuccess;
     for (int i = 0; i < 4 && e == hipSuccess; i++) {
-        e = hipFuncSetAttribute(decode[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kLdsStatic));
+        e = hipFuncSetAttribute(decode[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kDecodeStatic));
         if (e == hipSuccess) e = hipFuncSetAttribute(prefill[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLdsMax);
     }
     return e;

@@ -126,11 +126,10 @@ int program_check_handles(Model& m) {
 }
 
 // Splits of the absorbed attention: about one workgroup per CU over heads and rows, no more than a full context has chunks.
-static uint32_t decode_splits(const Model& m, const OxbLatentDims& d, int dt, uint32_t rows) {
-    const uint32_t tiles = (d.heads + 15) / 16, chunk = oxb_latent_chunk(d, dt), n_chunks = (m.d.max_seq + chunk - 1) / chunk;
+static uint32_t decode_splits(const Model& m, const OxbLatentDims& d, uint32_t rows) {
+    const uint32_t tiles = (d.heads + 15) / 16, most = oxb_latent_max_splits(m.d.max_seq);
     uint32_t s = (g_rt.n_cus + rows * tiles - 1) / (rows * tiles);
-    if (s > OXB_LATENT_MAX_SPLITS) s = OXB_LATENT_MAX_SPLITS;
-    if (s > n_chunks) s = n_chunks;
+    if (s > most) s = most;
     if (s > 8) s = s / 8 * 8;   // head tiles of a split then share an XCD's L2
     return s ? s : 1;
 }
@@ -283,7 +282,7 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
         lp.kv.n_layers = lp.kv.nkv = 1;
         lp.part_o = p.part_o;
         lp.part_ml = p.part_ml;
-        lp.n_splits = decode_splits(m, l.d, p.dt, M);
+        lp.n_splits = decode_splits(m, l.d, M);
         lp.out = a.attn;
         lp.ld_out = oxb_act_ld(l.d.heads * l.d.vdim_p);
         OXB_TRY_HIP(oxb_launch_latent_store(lp, absorbed, p.dt, st), "kernel launch failed: latent_store");
@@ -343,8 +342,8 @@ int program_decode_step(Model& m) {
     return OXB_HIP_OK;
 }
 
-// Portions up to this many tokens take the absorbed form and the few-row products.
-#define OXB_PROGRAM_SHORT OXB_DENSE_GEMV_MAX_ROWS
+// Portions up to this many tokens take the absorbed form.
+#define OXB_PROGRAM_SHORT 16u
 
 int program_prefill(Model& m, uint32_t seq, uint32_t M, uint32_t pos_start, const uint32_t* want, uint32_t n_want, float* d_logits) {
     Program& p = *m.prog;
@@ -667,7 +666,7 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
         if (l.has_mlp) grow(&p.ld_mid, oxb_act_ld(l.ff));
         const size_t tiles = (d.heads + 15) / 16;
         for (uint32_t r = 1; r <= R; r++) {
-            const size_t slots = (size_t)r * tiles * decode_splits(m, d, dt, r);
+            const size_t slots = (size_t)r * tiles * decode_splits(m, d, r);
             if (slots * 16 * d.rank_p > part) part = slots * 16 * d.rank_p;
             if (slots * 32 > ml) ml = slots * 32;
         }
