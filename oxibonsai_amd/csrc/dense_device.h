@@ -66,6 +66,16 @@ __device__ __forceinline__ void copy16_to_lds(const void* src, void* lds_base) {
     const uint32_t at = (uint32_t)__builtin_amdgcn_readfirstlane((int)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)lds_base);
     asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(at), "v"(src) : "m0");
 }
+// The same with the lane's address OFF bytes further on (an immediate of the instruction, which counts for the LDS address
+// too and is taken off there) and the LDS address as a number.
+template <int OFF>
+__device__ __forceinline__ void copy16_to_lds_at(const void* src, uint32_t lds_at) {
+    static_assert(OFF >= 0 && OFF < 4096, "immediate offset");
+    asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off offset:%2" ::"s"(lds_at - OFF), "v"(src), "n"(OFF) : "m0");
+}
+__device__ __forceinline__ uint32_t lds_address(const void* p) {
+    return (uint32_t)__builtin_amdgcn_readfirstlane((int)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)p);
+}
 // Staged units: 16 rows x 32 columns in LDS, filled by such copies from row-major memory.  Lane l brings columns
 // 8 stage_col(l) .. + 7 of row stage_row(l), so four lanes in turn read one row's 64 (128) contiguous bytes, and its 16 bytes
 // land in slot l: row r, column group g sits in slot 4 r + (g ^ (r >> 2)).  The exclusive-or keeps the operand reads of the

@@ -309,6 +309,13 @@ static hipError_t launch_gemv(const OxbDenseParams& p, hipStream_t st) {
     return hipGetLastError();
 }
 
+// Where the few-row kernel is the faster one (measured): always up to 16 rows; up to 32 unless the matrix alone fills the
+// GPU with GEMM tiles; up to 64 where it has few tiles and long rows.
+static bool few_rows(const OxbDenseParams& p, uint32_t n_cus) {
+    const uint32_t tiles = p.n_pad / 16;
+    return p.m <= 16 || (p.m <= 32 && tiles <= 4 * n_cus) || (p.m <= OXB_DENSE_GEMV_MAX_ROWS && tiles <= n_cus && p.k_pad >= 4096);
+}
+
 // Two row tiles per workgroup where the matrix has tiles enough for every CU to get several workgroups all the same; units
 // in flight per wave within what the registers of two workgroups per CU allow.
 template <typename T>
@@ -320,14 +327,14 @@ static hipError_t pick_gemv(const OxbDenseParams& p, uint32_t n_cus, hipStream_t
         if (many) return launch_gemv<T, 2, 1, 4 / S>(p, st);
         return per_wave > 2 ? launch_gemv<T, 1, 1, 8 / S>(p, st) : launch_gemv<T, 1, 1, 2>(p, st);
     }
-    if (p.m <= 32) return many ? launch_gemv<T, 2, 2, 4 / S>(p, st) : launch_gemv<T, 1, 2, 4 / S>(p, st);
+    if (p.m <= 32) return p.n_pad / 16 > n_cus ? launch_gemv<T, 2, 2, 4 / S>(p, st) : launch_gemv<T, 1, 2, 4 / S>(p, st);
     return launch_gemv<T, 1, 4, 2>(p, st);
 }
 
 hipError_t oxb_launch_dense(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st) {
     const hipError_t e = check(p, dt);
     if (e != hipSuccess) return e;
-    if (p.m <= OXB_DENSE_GEMV_MAX_ROWS) return dt == OXB_DT_BF16 ? pick_gemv<__bf16>(p, n_cus, st) : pick_gemv<float>(p, n_cus, st);
+    if (few_rows(p, n_cus)) return dt == OXB_DT_BF16 ? pick_gemv<__bf16>(p, n_cus, st) : pick_gemv<float>(p, n_cus, st);
     return dt == OXB_DT_BF16 ? pick_gemm<__bf16, false>(p, n_cus, st) : pick_gemm<float, false>(p, n_cus, st);
 }
 

@@ -68,6 +68,9 @@ hipError_t oxb_launch_latent_prefill(const OxbLatentParams& p, int dt, hipStream
 hipError_t oxb_latent_prepare(int dt);
 // Whether the kernels can take these sizes, and why not.
 const char* oxb_latent_check(const OxbLatentDims& d, int dt);
+// Head tiles (of 16 heads) a workgroup of the absorbed form takes: two share the cache reads where the rows alone keep the
+// GPU busy, one finishes a lone sequence sooner.
+static inline uint32_t oxb_latent_head_tiles(const OxbLatentDims& d, uint32_t rows) { return d.heads > 16 && rows >= 8 ? 2u : 1u; }
 // Splits of the absorbed form a context of max_seq positions can keep busy.
 uint32_t oxb_latent_max_splits(uint32_t max_seq);
 #define OXB_LATENT_MAX_SPLITS 128u

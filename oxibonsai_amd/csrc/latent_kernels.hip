@@ -101,10 +101,10 @@ __global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, ui
 // so a latent row is read once for all of them and serves as key and as value:
 //   S^T[key][head] = K[key] . q_abs[head]          operand reads of the staged rows
 //   O^T[r][head]  += c[key][r] P[head][key]        the same LDS rows through the transposing read
-// A split walks chunks of 32 keys through a ring of LDS buffers (memory -> LDS copies).  Wave w brings in and multiplies the
-// k units w / 2, w / 2 + 4, ... of key tile w % 2, so it starts on its own copies without a barrier; the partial scores of
-// the four k quarters meet in LDS behind the chunk's one barrier, every wave forms the same probabilities from them, and
-// takes its own eighth of the latent elements of O.  KSQ: k units per wave, NTW: accumulator tiles per wave.
+// A split walks chunks of 32 keys through a ring of LDS buffers (memory -> LDS copies, up to three chunks ahead).  HT head
+// tiles share a workgroup, 8 / HT waves each; of those, wave w multiplies key tile w % 2 with every (4 / HT)-th k unit, the
+// partial scores meet in LDS, every wave of the tile forms the same probabilities from them and takes its own share of the
+// latent elements of O.  KSQ: k units per wave, NTW: accumulator tiles per wave.
 // ---------------------------------------------------------------------------
 static constexpr uint32_t kChunk = 32;
 // Splits in use at a position: two chunks each at least.
@@ -130,34 +130,48 @@ __device__ __forceinline__ v8b value_frag(const __bf16* tile0, const __bf16* til
 }
 __device__ __forceinline__ v8f value_frag(const float* a, const float* b) { return (v8f){a[0], a[16], a[32], a[48], b[0], b[16], b[32], b[48]}; }
 
-template <typename T, int KSQ, int NTW>
+// Units 4 j, j < bring <= N, of a lane's row into the LDS units 4 j behind `at`.
+template <typename T, int N, int J>
+__device__ __forceinline__ void request_units(const T* row, uint32_t at, uint32_t bring) {
+    if constexpr (J < N) {
+        if ((uint32_t)J < bring) {
+            constexpr int PER = 4096 / (128 * (int)sizeof(T));   // units within an immediate offset
+            const T* base = row + J / PER * PER * 128;
+            copy16_to_lds_at<J % PER * 128 * (int)sizeof(T)>(base, at + J * 4 * Dt<T>::unit_bytes);
+            if constexpr (Dt<T>::sub == 2) copy16_to_lds_at<J % PER * 128 * (int)sizeof(T) + 16>(base, at + J * 4 * Dt<T>::unit_bytes + 1024);
+        }
+        request_units<T, N, J + 1>(row, at, bring);
+    }
+}
+
+template <typename T, int HT, int KSQ, int NTW>
 __global__ __launch_bounds__(512) void latent_decode_kernel(OxbLatentParams p, uint32_t n_buf) {
     typedef typename Dt<T>::frag frag;
-    constexpr float kLazy = 8.0f;   // the running maximum follows once it is 2^8 behind
+    constexpr float kLazy = 8.0f;                 // the running maximum follows once it is 2^8 behind
+    constexpr int WPT = 8 / HT, KSPLIT = 4 / HT;  // waves per head tile; waves sharing the k units of a key tile
+    constexpr int DQ = (KSQ + HT - 1) / HT;       // k units a wave brings in, at most (the copies are spread over all 8 waves)
+    constexpr int SUB = Dt<T>::sub;
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
-    __shared__ __attribute__((aligned(16))) float part_s[2][4][16][kChunk + 4];   // two chunks' worth: one barrier per chunk
+    __shared__ __attribute__((aligned(16))) float part_s[HT][KSPLIT][16][kChunk + 4];
     const OxbLatentDims& d = p.d;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
-    const uint32_t split = blockIdx.x, ht = blockIdx.y, m = blockIdx.z;
+    const uint32_t split = blockIdx.x, hw = wave / WPT, ht = blockIdx.y * HT + hw, m = blockIdx.z;
     const uint32_t pos = row_pos(p.rows, m), seq = row_seq(p.rows, m), used = latent_used_splits(pos, p.n_splits);
     if (split >= used) return;
     const uint32_t n_mine = (pos / kChunk - split) / used + 1;   // chunks split, split + used, ...
-    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, kt = wave & 1u, kq = wave >> 1, slot = staged_slot(qi, g);
-    const uint32_t mine = kq < ks ? (ks - kq + 3) / 4 : 0;       // this wave's k units (kq + 4 j)
+    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, kt = wave & 1u, kq = (wave >> 1) % KSPLIT, slot = staged_slot(qi, g);
+    const uint32_t dq = wave >> 1, bring = dq < ks ? (ks - dq + 3) / 4 : 0;   // this wave brings in units dq + 4 j of key tile kt
     T* lds = reinterpret_cast<T*>(smem);
-    const uint32_t buf_elems = 2 * ks * 512;
-    const T* cache = reinterpret_cast<const T*>(p.cache) + 8 * stage_col(lane);
+    const uint32_t buf_elems = 2 * ks * 512, lds0 = lds_address(smem) + (kt * ks + dq) * Dt<T>::unit_bytes;
+    const T* cache = reinterpret_cast<const T*>(p.cache) + 32 * dq + 8 * stage_col(lane);
     const float c2 = d.scale * 1.4426950408889634f;   // scores in units of log2(e)
-    auto unit_of = [&](int j) { return kq + 4 * min((uint32_t)j, mine - 1); };   // (past the end: the last one again)
     auto request = [&](uint32_t i) {
         // rows past the newest position repeat it; their scores are masked
         const uint32_t key = (split + i * used) * kChunk + kt * 16 + stage_row(lane);
         const T* row = cache + kv_row(p.kv, seq, 0, 0, min(key, pos)) * p.ld;
-        T* base = lds + (i % n_buf) * buf_elems + (size_t)kt * ks * 512;
-        if (mine)
-#pragma unroll
-            for (int j = 0; j < KSQ; j++) stage_unit(row + 32 * unit_of(j), base + (size_t)unit_of(j) * 512);
+        const uint32_t at = lds0 + (i % n_buf) * (2 * ks * Dt<T>::unit_bytes);
+        request_units<T, DQ, 0>(row, at, bring);
     };
     const uint32_t ahead = n_buf > 1 ? n_buf - 1 : 1;
     for (uint32_t i = 0; i < ahead && i < n_mine; i++) request(i);
@@ -167,45 +181,49 @@ __global__ __launch_bounds__(512) void latent_decode_kernel(OxbLatentParams p, u
         const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(ht * 16 + qi, d.heads - 1)) * p.ld + 8 * g;
 #pragma unroll
         for (int j = 0; j < KSQ; j++) {
-            q[j] = zero_frag((const T*)nullptr);
-            if ((uint32_t)j < mine) q[j] = load_row8(src + 32 * (kq + 4 * j));
+            const uint32_t s = kq + KSPLIT * j;
+            q[j] = load_row8(src + 32 * min(s, ks - 1));
+            if (s >= ks) q[j] = zero_frag((const T*)nullptr);
         }
     }
-    const uint32_t ntw = (nt + 7) / 8;
+    const uint32_t ntw = (nt + WPT - 1) / WPT, t0 = (wave % WPT) * ntw;
     uint32_t v_at[NTW];
     v4f O[NTW];
 #pragma unroll
     for (int i = 0; i < NTW; i++) {
-        v_at[i] = value_at<T>(min(wave * ntw + i, nt - 1), qi, g);
+        v_at[i] = value_at<T>(min(t0 + i, nt - 1), qi, g);
         O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
     }
-    float m_run = -INFINITY, l_run = 0.f;   // maximum (times c2) and this lane's share of the sum; the same in every wave
+    float m_run = -INFINITY, l_run = 0.f;   // maximum (times c2) and this lane's share of the sum; the same in every wave of a tile
 
     for (uint32_t i = 0; i < n_mine; i++) {
         const uint32_t key0 = (split + i * used) * kChunk;
         const T* kb = lds + (i % n_buf) * buf_elems;
         const T* tile = kb + (size_t)kt * ks * 512;
         // this chunk's copies have arrived; those of later chunks may stay in flight
-        if (n_buf == 3 && i + 1 < n_mine) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KSQ * Dt<T>::sub) : "memory");
-        else wait_lds_copies();
-        v4f s = {0.f, 0.f, 0.f, 0.f};
-        if (mine) {
-            frag k[KSQ];
-#pragma unroll
-            for (int j = 0; j < KSQ; j++) k[j] = load_staged(tile + (size_t)unit_of(j) * 512, slot);
-#pragma unroll
-            for (int j = 0; j < KSQ; j++) s = mfma32(k[j], q[j], s);
+        const uint32_t later = min(ahead - 1, n_mine - 1 - i);
+        if (later == 0 || n_buf == 1) wait_lds_copies();
+        else if (later == 1) {
+            if (bring == (uint32_t)DQ) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(DQ * SUB) : "memory");
+            else asm volatile("s_waitcnt vmcnt(%0)" ::"n"((DQ - 1) * SUB) : "memory");
+        } else {
+            if (bring == (uint32_t)DQ) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * DQ * SUB) : "memory");
+            else asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * (DQ - 1) * SUB) : "memory");
         }
-        *reinterpret_cast<v4f*>(&part_s[i & 1u][kq][qi][kt * 16 + 4 * g]) = s;
-        lds_barrier();   // scores and rows of the whole chunk are in LDS, and every wave is through with the chunk before
+        lds_barrier();   // for every wave; and every wave is through with the chunk before
         if (n_buf > 1 && i + ahead < n_mine) request(i + ahead);
+        v4f s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};   // (two chains of dependent products)
+#pragma unroll
+        for (int j = 0; j < KSQ; j++) s[j & 1] = mfma32(load_staged(tile + (size_t)min(kq + KSPLIT * j, ks - 1) * 512, slot), q[j], s[j & 1]);
+        *reinterpret_cast<v4f*>(&part_s[hw][kq][qi][kt * 16 + 4 * g]) = s[0] + s[1];
+        lds_barrier();
         float sv[8], mx = -INFINITY;
         {
-            v4f a = *reinterpret_cast<const v4f*>(&part_s[i & 1u][0][qi][4 * g]), b = *reinterpret_cast<const v4f*>(&part_s[i & 1u][0][qi][16 + 4 * g]);
+            v4f a = *reinterpret_cast<const v4f*>(&part_s[hw][0][qi][4 * g]), b = *reinterpret_cast<const v4f*>(&part_s[hw][0][qi][16 + 4 * g]);
 #pragma unroll
-            for (int k = 1; k < 4; k++) {
-                a += *reinterpret_cast<const v4f*>(&part_s[i & 1u][k][qi][4 * g]);
-                b += *reinterpret_cast<const v4f*>(&part_s[i & 1u][k][qi][16 + 4 * g]);
+            for (int k = 1; k < KSPLIT; k++) {
+                a += *reinterpret_cast<const v4f*>(&part_s[hw][k][qi][4 * g]);
+                b += *reinterpret_cast<const v4f*>(&part_s[hw][k][qi][16 + 4 * g]);
             }
 #pragma unroll
             for (int v = 0; v < 4; v++) sv[v] = a[v] * c2, sv[4 + v] = b[v] * c2;
@@ -235,26 +253,29 @@ __global__ __launch_bounds__(512) void latent_decode_kernel(OxbLatentParams p, u
         }
         frag hi, lo;
         split_hi_lo(pe, hi, lo);
+        frag v[NTW];
 #pragma unroll
-        for (int t = 0; t < NTW; t++) {
-            const frag a = value_frag(kb + v_at[t], kb + v_at[t] + (size_t)ks * 512);
-            O[t] = mfma32(a, hi, O[t]);
-            if constexpr (!Dt<T>::is_f32) O[t] = mfma32(a, lo, O[t]);
+        for (int t = 0; t < NTW; t++) v[t] = value_frag(kb + v_at[t], kb + v_at[t] + (size_t)ks * 512);
+#pragma unroll
+        for (int t = 0; t < NTW; t++) O[t] = mfma32(v[t], hi, O[t]);
+        if constexpr (!Dt<T>::is_f32) {
+#pragma unroll
+            for (int t = 0; t < NTW; t++) O[t] = mfma32(v[t], lo, O[t]);
         }
-        if (i + 1 < n_mine) {
-            if (n_buf == 1) {
-                lds_barrier();   // every wave is through with the buffer
-                request(i + 1);
-            }
+        if (n_buf == 1 && i + 1 < n_mine) {
+            lds_barrier();   // every wave is through with the buffer
+            request(i + 1);
         }
     }
-    const size_t part = ((size_t)m * gridDim.y + ht) * p.n_splits + split;
+    const uint32_t n_ht = (d.heads + 15) / 16;
+    if (ht >= n_ht) return;
+    const size_t part = ((size_t)m * n_ht + ht) * p.n_splits + split;
     float* po = p.part_o + part * 16 * d.rank_p + (size_t)qi * d.rank_p + 4 * g;
 #pragma unroll
     for (int t = 0; t < NTW; t++)
-        if ((uint32_t)t < ntw && wave * ntw + t < nt) *reinterpret_cast<v4f*>(po + 16 * (wave * ntw + t)) = O[t];
+        if ((uint32_t)t < ntw && t0 + t < nt) *reinterpret_cast<v4f*>(po + 16 * (t0 + t)) = O[t];
     l_run = sum_rows4(l_run);
-    if (wave == 0 && g == 0) {
+    if (wave % WPT == 0 && g == 0) {
         p.part_ml[part * 32 + qi * 2] = m_run;
         p.part_ml[part * 32 + qi * 2 + 1] = l_run;
     }
@@ -571,11 +592,11 @@ __global__ __launch_bounds__(256, QT == 2 && !Dt<T>::is_f32 ? 2 : 1) void latent
 }
 
 // ---------------------------------------------------------------------------
-static constexpr uint32_t kLdsMax = 160u << 10, kDecodeStatic = 2 * 4 * 16 * (kChunk + 4) * 4;   // (decode's partial scores)
+static constexpr uint32_t kLdsMax = 160u << 10, kDecodeStatic = 4 * 16 * (kChunk + 4) * 4;   // (decode's partial scores)
 
 static uint32_t decode_buffers(const OxbLatentDims& d, int dt) {
     const uint32_t n = (kLdsMax - kDecodeStatic) / (kChunk * (d.rank_p + d.rot_p) * oxb_dt_bytes(dt));
-    return n > 3 ? 3 : n;
+    return n > 4 ? 4 : n;
 }
 static uint32_t prefill_block_bytes(const OxbLatentDims& d, int dt) {
     return (2 * (d.dim_p + d.rot_p) / 32 + d.vdim_p / 16) * 512 * oxb_dt_bytes(dt);
@@ -614,20 +635,21 @@ hipError_t oxb_launch_latent_store(const OxbLatentParams& p, bool absorb, int dt
     return hipGetLastError();
 }
 
-template <typename T, int KSQ, int NTW>
+template <typename T, int HT, int KSQ, int NTW>
 static hipError_t launch_decode(const OxbLatentParams& p, uint32_t n_buf, hipStream_t st) {
-    hipLaunchKernelGGL((latent_decode_kernel<T, KSQ, NTW>), dim3(p.n_splits, (p.d.heads + 15) / 16, p.rows.m), dim3(512),
+    hipLaunchKernelGGL((latent_decode_kernel<T, HT, KSQ, NTW>), dim3(p.n_splits, (p.d.heads + 16 * HT - 1) / (16 * HT), p.rows.m), dim3(512),
                        n_buf * kChunk * p.ld * (uint32_t)sizeof(T), st, p, n_buf);
     return hipGetLastError();
 }
 
 template <typename T>
 static hipError_t pick_decode(const OxbLatentParams& p, uint32_t n_buf, hipStream_t st) {
-    const uint32_t nt = p.d.rank_p / 16, ks = p.ld / 32;   // ks - nt / 2 = rot_p / 32 <= 4
-    if (nt <= 8) return launch_decode<T, 2, 1>(p, n_buf, st);
-    if (nt <= 16) return launch_decode<T, 3, 2>(p, n_buf, st);
-    if (nt <= 32 && ks <= 20) return launch_decode<T, 5, 4>(p, n_buf, st);
-    return launch_decode<T, 9, 8>(p, n_buf, st);
+    const uint32_t nt = p.d.rank_p / 16;   // k units: nt / 2 + rot_p / 32, the latter <= 4
+    const bool two = oxb_latent_head_tiles(p.d, p.rows.m) == 2;
+    if (nt <= 8) return two ? launch_decode<T, 2, 4, 2>(p, n_buf, st) : launch_decode<T, 1, 2, 1>(p, n_buf, st);
+    if (nt <= 16) return two ? launch_decode<T, 2, 6, 4>(p, n_buf, st) : launch_decode<T, 1, 3, 2>(p, n_buf, st);
+    if (nt <= 32) return two ? launch_decode<T, 2, 10, 8>(p, n_buf, st) : launch_decode<T, 1, 5, 4>(p, n_buf, st);
+    return two ? launch_decode<T, 2, 18, 16>(p, n_buf, st) : launch_decode<T, 1, 9, 8>(p, n_buf, st);
 }
 
 hipError_t oxb_launch_latent_decode(const OxbLatentParams& p, int dt, hipStream_t st) {
@@ -669,15 +691,17 @@ static hipError_t pick_prefill(const OxbLatentParams& p, uint32_t bytes, hipStre
 // stream capture.
 template <typename T>
 static hipError_t raise_lds() {
-    const void* decode[] = {(const void*)&latent_decode_kernel<T, 2, 1>, (const void*)&latent_decode_kernel<T, 3, 2>,
-                            (const void*)&latent_decode_kernel<T, 5, 4>, (const void*)&latent_decode_kernel<T, 9, 8>};
+    const void* decode[] = {(const void*)&latent_decode_kernel<T, 1, 2, 1>, (const void*)&latent_decode_kernel<T, 1, 3, 2>,
+                            (const void*)&latent_decode_kernel<T, 1, 5, 4>, (const void*)&latent_decode_kernel<T, 1, 9, 8>,
+                            (const void*)&latent_decode_kernel<T, 2, 4, 2>, (const void*)&latent_decode_kernel<T, 2, 6, 4>,
+                            (const void*)&latent_decode_kernel<T, 2, 10, 8>, (const void*)&latent_decode_kernel<T, 2, 18, 16>};
     const void* prefill[] = {(const void*)&latent_prefill_kernel<T, 2, 4, 8>, (const void*)&latent_prefill_kernel<T, 2, 6, 8>,
                              (const void*)&latent_prefill_kernel<T, 1, 8, 16>, (const void*)&latent_prefill_kernel<T, 1, 16, 32>};
     hipError_t e = hipSuccess;
-    for (int i = 0; i < 4 && e == hipSuccess; i++) {
-        e = hipFuncSetAttribute(decode[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kDecodeStatic));
-        if (e == hipSuccess) e = hipFuncSetAttribute(prefill[i], hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLdsMax);
-    }
+    for (const void* f : decode)
+        if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kDecodeStatic));
+    for (const void* f : prefill)
+        if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLdsMax);
     return e;
 }
 hipError_t oxb_latent_prepare(int dt) { return dt == OXB_DT_BF16 ? raise_lds<__bf16>() : raise_lds<float>(); }

@@ -127,7 +127,7 @@ int program_check_handles(Model& m) {
 
 // Splits of the absorbed attention: about one workgroup per CU over heads and rows, no more than a full context has chunks.
 static uint32_t decode_splits(const Model& m, const OxbLatentDims& d, uint32_t rows) {
-    const uint32_t tiles = (d.heads + 15) / 16, most = oxb_latent_max_splits(m.d.max_seq);
+    const uint32_t per = 16 * oxb_latent_head_tiles(d, rows), tiles = (d.heads + per - 1) / per, most = oxb_latent_max_splits(m.d.max_seq);
     uint32_t s = (g_rt.n_cus + rows * tiles - 1) / (rows * tiles);
     if (s > most) s = most;
     if (s > 8) s = s / 8 * 8;   // head tiles of a split then share an XCD's L2
