@@ -3,6 +3,7 @@
 Independent of the product: no code, table or layout is shared with it.  Everything runs in float64 unless a dtype is
 given; weights come in as a dict name -> array (any float type), the configuration as the parsed config.json.
 
+    run_prompt(cfg, w, tokens)     -> logits [T, vocab] of a whole prompt in matrix form
     run(cfg, w, tokens)            -> Trace(logits [T, vocab], layers [runs, T, width])
     Sequence(cfg, w).step(tokens)  -> the same logits, portion by portion, from a per-pass history of latents
 """
@@ -134,3 +135,44 @@ def run(cfg, w, tokens):
     s = Sequence(cfg, w)
     rows = [s.token(t) for t in tokens]
     return Trace(np.stack([a for a, _ in rows]), np.stack([b for _, b in rows], axis=1))
+
+
+def run_prompt(cfg, w, tokens):
+    """The same equations for all positions of one prompt at once -> logits [T, vocab]; for prompts whose token-by-token run
+    would take minutes."""
+    w = {k: np.asarray(v, dtype=np.float64) for k, v in w.items()}
+    eps, n = cfg["norm"]["eps"], len(tokens)
+    x0 = w["embed"][np.asarray(tokens)]
+    x = x0
+    for L, t, first in schedule(cfg):
+        if first:
+            x = np.concatenate([x, x0], axis=1) @ w["loop.in"].T + w["loop.step"][t]
+        p, layer = f"l{L}.", cfg["layers"][L]
+        mix, m = layer["mixer"], p + "mix."
+        nh, dim, rot, vdim, half = mix["heads"], mix["dim"], mix["rot_dim"], mix["vdim"], mix["rot"]["dims"] // 2
+        angle = np.arange(n)[:, None] * float(mix["rot"]["base"]) ** (-2.0 * np.arange(half) / mix["rot"]["dims"])
+        cos, sin = np.cos(angle), np.sin(angle)
+
+        def turn(v):   # [T, ..., rot]
+            c, s = (a.reshape((n,) + (1,) * (v.ndim - 2) + (half,)) for a in (cos, sin))
+            a, b = v[..., :half], v[..., half:2 * half]
+            return np.concatenate([a * c - b * s, b * c + a * s, v[..., 2 * half:]], axis=-1)
+
+        h = norm(x, p + "norm1", w)
+        q = (h @ w[m + "q"].T).reshape(n, nh, dim + rot)
+        kv = h @ w[m + "dkv"].T
+        c = rms_norm(kv[:, :mix["kv_rank"]], w[m + "dkv.norm"], eps)
+        kr = turn(kv[:, mix["kv_rank"]:])
+        qr = turn(q[..., dim:])
+        outs = []
+        for j in range(nh):
+            s = (q[:, j, :dim] @ (c @ w[m + "uk"][j * dim:(j + 1) * dim].T).T + qr[:, j] @ kr.T) * mix["scale"]
+            s = np.where(np.tril(np.ones((n, n), dtype=bool)), s, -np.inf)
+            sink = float(w[m + "sink"][j])
+            top = np.maximum(s.max(axis=1), sink)
+            e = np.exp(s - top[:, None])
+            outs.append((e / (e.sum(axis=1) + np.exp(sink - top))[:, None]) @ (c @ w[m + "uv"][j * vdim:(j + 1) * vdim].T))
+        x = x + np.concatenate(outs, axis=1) @ w[m + "o"].T
+        if layer.get("mlp"):
+            x = x + gelu_tanh(norm(x, p + "norm2", w) @ w[p + "mlp.up"].T) @ w[p + "mlp.down"].T
+    return norm(x, "final.norm", w) @ w["embed"].T * cfg["logit_scale"]

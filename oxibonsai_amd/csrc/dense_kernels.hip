@@ -284,10 +284,10 @@ static hipError_t launch_gemm(const OxbDenseParams& p, hipStream_t st) {
 // Tile choice by measured cost (us for K = 4096): of a workgroup alone on its CU, and per workgroup where a CU gets several.
 template <typename T, bool SWAP>
 static hipError_t pick_gemm(const OxbDenseParams& p, uint32_t n_cus, hipStream_t st) {
-    struct { uint32_t rt, ct; double alone, each; } const opt[] = {{4, 8, 60, 64}, {2, 8, 42, 37.5}, {4, 4, 38, 38}, {2, 4, 28, 23.5}, {1, 8, 41, 28}, {1, 4, 24, 19}};
+    struct { uint32_t rt, ct; double alone, each; } const opt[] = {{4, 8, 60, 64}, {2, 8, 42, 37.5}, {4, 4, 38, 38}, {2, 4, 28, 23.5}, {1, 4, 24, 19}};
     int best = -1;
     double best_cost = 0;
-    for (int i = 0; i < 6; i++) {
+    for (int i = 0; i < 5; i++) {
         if (Dt<T>::is_f32 && opt[i].ct == 8) continue;   // (fp32 stages are twice as large)
         const uint64_t wgs = (uint64_t)((p.m + 16 * opt[i].ct - 1) / (16 * opt[i].ct)) * ((p.n_pad + 64 * opt[i].rt - 1) / (64 * opt[i].rt));
         const double busy = (double)((wgs + n_cus - 1) / n_cus) * opt[i].each, cost = busy > opt[i].alone ? busy : opt[i].alone;
@@ -296,7 +296,6 @@ static hipError_t pick_gemm(const OxbDenseParams& p, uint32_t n_cus, hipStream_t
     if constexpr (!Dt<T>::is_f32) {
         if (best == 0) return launch_gemm<T, 4, 8, SWAP>(p, st);
         if (best == 1) return launch_gemm<T, 2, 8, SWAP>(p, st);
-        if (best == 4) return launch_gemm<T, 1, 8, SWAP>(p, st);
     }
     if (best == 2) return launch_gemm<T, 4, 4, SWAP>(p, st);
     if (best == 3) return launch_gemm<T, 2, 4, SWAP>(p, st);

@@ -130,6 +130,10 @@ static uint32_t decode_splits(const Model& m, const OxbLatentDims& d, uint32_t r
     const uint32_t per = 16 * oxb_latent_head_tiles(d, rows), tiles = (d.heads + per - 1) / per, most = oxb_latent_max_splits(m.d.max_seq);
     uint32_t s = (g_rt.n_cus + rows * tiles - 1) / (rows * tiles);
     if (s > most) s = most;
+    if (const char* e = getenv("OXB_HIP_ATTN_SLOTS")) {  // measurement aid: a fixed slot count (long walks per workgroup)
+        const long v = strtol(e, nullptr, 10);
+        if (v > 0 && (uint32_t)v < s) s = (uint32_t)v;
+    }
     if (s > 8) s = s / 8 * 8;   // head tiles of a split then share an XCD's L2
     return s ? s : 1;
 }

@@ -109,6 +109,13 @@ def test_oracle_portions_and_schedule():
     assert t.layers.shape == (5, 14, cfg["width"])
 
 
+def test_oracle_matrix_form():
+    for cfg in (fm.MIXED, fm.PLAIN):
+        w = fm.values(fm.weights(cfg, 4))
+        ids = fm.tokens(cfg, 5, 25)
+        assert np.allclose(plain.run_prompt(cfg, w, ids), plain.run(cfg, w, ids).logits, atol=1e-10)
+
+
 def test_oracle_mechanisms():
     """Hand-checked values and invariants of the oracle's functions."""
     assert np.allclose(plain.dynamic_tanh(np.array([0.0, 1e9, -1e9]), 0.5, np.array([2.0, 2.0, 2.0]), np.array([1.0, 1.0, 1.0])), [1.0, 3.0, -1.0])

@@ -172,6 +172,55 @@ def test_prompt_lengths_at_tile_edges(make, n):
     assert fm.error(whole(m, e, ids), reference(cfg, bits, ids)) < TOL["float32"]
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("ff,n", [(3072, 512), (3072, 700), (3072, 1950), (2112, 1800), (520, 300), (3072, 40)])
+def test_products_at_every_tile_size(make, dtype, ff, n):
+    """Feed-forward alone at widths and prompt lengths that take the GEMM through its tile sizes, last tiles ragged."""
+    cfg = fm.config(200, 64, [fm.layer(1, 8, 4, 8, 16, ff=ff)])
+    bits = without_attention(fm.weights(cfg, 13))
+    ids = fm.tokens(cfg, 14, n)
+    m, e = make(cfg, bits, dtype, max_seq=2048)
+    w = {k: v.astype(np.float64) for k, v in fm.values(bits).items()}
+    x = w["embed"][ids]
+    x = x + plain.gelu_tanh(plain.norm(x, "l0.norm2", w) @ w["l0.mlp.up"].T) @ w["l0.mlp.down"].T
+    want = plain.norm(x, "final.norm", w) @ w["embed"].T * cfg["logit_scale"]
+    assert fm.error(whole(m, e, ids), want) < (5e-6 if dtype == "float32" else 2e-2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("heads,dim,rot,vdim,rank,n", [(24, 128, 64, 128, 512, 420), (16, 96, 32, 64, 256, 300), (9, 192, 64, 200, 130, 200)])
+def test_large_heads(make, dtype, heads, dim, rot, vdim, rank, n):
+    """Head and latent sizes of large models: prompt, short portions, decoding behind a long context."""
+    cfg = fm.config(192, 80, [fm.layer(heads, dim, rot, vdim, rank)])
+    bits = fm.weights(cfg, 15, sharp=1.5)
+    ids = fm.tokens(cfg, 16, n)
+    m, e = make(cfg, bits, dtype, max_seq=512)
+    want = plain.run_prompt(cfg, fm.values(bits), ids)
+    assert fm.error(whole(m, e, ids), want) < TOL[dtype]
+    got = np.concatenate([in_portions(m, e, ids[:n - 60], [150, 90])] +
+                         [m.forward_tokens(e, ids[at:at + k], at, want=range(k)) for at, k in ((n - 60, 16), (n - 44, 9), (n - 35, 3))] +
+                         [m.forward_tokens(e, [t], n - 32 + i) for i, t in enumerate(ids[n - 32:])])
+    assert fm.error(got, want) < TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("slots", [1, 3])
+def test_long_walks_of_the_decode_attention(make, monkeypatch, dtype, slots):
+    """Few splits, so that each walks many chunks of keys through its ring of buffers: lone rows and portions, one head tile
+    and two, latent sizes with rings of four buffers down to one."""
+    monkeypatch.setenv("OXB_HIP_ATTN_SLOTS", str(slots))
+    for layers in ([fm.layer(18, 32, 16, 24, 64, scale=0.4), fm.layer(3, 24, 8, 16, 300)], [fm.layer(2, 16, 8, 16, 640), fm.layer(20, 16, 8, 8, 500)]):
+        cfg = fm.config(64, 50, layers)
+        bits = fm.weights(cfg, 17, sharp=2.0)
+        ids = fm.tokens(cfg, 18, 330)
+        m, e = make(cfg, bits, dtype, max_seq=384)
+        want = plain.run_prompt(cfg, fm.values(bits), ids)
+        m.forward_tokens(e, ids[:250], 0, want=[])
+        got = np.concatenate([m.forward_tokens(e, ids[at:at + k], at, want=range(k)) for at, k in ((250, 16), (266, 8), (274, 2), (276, 16))] +
+                             [m.forward_tokens(e, [t], 292 + i) for i, t in enumerate(ids[292:])])
+        assert fm.error(got, want[250:]) < (5e-5 if dtype == "float32" else 0.12)
+
+
 def test_logits_of_chosen_tokens(make):
     cfg = fm.MIXED
     bits = fm.weights(cfg, 25)
