@@ -413,7 +413,7 @@ def fulirax_model(be, shape: dict, layers: int, vocab: int, max_seq: int, batch:
     return model, emb, macs
 
 
-def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, long_context: int, only: str = "") -> list:
+def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, long_context: int, only: str = "", which: int = -1) -> list:
     """Prefill and decode of both models from token ids, the token loops on the device; host-timed around whole calls."""
     from oxibonsai_amd import synth
     from oxibonsai_amd.model import Embedding, HipModel
@@ -468,7 +468,7 @@ def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, l
         return r
 
     out = []
-    for shape in FULIRAX_SHAPES:
+    for shape in FULIRAX_SHAPES if which < 0 else FULIRAX_SHAPES[which:which + 1]:
         cfg = dict(fmt=FMT_Q1, n_layers=layers, h=shape["width"], inter=shape["ff"], nq=shape["heads"], nkv=8, hd=128, vocab=vocab,
                    max_seq=0, eps=1e-6, rope_theta=1e6)
         row = {"shape": dict(shape, layers=layers, vocab=vocab, **FULIRAX_LATENT)}
@@ -582,6 +582,7 @@ def main() -> int:
     ap.add_argument("--fulirax", action="store_true",
                     help="instead of the default workload: prefill and decode of Fulirax at real layer sizes, next to the Q1 Qwen3 model of equal size")
     ap.add_argument("--fulirax-layers", type=int, default=8)
+    ap.add_argument("--fulirax-shape", type=int, default=-1, help="one of the shapes alone")
     ap.add_argument("--fulirax-only", choices=["", "fulirax", "qwen3"], default="", help="one of the two models alone (profiling)")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -601,7 +602,7 @@ def main() -> int:
     be = ox.NativeHipBackend(0)
     if args.fulirax:
         rows = fulirax_leg(be, args.fulirax_layers, 32768, args.decode_context, args.decode_tokens,
-                           tuple(int(b) for b in args.decode_batches.split(",") if b), args.long_context, args.fulirax_only)
+                           tuple(int(b) for b in args.decode_batches.split(",") if b), args.long_context, args.fulirax_only, args.fulirax_shape)
         print(json.dumps({"metric": "Fulirax prefill and decode", "n_gpus": 1, "dtype": "bf16", "data": "synthetic, random weights",
                           "prompt": args.decode_context, "steps": args.decode_tokens, "shapes": rows}), flush=True)
         return 0
