@@ -639,7 +639,6 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
     Program& p = *m.prog;
     Loader ld{tensors, dt, m};
     const uint32_t w = c.width;
-    const size_t es = oxb_dt_bytes(dt);
     OXB_TRY_HIP(oxb_latent_prepare(dt), "kernel preparation");
     const TensorView* emb;
     OXB_TRY(ld.get("embed", {c.vocab, w}, &emb));
@@ -697,7 +696,6 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
     OXB_TRY_HIP(hipHostMalloc((void**)&m.h_pos, B * 2 * 4, hipHostMallocCoherent), "pinned staging");
     m.h_tokens = m.h_pos + B;
     m.logits_cap = B * c.vocab;
-    (void)es;
     return oxb_hip_upload_embedding(embedding, emb->data, (size_t)emb->bytes, emb->type, c.vocab, w);
 }
 
