@@ -140,6 +140,15 @@ __device__ __forceinline__ v4f epilogue_resid(const OxbEpilogue& e, uint32_t m, 
 }
 // Four consecutive outputs through the epilogue; resid = epilogue_resid(e, m, n0).
 template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogue& e, uint32_t m, uint32_t n0, v4f y, v4f resid) {
+    if (e.glu_out && n0 >= e.glu) {
+        const uint32_t j = (n0 - e.glu) >> 1;
+        if (j >= e.n_glu) return;
+        y *= e.scale;
+        typedef T pair __attribute__((ext_vector_type(2)));
+        *reinterpret_cast<pair*>(reinterpret_cast<T*>(e.glu_out) + (size_t)m * e.ld_glu + j) =
+            (pair){(T)(gelu_tanh_of<T>(y[0]) * y[1]), (T)(gelu_tanh_of<T>(y[2]) * y[3])};
+        return;
+    }
     const uint32_t lim = e.n > e.fill ? e.n : e.fill;
     if (n0 >= lim) return;
     y *= e.scale;

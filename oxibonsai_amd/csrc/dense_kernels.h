@@ -44,6 +44,10 @@ struct OxbEpilogue {
     const float *nw, *nb;    // [n] norm weight and bias
     float alpha;             // dynamic tanh
     uint32_t n;              // valid columns
+    // gated pairs (null: none): columns glu .. hold (gate, up) pairs and only those; gelu_tanh(gate) * up -> glu_out[m][pair]
+    uint32_t glu;            // a multiple of 4, >= n
+    void* glu_out;           // weights' type
+    uint32_t ld_glu, n_glu;  // pairs, even
 };
 enum { OXB_ACT_NONE = 0, OXB_ACT_GELU_TANH = 1 };
 enum { OXB_NORM_NONE = 0, OXB_NORM_DYT = 1 };   // dynamic tanh: tanh(alpha x) * w + b, elementwise
@@ -64,8 +68,9 @@ struct OxbDenseParams {
 
 // src: row-major source elements on the device (gguf-style type ids: 0 F32, 1 F16, 30 BF16); element (n, k) of the packed
 // matrix is src[row_off[n] + col_off[k]], or zero where either offset is negative.  row_off [n_pad], col_off [k_pad].
-hipError_t oxb_launch_dense_pack(const void* src, int src_type, const int64_t* row_off, const int64_t* col_off, uint32_t n_pad,
-                                 uint32_t k_pad, int dt, void* dst, hipStream_t st);
+// With col_mul [k_pad] it is src[row_off[n] * col_mul[k] + col_off[k]]: columns out of matrices of different row lengths.
+hipError_t oxb_launch_dense_pack(const void* src, int src_type, const int64_t* row_off, const int64_t* col_off, const int64_t* col_mul,
+                                 uint32_t n_pad, uint32_t k_pad, int dt, void* dst, hipStream_t st);
 // y = W x for any m: up to OXB_DENSE_GEMV_MAX_ROWS through the few-row kernel (weights streamed once, K split over the waves of a
 // workgroup), more through the tiled GEMM.
 hipError_t oxb_launch_dense(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st);
@@ -76,3 +81,7 @@ hipError_t oxb_launch_stream_enter(const float* x, uint32_t width, uint32_t m, v
                                    uint32_t x0_fill, const OxbEpilogue& e, int dt, hipStream_t st);
 // out[i][0 .. ld) = in[rows[i]][0 .. ld)
 hipError_t oxb_launch_gather_rows(const void* in, uint32_t ld, const uint32_t* rows, uint32_t n, void* out, int dt, hipStream_t st);
+// RMS norm of fp32 rows x [m][width] into activation rows: out = x / sqrt(mean(x^2) + eps) * w, zeros up to `fill`.
+// in_scale != 1 multiplies x in front of it and is written back.
+hipError_t oxb_launch_row_norm(float* x, uint32_t width, uint32_t m, float in_scale, const float* w, float eps, void* out, uint32_t ld,
+                               uint32_t fill, int dt, hipStream_t st);

@@ -14,13 +14,14 @@
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(512) void dense_pack_kernel(const void* __restrict__ src, int type, const int64_t* __restrict__ row_off,
-                                                         const int64_t* __restrict__ col_off, uint32_t n_units_k, T* __restrict__ dst) {
+                                                         const int64_t* __restrict__ col_off, const int64_t* __restrict__ col_mul,
+                                                         uint32_t n_units_k, T* __restrict__ dst) {
     const uint32_t j = threadIdx.x, lane = j >> 3, e = j & 7u;
     const uint32_t tile = blockIdx.x / n_units_k, u = blockIdx.x % n_units_k;
     const int64_t ro = row_off[tile * 16 + (lane & 15u)], co = col_off[u * 32 + (lane >> 4) * 8 + e];
     float v = 0.f;
     if (ro >= 0 && co >= 0) {
-        const int64_t i = ro + co;
+        const int64_t i = (col_mul ? ro * col_mul[u * 32 + (lane >> 4) * 8 + e] : ro) + co;
         if (type == 0) v = static_cast<const float*>(src)[i];
         else if (type == 1) v = __half2float(static_cast<const __half*>(src)[i]);
         else v = __uint_as_float((uint32_t)static_cast<const uint16_t*>(src)[i] << 16);
@@ -30,17 +31,17 @@ __global__ __launch_bounds__(512) void dense_pack_kernel(const void* __restrict_
     else unit[lane * 8 + e] = (T)v;
 }
 
-hipError_t oxb_launch_dense_pack(const void* src, int src_type, const int64_t* row_off, const int64_t* col_off, uint32_t n_pad,
-                                 uint32_t k_pad, int dt, void* dst, hipStream_t st) {
+hipError_t oxb_launch_dense_pack(const void* src, int src_type, const int64_t* row_off, const int64_t* col_off, const int64_t* col_mul,
+                                 uint32_t n_pad, uint32_t k_pad, int dt, void* dst, hipStream_t st) {
     if (!src || !dst || !row_off || !col_off || n_pad % 16 || k_pad % 32 || !n_pad || !k_pad || (src_type != 0 && src_type != 1 && src_type != 30))
         return hipErrorInvalidValue;
     const uint32_t nu = k_pad / 32;
     const uint64_t grid = (uint64_t)(n_pad / 16) * nu;
     if (grid > 0x7FFFFFFFull) return hipErrorInvalidValue;
     if (dt == OXB_DT_BF16)
-        hipLaunchKernelGGL((dense_pack_kernel<__bf16>), dim3((uint32_t)grid), dim3(512), 0, st, src, src_type, row_off, col_off, nu, (__bf16*)dst);
+        hipLaunchKernelGGL((dense_pack_kernel<__bf16>), dim3((uint32_t)grid), dim3(512), 0, st, src, src_type, row_off, col_off, col_mul, nu, (__bf16*)dst);
     else
-        hipLaunchKernelGGL((dense_pack_kernel<float>), dim3((uint32_t)grid), dim3(512), 0, st, src, src_type, row_off, col_off, nu, (float*)dst);
+        hipLaunchKernelGGL((dense_pack_kernel<float>), dim3((uint32_t)grid), dim3(512), 0, st, src, src_type, row_off, col_off, col_mul, nu, (float*)dst);
     return hipGetLastError();
 }
 
@@ -271,6 +272,7 @@ static hipError_t check(const OxbDenseParams& p, int dt) {
     if (!p.w || !p.x || !p.m || !p.n_pad || !p.k_pad || p.n_pad % OXB_DENSE_PAD || p.k_pad % OXB_DENSE_PAD || p.ldx < p.k_pad || p.ldx % 8 ||
         (dt != OXB_DT_BF16 && dt != OXB_DT_F32) || p.e.n > p.n_pad || p.e.fill > p.n_pad || (p.row_table && (p.row_shift < 4 || p.row_shift > 7)))
         return hipErrorInvalidValue;
+    if (p.e.glu_out && (p.e.glu % 4 || p.e.glu < p.e.n || p.e.n_glu % 2 || p.e.ld_glu % 2 || p.e.n_glu > p.e.ld_glu || p.e.fill > p.e.glu)) return hipErrorInvalidValue;
     return hipSuccess;
 }
 
@@ -384,5 +386,90 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(const v4i* __restrict_
 hipError_t oxb_launch_gather_rows(const void* in, uint32_t ld, const uint32_t* rows, uint32_t n, void* out, int dt, hipStream_t st) {
     if (!in || !rows || !out || !n || ld % 8) return hipErrorInvalidValue;
     hipLaunchKernelGGL(gather_rows_kernel, dim3(n), dim3(256), 0, st, (const v4i*)in, ld * oxb_dt_bytes(dt) / 16, rows, (v4i*)out);
+    return hipGetLastError();
+}
+
+// Grid = rows, 256 threads; a thread keeps up to 16 of its row's values, longer rows are read again.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void row_norm_kernel(float* __restrict__ x, uint32_t width, float in_scale, const float* __restrict__ w,
+                                                       float eps, T* __restrict__ out, uint32_t ld, uint32_t fill) {
+    constexpr int STEP = VEC ? 4 : 1, KEEP = 16 / STEP;
+    __shared__ float red[4];
+    const uint32_t tid = threadIdx.x;
+    float* row = x + (size_t)blockIdx.x * width;
+    T* o = out + (size_t)blockIdx.x * ld;
+    float v[KEEP][STEP], ss = 0.f;
+    auto load = [&](uint32_t i, float (&y)[STEP]) {
+        if constexpr (VEC) {
+            const v4f q = *reinterpret_cast<const v4f*>(row + i);
+#pragma unroll
+            for (int e = 0; e < 4; e++) y[e] = q[e];
+        } else {
+            y[0] = row[i];
+        }
+    };
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+        const uint32_t i = (k * 256 + tid) * STEP;
+#pragma unroll
+        for (int e = 0; e < STEP; e++) v[k][e] = 0.f;
+        if (i < width) load(i, v[k]);
+    }
+#pragma unroll
+    for (int k = 0; k < KEEP; k++)
+#pragma unroll
+        for (int e = 0; e < STEP; e++) {
+            v[k][e] *= in_scale;
+            ss = fmaf(v[k][e], v[k][e], ss);
+        }
+    for (uint32_t i = (KEEP * 256 + tid) * STEP; i < width; i += 256 * STEP) {
+        float y[STEP];
+        load(i, y);
+#pragma unroll
+        for (int e = 0; e < STEP; e++) ss = fmaf(y[e] * in_scale, y[e] * in_scale, ss);
+    }
+    ss = wave_sum_f32(ss);
+    if ((tid & 63u) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)width + eps);
+    auto store = [&](uint32_t i, const float (&y)[STEP]) {
+        if constexpr (VEC) {
+            const v4f g = *reinterpret_cast<const v4f*>(w + i);
+            typename Dt<T>::quad q;
+#pragma unroll
+            for (int e = 0; e < 4; e++) q[e] = (T)(y[e] * inv * g[e]);
+            *reinterpret_cast<typename Dt<T>::quad*>(o + i) = q;
+            if (in_scale != 1.0f) *reinterpret_cast<v4f*>(row + i) = (v4f){y[0], y[1], y[2], y[3]};
+        } else {
+            o[i] = (T)(y[0] * inv * w[i]);
+            if (in_scale != 1.0f) row[i] = y[0];
+        }
+    };
+#pragma unroll
+    for (int k = 0; k < KEEP; k++) {
+        const uint32_t i = (k * 256 + tid) * STEP;
+        if (i < width) store(i, v[k]);
+    }
+    for (uint32_t i = (KEEP * 256 + tid) * STEP; i < width; i += 256 * STEP) {
+        float y[STEP];
+        load(i, y);
+#pragma unroll
+        for (int e = 0; e < STEP; e++) y[e] *= in_scale;
+        store(i, y);
+    }
+    for (uint32_t i = width + tid; i < fill; i += 256) o[i] = (T)0.f;
+}
+
+hipError_t oxb_launch_row_norm(float* x, uint32_t width, uint32_t m, float in_scale, const float* w, float eps, void* out, uint32_t ld,
+                               uint32_t fill, int dt, hipStream_t st) {
+    if (!x || !width || !m || !w || !out || fill > ld || ld < width || ld % 8) return hipErrorInvalidValue;
+    const bool vec = width % 4 == 0;
+    if (dt == OXB_DT_BF16) {
+        if (vec) hipLaunchKernelGGL((row_norm_kernel<__bf16, true>), dim3(m), dim3(256), 0, st, x, width, in_scale, w, eps, (__bf16*)out, ld, fill);
+        else hipLaunchKernelGGL((row_norm_kernel<__bf16, false>), dim3(m), dim3(256), 0, st, x, width, in_scale, w, eps, (__bf16*)out, ld, fill);
+    } else {
+        if (vec) hipLaunchKernelGGL((row_norm_kernel<float, true>), dim3(m), dim3(256), 0, st, x, width, in_scale, w, eps, (float*)out, ld, fill);
+        else hipLaunchKernelGGL((row_norm_kernel<float, false>), dim3(m), dim3(256), 0, st, x, width, in_scale, w, eps, (float*)out, ld, fill);
+    }
     return hipGetLastError();
 }

@@ -1,6 +1,8 @@
 // design.cpp — configuration readers and the registry of designs (see design.h).
 #include "design.h"
 
+#include <cmath>
+
 namespace oxb {
 
 namespace {
@@ -47,6 +49,25 @@ struct Fields {
     }
 };
 
+bool read_rope(Fields& f, uint32_t room, RopeConfig* out) {
+    Fields r = f.object("rot");
+    out->base = r.real("base");
+    out->dims = r.u32("dims", 2, 4096);
+    if (!f.ok || !r.ok) return false;
+    if (out->dims % 2 || out->dims > room) return r.bad("dims must be even and within the rotated part");
+    if (!(out->base > 0)) return r.bad("base must be positive");
+    const Json* scaling = r.j->get("scaling");
+    if (!scaling || scaling->is_null()) return true;
+    Fields s = r.object("scaling");
+    out->factor = s.real("factor");
+    out->low = s.real("low");
+    out->high = s.real("high");
+    out->original = s.real("original");
+    if (s.ok && (!(out->factor > 0) || !(out->low > 0) || !(out->high >= out->low) || !(out->original > 0)))
+        return s.bad("factor, low and original must be positive and high at least low");
+    return s.ok;
+}
+
 bool read_latent_attention(Fields f, MixerConfig* m) {
     m->kind = MixerKind::LatentAttention;
     m->heads = f.u32("heads", 1, 4096);
@@ -55,12 +76,56 @@ bool read_latent_attention(Fields f, MixerConfig* m) {
     m->vdim = f.u32("vdim", 1, 4096);
     m->kv_rank = f.u32("kv_rank", 1, 65536);
     m->scale = (float)f.real("scale");
-    Fields r = f.object("rot");
-    m->rot_base = r.real("base");
-    m->rot_dims = r.u32("dims", 2, 4096);
-    if (f.ok && r.ok && (m->rot_dims % 2 || m->rot_dims > m->rot_dim)) return r.bad("dims must be even and at most rot_dim");
-    if (f.ok && r.ok && !(m->rot_base > 0)) return r.bad("base must be positive");
-    return f.ok && r.ok;
+    if (!read_rope(f, m->rot_dim, &m->rope)) return false;
+    return f.ok;
+}
+
+bool read_grouped_attention(Fields f, MixerConfig* m) {
+    m->kind = MixerKind::GroupedAttention;
+    m->heads = f.u32("heads", 1, 4096);
+    m->kv_heads = f.u32("kv_heads", 1, 4096);
+    m->dim = f.u32("dim", 1, 4096);
+    m->vdim = f.u32("vdim", 1, 4096);
+    m->scale = (float)f.real("scale");
+    if (f.ok && m->heads % m->kv_heads) return f.bad("heads must be a multiple of kv_heads");
+    return f.ok && read_rope(f, m->dim, &m->rope);
+}
+
+bool read_state_space(Fields f, MixerConfig* m) {
+    m->kind = MixerKind::StateSpace;
+    m->heads = f.u32("heads", 1, 4096);
+    m->vdim = f.u32("vdim", 1, 4096);
+    m->state = f.u32("state", 1, 4096);
+    m->groups = f.u32("groups", 1, 4096);
+    m->norm_groups = f.u32("norm_groups", 1, 1u << 20);
+    m->conv = f.u32("conv", 1, 64);
+    if (f.ok && m->heads % m->groups) return f.bad("heads must be a multiple of groups");
+    if (f.ok && (m->heads * m->vdim) % m->norm_groups) return f.bad("norm_groups must divide heads x vdim");
+    return f.ok;
+}
+
+bool read_gated_delta(Fields f, MixerConfig* m) {
+    m->kind = MixerKind::GatedDelta;
+    m->heads = f.u32("heads", 1, 4096);
+    m->kv_heads = f.u32("kv_heads", 1, 4096);
+    m->dim = f.u32("dim", 1, 4096);
+    m->vdim = f.u32("vdim", 1, 4096);
+    m->conv = f.u32("conv", 1, 64);
+    if (f.ok && m->heads % m->kv_heads) return f.bad("heads must be a multiple of kv_heads");
+    return f.ok;
+}
+
+// Grouped attention (left) beside a state space (right).
+bool read_attention_and_state(Fields f, MixerConfig* m) {
+    m->kind = MixerKind::Parallel;
+    m->parts.resize(2);
+    Fields left = f.object("left");
+    if (!left.ok || !read_grouped_attention(left, &m->parts[0])) return false;
+    Fields right = f.object("right");
+    if (!right.ok || !read_state_space(right, &m->parts[1])) return false;
+    m->part_scales = {(float)f.real("left_scale"), (float)f.real("right_scale")};
+    m->part_names = {"left.", "right."};
+    return f.ok;
 }
 
 bool read_dense_mlp(Fields f, MlpConfig* m) {
@@ -69,17 +134,25 @@ bool read_dense_mlp(Fields f, MlpConfig* m) {
     return f.ok;
 }
 
-// The readers of the kinds a layer may name; designs share them.
-struct MixerReader { const char* name; bool (*read)(Fields, MixerConfig*); };
-const MixerReader kMixers[] = {{"latent_attention", read_latent_attention}};
-struct MlpReader { const char* name; bool (*read)(Fields, MlpConfig*); };
-const MlpReader kMlps[] = {{"dense", read_dense_mlp}};
+bool read_gated_mlp(Fields f, MlpConfig* m) {
+    m->kind = MlpKind::Gated;
+    m->ff = f.u32("ff");
+    return f.ok;
+}
 
-bool read_layer(Fields f, LayerConfig* l) {
+// The kinds a design's layers may name, with their readers.
+struct MixerReader { const char* name; bool (*read)(Fields, MixerConfig*); };
+struct MlpReader { const char* name; bool (*read)(Fields, MlpConfig*); };
+struct LayerKinds {
+    std::vector<MixerReader> mixers;
+    std::vector<MlpReader> mlps;
+};
+
+bool read_layer(Fields f, const LayerKinds& kinds, LayerConfig* l) {
     const std::string type = f.text("type");
     if (!f.ok) return false;
     const MixerReader* mr = nullptr;
-    for (const MixerReader& r : kMixers)
+    for (const MixerReader& r : kinds.mixers)
         if (type == r.name) mr = &r;
     if (!mr) return f.bad("type \"" + type + "\" is unknown");
     Fields mixer = f.object("mixer");
@@ -89,19 +162,15 @@ bool read_layer(Fields f, LayerConfig* l) {
     Fields ff = f.object("mlp");
     const std::string kind = ff.text("kind");
     if (!ff.ok) return false;
-    for (const MlpReader& r : kMlps)
+    for (const MlpReader& r : kinds.mlps)
         if (kind == r.name) return l->has_mlp = true, r.read(ff, &l->mlp);
     return ff.bad("kind \"" + kind + "\" is unknown");
 }
 
-// Fulirax: latent attention with sinks, dynamic-tanh norms, dense tanh-GELU feed-forwards, a loop that mixes the embedding
-// output back in, logits through the embedding table.
-bool read_fulirax(const Json& j, DesignConfig* c, std::string* err) {
-    Fields f{&j, "", err};
-    c->norm = NormKind::DynamicTanh;
+// Sizes, the norm's eps and the list of layers.
+bool read_common(Fields& f, const LayerKinds& kinds, DesignConfig* c) {
     c->vocab = f.u32("vocab");
     c->width = f.u32("width");
-    c->logit_scale = (float)f.real("logit_scale");
     Fields n = f.object("norm");
     if (f.ok && n.ok) c->eps = (float)n.real("eps");
     const Json* layers = f.need("layers");
@@ -109,9 +178,21 @@ bool read_fulirax(const Json& j, DesignConfig* c, std::string* err) {
     if (layers->type != Json::Array || layers->a.empty() || layers->a.size() > 4096) return f.bad("layers is not a list of layers");
     for (size_t i = 0; i < layers->a.size(); i++) {
         LayerConfig l;
-        if (!read_layer(Fields{&layers->a[i], "layers[" + std::to_string(i) + "].", err}, &l)) return false;
+        if (!read_layer(Fields{&layers->a[i], "layers[" + std::to_string(i) + "].", f.err}, kinds, &l)) return false;
         c->layers.push_back(l);
     }
+    return true;
+}
+
+// Fulirax: latent attention with sinks, dynamic-tanh norms, dense tanh-GELU feed-forwards, a loop that mixes the embedding
+// output back in, logits through the embedding table.
+bool read_fulirax(const Json& j, DesignConfig* c, std::string* err) {
+    static const LayerKinds kinds = {{{"latent_attention", read_latent_attention}}, {{"dense", read_dense_mlp}}};
+    Fields f{&j, "", err};
+    c->norm = NormKind::DynamicTanh;
+    c->block = BlockKind::Sequential;
+    c->logit_scale = (float)f.real("logit_scale");
+    if (!read_common(f, kinds, c)) return false;
     const Json* loop = j.get("loop");
     if (loop && !loop->is_null()) {
         Fields lf = f.object("loop");
@@ -124,10 +205,23 @@ bool read_fulirax(const Json& j, DesignConfig* c, std::string* err) {
     return true;
 }
 
+// Muvonex: layers of a gated delta rule, or of grouped attention beside a state space; mixer and gated feed-forward read one
+// norm and join the stream together; logits through the embedding table.
+bool read_muvonex(const Json& j, DesignConfig* c, std::string* err) {
+    static const LayerKinds kinds = {{{"delta", read_gated_delta}, {"parallel", read_attention_and_state}}, {{"dense", read_gated_mlp}}};
+    Fields f{&j, "", err};
+    c->norm = NormKind::RmsAroundOne;
+    c->block = BlockKind::Parallel;
+    c->residual_mult = (float)f.real("residual_mult");
+    Fields e = f.object("embedding");
+    if (f.ok && e.ok) c->embed_scale = (float)e.real("scale");
+    return e.ok && read_common(f, kinds, c);
+}
+
 }  // namespace
 
 const std::vector<Design>& designs() {
-    static const std::vector<Design> all = {{"Fulirax", read_fulirax}};
+    static const std::vector<Design> all = {{"Fulirax", read_fulirax}, {"Muvonex", read_muvonex}};
     return all;
 }
 
@@ -154,6 +248,16 @@ bool read_design(const std::string& text, DesignConfig* c, std::string* err) {
     for (const Design& d : designs()) known += std::string(known.empty() ? "" : ", ") + d.architecture;
     *err = "config.json: architecture \"" + a->s + "\" is unknown (known: " + known + ")";
     return false;
+}
+
+double rope_frequency(const RopeConfig& r, uint32_t i) {
+    const double f = std::pow(r.base, -2.0 * (double)i / (double)r.dims);
+    if (r.factor == 0) return f;
+    const double turn = 2.0 * 3.14159265358979323846 / f;   // positions per full turn
+    if (turn < r.original / r.high) return f;
+    if (turn > r.original / r.low) return f / r.factor;
+    const double s = (r.original / turn - r.low) / (r.high - r.low);
+    return (1.0 - s) * f / r.factor + s * f;
 }
 
 std::vector<LayerRun> layer_runs(const DesignConfig& c) {

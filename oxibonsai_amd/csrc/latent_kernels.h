@@ -14,20 +14,13 @@
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 
-#include "kv_quant_device.h"
-
-// Token rows of a launch: row r is the token of sequence seq0 + r * seq_step at position pos[r] (device) or pos0 + r.
-struct OxbRows {
-    const uint32_t* pos;
-    uint32_t pos0, seq0, seq_step, m;
-};
+#include "row_attention.h"
 
 struct OxbLatentDims {
     uint32_t heads, dim, dim_p, rot, rot_p, rank, rank_p, vdim, vdim_p;  // *_p: padded to multiples of 32
     uint32_t rot_dims;                                                    // rotated elements of the rot part (even)
     float scale, eps;
 };
-static inline uint32_t oxb_pad32(uint32_t n) { return (n + 31u) / 32u * 32u; }
 
 struct OxbLatentParams {
     OxbLatentDims d;
@@ -71,6 +64,3 @@ const char* oxb_latent_check(const OxbLatentDims& d, int dt);
 // Head tiles (of 16 heads) a workgroup of the absorbed form takes: two share the cache reads where the rows alone keep the
 // GPU busy, one finishes a lone sequence sooner.
 static inline uint32_t oxb_latent_head_tiles(const OxbLatentDims& d, uint32_t rows) { return d.heads > 16 && rows >= 8 ? 2u : 1u; }
-// Splits of the absorbed form a context of max_seq positions can keep busy.
-uint32_t oxb_latent_max_splits(uint32_t max_seq);
-#define OXB_LATENT_MAX_SPLITS 128u

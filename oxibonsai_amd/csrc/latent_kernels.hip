@@ -4,20 +4,11 @@
 // a weight keeps 16 bits; the fp32 kernels use fp32 operands throughout.
 #include <hip/hip_runtime.h>
 #include <stdint.h>
+#include <cstring>
 
 #include "dense_device.h"
 #include "latent_kernels.h"
-
-__device__ __forceinline__ uint32_t row_pos(const OxbRows& r, uint32_t m) { return r.pos ? r.pos[m] : r.pos0 + m; }
-__device__ __forceinline__ uint32_t row_seq(const OxbRows& r, uint32_t m) { return r.seq0 + m * r.seq_step; }
-
-// Element i of a rotated part v (rot elements, the first rot_dims of them in pairs (i, i + rot_dims / 2)).
-__device__ __forceinline__ float rotated(const float* v, uint32_t i, uint32_t rot_dims, const float* cs, const float* sn) {
-    const uint32_t half = rot_dims >> 1;
-    if (i < half) return v[i] * cs[i] - v[i + half] * sn[i];
-    if (i < rot_dims) return v[i] * cs[i - half] + v[i - half] * sn[i - half];
-    return v[i];
-}
+#include "row_attention_device.h"
 
 // ---------------------------------------------------------------------------
 // New tokens.  The first n_abs blocks of a grid row absorb queries (4 waves, one 16-row tile of (head, latent) each); the
@@ -97,191 +88,6 @@ __global__ __launch_bounds__(256) void latent_store_kernel(OxbLatentParams p, ui
 }
 
 // ---------------------------------------------------------------------------
-// Absorbed attention.  Grid (split, head tile, token row), 8 waves; the 16 heads of a tile are the columns of the products,
-// so a latent row is read once for all of them and serves as key and as value:
-//   S^T[key][head] = K[key] . q_abs[head]          operand reads of the staged rows
-//   O^T[r][head]  += c[key][r] P[head][key]        the same LDS rows through the transposing read
-// A split walks chunks of 32 keys through a ring of LDS buffers (memory -> LDS copies, up to three chunks ahead).  HT head
-// tiles share a workgroup, 8 / HT waves each; of those, wave w multiplies key tile w % 2 with every (4 / HT)-th k unit, the
-// partial scores meet in LDS, every wave of the tile forms the same probabilities from them and takes its own share of the
-// latent elements of O.  KSQ: k units per wave, NTW: accumulator tiles per wave.
-// ---------------------------------------------------------------------------
-static constexpr uint32_t kChunk = 32;
-// Splits in use at a position: two chunks each at least.
-__host__ __device__ static inline uint32_t latent_used_splits(uint32_t pos, uint32_t n_splits) {
-    const uint32_t pairs = (pos / kChunk + 2) / 2;
-    return pairs < n_splits ? pairs : n_splits;
-}
-
-// Value operand: keys 4 g .. 4 g + 3 of both key tiles, one latent element per lane.  `at` = value_at(..) of the tile.
-template <typename T> __device__ __forceinline__ uint32_t value_at(uint32_t sl, uint32_t qi, uint32_t g);
-template <> __device__ __forceinline__ uint32_t value_at<__bf16>(uint32_t sl, uint32_t qi, uint32_t g) {
-    // four consecutive halves per lane for the transposing read: row 4 g + qi / 4, columns 16 sl + 4 (qi % 4) ..
-    return (sl >> 1) * 512 + staged_slot(4 * g + (qi >> 2), (sl & 1u) * 2 + ((qi & 3u) >> 1)) * 8 + (qi & 1u) * 4;
-}
-template <> __device__ __forceinline__ uint32_t value_at<float>(uint32_t sl, uint32_t qi, uint32_t g) {
-    const uint32_t d = 16 * sl + qi, e = d & 7u;   // (the slots of rows 4 g .. 4 g + 3 lie four apart: they share r >> 2)
-    return (d >> 5) * 512 + (e >> 2) * 256 + staged_slot(4 * g, (d & 31u) >> 3) * 4 + (e & 3u);
-}
-__device__ __forceinline__ v8b value_frag(const __bf16* tile0, const __bf16* tile1) {
-    const v4b t0 = __builtin_bit_cast(v4b, lds_read_tr16(reinterpret_cast<const _Float16*>(tile0)));
-    const v4b t1 = __builtin_bit_cast(v4b, lds_read_tr16(reinterpret_cast<const _Float16*>(tile1)));
-    return (v8b){t0[0], t0[1], t0[2], t0[3], t1[0], t1[1], t1[2], t1[3]};
-}
-__device__ __forceinline__ v8f value_frag(const float* a, const float* b) { return (v8f){a[0], a[16], a[32], a[48], b[0], b[16], b[32], b[48]}; }
-
-// Units 4 j, j < bring <= N, of a lane's row into the LDS units 4 j behind `at`.
-template <typename T, int N, int J>
-__device__ __forceinline__ void request_units(const T* row, uint32_t at, uint32_t bring) {
-    if constexpr (J < N) {
-        if ((uint32_t)J < bring) {
-            constexpr int PER = 4096 / (128 * (int)sizeof(T));   // units within an immediate offset
-            const T* base = row + J / PER * PER * 128;
-            copy16_to_lds_at<J % PER * 128 * (int)sizeof(T)>(base, at + J * 4 * Dt<T>::unit_bytes);
-            if constexpr (Dt<T>::sub == 2) copy16_to_lds_at<J % PER * 128 * (int)sizeof(T) + 16>(base, at + J * 4 * Dt<T>::unit_bytes + 1024);
-        }
-        request_units<T, N, J + 1>(row, at, bring);
-    }
-}
-
-template <typename T, int HT, int KSQ, int NTW>
-__global__ __launch_bounds__(512) void latent_decode_kernel(OxbLatentParams p, uint32_t n_buf) {
-    typedef typename Dt<T>::frag frag;
-    constexpr float kLazy = 8.0f;                 // the running maximum follows once it is 2^8 behind
-    constexpr int WPT = 8 / HT, KSPLIT = 4 / HT;  // waves per head tile; waves sharing the k units of a key tile
-    constexpr int DQ = (KSQ + HT - 1) / HT;       // k units a wave brings in, at most (the copies are spread over all 8 waves)
-    constexpr int SUB = Dt<T>::sub;
-    extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
-    __shared__ __attribute__((aligned(16))) float part_s[HT][KSPLIT][16][kChunk + 4];
-    const OxbLatentDims& d = p.d;
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, qi = lane & 15u, g = lane >> 4;
-    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
-    const uint32_t split = blockIdx.x, hw = wave / WPT, ht = blockIdx.y * HT + hw, m = blockIdx.z;
-    const uint32_t pos = row_pos(p.rows, m), seq = row_seq(p.rows, m), used = latent_used_splits(pos, p.n_splits);
-    if (split >= used) return;
-    const uint32_t n_mine = (pos / kChunk - split) / used + 1;   // chunks split, split + used, ...
-    const uint32_t ks = p.ld / 32, nt = d.rank_p / 16, kt = wave & 1u, kq = (wave >> 1) % KSPLIT, slot = staged_slot(qi, g);
-    const uint32_t dq = wave >> 1, bring = dq < ks ? (ks - dq + 3) / 4 : 0;   // this wave brings in units dq + 4 j of key tile kt
-    T* lds = reinterpret_cast<T*>(smem);
-    const uint32_t buf_elems = 2 * ks * 512, lds0 = lds_address(smem) + (kt * ks + dq) * Dt<T>::unit_bytes;
-    const T* cache = reinterpret_cast<const T*>(p.cache) + 32 * dq + 8 * stage_col(lane);
-    const float c2 = d.scale * 1.4426950408889634f;   // scores in units of log2(e)
-    auto request = [&](uint32_t i) {
-        // rows past the newest position repeat it; their scores are masked
-        const uint32_t key = (split + i * used) * kChunk + kt * 16 + stage_row(lane);
-        const T* row = cache + kv_row(p.kv, seq, 0, 0, min(key, pos)) * p.ld;
-        const uint32_t at = lds0 + (i % n_buf) * (2 * ks * Dt<T>::unit_bytes);
-        request_units<T, DQ, 0>(row, at, bring);
-    };
-    const uint32_t ahead = n_buf > 1 ? n_buf - 1 : 1;
-    for (uint32_t i = 0; i < ahead && i < n_mine; i++) request(i);
-
-    frag q[KSQ];
-    {
-        const T* src = reinterpret_cast<const T*>(p.q_abs) + ((size_t)m * d.heads + min(ht * 16 + qi, d.heads - 1)) * p.ld + 8 * g;
-#pragma unroll
-        for (int j = 0; j < KSQ; j++) {
-            const uint32_t s = kq + KSPLIT * j;
-            q[j] = load_row8(src + 32 * min(s, ks - 1));
-            if (s >= ks) q[j] = zero_frag((const T*)nullptr);
-        }
-    }
-    const uint32_t ntw = (nt + WPT - 1) / WPT, t0 = (wave % WPT) * ntw;
-    uint32_t v_at[NTW];
-    v4f O[NTW];
-#pragma unroll
-    for (int i = 0; i < NTW; i++) {
-        v_at[i] = value_at<T>(min(t0 + i, nt - 1), qi, g);
-        O[i] = (v4f){0.f, 0.f, 0.f, 0.f};
-    }
-    float m_run = -INFINITY, l_run = 0.f;   // maximum (times c2) and this lane's share of the sum; the same in every wave of a tile
-
-    for (uint32_t i = 0; i < n_mine; i++) {
-        const uint32_t key0 = (split + i * used) * kChunk;
-        const T* kb = lds + (i % n_buf) * buf_elems;
-        const T* tile = kb + (size_t)kt * ks * 512;
-        // this chunk's copies have arrived; those of later chunks may stay in flight
-        const uint32_t later = min(ahead - 1, n_mine - 1 - i);
-        if (later == 0 || n_buf == 1) wait_lds_copies();
-        else if (later == 1) {
-            if (bring == (uint32_t)DQ) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(DQ * SUB) : "memory");
-            else asm volatile("s_waitcnt vmcnt(%0)" ::"n"((DQ - 1) * SUB) : "memory");
-        } else {
-            if (bring == (uint32_t)DQ) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * DQ * SUB) : "memory");
-            else asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * (DQ - 1) * SUB) : "memory");
-        }
-        lds_barrier();   // for every wave; and every wave is through with the chunk before
-        if (n_buf > 1 && i + ahead < n_mine) request(i + ahead);
-        v4f s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};   // (two chains of dependent products)
-#pragma unroll
-        for (int j = 0; j < KSQ; j++) s[j & 1] = mfma32(load_staged(tile + (size_t)min(kq + KSPLIT * j, ks - 1) * 512, slot), q[j], s[j & 1]);
-        *reinterpret_cast<v4f*>(&part_s[hw][kq][qi][kt * 16 + 4 * g]) = s[0] + s[1];
-        lds_barrier();
-        float sv[8], mx = -INFINITY;
-        {
-            v4f a = *reinterpret_cast<const v4f*>(&part_s[hw][0][qi][4 * g]), b = *reinterpret_cast<const v4f*>(&part_s[hw][0][qi][16 + 4 * g]);
-#pragma unroll
-            for (int k = 1; k < KSPLIT; k++) {
-                a += *reinterpret_cast<const v4f*>(&part_s[hw][k][qi][4 * g]);
-                b += *reinterpret_cast<const v4f*>(&part_s[hw][k][qi][16 + 4 * g]);
-            }
-#pragma unroll
-            for (int v = 0; v < 4; v++) sv[v] = a[v] * c2, sv[4 + v] = b[v] * c2;
-        }
-        if (key0 + kChunk - 1 > pos) {
-#pragma unroll
-            for (int v = 0; v < 4; v++) {
-                if (key0 + 4 * g + v > pos) sv[v] = -INFINITY;
-                if (key0 + 16 + 4 * g + v > pos) sv[4 + v] = -INFINITY;
-            }
-        }
-#pragma unroll
-        for (int e = 0; e < 8; e++) mx = fmaxf(mx, sv[e]);
-        mx = max_rows4(mx);  // finite: key0 <= pos
-        if (__any(mx > m_run + kLazy)) {
-            const float m_new = fmaxf(m_run, mx), alpha = exp2_of<T>(m_run - m_new);
-            m_run = m_new;
-            l_run *= alpha;
-#pragma unroll
-            for (int t = 0; t < NTW; t++) O[t] *= alpha;
-        }
-        float pe[8];
-#pragma unroll
-        for (int e = 0; e < 8; e++) {
-            pe[e] = exp2_of<T>(sv[e] - m_run);
-            l_run += pe[e];
-        }
-        frag hi, lo;
-        split_hi_lo(pe, hi, lo);
-        frag v[NTW];
-#pragma unroll
-        for (int t = 0; t < NTW; t++) v[t] = value_frag(kb + v_at[t], kb + v_at[t] + (size_t)ks * 512);
-#pragma unroll
-        for (int t = 0; t < NTW; t++) O[t] = mfma32(v[t], hi, O[t]);
-        if constexpr (!Dt<T>::is_f32) {
-#pragma unroll
-            for (int t = 0; t < NTW; t++) O[t] = mfma32(v[t], lo, O[t]);
-        }
-        if (n_buf == 1 && i + 1 < n_mine) {
-            lds_barrier();   // every wave is through with the buffer
-            request(i + 1);
-        }
-    }
-    const uint32_t n_ht = (d.heads + 15) / 16;
-    if (ht >= n_ht) return;
-    const size_t part = ((size_t)m * n_ht + ht) * p.n_splits + split;
-    float* po = p.part_o + part * 16 * d.rank_p + (size_t)qi * d.rank_p + 4 * g;
-#pragma unroll
-    for (int t = 0; t < NTW; t++)
-        if ((uint32_t)t < ntw && t0 + t < nt) *reinterpret_cast<v4f*>(po + 16 * (t0 + t)) = O[t];
-    l_run = sum_rows4(l_run);
-    if (wave % WPT == 0 && g == 0) {
-        p.part_ml[part * 32 + qi * 2] = m_run;
-        p.part_ml[part * 32 + qi * 2 + 1] = l_run;
-    }
-}
-
-// ---------------------------------------------------------------------------
 // Merge of one head's splits - the sink joins the denominator here, once - and the value product W_uv (sum p c).
 // Grid (head, token row), 8 waves, a tile of 16 value rows each; UN units of the product's weights are in flight per wave.
 // ---------------------------------------------------------------------------
@@ -290,12 +96,12 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(OxbLatentParams p) {
     typedef typename Dt<T>::frag frag;
     constexpr int UN = 8;
     extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
-    __shared__ float wgt[OXB_LATENT_MAX_SPLITS];
+    __shared__ float wgt[OXB_MAX_SPLITS];
     const OxbLatentDims& d = p.d;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, c = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
     const uint32_t head = blockIdx.x, m = blockIdx.y, ht = head / 16, col = head % 16, n_ht = (d.heads + 15) / 16;
-    const uint32_t used = latent_used_splits(row_pos(p.rows, m), p.n_splits);
+    const uint32_t used = oxb_used_splits(row_pos(p.rows, m), p.n_splits);
     const size_t slot0 = ((size_t)m * n_ht + ht) * p.n_splits;
     const float sink = p.sink[head] * 1.4426950408889634f;   // (maxima are in units of log2(e))
     const uint32_t nu = p.k_uv / 32, tiles = d.vdim_p / 16;
@@ -592,26 +398,17 @@ __global__ __launch_bounds__(256, QT == 2 && !Dt<T>::is_f32 ? 2 : 1) void latent
 }
 
 // ---------------------------------------------------------------------------
-static constexpr uint32_t kLdsMax = 160u << 10, kDecodeStatic = 4 * 16 * (kChunk + 4) * 4;   // (decode's partial scores)
+static constexpr uint32_t kLdsMax = 160u << 10;
 
-static uint32_t decode_buffers(const OxbLatentDims& d, int dt) {
-    const uint32_t n = (kLdsMax - kDecodeStatic) / (kChunk * (d.rank_p + d.rot_p) * oxb_dt_bytes(dt));
-    return n > 4 ? 4 : n;
-}
 static uint32_t prefill_block_bytes(const OxbLatentDims& d, int dt) {
     return (2 * (d.dim_p + d.rot_p) / 32 + d.vdim_p / 16) * 512 * oxb_dt_bytes(dt);
 }
-uint32_t oxb_latent_max_splits(uint32_t max_seq) {
-    const uint32_t n = latent_used_splits(max_seq - 1, OXB_LATENT_MAX_SPLITS);
-    return n;
-}
-
 const char* oxb_latent_check(const OxbLatentDims& d, int dt) {
     if (!d.heads || !d.dim || !d.rot || !d.rank || !d.vdim) return "a latent attention size is 0";
     if (d.rot_dims > d.rot || d.rot_dims % 2) return "rotated dimensions must be even and within the rotated part";
     if (d.rank > 1024 || d.rot > 128) return "latent size beyond 1024 or rotated part beyond 128";
     if (d.dim_p + d.rot_p > 512 || d.vdim > 512) return "head size beyond 512";
-    if (!decode_buffers(d, dt)) return "a block of latent rows exceeds the LDS";
+    if (const char* why = oxb_row_check((d.rank_p + d.rot_p) / 32, dt)) return why;
     if (prefill_block_bytes(d, dt) > kLdsMax) return "a block of keys and values exceeds the LDS";
     return nullptr;
 }
@@ -635,33 +432,29 @@ hipError_t oxb_launch_latent_store(const OxbLatentParams& p, bool absorb, int dt
     return hipGetLastError();
 }
 
-template <typename T, int HT, int KSQ, int NTW>
-static hipError_t launch_decode(const OxbLatentParams& p, uint32_t n_buf, hipStream_t st) {
-    hipLaunchKernelGGL((latent_decode_kernel<T, HT, KSQ, NTW>), dim3(p.n_splits, (p.d.heads + 16 * HT - 1) / (16 * HT), p.rows.m), dim3(512),
-                       n_buf * kChunk * p.ld * (uint32_t)sizeof(T), st, p, n_buf);
-    return hipGetLastError();
-}
-
-template <typename T>
-static hipError_t pick_decode(const OxbLatentParams& p, uint32_t n_buf, hipStream_t st) {
-    const uint32_t nt = p.d.rank_p / 16;   // k units: nt / 2 + rot_p / 32, the latter <= 4
-    const bool two = oxb_latent_head_tiles(p.d, p.rows.m) == 2;
-    if (nt <= 8) return two ? launch_decode<T, 2, 4, 2>(p, n_buf, st) : launch_decode<T, 1, 2, 1>(p, n_buf, st);
-    if (nt <= 16) return two ? launch_decode<T, 2, 6, 4>(p, n_buf, st) : launch_decode<T, 1, 3, 2>(p, n_buf, st);
-    if (nt <= 32) return two ? launch_decode<T, 2, 10, 8>(p, n_buf, st) : launch_decode<T, 1, 5, 4>(p, n_buf, st);
-    return two ? launch_decode<T, 2, 18, 16>(p, n_buf, st) : launch_decode<T, 1, 9, 8>(p, n_buf, st);
-}
-
 hipError_t oxb_launch_latent_decode(const OxbLatentParams& p, int dt, hipStream_t st) {
-    if (!rows_ok(p) || oxb_latent_check(p.d, dt) || !p.q_abs || !p.part_o || !p.part_ml || !p.n_splits || p.n_splits > OXB_LATENT_MAX_SPLITS)
-        return hipErrorInvalidValue;
-    const uint32_t n_buf = decode_buffers(p.d, dt);
-    return dt == OXB_DT_BF16 ? pick_decode<__bf16>(p, n_buf, st) : pick_decode<float>(p, n_buf, st);
+    if (!rows_ok(p) || oxb_latent_check(p.d, dt) || !p.q_abs) return hipErrorInvalidValue;
+    OxbRowAttnParams a;
+    memset(&a, 0, sizeof a);
+    a.rows = p.rows;
+    a.kv = p.kv;
+    a.q = p.q_abs;
+    a.heads = a.rep = p.d.heads;
+    a.cache = p.cache;
+    a.ld = p.ld;
+    a.ks = p.ld / 32;
+    a.nt = p.d.rank_p / 16;
+    a.scale = p.d.scale;
+    a.sink = p.sink;
+    a.part_o = p.part_o;
+    a.part_ml = p.part_ml;
+    a.n_splits = p.n_splits;
+    return oxb_launch_row_decode(a, oxb_latent_head_tiles(p.d, p.rows.m), dt, st);
 }
 
 hipError_t oxb_launch_latent_merge(const OxbLatentParams& p, int dt, hipStream_t st) {
     if (!rows_ok(p) || !p.part_o || !p.part_ml || !p.out || !p.w_uv || p.k_uv < p.d.rank_p || p.k_uv % 32 || p.ld_out < p.d.heads * p.d.vdim_p ||
-        !p.n_splits || p.n_splits > OXB_LATENT_MAX_SPLITS)
+        !p.n_splits || p.n_splits > OXB_MAX_SPLITS)
         return hipErrorInvalidValue;
     const dim3 grid(p.d.heads, p.rows.m);
     const uint32_t cols = p.d.rank_p / 4, shares = 512 / cols > 8 ? 8 : 512 / cols ? 512 / cols : 1;
@@ -691,20 +484,18 @@ static hipError_t pick_prefill(const OxbLatentParams& p, uint32_t bytes, hipStre
 // stream capture.
 template <typename T>
 static hipError_t raise_lds() {
-    const void* decode[] = {(const void*)&latent_decode_kernel<T, 1, 2, 1>, (const void*)&latent_decode_kernel<T, 1, 3, 2>,
-                            (const void*)&latent_decode_kernel<T, 1, 5, 4>, (const void*)&latent_decode_kernel<T, 1, 9, 8>,
-                            (const void*)&latent_decode_kernel<T, 2, 4, 2>, (const void*)&latent_decode_kernel<T, 2, 6, 4>,
-                            (const void*)&latent_decode_kernel<T, 2, 10, 8>, (const void*)&latent_decode_kernel<T, 2, 18, 16>};
     const void* prefill[] = {(const void*)&latent_prefill_kernel<T, 2, 4, 8>, (const void*)&latent_prefill_kernel<T, 2, 6, 8>,
                              (const void*)&latent_prefill_kernel<T, 1, 8, 16>, (const void*)&latent_prefill_kernel<T, 1, 16, 32>};
     hipError_t e = hipSuccess;
-    for (const void* f : decode)
-        if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kDecodeStatic));
     for (const void* f : prefill)
         if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLdsMax);
     return e;
 }
-hipError_t oxb_latent_prepare(int dt) { return dt == OXB_DT_BF16 ? raise_lds<__bf16>() : raise_lds<float>(); }
+hipError_t oxb_latent_prepare(int dt) {
+    const hipError_t e = oxb_row_attention_prepare(dt);
+    if (e != hipSuccess) return e;
+    return dt == OXB_DT_BF16 ? raise_lds<__bf16>() : raise_lds<float>();
+}
 
 hipError_t oxb_launch_latent_prefill(const OxbLatentParams& p, int dt, hipStream_t st) {
     if (!rows_ok(p) || oxb_latent_check(p.d, dt) || p.rows.pos || p.rows.seq_step || !p.k_exp || !p.v_exp_t || !p.out ||

@@ -276,10 +276,21 @@ static int kv_reserve(Model& m, uint32_t seq, uint64_t n_tokens) {
 }
 
 static void kv_release(Model& m, uint32_t seq) {  // PagedKvCache::drop_sequence (:362-375): pages go back to the pool
+    if (m.prog) program_commit(m, seq, 0);
     if (!m.n_pages) return;
     std::vector<uint32_t>& pg = m.seq_pages[seq];
     for (size_t i = pg.size(); i-- > 0;) m.free_pages.push_back(pg[i]);
     pg.clear();
+}
+
+// Recurrent memory of a program model: sequence `seq` takes n tokens from position pos on.  Between begin and end (reached only
+// when everything has run) it stands nowhere.
+static int memory_begin(Model& m, uint32_t seq, uint32_t pos) { return m.prog ? program_begin(m, seq, pos) : OXB_HIP_OK; }
+static void memory_open(Model& m, uint32_t seq) {
+    if (m.prog) program_commit(m, seq, kNoPosition);
+}
+static void memory_end(Model& m, uint32_t seq, uint32_t next) {
+    if (m.prog) program_commit(m, seq, next);
 }
 
 // The device copy of the page tables follows the host's before the next launch reads it (never inside a capture).
@@ -638,8 +649,10 @@ static uint32_t attn_slots(const Model& m, uint32_t kv_mode) {
 static int alloc_kv_cache(Model& m, uint32_t kv_mode, uint32_t page_size, uint32_t n_pages) {
     const oxb_model_desc& d = m.d;
     free_kv_cache(m);
+    if (m.prog)
+        for (uint32_t b = 0; b < d.batch; b++) program_commit(m, b, 0);
     m.row_stride = (d.max_seq + OXB_ATTN_CHUNK_POSITIONS - 1) / OXB_ATTN_CHUNK_POSITIONS * OXB_ATTN_CHUNK_POSITIONS;
-    // a layer program keeps latent rows, one region per layer run (program.hip), in k_cache alone
+    // a layer program keeps all its rows, one region per layer run (program.hip), in k_cache alone
     const size_t rows = m.prog ? (n_pages ? (size_t)n_pages * page_size : (size_t)d.batch * m.row_stride)
                                : (n_pages ? (size_t)n_pages * d.n_layers * d.nkv * page_size : (size_t)d.batch * d.n_layers * d.nkv * m.row_stride);
     const size_t bytes = m.prog ? rows * program_cache_row_bytes(*m.prog) : rows * d.hd * (kv_mode == OXB_KV_F16 ? 2 : 1);
@@ -649,8 +662,8 @@ static int alloc_kv_cache(Model& m, uint32_t kv_mode, uint32_t page_size, uint32
         return fail(OXB_HIP_OUT_OF_MEMORY, "out of device memory: requested %zu bytes of KV cache on device %d", n, g_rt.device);
     };
     OXB_TRY(grab(&m.k_cache, bytes));
-    if (m.prog) OXB_TRY_HIP(hipMemset(m.k_cache, 0, bytes), "cache clear");   // rows are written whole; nothing unwritten may be a NaN
-    else OXB_TRY(grab(&m.v_cache, bytes));
+    if (m.prog && bytes) OXB_TRY_HIP(hipMemset(m.k_cache, 0, bytes), "cache clear");   // rows are written whole; nothing unwritten may be a NaN
+    if (!m.prog) OXB_TRY(grab(&m.v_cache, bytes));
     if (kv_mode != OXB_KV_F16) {
         const size_t sb = rows * sizeof(float);
         OXB_TRY(grab((void**)&m.k_scale, sb));
@@ -793,7 +806,7 @@ int oxb_hip_model_set_attention(uint64_t model, const oxb_attention_options* opt
     if (opt->kv_dtype != OXB_KV_DTYPE_F16 && opt->kv_dtype != OXB_KV_DTYPE_I8 && opt->kv_dtype != OXB_KV_DTYPE_FP8_E4M3)
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: unknown KV cache type %d", opt->kv_dtype);
     if (m->prog && (opt->kv_dtype != OXB_KV_DTYPE_F16 || opt->window_size))
-        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: a latent cache keeps its rows in the model's own type and has no window (paging is available)");
+        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: a configured design keeps its cache rows in the model's own type and has no window (paging is available)");
     OXB_TRY_HIP(hipStreamSynchronize(g_rt.stream), "synchronize");
     // the captured decode step holds the cache pointers and the options: it is captured again on the next step
     if (m->graph_exec) (void)hipGraphExecDestroy(m->graph_exec);
@@ -839,7 +852,7 @@ int oxb_hip_model_read_kv(uint64_t model, uint32_t seq, uint32_t layer, uint32_t
     Model* m = find_model(model);
     if (!m) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: unknown model %llu", (unsigned long long)model);
     const oxb_model_desc& d = m->d;
-    if (m->prog) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the rows of a latent cache are not key / value rows");
+    if (m->prog) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the cache rows of a configured design are its own");
     if (seq >= d.batch || layer >= d.n_layers || kv_head >= d.nkv || (uint64_t)pos + n_pos > d.max_seq)
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: cache rows (sequence %u, layer %u, head %u, positions %u..%llu) out of range",
                     seq, layer, kv_head, pos, (unsigned long long)pos + n_pos);
@@ -1060,9 +1073,11 @@ int oxb_hip_decode(uint64_t model, const float* hidden, const uint32_t* pos, flo
     for (uint32_t b = 0; b < d.batch; b++)
         if (pos[b] >= d.max_seq)
             return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: position %u exceeds the context of %u", pos[b], d.max_seq);
+    for (uint32_t b = 0; b < d.batch; b++) OXB_TRY(memory_begin(m, b, pos[b]));
     for (uint32_t b = 0; b < d.batch; b++) OXB_TRY(kv_reserve(m, b, (uint64_t)pos[b] + 1));
     OXB_TRY(kv_sync_table(m));
     hipStream_t st = g_rt.stream;
+    for (uint32_t b = 0; b < d.batch; b++) memory_open(m, b);
     // (the previous call ended with a stream synchronisation, so the staging buffers are free)
     memcpy(m.h_hidden, hidden, (size_t)d.batch * d.h * 4);
     memcpy(m.h_pos, pos, (size_t)d.batch * 4);
@@ -1073,6 +1088,7 @@ int oxb_hip_decode(uint64_t model, const float* hidden, const uint32_t* pos, flo
         OXB_TRY_HIP(hipMemcpyAsync(logits_or_null, m.logits, (size_t)d.batch * d.vocab * 4, hipMemcpyDeviceToHost, st), "logits download");
     hipError_t e = hipStreamSynchronize(st);
     if (e != hipSuccess) return fail(OXB_HIP_SYNC_FAILED, "device synchronization failed: decode: %s", hipGetErrorString(e));
+    for (uint32_t b = 0; b < d.batch; b++) memory_end(m, b, pos[b] + 1);
     if (token_out) memcpy(token_out, m.h_tokens, (size_t)d.batch * 4);
     return OXB_HIP_OK;
     OXB_API_END
@@ -1190,17 +1206,20 @@ int oxb_hip_prefill(uint64_t model, uint32_t seq, const float* hidden, uint32_t 
     if ((uint64_t)pos_start + n_tokens > d.max_seq)
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: positions %u..%llu exceed the context of %u", pos_start,
                     (unsigned long long)pos_start + n_tokens - 1, d.max_seq);
+    OXB_TRY(memory_begin(m, seq, pos_start));
     OXB_TRY(kv_reserve(m, seq, (uint64_t)pos_start + n_tokens));
     OXB_TRY(kv_sync_table(m));
     OXB_TRY(ensure_prefill_buffers(m, n_tokens, pos_start));
     hipStream_t st = g_rt.stream;
     OXB_TRY_HIP(hipMemcpyAsync(m.pf_hidden, hidden, (size_t)n_tokens * d.h * 4, hipMemcpyHostToDevice, st), "hidden upload");
+    memory_open(m, seq);
     OXB_TRY(encode_prefill(m, seq, n_tokens, pos_start));
     if (token_out_or_null) OXB_TRY_HIP(hipMemcpyAsync(token_out_or_null, m.tokens + seq, 4, hipMemcpyDeviceToHost, st), "token download");
     if (logits_or_null)
         OXB_TRY_HIP(hipMemcpyAsync(logits_or_null, m.logits + (size_t)seq * d.vocab, (size_t)d.vocab * 4, hipMemcpyDeviceToHost, st), "logits download");
     hipError_t e = hipStreamSynchronize(st);
     if (e != hipSuccess) return fail(OXB_HIP_SYNC_FAILED, "device synchronization failed: prefill: %s", hipGetErrorString(e));
+    memory_end(m, seq, pos_start + n_tokens);
     return OXB_HIP_OK;
     OXB_API_END
 }
@@ -1380,6 +1399,7 @@ static int decode_tokens_impl(uint64_t model, uint64_t embedding, const uint32_t
         if ((uint64_t)pos[b] + n_steps > d.max_seq)
             return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: positions %u..%llu exceed the context of %u", pos[b],
                         (unsigned long long)pos[b] + n_steps - 1, d.max_seq);
+    for (uint32_t b = 0; b < d.batch; b++) OXB_TRY(memory_begin(m, b, pos[b]));
     for (uint32_t b = 0; b < d.batch; b++) OXB_TRY(kv_reserve(m, b, (uint64_t)pos[b] + n_steps));
     OXB_TRY(kv_sync_table(m));
     const bool sampled = sp && sp->temperature >= 1e-6f;  // below: greedy (sampling.rs:89-92)
@@ -1395,6 +1415,8 @@ static int decode_tokens_impl(uint64_t model, uint64_t embedding, const uint32_t
     uint32_t* hist = (uint32_t*)m.tok_hist.ptr;
     OXB_TRY_HIP(hipMemcpyAsync(m.tokens, tokens, (size_t)d.batch * 4, hipMemcpyHostToDevice, st), "token upload");
     OXB_TRY_HIP(hipMemcpyAsync(m.pos, pos, (size_t)d.batch * 4, hipMemcpyHostToDevice, st), "position upload");
+    if (n_steps)
+        for (uint32_t b = 0; b < d.batch; b++) memory_open(m, b);
     for (uint32_t i = 0; i < n_steps; i++) {
         OXB_TRY_HIP(oxb_launch_embedding_gather(e->d, e->type, e->vocab, d.h, m.tokens, d.batch, m.hidden, st),
                     "kernel launch failed: embedding_gather");
@@ -1409,6 +1431,8 @@ static int decode_tokens_impl(uint64_t model, uint64_t embedding, const uint32_t
     if (sampled) OXB_TRY_HIP(hipMemcpyAsync(rng_state, m.rng.ptr, (size_t)d.batch * 8, hipMemcpyDeviceToHost, st), "rng state download");
     hipError_t he = hipStreamSynchronize(st);
     if (he != hipSuccess) return fail(OXB_HIP_SYNC_FAILED, "device synchronization failed: decode_tokens: %s", hipGetErrorString(he));
+    if (n_steps)
+        for (uint32_t b = 0; b < d.batch; b++) memory_end(m, b, pos[b] + n_steps);
     return OXB_HIP_OK;
 }
 
@@ -1497,6 +1521,7 @@ int oxb_hip_prefill_tokens(uint64_t model, uint64_t embedding, uint32_t seq, con
         return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: positions %u..%llu exceed the context of %u", pos_start,
                     (unsigned long long)pos_start + n_tokens - 1, d.max_seq);
     OXB_TRY(check_ids(*e, ids, n_tokens));
+    OXB_TRY(memory_begin(m, seq, pos_start));
     OXB_TRY(kv_reserve(m, seq, (uint64_t)pos_start + n_tokens));
     OXB_TRY(kv_sync_table(m));
     OXB_TRY(ensure_prefill_buffers(m, n_tokens, pos_start));
@@ -1505,12 +1530,14 @@ int oxb_hip_prefill_tokens(uint64_t model, uint64_t embedding, uint32_t seq, con
     OXB_TRY_HIP(hipMemcpyAsync(m.tok_ids.ptr, ids, (size_t)n_tokens * 4, hipMemcpyHostToDevice, st), "token id upload");
     OXB_TRY_HIP(oxb_launch_embedding_gather(e->d, e->type, e->vocab, d.h, (const uint32_t*)m.tok_ids.ptr, n_tokens, m.pf_hidden, st),
                 "kernel launch failed: embedding_gather");
+    memory_open(m, seq);
     OXB_TRY(encode_prefill(m, seq, n_tokens, pos_start));
     if (token_out_or_null) OXB_TRY_HIP(hipMemcpyAsync(token_out_or_null, m.tokens + seq, 4, hipMemcpyDeviceToHost, st), "token download");
     if (logits_or_null)
         OXB_TRY_HIP(hipMemcpyAsync(logits_or_null, m.logits + (size_t)seq * d.vocab, (size_t)d.vocab * 4, hipMemcpyDeviceToHost, st), "logits download");
     hipError_t he = hipStreamSynchronize(st);
     if (he != hipSuccess) return fail(OXB_HIP_SYNC_FAILED, "device synchronization failed: prefill_tokens: %s", hipGetErrorString(he));
+    memory_end(m, seq, pos_start + n_tokens);
     return OXB_HIP_OK;
     OXB_API_END
 }
@@ -1784,9 +1811,11 @@ int oxb_hip_forward_tokens(uint64_t model, uint64_t embedding, uint32_t seq, con
                     (unsigned long long)pos_start + n_tokens - 1, d.max_seq);
     if (m.checked_gen != g_rt.weights_gen) OXB_TRY(check_model_handles(m));
     OXB_TRY(check_ids(*e, ids, n_tokens));
+    OXB_TRY(memory_begin(m, seq, pos_start));
     OXB_TRY(kv_reserve(m, seq, (uint64_t)pos_start + n_tokens));
     OXB_TRY(kv_sync_table(m));
     hipStream_t st = g_rt.stream;
+    memory_open(m, seq);
     if (n_tokens == 1 && d.batch == 1) {   // a decode step, the one the token loops replay
         OXB_TRY_HIP(hipMemcpyAsync(m.tokens, ids, 4, hipMemcpyHostToDevice, st), "token upload");
         OXB_TRY_HIP(hipMemcpyAsync(m.pos, &pos_start, 4, hipMemcpyHostToDevice, st), "position upload");
@@ -1805,6 +1834,7 @@ int oxb_hip_forward_tokens(uint64_t model, uint64_t embedding, uint32_t seq, con
     }
     hipError_t he = hipStreamSynchronize(st);
     if (he != hipSuccess) return fail(OXB_HIP_SYNC_FAILED, "device synchronization failed: forward_tokens: %s", hipGetErrorString(he));
+    memory_end(m, seq, pos_start + n_tokens);
     return OXB_HIP_OK;
     OXB_API_END
 }

@@ -7,6 +7,8 @@
 
 namespace oxb {
 
+static constexpr uint32_t kNoPosition = 0xFFFFFFFFu;
+
 // Uploads the tensors, creates the model and its embedding table.  dt: OXB_DT_*.
 int program_create(const DesignConfig& c, const TensorMap& tensors, int dt, uint32_t max_seq, uint32_t batch, uint64_t* model,
                    uint64_t* embedding);
@@ -18,6 +20,10 @@ int program_prefill_buffers(Model& m, uint32_t rows, uint32_t pos_start);
 // M tokens of one sequence, embedding rows in m.pf_hidden.  Logits of the wanted rows (host indices into the portion; null:
 // the last row only) -> d_logits [n_want][vocab]; n_want 0: none.
 int program_prefill(Model& m, uint32_t seq, uint32_t M, uint32_t pos_start, const uint32_t* want, uint32_t n_want, float* d_logits);
+// Recurrent memory: whether sequence `seq` can take tokens from position `pos` on, and where it stands afterwards
+// (kNoPosition while a call is under way; 0 once its slot is free).
+int program_begin(Model& m, uint32_t seq, uint32_t pos);
+void program_commit(Model& m, uint32_t seq, uint32_t next);
 // Bytes of cache per position over all layer runs.
 size_t program_cache_row_bytes(const Program& p);
 

@@ -7,76 +7,20 @@
 // nothing else.  A repeated layer's runs share weights and differ in their cache regions.
 #include <hip/hip_runtime.h>
 
-#include <hip/hip_fp16.h>
-
+#include <algorithm>
 #include <cmath>
 #include <cstdlib>
 #include <cstring>
 
-#include "dense_kernels.h"
-#include "gguf.h"
-#include "latent_kernels.h"
 #include "layer_kernels.h"
-#include "program.h"
+#include "program_internal.h"
 
 namespace oxb {
-
-struct ProgramNorm {
-    uint64_t w = 0, b = 0;
-    float alpha = 1.0f;
-};
-
-struct ProgramLayer {
-    bool has_mlp = false;
-    OxbLatentDims d;
-    uint32_t n_qkv = 0, ff = 0;           // columns of the input product; feed-forward width
-    ProgramNorm norm1, norm2;
-    uint64_t qkv = 0, uk_t = 0, uk = 0, uv = 0, o = 0, up = 0, down = 0;   // dense matrices
-    uint64_t c_norm = 0, sink = 0;        // vectors
-    uint32_t rope = 0;                    // index into Program::rope
-};
-
-struct ProgramRun {
-    LayerRun r;
-    size_t cache_off = 0;                 // elements in front of this run's rows, per cache row slot (times row count)
-    uint32_t ld = 0;                      // elements per cache row
-};
-
-struct RopeTable {
-    double base;
-    uint32_t dims;
-    float *cos_t, *sin_t;                 // [max_seq][dims / 2]
-};
-
-// Activations of up to `rows` token rows.
-struct ActBuf {
-    uint32_t rows = 0;
-    void *act = nullptr, *cat = nullptr, *q_abs = nullptr, *attn = nullptr, *mid = nullptr;
-    float* qkv = nullptr;
-};
-
-struct Program {
-    DesignConfig c;
-    int dt = OXB_DT_BF16;
-    std::vector<ProgramLayer> layers;
-    std::vector<ProgramRun> runs;
-    std::vector<RopeTable> rope;
-    ProgramNorm final_norm;
-    uint64_t loop_in = 0;
-    std::vector<uint64_t> loop_step;      // one vector per pass
-    uint64_t head = 0;                    // embedding table as the output product
-    uint32_t ld_act = 0, ld_cat = 0, ld_mid = 0, ld_attn = 0, ld_qkv = 0, n_q_abs = 0;
-    size_t row_elems = 0;                 // cache elements per position over all runs
-    ActBuf dec, pf;
-    std::vector<void*> pf_allocs;
-    float *part_o = nullptr, *part_ml = nullptr;
-    DevBuf k_exp, v_exp, want_act;
-};
 
 Model::Model() = default;
 Model::~Model() = default;
 
-static const DenseWeight* dense_ptr(uint64_t id, const char* what, int* rc) {
+const DenseWeight* dense_ptr(uint64_t id, const char* what, int* rc) {
     auto it = g_rt.dense.find(id);
     if (it != g_rt.dense.end()) return &it->second;
     if (!*rc) *rc = fail(OXB_HIP_WEIGHT_NOT_FOUND, "weight handle %llu (%s) not found", (unsigned long long)id, what);
@@ -87,10 +31,27 @@ void program_release(Program& p) {
     p.k_exp.release();
     p.v_exp.release();
     p.want_act.release();
+    p.scan_ws.release();
     for (void* q : p.pf_allocs) (void)hipFree(q);
     p.pf_allocs.clear();
     p.pf = ActBuf();
 }
+
+// ---------------------------------------------------------------------------
+// Recurrent memory follows its sequence: it can go on where it stands, or start again at position 0.
+// ---------------------------------------------------------------------------
+int program_begin(Model& m, uint32_t seq, uint32_t pos) {
+    Program& p = *m.prog;
+    if (!p.memory_floats) return OXB_HIP_OK;
+    if (pos && p.at[seq] != pos) {
+        if (p.at[seq] == kNoPosition)
+            return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the recurrent state of sequence %u was lost in a failed call: it starts again at position 0", seq);
+        return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: the recurrent state of sequence %u stands at position %u: it goes on there or starts again at 0, not at %u",
+                    seq, p.at[seq], pos);
+    }
+    return OXB_HIP_OK;
+}
+void program_commit(Model& m, uint32_t seq, uint32_t next) { m.prog->at[seq] = next; }
 
 size_t program_cache_row_bytes(const Program& p) { return p.row_elems * oxb_dt_bytes(p.dt); }
 
@@ -100,10 +61,14 @@ int program_check_handles(Model& m) {
     int rc = OXB_HIP_OK;
     auto norm = [&](const ProgramNorm& n, const char* what) {
         if (!rc) vec_ptr(n.w, w, what, &rc);
-        if (!rc) vec_ptr(n.b, w, what, &rc);
+        if (!rc && p.c.norm == NormKind::DynamicTanh) vec_ptr(n.b, w, what, &rc);
     };
     for (const ProgramLayer& l : p.layers) {
         norm(l.norm1, "norm1");
+        if (p.c.block == BlockKind::Parallel) {
+            if (!rc) rc = check_parallel_layer(p, l);
+            continue;
+        }
         if (l.has_mlp) norm(l.norm2, "norm2");
         if (!rc) vec_ptr(l.c_norm, l.d.rank, "latent norm", &rc);
         if (!rc) vec_ptr(l.sink, l.d.heads, "sink", &rc);
@@ -125,10 +90,9 @@ int program_check_handles(Model& m) {
     return rc;
 }
 
-// Splits of the absorbed attention: about one workgroup per CU over heads and rows, no more than a full context has chunks.
-static uint32_t decode_splits(const Model& m, const OxbLatentDims& d, uint32_t rows) {
-    const uint32_t per = 16 * oxb_latent_head_tiles(d, rows), tiles = (d.heads + per - 1) / per, most = oxb_latent_max_splits(m.d.max_seq);
-    uint32_t s = (g_rt.n_cus + rows * tiles - 1) / (rows * tiles);
+uint32_t decode_splits(const Model& m, uint32_t wgs, uint32_t rows) {
+    const uint32_t most = oxb_max_splits(m.d.max_seq);
+    uint32_t s = (wgs + rows - 1) / rows;
     if (s > most) s = most;
     if (const char* e = getenv("OXB_HIP_ATTN_SLOTS")) {  // measurement aid: a fixed slot count (long walks per workgroup)
         const long v = strtol(e, nullptr, 10);
@@ -137,8 +101,12 @@ static uint32_t decode_splits(const Model& m, const OxbLatentDims& d, uint32_t r
     if (s > 8) s = s / 8 * 8;   // head tiles of a split then share an XCD's L2
     return s ? s : 1;
 }
+static uint32_t latent_splits(const Model& m, const OxbLatentDims& d, uint32_t rows) {
+    const uint32_t per = 16 * oxb_latent_head_tiles(d, rows), tiles = (d.heads + per - 1) / per;
+    return decode_splits(m, g_rt.n_cus, rows * tiles);
+}
 
-static OxbEpilogue epilogue(uint32_t n) {
+OxbEpilogue epilogue(uint32_t n) {
     OxbEpilogue e;
     memset(&e, 0, sizeof e);
     e.scale = 1.0f;
@@ -170,7 +138,7 @@ static int feed_next(const Program& p, int i, const ActBuf& a, OxbEpilogue* e) {
     return rc;
 }
 
-static int product(const Program& p, uint64_t id, const void* x, uint32_t ldx, uint32_t m, const OxbEpilogue& e, const char* what) {
+int product(const Program& p, uint64_t id, const void* x, uint32_t ldx, uint32_t m, const OxbEpilogue& e, const char* what) {
     int rc = OXB_HIP_OK;
     const DenseWeight* w = dense_ptr(id, what, &rc);
     if (rc) return rc;
@@ -233,6 +201,7 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
     hipStream_t st = g_rt.stream;
     const uint32_t w = p.c.width, M = rows.m;
     int rc = OXB_HIP_OK;
+    if (p.c.block == BlockKind::Parallel) return encode_parallel_layers(m, a, x, rows, absorbed);
     {
         OxbEpilogue e = epilogue(w);
         OXB_TRY(feed_next(p, -1, a, &e));
@@ -286,7 +255,7 @@ static int encode_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, boo
         lp.kv.n_layers = lp.kv.nkv = 1;
         lp.part_o = p.part_o;
         lp.part_ml = p.part_ml;
-        lp.n_splits = decode_splits(m, l.d, M);
+        lp.n_splits = latent_splits(m, l.d, M);
         lp.out = a.attn;
         lp.ld_out = oxb_act_ld(l.d.heads * l.d.vdim_p);
         OXB_TRY_HIP(oxb_launch_latent_store(lp, absorbed, p.dt, st), "kernel launch failed: latent_store");
@@ -373,7 +342,7 @@ static int alloc_act(const Program& p, ActBuf* a, uint32_t rows, bool absorbed, 
     const size_t es = oxb_dt_bytes(p.dt), R = rows;
     struct { void** ptr; size_t bytes; } bufs[] = {{&a->act, R * p.ld_act * es}, {&a->cat, p.loop_in ? R * p.ld_cat * es : 0},
                                                   {&a->q_abs, absorbed ? R * p.n_q_abs * es : 0}, {&a->attn, R * p.ld_attn * es},
-                                                  {&a->mid, R * p.ld_mid * es}, {(void**)&a->qkv, R * p.ld_qkv * 4}};
+                                                  {&a->mid, R * p.ld_mid * es}, {(void**)&a->qkv, R * p.ld_qkv * 4}, {(void**)&a->rec, R * p.n_rec * 4}};
     for (auto& b : bufs) {
         *b.ptr = nullptr;
         if (!b.bytes) continue;
@@ -407,13 +376,22 @@ int program_prefill_buffers(Model& m, uint32_t rows, uint32_t pos_start) {
         p.pf_allocs.clear();
         p.pf = ActBuf();
         ActBuf a;
-        const int rc = alloc_act(p, &a, (rows + 127u) / 128u * 128u, false, &p.pf_allocs);
+        const int rc = alloc_act(p, &a, (rows + 127u) / 128u * 128u, p.c.block == BlockKind::Parallel, &p.pf_allocs);
         if (rc) {
             for (void* q : p.pf_allocs) (void)hipFree(q);
             p.pf_allocs.clear();
             return rc;
         }
         p.pf = a;
+    }
+    if (p.c.block == BlockKind::Parallel) {
+        size_t floats = 0;
+        for (const ProgramLayer& l : p.layers)
+            for (const ProgramBranch& b : l.branches)
+                if (b.kind != MixerKind::GroupedAttention)
+                    floats = std::max(floats, oxb_recur_scratch(b.r, std::min(rows, OXB_RECUR_SEGMENT), nullptr, nullptr));
+        OXB_TRY_HIP(hipStreamSynchronize(g_rt.stream), "synchronize");
+        return floats ? p.scan_ws.ensure(floats * 4) : OXB_HIP_OK;
     }
     const size_t keys = ((size_t)pos_start + rows + 127) / 128 * 128, es = oxb_dt_bytes(p.dt);
     size_t k = 0, v = 0;
@@ -431,122 +409,6 @@ int program_prefill_buffers(Model& m, uint32_t rows, uint32_t pos_start) {
 // ---------------------------------------------------------------------------
 // Loading
 // ---------------------------------------------------------------------------
-static std::string shape_text(const std::vector<uint64_t>& s) {
-    std::string t = "[";
-    for (size_t i = 0; i < s.size(); i++) t += (i ? ", " : "") + std::to_string(s[i]);
-    return t + "]";
-}
-
-struct Loader {
-    const TensorMap& tensors;
-    int dt;
-    Model& owner;   // collects what was uploaded
-
-    int get(const std::string& name, const std::vector<uint64_t>& shape, const TensorView** out) {
-        auto it = tensors.find(name);
-        if (it == tensors.end()) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: tensor not found: %s", name.c_str());
-        const TensorView& t = it->second;
-        if (t.type != (int)GGUF_F32 && t.type != (int)GGUF_F16 && t.type != (int)GGUF_BF16)
-            return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: tensor %s is not of a floating-point type this tier reads", name.c_str());
-        if (t.shape != shape || !t.data || t.bytes != t.elements() * tensor_type_bytes(t.type))
-            return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: tensor %s has shape %s, expected %s", name.c_str(), shape_text(t.shape).c_str(),
-                        shape_text(shape).c_str());
-        *out = &t;
-        return OXB_HIP_OK;
-    }
-    static float element(const TensorView& t, uint64_t i) {
-        if (t.type == (int)GGUF_F32) {
-            float f;
-            memcpy(&f, t.data + 4 * i, 4);
-            return f;
-        }
-        uint16_t h;
-        memcpy(&h, t.data + 2 * i, 2);
-        if (t.type == (int)GGUF_F16) return __half2float(__ushort_as_half(h));
-        const uint32_t b = (uint32_t)h << 16;
-        float f;
-        memcpy(&f, &b, 4);
-        return f;
-    }
-    int upload_vector(const TensorView& t, uint64_t first, uint32_t n, uint64_t* id) {
-        std::vector<float> v(n);
-        for (uint32_t i = 0; i < n; i++) v[i] = element(t, first + i);
-        *id = 0;
-        OXB_TRY(oxb_hip_upload_f32(id, v.data(), n));
-        owner.owned_vecs.push_back(*id);
-        return OXB_HIP_OK;
-    }
-    int vector(const std::string& name, uint32_t n, uint64_t* id) {
-        const TensorView* t;
-        OXB_TRY(get(name, {n}, &t));
-        return upload_vector(*t, 0, n, id);
-    }
-    int norm(const std::string& name, uint32_t n, ProgramNorm* out) {
-        const TensorView* t;
-        OXB_TRY(vector(name, n, &out->w));
-        OXB_TRY(vector(name + ".b", n, &out->b));
-        auto a = tensors.find(name + ".alpha");   // a scalar; a vector of one value will do
-        const bool one = a != tensors.end() && a->second.shape.size() == 1;
-        OXB_TRY(get(name + ".alpha", one ? std::vector<uint64_t>{1} : std::vector<uint64_t>{}, &t));
-        out->alpha = element(*t, 0);
-        return OXB_HIP_OK;
-    }
-    // Packed matrix from the concatenated source tensors (all of one type): element (n, k) = source[row_off[n] + col_off[k]].
-    int matrix(const std::vector<const TensorView*>& src, const std::vector<int64_t>& rows, const std::vector<int64_t>& cols, uint64_t* id) {
-        const uint32_t n_pad = oxb_dense_pad((uint32_t)rows.size()), k_pad = oxb_dense_pad((uint32_t)cols.size());
-        std::vector<int64_t> ro(rows), co(cols);
-        ro.resize(n_pad, -1);
-        co.resize(k_pad, -1);
-        size_t bytes = 0;
-        for (const TensorView* t : src) {
-            if (t->type != src[0]->type) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: matrices that are packed together differ in type");
-            bytes += t->bytes;
-        }
-        DevBuf raw, off;
-        DenseWeight w;
-        w.dt = dt;
-        w.n_pad = n_pad;
-        w.k_pad = k_pad;
-        int rc = OXB_HIP_OK;
-        if (!(rc = raw.ensure(bytes)) && !(rc = off.ensure(((size_t)n_pad + k_pad) * 8))) {
-            hipError_t e = hipSuccess;
-            size_t at = 0;
-            for (const TensorView* t : src) {
-                if (e == hipSuccess) e = hipMemcpy((uint8_t*)raw.ptr + at, t->data, t->bytes, hipMemcpyHostToDevice);
-                at += t->bytes;
-            }
-            int64_t* d_ro = (int64_t*)off.ptr;
-            if (e == hipSuccess) e = hipMemcpy(d_ro, ro.data(), (size_t)n_pad * 8, hipMemcpyHostToDevice);
-            if (e == hipSuccess) e = hipMemcpy(d_ro + n_pad, co.data(), (size_t)k_pad * 8, hipMemcpyHostToDevice);
-            if (e == hipSuccess && hipMalloc(&w.d, (n_pad / 16) * oxb_tile_stride(k_pad, oxb_dt_bytes(dt)) * oxb_dt_bytes(dt)) != hipSuccess)
-                rc = fail(OXB_HIP_OUT_OF_MEMORY, "out of device memory: a %u x %u matrix on device %d", n_pad, k_pad, g_rt.device);
-            if (!rc && e == hipSuccess) e = oxb_launch_dense_pack(raw.ptr, src[0]->type, d_ro, d_ro + n_pad, n_pad, k_pad, dt, w.d, g_rt.stream);
-            if (e == hipSuccess) e = hipStreamSynchronize(g_rt.stream);
-            if (!rc && e != hipSuccess) rc = hip_fail(e, "matrix upload");
-        }
-        raw.release();
-        off.release();
-        if (rc) {
-            if (w.d) (void)hipFree(w.d);
-            return rc;
-        }
-        *id = g_rt.next_id++;
-        g_rt.dense[*id] = w;
-        owner.owned_mats.push_back(*id);
-        return OXB_HIP_OK;
-    }
-    static std::vector<int64_t> range(uint32_t n, int64_t stride) {
-        std::vector<int64_t> v(n);
-        for (uint32_t i = 0; i < n; i++) v[i] = (int64_t)i * stride;
-        return v;
-    }
-    int plain(const std::string& name, uint32_t n, uint32_t k, uint64_t* id) {
-        const TensorView* t;
-        OXB_TRY(get(name, {n, k}, &t));
-        return matrix({t}, range(n, k), range(k, 1), id);
-    }
-};
-
 static int load_layer(Loader& ld, Program& p, const LayerConfig& c, const std::string& name, ProgramLayer* l) {
     const MixerConfig& mx = c.mixer;
     const uint32_t w = p.c.width;
@@ -557,7 +419,7 @@ static int load_layer(Loader& ld, Program& p, const LayerConfig& c, const std::s
     d.rot = mx.rot_dim, d.rot_p = oxb_pad32(mx.rot_dim);
     d.rank = mx.kv_rank, d.rank_p = oxb_pad32(mx.kv_rank);
     d.vdim = mx.vdim, d.vdim_p = oxb_pad32(mx.vdim);
-    d.rot_dims = mx.rot_dims;
+    d.rot_dims = mx.rope.dims;
     d.scale = mx.scale;
     d.eps = p.c.eps;
     if (const char* why = oxb_latent_check(d, p.dt)) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: %s: %s", name.c_str(), why);
@@ -609,23 +471,23 @@ static int load_layer(Loader& ld, Program& p, const LayerConfig& c, const std::s
     return OXB_HIP_OK;
 }
 
-// Angles position * base^(-2 i / dims), formed in double and rounded once.
-static int rope_table(Model& m, Program& p, double base, uint32_t dims, uint32_t* index) {
+// Angles position * frequency, formed in double and rounded once.
+int rope_table(Model& m, Program& p, const RopeConfig& r, uint32_t* index) {
     for (size_t i = 0; i < p.rope.size(); i++)
-        if (p.rope[i].base == base && p.rope[i].dims == dims) {
+        if (p.rope[i].r == r) {
             *index = (uint32_t)i;
             return OXB_HIP_OK;
         }
-    const size_t half = dims / 2, n = (size_t)m.d.max_seq * half;
+    const size_t half = r.dims / 2, n = (size_t)m.d.max_seq * half;
     std::vector<float> c(n), s(n);
     for (size_t i = 0; i < half; i++) {
-        const double f = pow(base, -2.0 * (double)i / (double)dims);
+        const double f = rope_frequency(r, (uint32_t)i);
         for (size_t pos = 0; pos < m.d.max_seq; pos++) {
             c[pos * half + i] = (float)cos((double)pos * f);
             s[pos * half + i] = (float)sin((double)pos * f);
         }
     }
-    RopeTable t = {base, dims, nullptr, nullptr};
+    RopeTable t = {r, nullptr, nullptr};
     OXB_TRY(dev_alloc(m, (void**)&t.cos_t, n * 4));
     OXB_TRY(dev_alloc(m, (void**)&t.sin_t, n * 4));
     OXB_TRY_HIP(hipMemcpy(t.cos_t, c.data(), n * 4, hipMemcpyHostToDevice), "rope table upload");
@@ -639,11 +501,13 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
     Program& p = *m.prog;
     Loader ld{tensors, dt, m};
     const uint32_t w = c.width;
-    OXB_TRY_HIP(oxb_latent_prepare(dt), "kernel preparation");
+    OXB_TRY_HIP(c.block == BlockKind::Parallel ? oxb_row_attention_prepare(dt) : oxb_latent_prepare(dt), "kernel preparation");
     const TensorView* emb;
     OXB_TRY(ld.get("embed", {c.vocab, w}, &emb));
     OXB_TRY(ld.plain("embed", c.vocab, w, &p.head));
-    OXB_TRY(ld.norm("final.norm", w, &p.final_norm));
+    const bool parallel = c.block == BlockKind::Parallel;
+    if (parallel) OXB_TRY(ld.vector("final.norm", w, [](double v) { return 1.0 + v; }, &p.final_norm.w));
+    else OXB_TRY(ld.norm("final.norm", w, &p.final_norm));
     if (c.loop.times) {
         OXB_TRY(ld.plain("loop.in", w, 2 * w, &p.loop_in));
         const TensorView* step;
@@ -653,23 +517,45 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
     }
     p.layers.resize(c.layers.size());
     for (size_t i = 0; i < c.layers.size(); i++) {
-        OXB_TRY(load_layer(ld, p, c.layers[i], "l" + std::to_string(i) + ".", &p.layers[i]));
-        OXB_TRY(rope_table(m, p, c.layers[i].mixer.rot_base, c.layers[i].mixer.rot_dims, &p.layers[i].rope));
+        const std::string name = "l" + std::to_string(i) + ".";
+        if (parallel) {
+            OXB_TRY(load_parallel_layer(ld, m, c.layers[i], name, &p.layers[i]));
+            continue;
+        }
+        OXB_TRY(load_layer(ld, p, c.layers[i], name, &p.layers[i]));
+        OXB_TRY(rope_table(m, p, c.layers[i].mixer.rope, &p.layers[i].rope));
     }
     p.ld_act = oxb_act_ld(w);
     p.ld_cat = oxb_act_ld(2 * w);
     const size_t R = m.d.batch > OXB_PROGRAM_SHORT ? m.d.batch : OXB_PROGRAM_SHORT;
     size_t part = 0, ml = 0;
+    auto grow = [](auto* v, size_t n) { if (n > *v) *v = (std::remove_pointer_t<decltype(v)>)n; };
     for (const ProgramLayer& l : p.layers) {
+        if (parallel) {
+            grow(&p.ld_qkv, oxb_dense_pad(l.n_lin));
+            grow(&p.ld_attn, oxb_act_ld(l.n_out));
+            for (const ProgramBranch& b : l.branches) {
+                if (b.kind != MixerKind::GroupedAttention) {
+                    grow(&p.n_rec, (size_t)b.r.heads * b.r.dv);
+                    continue;
+                }
+                grow(&p.n_q_abs, (size_t)b.heads * b.dim_p);
+                for (uint32_t r = 1; r <= R; r++) {
+                    const size_t slots = (size_t)r * b.kv_heads * oxb_row_head_tiles(b.heads / b.kv_heads) * grouped_splits(m, b, r);
+                    grow(&part, slots * 16 * b.vdim_p);
+                    grow(&ml, slots * 32);
+                }
+            }
+            continue;
+        }
         const OxbLatentDims& d = l.d;
-        auto grow = [](uint32_t* v, uint32_t n) { if (n > *v) *v = n; };
         grow(&p.ld_qkv, oxb_dense_pad(l.n_qkv));
         grow(&p.ld_attn, oxb_act_ld(d.heads * d.vdim_p));
         grow(&p.n_q_abs, d.heads * (d.rank_p + d.rot_p));
         if (l.has_mlp) grow(&p.ld_mid, oxb_act_ld(l.ff));
         const size_t tiles = (d.heads + 15) / 16;
         for (uint32_t r = 1; r <= R; r++) {
-            const size_t slots = (size_t)r * tiles * decode_splits(m, d, r);
+            const size_t slots = (size_t)r * tiles * latent_splits(m, d, r);
             if (slots * 16 * d.rank_p > part) part = slots * 16 * d.rank_p;
             if (slots * 32 > ml) ml = slots * 32;
         }
@@ -680,12 +566,14 @@ static int load_all(Model& m, const DesignConfig& c, const TensorMap& tensors, i
         run.r = r;
         run.cache_off = p.row_elems;
         run.ld = d.rank_p + d.rot_p;
-        p.row_elems += run.ld;
+        if (!parallel) p.row_elems += run.ld;   // (a parallel block's branches have taken theirs)
         p.runs.push_back(run);
     }
     OXB_TRY(alloc_act(p, &p.dec, (uint32_t)R, true, &m.allocs));
-    OXB_TRY(dev_alloc(m, (void**)&p.part_o, part * 4));
-    OXB_TRY(dev_alloc(m, (void**)&p.part_ml, ml * 4));
+    OXB_TRY(dev_alloc(m, (void**)&p.part_o, std::max<size_t>(part, 4) * 4));
+    OXB_TRY(dev_alloc(m, (void**)&p.part_ml, std::max<size_t>(ml, 4) * 4));
+    if (p.memory_floats) OXB_TRY(dev_alloc(m, (void**)&p.memory, m.d.batch * p.memory_floats * 4));
+    p.at.assign(m.d.batch, 0);
     const size_t B = m.d.batch;
     OXB_TRY(dev_alloc(m, (void**)&m.hidden, B * w * 4));
     OXB_TRY(dev_alloc(m, (void**)&m.logits, B * c.vocab * 4));
