@@ -413,16 +413,72 @@ def fulirax_model(be, shape: dict, layers: int, vocab: int, max_seq: int, batch:
     return model, emb, macs
 
 
-def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, long_context: int, only: str = "", which: int = -1) -> list:
-    """Prefill and decode of both models from token ids, the token loops on the device; host-timed around whole calls."""
+MUVONEX_SHAPES = [dict(width=2048, heads=16, kv_heads=8, ff=6144), dict(width=4096, heads=32, kv_heads=8, ff=12288)]
+
+
+def muvonex_model(be, shape: dict, layers: int, vocab: int, max_seq: int, batch: int):
+    """Random weights as above: three gated-delta layers for one of grouped attention beside a state space, heads of 128 (64
+    in the state space, twice as many, 128 states)."""
+    from oxibonsai_amd.model import HipModel
+    w, ff, h, g = shape["width"], shape["ff"], shape["heads"], shape["kv_heads"]
+    base = np.random.default_rng(0xF02).standard_normal(1 << 22, dtype=np.float32)
+
+    def tensor(*dims, std):
+        n = int(np.prod(dims))
+        return np.resize((base * std).view(np.uint32) >> 16, n).astype(np.uint16).reshape(dims)
+
+    def flat(n, value):
+        return np.full(n, np.float32(value).view(np.uint32) >> 16, np.uint16)
+
+    delta = {"heads": h, "kv_heads": h, "dim": 128, "vdim": 128, "conv": 4}
+    left = {"heads": h, "kv_heads": g, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+            "rot": {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    right = {"heads": 2 * h, "vdim": 64, "state": 128, "groups": 1, "norm_groups": 1, "conv": 4}
+    inner, channels = 128 * h, 128 * h + 256
+    kinds = {"mlp.gate": (ff, w), "mlp.up": (ff, w), "mlp.down": (w, ff)}
+    d_kinds = {"mix." + k: (inner, w) for k in "qkvg"} | {"mix.b": (h, w), "mix.a": (h, w), "mix.o": (w, inner)}
+    p_kinds = {"mix.left.q": (inner, w), "mix.left.k": (128 * g, w), "mix.left.v": (128 * g, w), "mix.left.o": (w, inner),
+               "mix.right.in": (inner + channels + 2 * h, w), "mix.right.o": (w, inner)}
+    shared = {k: tensor(*d, std=d[1] ** -0.5) for k, d in (kinds | d_kinds | p_kinds).items()}
+    shared |= {f"mix.{k}.conv": tensor(inner, 4, std=0.5) for k in "qkv"} | {"mix.right.conv": tensor(channels, 4, std=0.5)}
+    t = {"embed": tensor(vocab, w, std=1.0), "final.norm": flat(w, 0.0)}
+    cfg_layers, macs = [], 0
+    for i in range(layers):
+        p, parallel = f"l{i}.", i % 4 == 3
+        t[p + "norm1"] = flat(w, 0.0)
+        names = kinds | (p_kinds if parallel else d_kinds)
+        macs += sum(a * b for a, b in names.values())
+        for k in names:
+            t[p + k] = shared[k]
+        if parallel:
+            t |= {p + "mix.left.sink": flat(h, 0.0), p + "mix.right.conv": shared["mix.right.conv"], p + "mix.right.conv.b": flat(channels, 0.0),
+                  p + "mix.right.dt_bias": flat(2 * h, -2.0), p + "mix.right.A_log": flat(2 * h, -1.0), p + "mix.right.D": flat(2 * h, 1.0),
+                  p + "mix.right.norm": flat(inner, 1.0)}
+        else:
+            t |= {p + f"mix.{k}.conv": shared[f"mix.{k}.conv"] for k in "qkv"}
+            t |= {p + "mix.A_log": flat(h, -1.0), p + "mix.dt_bias": flat(h, -2.0), p + "mix.norm": flat(128, 1.0)}
+        cfg_layers.append({"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7}} if parallel
+                          else {"type": "delta", "mixer": delta})
+        cfg_layers[-1]["mlp"] = {"kind": "dense", "ff": ff}
+    cfg = {"architecture": "Muvonex", "width": w, "vocab": vocab, "layers": cfg_layers, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+           "residual_mult": 0.5}
+    model, emb = HipModel.from_tensors(be, cfg, t, max_seq=max_seq, batch=batch)
+    return model, emb, macs
+
+
+def design_leg(be, name: str, layers: int, vocab: int, prompt: int, steps: int, batches, long_context: int, only: str = "", which: int = -1) -> list:
+    """Prefill and decode of a configured design and of the Q1 Qwen3 model of equal size from token ids, the token loops on the device; host-timed around whole calls."""
     from oxibonsai_amd import synth
     from oxibonsai_amd.model import Embedding, HipModel
     ids = (synth.splitmix64(0xF0120F, max(prompt, long_context)) % np.uint64(vocab)).astype(np.int64)
     chunk = 2048
 
-    def fill(m, e, n, seq):
-        for at in range(0, n, chunk):
+    def fill(m, e, n, seq, first=0):
+        t0 = 0.0
+        for at in range(first, n, chunk):
+            t0 = time.perf_counter()
             m.prefill_tokens(e, ids[at:min(n, at + chunk)], at, seq, want_logits=False)
+        return time.perf_counter() - t0
 
     def measure(build) -> dict:
         r = {}
@@ -437,10 +493,9 @@ def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, l
         r["prefill_ms"], r["prefill_tok_per_s"] = round(t * 1e3, 3), round(prompt / t, 1)
 
         def decode(m, e, n, batch):
-            pos = np.full(batch, n)
-            m.generate(e, np.arange(batch), pos, 2)
+            m.generate(e, np.arange(batch), np.full(batch, n), 2)
             t0 = time.perf_counter()
-            m.generate(e, np.arange(batch), pos, steps)
+            m.generate(e, np.arange(batch), np.full(batch, n + 2), steps)
             return (time.perf_counter() - t0) / steps
 
         t = decode(m, e, prompt, 1)
@@ -456,10 +511,8 @@ def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, l
             e2.close()
         if long_context:
             m3, e3 = build(long_context + 2 * steps, 1)
-            fill(m3, e3, long_context, 0)
-            t0 = time.perf_counter()
-            m3.prefill_tokens(e3, ids[long_context - chunk:long_context], long_context - chunk, 0, want_logits=False)
-            tp = time.perf_counter() - t0
+            fill(m3, e3, long_context - chunk, 0)
+            tp = fill(m3, e3, long_context, 0, long_context - chunk)
             t = decode(m3, e3, long_context, 1)
             r[f"context_{long_context}"] = {"last_2048_prefill_ms": round(tp * 1e3, 3), "decode_ms_per_step": round(t * 1e3, 4)}
             m3.close()
@@ -468,20 +521,24 @@ def fulirax_leg(be, layers: int, vocab: int, prompt: int, steps: int, batches, l
         return r
 
     out = []
-    for shape in FULIRAX_SHAPES if which < 0 else FULIRAX_SHAPES[which:which + 1]:
+    shapes, build = (FULIRAX_SHAPES, fulirax_model) if name == "fulirax" else (MUVONEX_SHAPES, muvonex_model)
+    for shape in shapes if which < 0 else shapes[which:which + 1]:
         cfg = dict(fmt=FMT_Q1, n_layers=layers, h=shape["width"], inter=shape["ff"], nq=shape["heads"], nkv=8, hd=128, vocab=vocab,
                    max_seq=0, eps=1e-6, rope_theta=1e6)
-        row = {"shape": dict(shape, layers=layers, vocab=vocab, **FULIRAX_LATENT)}
+        row = {"shape": dict(shape, layers=layers, vocab=vocab)}
         if only != "qwen3":
-            macs = fulirax_model(be, shape, 1, 64, 64, 1)
-            macs[0].close()
-            macs[1].close()
-            row["fulirax"] = measure(lambda n, b: fulirax_model(be, shape, layers, vocab, n, b)[:2])
-            flop = 2.0 * prompt * layers * macs[2] + 2.0 * layers * shape["heads"] * (192 + 128) * prompt * (prompt + 1) / 2
-            row["fulirax"]["prefill_TFLOPs"] = round(flop / row["fulirax"]["prefill_ms"] / 1e9, 1)
-            row["fulirax"]["weight_bytes_per_token"] = 2 * (layers * macs[2] + vocab * shape["width"] + 2 * shape["width"] ** 2)
-            row["fulirax"]["cache_bytes_per_position"] = 2 * layers * (FULIRAX_LATENT["kv_rank"] + FULIRAX_LATENT["rot_dim"])
-        if only != "fulirax":
+            n = 1 if name == "fulirax" else layers
+            m, e, macs = build(be, shape, n, 64, 64, 1)
+            m.close()
+            e.close()
+            macs *= layers // n
+            row[name] = measure(lambda n, b: build(be, shape, layers, vocab, n, b)[:2])
+            # products of attention alone beside the matrices (a recurrence's own are not counted)
+            per_layer = layers * (192 + 128) if name == "fulirax" else (layers // 4) * 256
+            flop = 2.0 * prompt * macs + 2.0 * per_layer * shape["heads"] * prompt * (prompt + 1) / 2
+            row[name]["prefill_TFLOPs"] = round(flop / row[name]["prefill_ms"] / 1e9, 1)
+            row[name]["weight_bytes_per_token"] = 2 * (macs + vocab * shape["width"] + (2 * shape["width"] ** 2 if name == "fulirax" else 0))
+        if only != name:
             weights = synth.make_model(dict(cfg, max_seq=prompt), 0xF012)
             table = synth.make_q1_blocks(0xF0E, vocab * (shape["width"] // 128), 0.01, 0.1)
             row["qwen3_q1"] = measure(lambda n, b: (HipModel(be, dict(cfg, max_seq=n), weights, batch=b), Embedding(table, 41, vocab, shape["width"])))
@@ -581,9 +638,10 @@ def main() -> int:
     ap.add_argument("--no-ternary", action="store_true", help="skip the ternary 1.7B-shape decode leg")
     ap.add_argument("--fulirax", action="store_true",
                     help="instead of the default workload: prefill and decode of Fulirax at real layer sizes, next to the Q1 Qwen3 model of equal size")
-    ap.add_argument("--fulirax-layers", type=int, default=8)
-    ap.add_argument("--fulirax-shape", type=int, default=-1, help="one of the shapes alone")
-    ap.add_argument("--fulirax-only", choices=["", "fulirax", "qwen3"], default="", help="one of the two models alone (profiling)")
+    ap.add_argument("--muvonex", action="store_true", help="the same for Muvonex")
+    ap.add_argument("--design-layers", "--fulirax-layers", type=int, default=8)
+    ap.add_argument("--design-shape", "--fulirax-shape", type=int, default=-1, help="one of the shapes alone")
+    ap.add_argument("--design-only", choices=["", "design", "qwen3"], default="", help="one of the two models alone (profiling)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build targets one GPU; run with --gpus 1 (multi-GPU sharding is design-only)",
@@ -600,10 +658,12 @@ def main() -> int:
         return 1
     torch.cuda.set_device(0)
     be = ox.NativeHipBackend(0)
-    if args.fulirax:
-        rows = fulirax_leg(be, args.fulirax_layers, 32768, args.decode_context, args.decode_tokens,
-                           tuple(int(b) for b in args.decode_batches.split(",") if b), args.long_context, args.fulirax_only, args.fulirax_shape)
-        print(json.dumps({"metric": "Fulirax prefill and decode", "n_gpus": 1, "dtype": "bf16", "data": "synthetic, random weights",
+    if args.fulirax or args.muvonex:
+        design = "fulirax" if args.fulirax else "muvonex"
+        rows = design_leg(be, design, args.design_layers, 32768, args.decode_context, args.decode_tokens,
+                          tuple(int(b) for b in args.decode_batches.split(",") if b), args.long_context,
+                          design if args.design_only == "design" else args.design_only, args.design_shape)
+        print(json.dumps({"metric": f"{design.capitalize()} prefill and decode", "n_gpus": 1, "dtype": "bf16", "data": "synthetic, random weights",
                           "prompt": args.decode_context, "steps": args.decode_tokens, "shapes": rows}), flush=True)
         return 0
     L = _lib.lib()

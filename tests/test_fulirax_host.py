@@ -43,7 +43,7 @@ def test_checkpoint_info(tmp_path):
 
 
 @pytest.mark.parametrize("text,says", [
-    (changed(architecture="Nothing"), "unknown (known: Fulirax)"), (changed(architecture=KeyError), "architecture is missing"),
+    (changed(architecture="Nothing"), "unknown (known: Fulirax"), (changed(architecture=KeyError), "architecture is missing"),
     (changed(width=0), "width"), (changed(vocab=1.5), "vocab"), (changed(layers=[]), "layers"),
     (changed(layers__1__type="mystery"), 'layers[1].type "mystery"'), (changed(layers__2__mixer__kv_rank=KeyError), "layers[2].mixer.kv_rank"),
     (changed(layers__0__mlp__kind="routed"), 'layers[0].mlp.kind "routed"'), (changed(layers__0__mixer__rot__dims=7), "rot.dims"),
