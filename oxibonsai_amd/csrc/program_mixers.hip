@@ -117,7 +117,8 @@ static int encode_recurrent(Model& m, const ProgramBranch& b, ActBuf& a, const O
     r.out_col = b.out_col;
     r.out_fill = b.out_fill;
     if (step) {
-        OXB_TRY_HIP(oxb_launch_recur_step(r, st), "kernel launch failed: recur_step");
+        OXB_TRY_HIP(oxb_launch_recur_step(r, p.dt, st), "kernel launch failed: recur_step");
+        if (oxb_recur_step_finishes(b.r)) return OXB_HIP_OK;
     } else {
         for (uint32_t at = 0; at < rows.m; at += OXB_RECUR_SEGMENT) {
             r.first = at;
@@ -244,7 +245,8 @@ int finish_recurrent(BlockMaps& b, Program& p, const std::string& name, ProgramB
     OxbRecurDims& d = o->r;
     d.dk_p = oxb_pad32(d.dk);
     d.slices = (d.dv + 31) / 32;
-    d.ring = d.taps - 1 + OXB_RECUR_STEP_TOKENS;
+    d.ring = 1;
+    while (d.ring < d.taps - 1 + OXB_RECUR_STEP_TOKENS) d.ring *= 2;
     d.eps = p.c.eps;
     d.out_scale = o->scale;
     if (const char* why = oxb_recur_check(d)) return fail(OXB_HIP_INVALID_ARGUMENT, "invalid argument: %s: %s", name.c_str(), why);

@@ -7,12 +7,12 @@
 // with a scalar decay a per token and head.  Everything in them is fp32 in every compute type, products included.
 //
 // What a sequence keeps, per layer (floats): the states [heads][dv / 32 slices][dk_p][32], then a ring of convolution inputs
-// [ring][channels], the inputs of position p in row p % ring.  Neither is ever cleared: position 0 starts from zeros without
+// [ring][channels], the inputs of position p in row p % ring (ring a power of two).  Neither is ever cleared: position 0 starts from zeros without
 // reading, and a convolution reads no position before 0.
 //
 // Forms:
-//   step   a workgroup per (sequence, head, 32 columns) walks its tokens with the state in registers: decode steps, portions
-//          of up to OXB_RECUR_STEP_TOKENS.
+//   step   a workgroup per sequence and head (or 32 columns of one) walks its tokens with the state in registers: decode
+//          steps, portions of up to OXB_RECUR_STEP_TOKENS.
 //   chunks of 64 tokens: `prepare` (convolutions, unit norms, decays), `chunk` (what needs no state, all chunks at once: decay
 //          matrices, and for the delta rule the inverse of its unit lower triangular system), `scan` (chunk after chunk, a
 //          workgroup per head and 16 columns): prompts.
@@ -74,7 +74,9 @@ struct OxbRecurParams {
 };
 
 // One token per sequence (rows.seq_step 1), or all rows.m <= OXB_RECUR_STEP_TOKENS of one sequence (seq_step 0).
-hipError_t oxb_launch_recur_step(const OxbRecurParams& p, hipStream_t st);
+// Where it finishes a head's output by itself (oxb_recur_step_finishes) p.out is written and no `finish` follows.
+hipError_t oxb_launch_recur_step(const OxbRecurParams& p, int dt, hipStream_t st);
+bool oxb_recur_step_finishes(const OxbRecurDims& d);
 hipError_t oxb_launch_recur_chunked(const OxbRecurParams& p, hipStream_t st);
 // keep_conv: also bring the last convolution inputs of a chunked portion into the ring.
 hipError_t oxb_launch_recur_finish(const OxbRecurParams& p, bool keep_conv, int dt, hipStream_t st);

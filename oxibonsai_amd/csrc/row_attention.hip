@@ -8,37 +8,63 @@
 #include "row_attention_device.h"
 
 // ---------------------------------------------------------------------------
-// Grouped heads, new tokens: a wave per (row, head): queries and keys are rotated, then divided by their root mean square;
-// values are copied.  Grid (row, heads / 4).
+// Grouped heads, new tokens: a wave per head and ROWS rows, E elements per lane: queries and keys are rotated, then divided by
+// their root mean square; values are copied.  Grid (rows / ROWS, heads / 4).
 // ---------------------------------------------------------------------------
-template <typename T>
+template <typename T, int E, int ROWS>
 __global__ __launch_bounds__(256) void grouped_store_kernel(OxbGroupedStore p) {
-    const uint32_t lane = threadIdx.x & 63u, m = blockIdx.x, hd = blockIdx.y * 4 + (threadIdx.x >> 6);
+    const uint32_t lane = threadIdx.x & 63u, hd = blockIdx.y * 4 + (threadIdx.x >> 6);
     if (hd >= p.heads + 2 * p.kv_heads) return;
-    const uint32_t pos = row_pos(p.rows, m), half = p.rot_dims >> 1;
-    const float* row = p.lin + (size_t)m * p.ld_lin;
-    const bool is_q = hd < p.heads;
-    const uint32_t kvh = is_q ? 0 : (hd - p.heads) % p.kv_heads;
-    T* dst = is_q ? reinterpret_cast<T*>(p.q) + ((size_t)m * p.heads + hd) * p.dim_p
-                  : reinterpret_cast<T*>(p.cache) + kv_row(p.kv, row_seq(p.rows, m), 0, kvh, pos) * (p.dim_p + p.vdim_p);
-    if (hd >= p.heads + p.kv_heads) {
-        for (uint32_t i = lane; i < p.vdim_p; i += 64) dst[p.dim_p + i] = i < p.vdim ? (T)row[p.col_v + kvh * p.vdim + i] : (T)0.f;
-        return;
-    }
-    const float* src = row + (is_q ? p.col_q + hd * p.dim : p.col_k + kvh * p.dim);
-    const float* cs = p.cos_t + (size_t)pos * half;
-    const float* sn = p.sin_t + (size_t)pos * half;
-    float x[8], ss = 0.f;
+    const uint32_t half = p.rot_dims >> 1, kvh = hd < p.heads ? 0 : (hd - p.heads) % p.kv_heads;
+    const bool is_q = hd < p.heads, is_v = hd >= p.heads + p.kv_heads;
+    const uint32_t len = is_v ? p.vdim : p.dim, pad = is_v ? p.vdim_p : p.dim_p;
+    const uint32_t col = is_q ? p.col_q + hd * p.dim : is_v ? p.col_v + kvh * p.vdim : p.col_k + kvh * p.dim;
+    // the partner of each element in its rotation, the sign of the partner's share, and the angle's index
+    uint32_t partner[E], angle[E];
+    float sign[E];
 #pragma unroll
-    for (int e = 0; e < 8; e++) {
+    for (int e = 0; e < E; e++) {
         const uint32_t i = lane + 64 * e;
-        x[e] = i < p.dim ? rotated(src, i, p.rot_dims, cs, sn) : 0.f;
-        ss = fmaf(x[e], x[e], ss);
+        const bool low = i < half, turns = !is_v && i < p.rot_dims;
+        partner[e] = turns ? (low ? i + half : i - half) : min(i, len - 1);
+        angle[e] = turns ? (low ? i : i - half) : 0;
+        sign[e] = turns ? (low ? -1.f : 1.f) : 0.f;
     }
-    const float inv = 1.0f / sqrtf(wave_sum_f32(ss) / (float)p.dim + p.eps);
+    float x[ROWS][E], y[ROWS][E], cs[ROWS][E], sn[ROWS][E];
 #pragma unroll
-    for (int e = 0; e < 8; e++)
-        if (lane + 64 * e < p.dim_p) dst[lane + 64 * e] = (T)(x[e] * inv);
+    for (int t = 0; t < ROWS; t++) {
+        const uint32_t m = min(blockIdx.x * ROWS + t, p.rows.m - 1);
+        const size_t at = (size_t)row_pos(p.rows, m) * half;
+        const float* src = p.lin + (size_t)m * p.ld_lin + col;
+#pragma unroll
+        for (int e = 0; e < E; e++) {
+            x[t][e] = src[min(lane + 64 * e, len - 1)];
+            if (is_v) continue;
+            y[t][e] = src[partner[e]];
+            cs[t][e] = p.cos_t[at + angle[e]];
+            sn[t][e] = p.sin_t[at + angle[e]];
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < ROWS; t++) {
+        const uint32_t m = blockIdx.x * ROWS + t;
+        float f = 1.0f;
+        if (!is_v) {
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < E; e++) {
+                if (sign[e] != 0.f) x[t][e] = x[t][e] * cs[t][e] + sign[e] * y[t][e] * sn[t][e];
+                if (lane + 64 * e < len) ss = fmaf(x[t][e], x[t][e], ss);
+            }
+            f = 1.0f / sqrtf(wave_sum_f32(ss) / (float)len + p.eps);
+        }
+        if (m >= p.rows.m) continue;
+        T* dst = is_q ? reinterpret_cast<T*>(p.q) + ((size_t)m * p.heads + hd) * p.dim_p
+                      : reinterpret_cast<T*>(p.cache) + kv_row(p.kv, row_seq(p.rows, m), 0, kvh, row_pos(p.rows, m)) * (p.dim_p + p.vdim_p) + (is_v ? p.dim_p : 0);
+#pragma unroll
+        for (int e = 0; e < E; e++)
+            if (lane + 64 * e < pad) dst[lane + 64 * e] = lane + 64 * e < len ? (T)(x[t][e] * f) : (T)0.f;
+    }
 }
 
 // ---------------------------------------------------------------------------
@@ -447,13 +473,26 @@ const char* oxb_grouped_check(uint32_t heads, uint32_t kv_heads, uint32_t dim, u
     return oxb_row_check(units, dt);
 }
 
+template <typename T, int E>
+static void launch_store_rows(const OxbGroupedStore& p, hipStream_t st) {
+    const uint32_t y = (p.heads + 2 * p.kv_heads + 3) / 4;
+    if (p.rows.m < 64) hipLaunchKernelGGL((grouped_store_kernel<T, E, 1>), dim3(p.rows.m, y), dim3(256), 0, st, p);
+    else hipLaunchKernelGGL((grouped_store_kernel<T, E, 4>), dim3((p.rows.m + 3) / 4, y), dim3(256), 0, st, p);
+}
+template <typename T>
+static void launch_store(const OxbGroupedStore& p, uint32_t widest, hipStream_t st) {
+    if (widest <= 64) launch_store_rows<T, 1>(p, st);
+    else if (widest <= 128) launch_store_rows<T, 2>(p, st);
+    else launch_store_rows<T, 4>(p, st);
+}
+
 hipError_t oxb_launch_grouped_store(const OxbGroupedStore& p, int dt, hipStream_t st) {
     if (!p.rows.m || !p.lin || !p.q || !p.cache || !p.cos_t || !p.sin_t || p.dim_p != oxb_pad32(p.dim) || p.vdim_p != oxb_pad32(p.vdim) ||
         oxb_grouped_check(p.heads, p.kv_heads, p.dim, p.vdim, p.rot_dims, dt) || p.kv.n_layers != 1 || p.kv.nkv != p.kv_heads)
         return hipErrorInvalidValue;
-    const dim3 grid(p.rows.m, (p.heads + 2 * p.kv_heads + 3) / 4);
-    if (dt == OXB_DT_BF16) hipLaunchKernelGGL((grouped_store_kernel<__bf16>), grid, dim3(256), 0, st, p);
-    else hipLaunchKernelGGL((grouped_store_kernel<float>), grid, dim3(256), 0, st, p);
+    const uint32_t widest = p.dim_p > p.vdim_p ? p.dim_p : p.vdim_p;
+    if (dt == OXB_DT_BF16) launch_store<__bf16>(p, widest, st);
+    else launch_store<float>(p, widest, st);
     return hipGetLastError();
 }
 
