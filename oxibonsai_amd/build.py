@@ -16,7 +16,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 OUT = os.path.join(HERE, "lib")
 SOURCES = ["runtime.hip", "gemv_kernels.hip", "gemm_kernels.hip", "layer_kernels.hip", "prefill_kernels.hip", "token_kernels.hip", "dense_kernels.hip",
-           "latent_kernels.hip", "row_attention.hip", "recurrent_kernels.hip", "model.hip", "program.hip", "program_mixers.hip", "repack.cpp", "gguf.cpp", "json.cpp", "safetensors.cpp", "design.cpp"]
+           "latent_kernels.hip", "row_attention.hip", "recurrent_kernels.hip", "mixer_kernels.hip", "model.hip", "program.hip", "program_mixers.hip",
+           "repack.cpp", "gguf.cpp", "json.cpp", "safetensors.cpp", "design.cpp"]
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function",
          # packed-FP32 VALU forms are kept out of every kernel

@@ -138,20 +138,22 @@ __device__ __forceinline__ v4f epilogue_resid(const OxbEpilogue& e, uint32_t m, 
     if (!e.resid || !epilogue_whole(e, n0)) return (v4f){0.f, 0.f, 0.f, 0.f};
     return *reinterpret_cast<const v4f*>(e.resid + (size_t)m * e.ld32 + n0);
 }
-// Four consecutive outputs through the epilogue; resid = epilogue_resid(e, m, n0).
-template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogue& e, uint32_t m, uint32_t n0, v4f y, v4f resid) {
+// Four consecutive outputs through the epilogue; resid = epilogue_resid(e, m, n0).  -> the outputs in front of the norm, zeros
+// past the last column.
+template <typename T> __device__ __forceinline__ v4f epilogue4(const OxbEpilogue& e, uint32_t m, uint32_t n0, v4f y, v4f resid) {
     if (e.glu_out && n0 >= e.glu) {
         const uint32_t j = (n0 - e.glu) >> 1;
-        if (j >= e.n_glu) return;
+        if (j >= e.n_glu) return y;
         y *= e.scale;
         typedef T pair __attribute__((ext_vector_type(2)));
         *reinterpret_cast<pair*>(reinterpret_cast<T*>(e.glu_out) + (size_t)m * e.ld_glu + j) =
             (pair){(T)(gelu_tanh_of<T>(y[0]) * y[1]), (T)(gelu_tanh_of<T>(y[2]) * y[3])};
-        return;
+        return y;
     }
     const uint32_t lim = e.n > e.fill ? e.n : e.fill;
-    if (n0 >= lim) return;
+    if (n0 >= lim) return (v4f){0.f, 0.f, 0.f, 0.f};
     y *= e.scale;
+    v4f sum = {0.f, 0.f, 0.f, 0.f};
     if (epilogue_whole(e, n0)) {
         if (e.add) y += *reinterpret_cast<const v4f*>(e.add + n0);
         if (e.act == OXB_ACT_GELU_TANH) {
@@ -160,8 +162,10 @@ template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogu
         }
         const size_t o = (size_t)m * e.ld32 + n0;
         y += resid;
+        sum = y;
         if (e.out32) *reinterpret_cast<v4f*>(e.out32 + o) = y;
-        if (!e.out_t) return;
+        if (!e.out_t) return sum;
+        if (e.norm == OXB_NORM_SCALE) y *= *reinterpret_cast<const v4f*>(e.nw + n0);
         if (e.norm == OXB_NORM_DYT) {
             const v4f w = *reinterpret_cast<const v4f*>(e.nw + n0), b = *reinterpret_cast<const v4f*>(e.nb + n0);
 #pragma unroll
@@ -180,11 +184,13 @@ template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogu
             if (e.act == OXB_ACT_GELU_TANH) v = gelu_tanh_of<T>(v);
             const size_t o = (size_t)m * e.ld32 + n;
             if (e.resid) v += e.resid[o];
+            sum[i] = v;
             if (e.out32) e.out32[o] = v;
+            if (e.norm == OXB_NORM_SCALE) v *= e.nw[n];
             if (e.norm == OXB_NORM_DYT) v = tanh_of<T>(e.alpha * v) * e.nw[n] + e.nb[n];
             y[i] = v;
         }
-        if (!e.out_t) return;
+        if (!e.out_t) return sum;
     }
     T* t = reinterpret_cast<T*>(e.out_t) + (size_t)m * e.ld_t + n0;
     if (n0 + 4 <= e.fill && (((uintptr_t)t) & (sizeof(T) * 4 - 1)) == 0) {
@@ -197,4 +203,5 @@ template <typename T> __device__ __forceinline__ void epilogue4(const OxbEpilogu
         for (int i = 0; i < 4; i++)
             if (n0 + i < e.fill) t[i] = (T)y[i];
     }
+    return sum;
 }

@@ -44,13 +44,20 @@ struct OxbEpilogue {
     const float *nw, *nb;    // [n] norm weight and bias
     float alpha;             // dynamic tanh
     uint32_t n;              // valid columns
+    // RMS norm over a whole row, its two halves in the products on either side (few-row kernel): the one that completes the
+    // row leaves y * nw in out_t and sums of squares, one per 16 columns, in ssq_out[m][n_pad / 16]; the one that consumes
+    // it multiplies its products by 1 / sqrt(sum(ssq_in[m][0 .. n_ssq)) / ssq_width + ssq_eps) in front of everything else.
+    float* ssq_out;
+    const float* ssq_in;
+    uint32_t n_ssq, ssq_width;
+    float ssq_eps;
     // gated pairs (null: none): columns glu .. hold (gate, up) pairs and only those; gelu_tanh(gate) * up -> glu_out[m][pair]
     uint32_t glu;            // a multiple of 4, >= n
     void* glu_out;           // weights' type
     uint32_t ld_glu, n_glu;  // pairs, even
 };
 enum { OXB_ACT_NONE = 0, OXB_ACT_GELU_TANH = 1 };
-enum { OXB_NORM_NONE = 0, OXB_NORM_DYT = 1 };   // dynamic tanh: tanh(alpha x) * w + b, elementwise
+enum { OXB_NORM_NONE = 0, OXB_NORM_DYT = 1, OXB_NORM_SCALE = 2 };   // dynamic tanh: tanh(alpha x) * w + b, elementwise; x * w
 
 struct OxbDenseParams {
     const void* w;           // operand units
@@ -74,6 +81,8 @@ hipError_t oxb_launch_dense_pack(const void* src, int src_type, const int64_t* r
 // y = W x for any m: up to OXB_DENSE_GEMV_MAX_ROWS through the few-row kernel (weights streamed once, K split over the waves of a
 // workgroup), more through the tiled GEMM.
 hipError_t oxb_launch_dense(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st);
+// Whether a product of this size takes the few-row kernel, for m rows.
+bool oxb_dense_few_rows(uint32_t n_pad, uint32_t k_pad, uint32_t m, uint32_t n_cus);
 hipError_t oxb_launch_dense_gemm_t(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st);
 // Start of a forward on fp32 rows x [m][width]: optional copy of the rows into the second half of a [x; x0] buffer
 // (x0_out + column x0_col, padded with zeros to x0_fill), and the first consumer's activation through the epilogue.

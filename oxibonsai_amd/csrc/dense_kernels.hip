@@ -60,6 +60,7 @@ template <typename T, int RT, int CT, int UN>
 __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
     typedef typename Dt<T>::frag frag;
     __shared__ __attribute__((aligned(16))) float red[8][RT * CT][16][20];
+    __shared__ float row_scale[16 * CT];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, c = lane & 15u, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
     const uint32_t nu = p.k_pad / 32, n_tiles = p.n_pad / 16;
@@ -74,6 +75,17 @@ __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
     for (int r = 0; r < RT; r++)
 #pragma unroll
         for (int t = 0; t < CT; t++) acc[r][t] = (v4f){0.f, 0.f, 0.f, 0.f};
+    // sums of squares of a consumed norm: the first token's are on their way under the products
+    constexpr int PRE = 4;
+    float sq[PRE];
+    auto load_ssq = [&](uint32_t m, uint32_t i0) {
+#pragma unroll
+        for (int k = 0; k < PRE; k++) {
+            const uint32_t i = i0 + 64 * k + lane;
+            sq[k] = i < p.e.n_ssq ? p.e.ssq_in[(size_t)m * p.e.n_ssq + i] : 0.f;
+        }
+    };
+    if (p.e.ssq_in && wave < p.m) load_ssq(wave, 0);
     for (uint32_t u0 = wave; u0 < nu; u0 += 8 * UN) {
         frag b[UN][CT], a[UN][RT];
 #pragma unroll
@@ -103,12 +115,31 @@ __global__ __launch_bounds__(512) void dense_gemv_kernel(OxbDenseParams p) {
     for (int r = 0; r < RT; r++)
 #pragma unroll
         for (int t = 0; t < CT; t++) *reinterpret_cast<v4f*>(&red[wave][r * CT + t][c][4 * g]) = acc[r][t];
+    if (p.e.ssq_in) {
+        for (uint32_t m = wave; m < p.m; m += 8) {
+            float ss = 0.f;
+            for (uint32_t i0 = 0; i0 < p.e.n_ssq; i0 += 64 * PRE) {
+                if (m != wave || i0) load_ssq(m, i0);
+#pragma unroll
+                for (int k = 0; k < PRE; k++) ss += sq[k];
+            }
+            ss = wave_sum_f32(ss);
+            if (lane == 0) row_scale[m] = 1.0f / sqrtf(ss / (float)p.e.ssq_width + p.e.ssq_eps);
+        }
+    }
     __syncthreads();
     if (finish) {
         v4f y = *reinterpret_cast<const v4f*>(&red[0][f][ft & 15u][4 * fq]);
 #pragma unroll
         for (int i = 1; i < 8; i++) y += *reinterpret_cast<const v4f*>(&red[i][f][ft & 15u][4 * fq]);
-        epilogue4<T>(p.e, ft, fn, y, resid);
+        if (p.e.ssq_in) y *= row_scale[ft];
+        y = epilogue4<T>(p.e, ft, fn, y, resid);
+        if (p.e.ssq_out) {
+            float ss = y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3];   // (the tile's four quads are four neighbouring lanes)
+            ss += dpp_f32<0xB1>(ss);
+            ss += dpp_f32<0x4E>(ss);
+            if (fq == 0) p.e.ssq_out[(size_t)ft * n_tiles + fn / 16] = ss;
+        }
     }
 }
 
@@ -312,9 +343,9 @@ static hipError_t launch_gemv(const OxbDenseParams& p, hipStream_t st) {
 
 // Where the few-row kernel is the faster one (measured): always up to 16 rows; up to 32 unless the matrix alone fills the
 // GPU with GEMM tiles; up to 64 where it has few tiles and long rows.
-static bool few_rows(const OxbDenseParams& p, uint32_t n_cus) {
-    const uint32_t tiles = p.n_pad / 16;
-    return p.m <= 16 || (p.m <= 32 && tiles <= 4 * n_cus) || (p.m <= OXB_DENSE_GEMV_MAX_ROWS && tiles <= n_cus && p.k_pad >= 4096);
+bool oxb_dense_few_rows(uint32_t n_pad, uint32_t k_pad, uint32_t m, uint32_t n_cus) {
+    const uint32_t tiles = n_pad / 16;
+    return m <= 16 || (m <= 32 && tiles <= 4 * n_cus) || (m <= OXB_DENSE_GEMV_MAX_ROWS && tiles <= n_cus && k_pad >= 4096);
 }
 
 // Two row tiles per workgroup where the matrix has tiles enough for every CU to get several workgroups all the same; units
@@ -335,7 +366,8 @@ static hipError_t pick_gemv(const OxbDenseParams& p, uint32_t n_cus, hipStream_t
 hipError_t oxb_launch_dense(const OxbDenseParams& p, int dt, uint32_t n_cus, hipStream_t st) {
     const hipError_t e = check(p, dt);
     if (e != hipSuccess) return e;
-    if (few_rows(p, n_cus)) return dt == OXB_DT_BF16 ? pick_gemv<__bf16>(p, n_cus, st) : pick_gemv<float>(p, n_cus, st);
+    if (oxb_dense_few_rows(p.n_pad, p.k_pad, p.m, n_cus)) return dt == OXB_DT_BF16 ? pick_gemv<__bf16>(p, n_cus, st) : pick_gemv<float>(p, n_cus, st);
+    if (p.e.ssq_in || p.e.ssq_out) return hipErrorInvalidValue;   // (the few-row kernel's)
     return dt == OXB_DT_BF16 ? pick_gemm<__bf16, false>(p, n_cus, st) : pick_gemm<float, false>(p, n_cus, st);
 }
 

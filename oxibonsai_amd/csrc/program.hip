@@ -342,7 +342,8 @@ static int alloc_act(const Program& p, ActBuf* a, uint32_t rows, bool absorbed, 
     const size_t es = oxb_dt_bytes(p.dt), R = rows;
     struct { void** ptr; size_t bytes; } bufs[] = {{&a->act, R * p.ld_act * es}, {&a->cat, p.loop_in ? R * p.ld_cat * es : 0},
                                                   {&a->q_abs, absorbed ? R * p.n_q_abs * es : 0}, {&a->attn, R * p.ld_attn * es},
-                                                  {&a->mid, R * p.ld_mid * es}, {(void**)&a->qkv, R * p.ld_qkv * 4}, {(void**)&a->rec, R * p.n_rec * 4}};
+                                                  {&a->mid, R * p.ld_mid * es}, {(void**)&a->qkv, R * p.ld_qkv * 4}, {(void**)&a->rec, R * p.n_rec * 4},
+                                                  {(void**)&a->ssq, R * (oxb_dense_pad(p.c.width) / 16) * 4}};
     for (auto& b : bufs) {
         *b.ptr = nullptr;
         if (!b.bytes) continue;

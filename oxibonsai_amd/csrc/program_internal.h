@@ -68,6 +68,7 @@ struct ActBuf {
     uint32_t rows = 0;
     void *act = nullptr, *cat = nullptr, *q_abs = nullptr, *attn = nullptr, *mid = nullptr;
     float *qkv = nullptr, *rec = nullptr;   // input product; outputs of a recurrence
+    float* ssq = nullptr;                   // sums of squares of a norm between two products
 };
 
 struct Program {

@@ -9,6 +9,7 @@
 #include <algorithm>
 #include <cmath>
 
+#include "mixer_kernels.h"
 #include "program_internal.h"
 
 namespace oxb {
@@ -39,83 +40,95 @@ int check_parallel_layer(const Program& p, const ProgramLayer& l) {
     return rc;
 }
 
-static int encode_attention(Model& m, const ProgramBranch& b, ActBuf& a, const OxbRows& rows, bool step) {
+// Parameters of a grouped attention branch: the new tokens' store, and the attention with what follows it.
+static int attention_params(Model& m, const ProgramBranch& b, ActBuf& a, const OxbRows& rows, OxbGroupedStore* s, OxbRowAttnParams* q) {
     Program& p = *m.prog;
-    hipStream_t st = g_rt.stream;
     int rc = OXB_HIP_OK;
-    OxbRowAttnParams q;
-    memset(&q, 0, sizeof q);
-    q.sink = vec_ptr(b.sink, b.heads, "sink", &rc);
+    memset(s, 0, sizeof *s);
+    memset(q, 0, sizeof *q);
+    q->sink = vec_ptr(b.sink, b.heads, "sink", &rc);
     if (rc) return rc;
     const size_t slots = m.n_pages ? (size_t)m.n_pages << m.page_shift : (size_t)m.d.batch * m.row_stride;
+    s->rows = q->rows = rows;
+    s->lin = a.qkv;
+    s->ld_lin = p.ld_qkv;
+    s->col_q = b.col_q, s->col_k = b.col_k, s->col_v = b.col_v;
+    s->heads = b.heads, s->kv_heads = b.kv_heads;
+    s->dim = b.dim, s->dim_p = b.dim_p, s->vdim = b.vdim, s->vdim_p = b.vdim_p;
+    s->rot_dims = p.rope[b.rope].r.dims;
+    s->eps = p.c.eps;
+    s->cos_t = p.rope[b.rope].cos_t;
+    s->sin_t = p.rope[b.rope].sin_t;
+    s->q = a.q_abs;
+    s->cache = (uint8_t*)m.k_cache + b.cache_off * slots * oxb_dt_bytes(p.dt);
+    s->kv = kv_layout(m);
+    s->kv.n_layers = 1;
+    s->kv.nkv = b.kv_heads;
+    q->kv = s->kv;
+    q->q = a.q_abs;
+    q->heads = b.heads;
+    q->rep = b.heads / b.kv_heads;
+    q->cache = s->cache;
+    q->ld = b.dim_p + b.vdim_p;
+    q->ks = q->v0 = b.dim_p / 32;
+    q->nt = b.vdim_p / 16;
+    q->scale = b.att_scale;
+    q->part_o = p.part_o;
+    q->part_ml = p.part_ml;
+    q->n_splits = grouped_splits(m, b, rows.m);
+    q->out = a.attn;
+    q->ld_out = p.ld_attn;
+    q->out_col = b.out_col;
+    q->out_scale = b.scale;
+    return OXB_HIP_OK;
+}
+
+static int recurrent_params(Model& m, const ProgramBranch& b, ActBuf& a, const OxbRows& rows, OxbRecurParams* r) {
+    Program& p = *m.prog;
+    int rc = OXB_HIP_OK;
+    auto vec = [&](uint64_t id, uint32_t n, const char* what) { return rc || !id ? nullptr : vec_ptr(id, n, what, &rc); };
+    memset(r, 0, sizeof *r);
+    r->d = b.r;
+    r->rows = rows;
+    r->lin = a.qkv;
+    r->ld_lin = p.ld_qkv;
+    r->conv_w = vec(b.conv_w, b.r.channels * b.r.taps, "convolution");
+    r->conv_b = vec(b.conv_b, b.r.channels, "convolution bias");
+    r->neg_a = vec(b.neg_a, b.r.heads, "decay");
+    r->dt_bias = vec(b.dt_bias, b.r.heads, "decay bias");
+    r->skip = vec(b.skip, b.r.heads, "skip");
+    r->norm_w = vec(b.norm_w, b.r.norm_shared ? b.r.norm_len : b.r.heads * b.r.dv, "output norm");
+    r->memory = p.memory + b.memory_off;
+    r->seq_stride = p.memory_floats;
+    r->o = a.rec;
+    r->out = a.attn;
+    r->ld_out = p.ld_attn;
+    r->out_col = b.out_col;
+    r->out_fill = b.out_fill;
+    return rc;
+}
+
+static int encode_attention(Model& m, const ProgramBranch& b, ActBuf& a, const OxbRows& rows, bool step) {
+    const int dt = m.prog->dt;
+    hipStream_t st = g_rt.stream;
     OxbGroupedStore s;
-    memset(&s, 0, sizeof s);
-    s.rows = q.rows = rows;
-    s.lin = a.qkv;
-    s.ld_lin = p.ld_qkv;
-    s.col_q = b.col_q, s.col_k = b.col_k, s.col_v = b.col_v;
-    s.heads = b.heads, s.kv_heads = b.kv_heads;
-    s.dim = b.dim, s.dim_p = b.dim_p, s.vdim = b.vdim, s.vdim_p = b.vdim_p;
-    s.rot_dims = p.rope[b.rope].r.dims;
-    s.eps = p.c.eps;
-    s.cos_t = p.rope[b.rope].cos_t;
-    s.sin_t = p.rope[b.rope].sin_t;
-    s.q = a.q_abs;
-    s.cache = (uint8_t*)m.k_cache + b.cache_off * slots * oxb_dt_bytes(p.dt);
-    s.kv = kv_layout(m);
-    s.kv.n_layers = 1;
-    s.kv.nkv = b.kv_heads;
-    OXB_TRY_HIP(oxb_launch_grouped_store(s, p.dt, st), "kernel launch failed: grouped_store");
-    q.kv = s.kv;
-    q.q = a.q_abs;
-    q.heads = b.heads;
-    q.rep = b.heads / b.kv_heads;
-    q.cache = s.cache;
-    q.ld = b.dim_p + b.vdim_p;
-    q.ks = q.v0 = b.dim_p / 32;
-    q.nt = b.vdim_p / 16;
-    q.scale = b.att_scale;
-    q.part_o = p.part_o;
-    q.part_ml = p.part_ml;
-    q.n_splits = grouped_splits(m, b, rows.m);
-    q.out = a.attn;
-    q.ld_out = p.ld_attn;
-    q.out_col = b.out_col;
-    q.out_scale = b.scale;
+    OxbRowAttnParams q;
+    OXB_TRY(attention_params(m, b, a, rows, &s, &q));
+    OXB_TRY_HIP(oxb_launch_grouped_store(s, dt, st), "kernel launch failed: grouped_store");
     if (!step) {
-        OXB_TRY_HIP(oxb_launch_row_prefill(q, p.dt, st), "kernel launch failed: row_prefill");
+        OXB_TRY_HIP(oxb_launch_row_prefill(q, dt, st), "kernel launch failed: row_prefill");
         return OXB_HIP_OK;
     }
-    OXB_TRY_HIP(oxb_launch_row_decode(q, 1, p.dt, st), "kernel launch failed: row_decode");
-    OXB_TRY_HIP(oxb_launch_row_merge(q, p.dt, st), "kernel launch failed: row_merge");
+    OXB_TRY_HIP(oxb_launch_row_decode(q, 1, dt, st), "kernel launch failed: row_decode");
+    OXB_TRY_HIP(oxb_launch_row_merge(q, dt, st), "kernel launch failed: row_merge");
     return OXB_HIP_OK;
 }
 
 static int encode_recurrent(Model& m, const ProgramBranch& b, ActBuf& a, const OxbRows& rows, bool step) {
     Program& p = *m.prog;
     hipStream_t st = g_rt.stream;
-    int rc = OXB_HIP_OK;
-    auto vec = [&](uint64_t id, uint32_t n, const char* what) { return rc || !id ? nullptr : vec_ptr(id, n, what, &rc); };
     OxbRecurParams r;
-    memset(&r, 0, sizeof r);
-    r.d = b.r;
-    r.rows = rows;
-    r.lin = a.qkv;
-    r.ld_lin = p.ld_qkv;
-    r.conv_w = vec(b.conv_w, b.r.channels * b.r.taps, "convolution");
-    r.conv_b = vec(b.conv_b, b.r.channels, "convolution bias");
-    r.neg_a = vec(b.neg_a, b.r.heads, "decay");
-    r.dt_bias = vec(b.dt_bias, b.r.heads, "decay bias");
-    r.skip = vec(b.skip, b.r.heads, "skip");
-    r.norm_w = vec(b.norm_w, b.r.norm_shared ? b.r.norm_len : b.r.heads * b.r.dv, "output norm");
-    if (rc) return rc;
-    r.memory = p.memory + b.memory_off;
-    r.seq_stride = p.memory_floats;
-    r.o = a.rec;
-    r.out = a.attn;
-    r.ld_out = p.ld_attn;
-    r.out_col = b.out_col;
-    r.out_fill = b.out_fill;
+    OXB_TRY(recurrent_params(m, b, a, rows, &r));
     if (step) {
         OXB_TRY_HIP(oxb_launch_recur_step(r, p.dt, st), "kernel launch failed: recur_step");
         if (oxb_recur_step_finishes(b.r)) return OXB_HIP_OK;
@@ -131,6 +144,30 @@ static int encode_recurrent(Model& m, const ProgramBranch& b, ActBuf& a, const O
     return OXB_HIP_OK;
 }
 
+// All mixers of a block.  A decode step of attention beside a recurrence shares launches between the two.
+static int encode_branches(Model& m, const ProgramLayer& l, ActBuf& a, const OxbRows& rows, bool step) {
+    const int dt = m.prog->dt;
+    hipStream_t st = g_rt.stream;
+    if (step && l.branches.size() == 2 && l.branches[0].kind == MixerKind::GroupedAttention && l.branches[1].kind != MixerKind::GroupedAttention) {
+        OxbGroupedStore s;
+        OxbRowAttnParams q;
+        OxbRecurParams r;
+        OXB_TRY(attention_params(m, l.branches[0], a, rows, &s, &q));
+        OXB_TRY(recurrent_params(m, l.branches[1], a, rows, &r));
+        if (oxb_pair_ok(s, r)) {
+            OXB_TRY_HIP(oxb_launch_pair_enter(s, r, dt, st), "kernel launch failed: pair_enter");
+            OXB_TRY_HIP(oxb_launch_row_decode(q, 1, dt, st), "kernel launch failed: row_decode");
+            OXB_TRY_HIP(oxb_launch_pair_leave(q, r, dt, st), "kernel launch failed: pair_leave");
+            return OXB_HIP_OK;
+        }
+    }
+    for (const ProgramBranch& b : l.branches) {
+        if (b.kind == MixerKind::GroupedAttention) OXB_TRY(encode_attention(m, b, a, rows, step));
+        else OXB_TRY(encode_recurrent(m, b, a, rows, step));
+    }
+    return OXB_HIP_OK;
+}
+
 int encode_parallel_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, bool step) {
     Program& p = *m.prog;
     const uint32_t w = p.c.width;
@@ -141,12 +178,25 @@ int encode_parallel_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, b
         OXB_TRY_HIP(oxb_launch_row_norm(x, w, rows.m, in_scale, nw, p.c.eps, a.act, p.ld_act, oxb_dense_pad(w), p.dt, g_rt.stream), "kernel launch failed: row_norm");
         return OXB_HIP_OK;
     };
+    // The norm between two layers is split over the products on either side where both take the few-row kernel.
+    const uint32_t w_pad = oxb_dense_pad(w);
+    auto few = [&](uint64_t id) {
+        const DenseWeight* d = dense_ptr(id, "weight", &rc);
+        return d && oxb_dense_few_rows(d->n_pad, d->k_pad, rows.m, g_rt.n_cus);
+    };
+    bool half_normed = false;   // a.act holds x * weight, a.ssq the sums of squares
     for (size_t i = 0; i < p.layers.size(); i++) {
         const ProgramLayer& l = p.layers[i];
-        OXB_TRY(norm(l.norm1, i ? 1.0f : p.c.embed_scale));
+        if (!half_normed) OXB_TRY(norm(l.norm1, i ? 1.0f : p.c.embed_scale));
         OxbEpilogue e = epilogue(l.n_lin);
         e.out32 = a.qkv;
         e.ld32 = p.ld_qkv;
+        if (half_normed) {
+            e.ssq_in = a.ssq;
+            e.n_ssq = w_pad / 16;
+            e.ssq_width = w;
+            e.ssq_eps = p.c.eps;
+        }
         if (l.has_mlp) {
             e.glu = l.n_lin;
             e.glu_out = (uint8_t*)a.attn + (size_t)l.mid_col * oxb_dt_bytes(p.dt);
@@ -154,14 +204,21 @@ int encode_parallel_layers(Model& m, ActBuf& a, float* x, const OxbRows& rows, b
             e.n_glu = oxb_dense_pad(l.ff);
         }
         OXB_TRY(product(p, l.in, a.act, p.ld_act, rows.m, e, "kernel launch failed: input product"));
-        for (const ProgramBranch& b : l.branches) {
-            if (b.kind == MixerKind::GroupedAttention) OXB_TRY(encode_attention(m, b, a, rows, step));
-            else OXB_TRY(encode_recurrent(m, b, a, rows, step));
-        }
+        OXB_TRY(encode_branches(m, l, a, rows, step));
         OxbEpilogue o = epilogue(w);
         o.scale = p.c.residual_mult;
         o.resid = o.out32 = x;
         o.ld32 = w;
+        half_normed = i + 1 < p.layers.size() && few(l.out) && few(p.layers[i + 1].in);
+        if (half_normed) {
+            o.nw = vec_ptr(p.layers[i + 1].norm1.w, w, "norm", &rc);
+            o.norm = OXB_NORM_SCALE;
+            o.out_t = a.act;
+            o.ld_t = p.ld_act;
+            o.fill = w_pad;
+            o.ssq_out = a.ssq;
+        }
+        if (rc) return rc;
         OXB_TRY(product(p, l.out, a.attn, p.ld_attn, rows.m, o, "kernel launch failed: output product"));
     }
     return norm(p.final_norm, 1.0f);

@@ -80,4 +80,6 @@ bool oxb_recur_step_finishes(const OxbRecurDims& d);
 hipError_t oxb_launch_recur_chunked(const OxbRecurParams& p, hipStream_t st);
 // keep_conv: also bring the last convolution inputs of a chunked portion into the ring.
 hipError_t oxb_launch_recur_finish(const OxbRecurParams& p, bool keep_conv, int dt, hipStream_t st);
+bool oxb_recur_params_ok(const OxbRecurParams& p);
+bool oxb_recur_finish_ok(const OxbRecurParams& p);
 const char* oxb_recur_check(const OxbRecurDims& d);

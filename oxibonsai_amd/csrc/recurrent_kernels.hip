@@ -2,166 +2,11 @@
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 
-#include "dense_device.h"
-#include "recurrent_kernels.h"
+#include "recurrent_device.h"
 
-__device__ __forceinline__ float silu_of(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_of(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-__device__ __forceinline__ v4f load4(const float* p) { return *reinterpret_cast<const v4f*>(p); }
-
-// Short convolution and its activation: channel ch of the token in row `row` of the input product, at position pos; `back`
-// earlier rows of the same sequence lie in front of it there, older inputs in the ring.
-__device__ __forceinline__ float conv_of(const OxbRecurParams& p, const float* ring, uint32_t row, uint32_t back, uint32_t pos, uint32_t ch) {
-    const OxbRecurDims& d = p.d;
-    const float* w = p.conv_w + (size_t)ch * d.taps;
-    const float* x = p.lin + (size_t)row * p.ld_lin + d.col_conv + ch;
-    auto past = [&](uint32_t j) {
-        const float* at = j <= back ? x - (size_t)j * p.ld_lin : ring + (size_t)((pos - j) & (d.ring - 1u)) * d.channels + ch;
-        return *at * w[d.taps - 1 - j];
-    };
-    const uint32_t n = min(d.taps - 1, pos);   // inputs there are behind this one
-    const float x0 = x[0] * w[d.taps - 1], x1 = n >= 1 ? past(1) : 0.f, x2 = n >= 2 ? past(2) : 0.f, x3 = n >= 3 ? past(3) : 0.f;
-    float v = (p.conv_b ? p.conv_b[ch] : 0.f) + x0 + x1 + x2 + x3;
-#pragma unroll 1
-    for (uint32_t j = 4; j <= n; j++) v += past(j);
-    return silu_of(v);
-}
-
-// Logarithm of the decay and beta of one head from its columns of the input product.
-__device__ __forceinline__ void gates_of(const OxbRecurParams& p, uint32_t row, uint32_t head, float* la, float* beta) {
-    const float* x = p.lin + (size_t)row * p.ld_lin;
-    const float sp = softplus_of(x[p.d.col_a + head] + p.dt_bias[head]);
-    *la = p.neg_a[head] * sp;
-    *beta = p.d.delta ? 1.0f / (1.0f + expf(-x[p.d.col_b + head])) : sp;
-}
-
-// ---------------------------------------------------------------------------
-// Step.  Grid (head x slice group, sequence), 256 threads per slice of 32 columns: thread (rg, cl) = (tid / 8 % 32, tid % 8)
-// holds rows rg + 32 j and columns 4 cl .. + 3 of its slice of the state.  S^T k and S^T q come out of the state as it was, in
-// one pass: with the write k u^T, o = a (S^T q) + (k . q) u.  With every slice of a head in the workgroup (FINISH) the head's
-// output is gated and normed here as well.
-// ---------------------------------------------------------------------------
 template <typename T, int RPT, int SL, bool FINISH, bool ONE>
-__global__ __launch_bounds__(256 * SL, ONE && RPT <= 4 ? 8 : 4) void recur_step_kernel(OxbRecurParams p, uint32_t n_tokens) {
-    const OxbRecurDims& d = p.d;
-    const uint32_t tokens = ONE ? 1 : n_tokens;
-    __shared__ __attribute__((aligned(16))) float qs[256], ks[256], vs[32 * SL], os[32 * SL];
-    __shared__ __attribute__((aligned(16))) float part[4 * SL][8][8];
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, cl = tid & 7u, rg = (tid >> 3) & 31u;
-    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6)), mine = wave >> 2;   // slice of the workgroup's
-    const uint32_t groups = (d.slices + SL - 1) / SL, head = blockIdx.x / groups, slice = blockIdx.x % groups * SL + mine;
-    const uint32_t row0 = blockIdx.y * tokens, rep = d.heads / d.qk_heads, qk = head / rep, pos0 = row_pos(p.rows, row0);
-    float* mem = p.memory + (size_t)row_seq(p.rows, row0) * p.seq_stride;
-    float* state = mem + ((size_t)head * d.slices + min(slice, d.slices - 1)) * d.dk_p * 32 + rg * 32 + 4 * cl;
-    float* ring = mem + oxb_recur_state(d);
-    v4f s[RPT];
-#pragma unroll
-    for (int j = 0; j < RPT; j++) s[j] = pos0 && 32u * j < d.dk_p ? load4(state + 1024 * j) : (v4f){0.f, 0.f, 0.f, 0.f};
-    const bool own_qk = head % rep == 0 && blockIdx.x % groups == 0;
-    // which convolutions a thread brings: queries, keys, values in turn, spread over the workgroup
-    const uint32_t qi = tid, ki = SL > 1 ? tid - 256u : tid, vi = SL > 2 ? tid - 512u : 256u * SL - 1 - tid;
-    const uint32_t vcol = blockIdx.x % groups * SL * 32 + vi;
-    for (uint32_t t = 0; t < tokens; t++) {
-        const uint32_t row = row0 + t, pos = pos0 + t;
-        const float* lin = p.lin + (size_t)row * p.ld_lin;
-        float z[FINISH ? (SL + 1) / 2 : 1], nw[FINISH ? (SL + 1) / 2 : 1];
-        if constexpr (FINISH) {
-            if (wave == 0) {
-#pragma unroll
-                for (int e = 0; e < (SL + 1) / 2; e++) {
-                    const uint32_t i = min(lane + 64 * e, d.dv - 1);
-                    z[e] = lin[d.col_z + head * d.dv + i];
-                    nw[e] = p.norm_w[i];
-                }
-            }
-        }
-        float la, beta;
-        gates_of(p, row, head, &la, &beta);
-        const float a = expf(la);
-        if (qi < d.dk_p) qs[qi] = qi < d.dk ? conv_of(p, ring, row, t, pos, d.ch_q + qk * d.dk + qi) : 0.f;
-        if (ki < d.dk_p) ks[ki] = ki < d.dk ? conv_of(p, ring, row, t, pos, d.ch_k + qk * d.dk + ki) : 0.f;
-        if (vi < 32 * SL) vs[vi] = vcol < d.dv ? conv_of(p, ring, row, t, pos, d.ch_v + head * d.dv + vcol) : 0.f;
-        if (d.taps > 1 && t + d.taps > tokens) {   // inputs that later tokens convolve
-            float* keep = ring + (size_t)(pos & (d.ring - 1u)) * d.channels;
-            const float* x = lin + d.col_conv;
-            if (own_qk && qi < d.dk) keep[d.ch_q + qk * d.dk + qi] = x[d.ch_q + qk * d.dk + qi];
-            if (own_qk && ki < d.dk) keep[d.ch_k + qk * d.dk + ki] = x[d.ch_k + qk * d.dk + ki];
-            if (vi < 32 * SL && vcol < d.dv) keep[d.ch_v + head * d.dv + vcol] = x[d.ch_v + head * d.dv + vcol];
-        }
-        __syncthreads();
-        float qq = 0.f, kk = 0.f, kq = 0.f;   // (every wave for itself)
-        #pragma unroll 1
-        for (uint32_t i = lane; i < d.dk_p; i += 64) {
-            const float q = qs[i], k = ks[i];
-            qq = fmaf(q, q, qq), kk = fmaf(k, k, kk), kq = fmaf(k, q, kq);
-        }
-        float rq = 1.0f, rk = 1.0f;
-        if (d.delta) {
-            rq = d.q_scale / sqrtf(wave_sum_f32(qq) + 1e-6f);
-            rk = 1.0f / sqrtf(wave_sum_f32(kk) + 1e-6f);
-        }
-        const float dot = wave_sum_f32(kq) * rq * rk;
-        v4f sk = {0.f, 0.f, 0.f, 0.f}, sq = sk;
-#pragma unroll
-        for (int j = 0; j < RPT; j++)
-            if (32u * j < d.dk_p) {
-                sk += s[j] * ks[rg + 32 * j];
-                sq += s[j] * qs[rg + 32 * j];
-            }
-#pragma unroll
-        for (int i = 0; i < 4; i++) {   // over the wave's eight row groups
-            sk[i] = sum_rows4(sk[i] + dpp_f32<0x128>(sk[i]));
-            sq[i] = sum_rows4(sq[i] + dpp_f32<0x128>(sq[i]));
-        }
-        if (lane < 8) {
-            *reinterpret_cast<v4f*>(&part[wave][cl][0]) = sk;
-            *reinterpret_cast<v4f*>(&part[wave][cl][4]) = sq;
-        }
-        __syncthreads();
-        const uint32_t w0 = 4 * mine;
-        sk = load4(&part[w0][cl][0]) + load4(&part[w0 + 1][cl][0]) + load4(&part[w0 + 2][cl][0]) + load4(&part[w0 + 3][cl][0]);
-        sq = load4(&part[w0][cl][4]) + load4(&part[w0 + 1][cl][4]) + load4(&part[w0 + 2][cl][4]) + load4(&part[w0 + 3][cl][4]);
-        const v4f v = load4(&vs[32 * mine + 4 * cl]);
-        const v4f u = d.delta ? (v - sk * (a * rk)) * beta : v * beta, uk = u * rk;
-#pragma unroll
-        for (int j = 0; j < RPT; j++)
-            if (32u * j < d.dk_p) s[j] = s[j] * a + uk * ks[rg + 32 * j];
-        if (rg == 0) {
-            v4f o = sq * (a * rq) + u * dot;
-            if (p.skip) o += v * p.skip[head];
-            if constexpr (FINISH) {
-                *reinterpret_cast<v4f*>(&os[32 * mine + 4 * cl]) = o;
-            } else {
-                float* dst = p.o + (size_t)row * d.heads * d.dv + head * d.dv + slice * 32 + 4 * cl;
-#pragma unroll
-                for (int i = 0; i < 4; i++)
-                    if (slice * 32 + 4 * cl + i < d.dv) dst[i] = o[i];
-            }
-        }
-        if (FINISH || t + 1 < tokens) __syncthreads();
-        if constexpr (FINISH) {
-            if (wave == 0) {
-                float y[(SL + 1) / 2], ss = 0.f;
-#pragma unroll
-                for (int e = 0; e < (SL + 1) / 2; e++) {
-                    y[e] = lane + 64 * e < d.dv ? os[lane + 64 * e] : 0.f;
-                    ss = fmaf(y[e], y[e], ss);
-                }
-                const float inv = d.out_scale / sqrtf(wave_sum_f32(ss) / (float)d.dv + d.eps);
-                T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ld_out + p.out_col;
-#pragma unroll
-                for (int e = 0; e < (SL + 1) / 2; e++)
-                    if (lane + 64 * e < d.dv) out[head * d.dv + lane + 64 * e] = (T)(y[e] * inv * nw[e] * silu_of(z[e]));
-                if (head == 0)
-                    for (uint32_t i = d.heads * d.dv + lane; i < p.out_fill; i += 64) out[i] = (T)0.f;
-            }
-        }
-    }
-    if (slice < d.slices) {
-#pragma unroll
-        for (int j = 0; j < RPT; j++)
-            if (32u * j < d.dk_p) *reinterpret_cast<v4f*>(state + 1024 * j) = s[j];
-    }
+__global__ __launch_bounds__(256 * SL, ONE && RPT <= 4 ? (SL == 4 ? 8 : 7) : 4) void recur_step_kernel(OxbRecurParams p, uint32_t tokens) {   // grid (head x slice group, sequence)
+    recur_step<T, RPT, SL, FINISH, ONE>(p, tokens, blockIdx.x, blockIdx.y);
 }
 
 // ---------------------------------------------------------------------------
@@ -415,10 +260,10 @@ __global__ __launch_bounds__(256) void recur_chunk_kernel(OxbRecurParams p, uint
 // Scan.  Grid (head x 16 columns, the tiles of a head on one XCD: they share its L2), 4 waves: wave w takes token rows 16 w .. of every chunk and the state's row tiles w, w + 4,
 // ..; per chunk, with S the state at its start,
 //   U = U0 - W S        o = e^c (Q S) + P U        S <- e^(c_end) S + K^T diag(e^(c_end - c)) U
-// The operands of the next chunk are requested as soon as this chunk's have been used; the barriers order LDS alone.
+// The operands of a later chunk are requested as soon as this chunk's have been used; the barriers order LDS alone.
 // ---------------------------------------------------------------------------
 template <int DKU, bool DELTA>
-__global__ __launch_bounds__(256) void recur_scan_kernel(OxbRecurParams p, uint32_t dv_p) {
+__global__ __launch_bounds__(256, 1) void recur_scan_kernel(OxbRecurParams p, uint32_t dv_p) {
     const OxbRecurDims& d = p.d;
     constexpr int DK = 32 * DKU, TPW = (2 * DKU + 3) / 4;
     __shared__ __attribute__((aligned(16))) float Sx[16][DK + 4], Ux[16][kLdT], Uf[16][kLdT];
@@ -443,76 +288,85 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(OxbRecurParams p, uint3
             *reinterpret_cast<v4f*>(&Sx[c][r0]) = S[j];
         }
     }
-    v8f qf[DKU], wf[DELTA ? DKU : 1], pf[2], kf[TPW][2];
-    v4f u0, gam, fwd;
-    float g_end;
-    auto load_qw = [&](uint32_t ch) {
-        const float* q = p.s.q + ((size_t)min(ch * 64 + 16 * w + c, last) * d.qk_heads + qk) * DK + 4 * g;
-        const float* W = p.s.W + ((size_t)ch * d.heads + head) * 64 * DK + (size_t)w * 16 * DK;
-#pragma unroll
-        for (int u = 0; u < DKU; u++) {
-            qf[u] = join(load4(q + 32 * u), load4(q + 32 * u + 16));
-            if constexpr (DELTA) wf[u] = load_unit(W + u * 512, lane);
-        }
+    constexpr int NS = DKU <= 4 ? 2 : 1;   // chunks whose operands of the first two products are on their way or in registers
+    v8f qf[NS][DKU], wf[NS][DELTA ? DKU : 1], pf[2], kf[TPW][2];
+    v4f u0[NS], gam[NS], fwd[NS], beta[NS];
+    float g_end[NS];
+    auto q_at = [&](uint32_t ch) { return p.s.q + ((size_t)min(min(ch, n_chunks - 1) * 64 + 16 * w + c, last) * d.qk_heads + qk) * DK + 4 * g; };
+    auto w_at = [&](uint32_t ch) { return p.s.W + ((size_t)min(ch, n_chunks - 1) * d.heads + head) * 64 * DK + (size_t)w * 16 * DK; };
+    auto load_qw = [&](const float* q, const float* W, int set, int u) {
+        qf[set][u] = join(load4(q + 32 * u), load4(q + 32 * u + 16));
+        if constexpr (DELTA) wf[set][u] = load_unit(W + u * 512, lane);
     };
-    auto load_rest = [&](uint32_t ch) {
+    auto load_u = [&](uint32_t c0, int set) {
+        const uint32_t ch = min(c0, n_chunks - 1);
         const size_t slot = (size_t)ch * d.heads + head;
-        const float* P = p.s.P + slot * 4096 + w * 1024;
-        const float* kt = p.s.Kt + ((size_t)ch * d.qk_heads + qk) * (2 * DKU) * 1024;
-#pragma unroll
-        for (int u = 0; u < 2; u++) {
-            pf[u] = load_unit(P + u * 512, lane);
-#pragma unroll
-            for (int j = 0; j < TPW; j++) kf[j][u] = load_unit(kt + (size_t)min(w + 4 * j, 2u * DKU - 1) * 1024 + u * 512, lane);
-        }
-    };
-    auto load_u = [&](uint32_t ch) {
-        const size_t slot = (size_t)ch * d.heads + head;
-        gam = load4(p.s.gam + slot * 64 + 16 * w + 4 * g);
-        fwd = load4(p.s.fwd + slot * 64 + 16 * w + 4 * g);
-        g_end = p.s.gam[slot * 64 + 63];
+        gam[set] = load4(p.s.gam + slot * 64 + 16 * w + 4 * g);
+        fwd[set] = load4(p.s.fwd + slot * 64 + 16 * w + 4 * g);
+        g_end[set] = p.s.gam[slot * 64 + 63];
         if constexpr (DELTA) {
-            u0 = load4(p.s.U0 + (slot * dvt + tile) * 1024 + w * 256 + lane * 4);
+            u0[set] = load4(p.s.U0 + (slot * dvt + tile) * 1024 + w * 256 + lane * 4);
         } else {
-#pragma unroll
-            for (int v = 0; v < 4; v++) u0[v] = p.s.v[((size_t)min(ch * 64 + 16 * w + 4 * g + v, last) * d.heads + head) * dv_p + col];
-        }
-    };
-    v4f beta = {0.f, 0.f, 0.f, 0.f};
-    auto load_beta = [&](uint32_t ch) {
-        if constexpr (!DELTA) {
 #pragma unroll
             for (int v = 0; v < 4; v++) {
                 const uint32_t m = ch * 64 + 16 * w + 4 * g + v;
-                beta[v] = m < p.n ? p.s.beta[(size_t)m * d.heads + head] : 0.f;
+                u0[set][v] = p.s.v[((size_t)min(m, last) * d.heads + head) * dv_p + col];
+                beta[set][v] = m < p.n ? p.s.beta[(size_t)m * d.heads + head] : 0.f;
             }
         }
     };
-    load_qw(0);
-    load_u(0);
-    load_beta(0);
-    load_rest(0);
+    auto p_at = [&](uint32_t ch) { return p.s.P + ((size_t)min(ch, n_chunks - 1) * d.heads + head) * 4096 + w * 1024; };
+    auto k_at = [&](uint32_t ch) { return p.s.Kt + ((size_t)min(ch, n_chunks - 1) * d.qk_heads + qk) * (2 * DKU) * 1024; };
+    auto load_pk = [&](const float* P, const float* kt, int u) {
+        pf[u] = load_unit(P + u * 512, lane);
+#pragma unroll
+        for (int j = 0; j < TPW; j++) kf[j][u] = load_unit(kt + (size_t)min(w + 4 * j, 2u * DKU - 1) * 1024 + u * 512, lane);
+    };
+#pragma unroll
+    for (int i = 0; i < NS; i++) {
+#pragma unroll
+        for (int u = 0; u < DKU; u++) load_qw(q_at(i), w_at(i), i, u);
+        load_u(i, i);
+    }
+    load_pk(p_at(0), k_at(0), 0);
+    load_pk(p_at(0), k_at(0), 1);
     const float skip = p.skip ? p.skip[head] : 0.f;
-    for (uint32_t ch = 0; ch < n_chunks; ch++) {
+    // Stores behind the end fall outside the buffer and are dropped: no branch, so the count of requests in flight stays known
+    // and a chunk waits for its own operands alone.
+    const uint32_t inner = d.heads * d.dv, o_bytes = p.n * inner * 4u;
+    const __amdgpu_buffer_rsrc_t out = make_rsrc(p.o + (size_t)p.first * inner, o_bytes);
+    const uint32_t o_at = ((16 * w + 4 * g) * inner + head * d.dv + col) * 4u;
+    auto step = [&](uint32_t ch, int set) {
+        const bool live = ch < n_chunks;   // (the last group of NS chunks may run over the end)
         lds_barrier();
         v4f oq = {0.f, 0.f, 0.f, 0.f}, ws = oq;
+        const float *qn = q_at(ch + NS), *wn = w_at(ch + NS), *pn = p_at(ch + 1), *kn = k_at(ch + 1);
+        // an operand's successor is requested right behind its last product, so that the requests spread over the products
 #pragma unroll
         for (int u = 0; u < DKU; u++) {
             const v8f sb = join(load4(&Sx[c][32 * u + 4 * g]), load4(&Sx[c][32 * u + 16 + 4 * g]));
-            if constexpr (DELTA) ws = mfma32(wf[u], sb, ws);
-            oq = mfma32(qf[u], sb, oq);
+            if constexpr (DELTA) ws = mfma32(wf[set][u], sb, ws);
+            oq = mfma32(qf[set][u], sb, oq);
+            load_qw(qn, wn, set, u);
         }
-        const uint32_t next = min(ch + 1, n_chunks - 1);
-        load_qw(next);
-        const v4f v = u0, U = DELTA ? u0 - ws : u0 * beta, gc = gam, ge = {g_end, g_end, g_end, g_end};
-        *reinterpret_cast<v4f*>(&Ux[c][16 * w + 4 * g]) = U;
-        *reinterpret_cast<v4f*>(&Uf[c][16 * w + 4 * g]) = U * fwd;
-        load_u(next);
-        load_beta(next);
-        lds_barrier();
-        v4f o = oq * gc;
 #pragma unroll
-        for (int j = 0; j < TPW; j++) S[j] *= ge;
+        for (int u = 0; u < DKU; u++) {
+            __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);                 // LDS read
+            __builtin_amdgcn_sched_group_barrier(0x008, DELTA ? 16 : 8, 0);    // matrix core
+            __builtin_amdgcn_sched_group_barrier(0x020, DELTA ? 4 : 2, 0);     // request
+        }
+        __builtin_amdgcn_sched_barrier(0);
+        const v4f v = u0[set];
+        v4f U = DELTA ? u0[set] - ws : u0[set] * beta[set];
+        if (!live) U = (v4f){0.f, 0.f, 0.f, 0.f};
+        *reinterpret_cast<v4f*>(&Ux[c][16 * w + 4 * g]) = U;
+        *reinterpret_cast<v4f*>(&Uf[c][16 * w + 4 * g]) = U * fwd[set];
+        v4f o = oq * gam[set];
+        const float end = live ? g_end[set] : 1.0f;
+#pragma unroll
+        for (int j = 0; j < TPW; j++) S[j] *= end;
+        load_u(ch + NS, set);
+        lds_barrier();
 #pragma unroll
         for (int u = 0; u < 2; u++) {
             const v8f ub = join(load4(&Ux[c][32 * u + 4 * g]), load4(&Ux[c][32 * u + 16 + 4 * g]));
@@ -520,21 +374,30 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(OxbRecurParams p, uint3
             o = mfma32(pf[u], ub, o);
 #pragma unroll
             for (int j = 0; j < TPW; j++) S[j] = mfma32(kf[j][u], uf, S[j]);
+            load_pk(pn, kn, u);
         }
-        load_rest(next);
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
+            __builtin_amdgcn_sched_group_barrier(0x008, 8 * (1 + TPW), 0);
+            __builtin_amdgcn_sched_group_barrier(0x020, 2 * (1 + TPW), 0);
+        }
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int j = 0; j < TPW; j++) {
             const uint32_t r0 = 16 * (w + 4 * j) + 4 * g;
-            if (r0 < DK) *reinterpret_cast<v4f*>(&Sx[c][r0]) = S[j];
+            if (4 * (j + 1) <= 2 * DKU || r0 < DK) *reinterpret_cast<v4f*>(&Sx[c][r0]) = S[j];
         }
-        if (col < d.dv) {
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const uint32_t m = ch * 64 + 16 * w + 4 * g + i;
-                if (m < p.n) p.o[(size_t)(p.first + m) * d.heads * d.dv + head * d.dv + col] = o[i] + (DELTA ? 0.f : skip * v[i]);
-            }
+        for (int i = 0; i < 4; i++) {
+            const uint32_t m = ch * 64 + 16 * w + 4 * g + i;
+            __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(o[i] + (DELTA ? 0.f : skip * v[i])), out,
+                                                  (int)(m < p.n && col < d.dv ? o_at + (ch * 64 + i) * inner * 4u : OXB_OOB), 0, 0);
         }
-    }
+    };
+    for (uint32_t ch = 0; ch < n_chunks; ch += NS)
+#pragma unroll
+        for (int i = 0; i < NS; i++) step(ch + i, i);
 #pragma unroll
     for (int j = 0; j < TPW; j++) {
         const uint32_t r0 = 16 * (w + 4 * j) + 4 * g;
@@ -546,100 +409,19 @@ __global__ __launch_bounds__(256) void recur_scan_kernel(OxbRecurParams p, uint3
 }
 
 // ---------------------------------------------------------------------------
-// Finish: gate and norm of each part of a row's outputs, values in registers.  Short parts (E values per lane): a wave per
-// part, four rows each, grid (rows / 4, parts / 4).  Long ones: 1024 threads per part, eight values each (parts beyond 8192 are
-// read again), grid (row, part).  Blocks behind the token rows bring the portion's last convolution inputs into the ring.
+// Finish.  Blocks behind the token rows bring the portion's last convolution inputs into the ring.
 // ---------------------------------------------------------------------------
-__device__ __forceinline__ void keep_inputs(const OxbRecurParams& p, uint32_t back, uint32_t first, uint32_t step) {
-    const uint32_t row = p.rows.m - 1 - back, pos = p.rows.pos0 + row;
-    float* keep = p.memory + (size_t)p.rows.seq0 * p.seq_stride + oxb_recur_state(p.d) + (size_t)(pos & (p.d.ring - 1u)) * p.d.channels;
-    const float* x = p.lin + (size_t)row * p.ld_lin + p.d.col_conv;
-    for (uint32_t i = first; i < p.d.channels; i += step) keep[i] = x[i];
-}
-
 template <typename T, int E, int ROWS>
-__global__ __launch_bounds__(256) void recur_finish_kernel(OxbRecurParams p) {
-    const OxbRecurDims& d = p.d;
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, inner = d.heads * d.dv, parts = inner / d.norm_len, n_rb = (p.rows.m + ROWS - 1) / ROWS;
-    if (blockIdx.x >= n_rb) return keep_inputs(p, blockIdx.x - n_rb, blockIdx.y * 256 + tid, gridDim.y * 256);
-    const uint32_t row0 = blockIdx.x * ROWS, part = blockIdx.y * 4 + (tid >> 6);
-    if (blockIdx.y == 0)
-        for (uint32_t t = 0; t < ROWS && row0 + t < p.rows.m; t++)
-            for (uint32_t i = inner + tid; i < p.out_fill; i += 256) reinterpret_cast<T*>(p.out)[(size_t)(row0 + t) * p.ld_out + p.out_col + i] = (T)0.f;
-    if (part >= parts) return;
-    float o[ROWS][E], z[ROWS][E], w[E];
-#pragma unroll
-    for (int t = 0; t < ROWS; t++) {
-        const uint32_t row = min(row0 + t, p.rows.m - 1);
-#pragma unroll
-        for (int e = 0; e < E; e++) {
-            const uint32_t i = min(lane + 64 * e, d.norm_len - 1);
-            o[t][e] = p.o[(size_t)row * inner + (size_t)part * d.norm_len + i];
-            z[t][e] = p.lin[(size_t)row * p.ld_lin + d.col_z + (size_t)part * d.norm_len + i];
-        }
-    }
-#pragma unroll
-    for (int e = 0; e < E; e++) w[e] = p.norm_w[(d.norm_shared ? 0 : (size_t)part * d.norm_len) + min(lane + 64 * e, d.norm_len - 1)];
-#pragma unroll
-    for (int t = 0; t < ROWS; t++) {
-        float ss = 0.f;
-#pragma unroll
-        for (int e = 0; e < E; e++) {
-            z[t][e] = silu_of(z[t][e]);
-            const float y = d.gate_first ? o[t][e] * z[t][e] : o[t][e];
-            if (lane + 64 * e < d.norm_len) ss = fmaf(y, y, ss);
-        }
-        const float inv = d.out_scale / sqrtf(wave_sum_f32(ss) / (float)d.norm_len + d.eps);
-        if (row0 + t >= p.rows.m) continue;
-        T* out = reinterpret_cast<T*>(p.out) + (size_t)(row0 + t) * p.ld_out + p.out_col + (size_t)part * d.norm_len;
-#pragma unroll
-        for (int e = 0; e < E; e++)
-            if (lane + 64 * e < d.norm_len) out[lane + 64 * e] = (T)(o[t][e] * inv * w[e] * z[t][e]);
-    }
+__global__ __launch_bounds__(256) void recur_finish_kernel(OxbRecurParams p) {   // grid (rows / ROWS, parts / 4)
+    const uint32_t n_rb = (p.rows.m + ROWS - 1) / ROWS;
+    if (blockIdx.x >= n_rb) return keep_inputs(p, blockIdx.x - n_rb, blockIdx.y * 256 + threadIdx.x, gridDim.y * 256);
+    recur_finish<T, E, ROWS>(p, blockIdx.x, blockIdx.y);
 }
 
 template <typename T>
-__global__ __launch_bounds__(1024) void recur_finish_long_kernel(OxbRecurParams p) {
-    constexpr int KEEP = 8;
-    const OxbRecurDims& d = p.d;
-    __shared__ float red[16];
-    const uint32_t tid = threadIdx.x, lane = tid & 63u, inner = d.heads * d.dv, row = blockIdx.x, part = blockIdx.y;
-    if (row >= p.rows.m) return keep_inputs(p, row - p.rows.m, blockIdx.y * 1024 + tid, gridDim.y * 1024);
-    T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ld_out + p.out_col;
-    if (part == 0)
-        for (uint32_t i = inner + tid; i < p.out_fill; i += 1024) out[i] = (T)0.f;
-    const float* o = p.o + (size_t)row * inner + (size_t)part * d.norm_len;
-    const float* z = p.lin + (size_t)row * p.ld_lin + d.col_z + (size_t)part * d.norm_len;
-    const float* w = p.norm_w + (d.norm_shared ? 0 : (size_t)part * d.norm_len);
-    float y[KEEP], g[KEEP], nw[KEEP], ss = 0.f;
-#pragma unroll
-    for (int k = 0; k < KEEP; k++) {
-        const uint32_t i = tid + 1024 * k;
-        y[k] = g[k] = nw[k] = 0.f;
-        if (i < d.norm_len) y[k] = o[i], g[k] = z[i], nw[k] = w[i];
-    }
-#pragma unroll
-    for (int k = 0; k < KEEP; k++) {
-        g[k] = silu_of(g[k]);
-        const float v = d.gate_first ? y[k] * g[k] : y[k];
-        ss = fmaf(v, v, ss);
-    }
-    for (uint32_t i = tid + 1024 * KEEP; i < d.norm_len; i += 1024) {
-        const float v = d.gate_first ? o[i] * silu_of(z[i]) : o[i];
-        ss = fmaf(v, v, ss);
-    }
-    ss = wave_sum_f32(ss);
-    if (lane == 0) red[tid >> 6] = ss;
-    __syncthreads();
-    ss = 0.f;
-#pragma unroll
-    for (int k = 0; k < 16; k++) ss += red[k];
-    const float inv = d.out_scale / sqrtf(ss / (float)d.norm_len + d.eps);
-    out += (size_t)part * d.norm_len;
-#pragma unroll
-    for (int k = 0; k < KEEP; k++)
-        if (tid + 1024 * k < d.norm_len) out[tid + 1024 * k] = (T)(y[k] * inv * nw[k] * g[k]);
-    for (uint32_t i = tid + 1024 * KEEP; i < d.norm_len; i += 1024) out[i] = (T)(o[i] * inv * w[i] * silu_of(z[i]));
+__global__ __launch_bounds__(1024) void recur_finish_long_kernel(OxbRecurParams p) {   // grid (row, part)
+    if (blockIdx.x >= p.rows.m) return keep_inputs(p, blockIdx.x - p.rows.m, blockIdx.y * 1024 + threadIdx.x, gridDim.y * 1024);
+    recur_finish_long<T>(p, blockIdx.x, blockIdx.y);
 }
 
 // ---------------------------------------------------------------------------
@@ -674,11 +456,11 @@ const char* oxb_recur_check(const OxbRecurDims& d) {
     if (d.dk > 256 || d.dv > 256) return "recurrent head size beyond 256";
     if (d.taps > 64 || d.ring < d.taps - 1 + OXB_RECUR_STEP_TOKENS || (d.ring & (d.ring - 1))) return "convolution taps beyond 64";
     if ((d.heads * d.dv) % d.norm_len) return "norm parts must divide the outputs";
-    if (d.heads > 65535) return "too many heads";
+    if (d.heads > 65535 || (uint64_t)d.heads * d.dv > (1u << 18)) return "too many heads";
     return nullptr;
 }
 
-static bool params_ok(const OxbRecurParams& p) {
+bool oxb_recur_params_ok(const OxbRecurParams& p) {
     return p.rows.m && p.lin && p.conv_w && p.neg_a && p.dt_bias && p.norm_w && p.memory && p.o && !oxb_recur_check(p.d) &&
            p.d.slices == (p.d.dv + 31) / 32 && p.d.dk_p == oxb_pad32(p.d.dk) && p.ld_lin >= p.d.col_conv + p.d.channels;
 }
@@ -710,8 +492,8 @@ static void pick_step(const OxbRecurParams& p, uint32_t tokens, hipStream_t st) 
 
 hipError_t oxb_launch_recur_step(const OxbRecurParams& p, int dt, hipStream_t st) {
     const uint32_t tokens = p.rows.seq_step ? 1 : p.rows.m;
-    if (!params_ok(p) || tokens > OXB_RECUR_STEP_TOKENS || p.rows.m / tokens > 65535) return hipErrorInvalidValue;
-    if (oxb_recur_step_finishes(p.d) && (!p.out || p.out_fill < p.d.heads * p.d.dv || p.out_col + p.out_fill > p.ld_out)) return hipErrorInvalidValue;
+    if (!oxb_recur_params_ok(p) || tokens > OXB_RECUR_STEP_TOKENS || p.rows.m / tokens > 65535) return hipErrorInvalidValue;
+    if (oxb_recur_step_finishes(p.d) && !oxb_recur_finish_ok(p)) return hipErrorInvalidValue;
     if (dt == OXB_DT_BF16) pick_step<__bf16>(p, tokens, st);
     else pick_step<float>(p, tokens, st);
     return hipGetLastError();
@@ -737,7 +519,7 @@ static void launch_prepare(const OxbRecurParams& p, uint32_t dv_p, dim3 grid, hi
 
 hipError_t oxb_launch_recur_chunked(const OxbRecurParams& p, hipStream_t st) {
     const OxbRecurDims& d = p.d;
-    if (!params_ok(p) || p.rows.pos || p.rows.seq_step || !p.n || p.first + p.n > p.rows.m || p.n > OXB_RECUR_SEGMENT || !p.s.q) return hipErrorInvalidValue;
+    if (!oxb_recur_params_ok(p) || p.rows.pos || p.rows.seq_step || !p.n || p.first + p.n > p.rows.m || p.n > OXB_RECUR_SEGMENT || !p.s.q) return hipErrorInvalidValue;
     const uint32_t dv_p = pad16(d.dv), n_vec = 2 * d.qk_heads + d.heads + 1;
     const uint32_t widest = d.dk_p > dv_p ? d.dk_p : dv_p;
     const dim3 prep((p.n + 7) / 8, (n_vec + 3) / 4);
@@ -772,9 +554,12 @@ static void launch_finish(const OxbRecurParams& p, uint32_t extra, hipStream_t s
     else hipLaunchKernelGGL((recur_finish_long_kernel<T>), dim3(p.rows.m + extra, p.d.heads * p.d.dv / p.d.norm_len), dim3(1024), 0, st, p);
 }
 
+bool oxb_recur_finish_ok(const OxbRecurParams& p) {
+    return oxb_recur_params_ok(p) && p.out && p.out_fill >= p.d.heads * p.d.dv && p.out_col + p.out_fill <= p.ld_out;
+}
+
 hipError_t oxb_launch_recur_finish(const OxbRecurParams& p, bool keep_conv, int dt, hipStream_t st) {
-    if (!params_ok(p) || !p.out || p.out_fill < p.d.heads * p.d.dv || p.out_col + p.out_fill > p.ld_out || (keep_conv && (p.rows.pos || p.rows.seq_step)))
-        return hipErrorInvalidValue;
+    if (!oxb_recur_finish_ok(p) || (keep_conv && (p.rows.pos || p.rows.seq_step))) return hipErrorInvalidValue;
     uint32_t extra = keep_conv ? p.d.taps - 1 : 0;
     if (extra > p.rows.m) extra = p.rows.m;
     if (dt == OXB_DT_BF16) launch_finish<__bf16>(p, extra, st);

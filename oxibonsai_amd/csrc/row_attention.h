@@ -50,6 +50,8 @@ hipError_t oxb_launch_grouped_store(const OxbGroupedStore& p, int dt, hipStream_
 hipError_t oxb_launch_row_decode(const OxbRowAttnParams& p, uint32_t head_tiles, int dt, hipStream_t st);
 hipError_t oxb_launch_row_merge(const OxbRowAttnParams& p, int dt, hipStream_t st);
 hipError_t oxb_launch_row_prefill(const OxbRowAttnParams& p, int dt, hipStream_t st);
+bool oxb_grouped_store_ok(const OxbGroupedStore& p, int dt);
+bool oxb_row_merge_ok(const OxbRowAttnParams& p, int dt);
 // Once per process and type, before the first launch.
 hipError_t oxb_row_attention_prepare(int dt);
 // Whether rows of `units` 32-element units and grouped heads of these sizes fit the kernels, and why not.
