@@ -297,6 +297,15 @@ int load_attention(BlockMaps& b, Model& m, const MixerConfig& c, const std::stri
     return rope_table(m, p, c.rope, &o->rope);
 }
 
+// Convolution weights [channels][taps] -> [taps][channels].
+int upload_taps(BlockMaps& b, const std::vector<float>& w, uint32_t taps, uint64_t* id) {
+    std::vector<float> t(w.size());
+    const size_t channels = w.size() / taps;
+    for (size_t c = 0; c < channels; c++)
+        for (size_t k = 0; k < taps; k++) t[k * channels + c] = w[c * taps + k];
+    return b.ld.upload(t, id);
+}
+
 // Sizes both recurrent mixers derive from the ones their configuration gives.
 int finish_recurrent(BlockMaps& b, Program& p, const std::string& name, ProgramBranch* o) {
     OxbRecurDims& d = o->r;
@@ -333,7 +342,7 @@ int load_state_space(BlockMaps& b, Program& p, const MixerConfig& c, const std::
     d.col_a = d.col_b = b.columns(in, (uint64_t)inner + d.channels, c.heads);
     std::vector<float> w;
     OXB_TRY(b.ld.values(name + "conv", {d.channels, d.taps}, plain_value, &w));
-    OXB_TRY(b.ld.upload(w, &o->conv_w));
+    OXB_TRY(upload_taps(b, w, d.taps, &o->conv_w));
     OXB_TRY(b.ld.vector(name + "conv.b", d.channels, &o->conv_b));
     OXB_TRY(b.ld.vector(name + "D", c.heads, &o->skip));
     return finish_recurrent(b, p, name, o);
@@ -365,7 +374,7 @@ int load_gated_delta(BlockMaps& b, Program& p, const MixerConfig& c, const std::
     OXB_TRY(b.ld.values(name + "q.conv", {qk, d.taps}, plain_value, &w));
     OXB_TRY(b.ld.values(name + "k.conv", {qk, d.taps}, plain_value, &w));
     OXB_TRY(b.ld.values(name + "v.conv", {inner, d.taps}, plain_value, &w));
-    OXB_TRY(b.ld.upload(w, &o->conv_w));
+    OXB_TRY(upload_taps(b, w, d.taps, &o->conv_w));
     return finish_recurrent(b, p, name, o);
 }
 

@@ -11,15 +11,18 @@ __device__ __forceinline__ v4f load4(const float* p) { return *reinterpret_cast<
 // Short convolution and its activation: channel ch of the token in row `row` of the input product, at position pos; `back`
 // earlier rows of the same sequence lie in front of it there, older inputs in the ring.
 __device__ __forceinline__ float conv_of(const OxbRecurParams& p, const float* ring, uint32_t row, uint32_t back, uint32_t pos, uint32_t ch) {
+    // (bases are the same for all lanes, the channel is every load's offset)
     const OxbRecurDims& d = p.d;
-    const float* w = p.conv_w + (size_t)ch * d.taps;
-    const float* x = p.lin + (size_t)row * p.ld_lin + d.col_conv + ch;
-    auto past = [&](uint32_t j) {
-        const float* at = j <= back ? x - (size_t)j * p.ld_lin : ring + (size_t)((pos - j) & (d.ring - 1u)) * d.channels + ch;
-        return *at * w[d.taps - 1 - j];
-    };
+    const float* x = p.lin + (size_t)row * p.ld_lin + d.col_conv;
+    const float* w = p.conv_w + (size_t)(d.taps - 1) * d.channels;
     const uint32_t n = min(d.taps - 1, pos);   // inputs there are behind this one
-    const float x0 = x[0] * w[d.taps - 1], x1 = n >= 1 ? past(1) : 0.f, x2 = n >= 2 ? past(2) : 0.f, x3 = n >= 3 ? past(3) : 0.f;
+    auto past = [&](uint32_t j) {   // (no branch around the loads: they all travel together)
+        const uint32_t k = min(j, n);
+        const float* at = k <= back ? x - (size_t)k * p.ld_lin : ring + (size_t)((pos - k) & (d.ring - 1u)) * d.channels;
+        const float y = at[ch] * (w - (size_t)k * d.channels)[ch];
+        return j <= n ? y : 0.f;
+    };
+    const float x0 = x[ch] * w[ch], x1 = past(1), x2 = past(2), x3 = past(3);
     float v = (p.conv_b ? p.conv_b[ch] : 0.f) + x0 + x1 + x2 + x3;
 #pragma unroll 1
     for (uint32_t j = 4; j <= n; j++) v += past(j);
@@ -44,8 +47,9 @@ template <typename T, int RPT, int SL, bool FINISH, bool ONE>
 __device__ __forceinline__ void recur_step(const OxbRecurParams& p, uint32_t n_tokens, uint32_t hb, uint32_t sb) {
     const OxbRecurDims& d = p.d;
     const uint32_t tokens = ONE ? 1 : n_tokens;
-    __shared__ __attribute__((aligned(16))) float qs[256], ks[256], vs[32 * SL], os[32 * SL];
+    __shared__ __attribute__((aligned(16))) float conv[512 + 32 * SL], os[32 * SL];   // queries, keys, values behind their convolutions
     __shared__ __attribute__((aligned(16))) float part[4 * SL][8][8];
+    __shared__ float gates[2];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, cl = tid & 7u, rg = (tid >> 3) & 31u;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6)), mine = wave >> 2;   // slice of the workgroup's
     const uint32_t groups = (d.slices + SL - 1) / SL, head = hb / groups, slice = hb % groups * SL + mine;
@@ -55,39 +59,51 @@ __device__ __forceinline__ void recur_step(const OxbRecurParams& p, uint32_t n_t
     float* ring = mem + oxb_recur_state(d);
     v4f s[RPT];
 #pragma unroll
-    for (int j = 0; j < RPT; j++) s[j] = pos0 && 32u * j < d.dk_p ? load4(state + 1024 * j) : (v4f){0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < RPT; j++) s[j] = load4(state + min(1024u * j, (d.dk_p - 32) * 32));
     const bool own_qk = head % rep == 0 && hb % groups == 0;
-    // which convolutions a thread brings: queries, keys, values in turn, spread over the workgroup
-    const uint32_t qi = tid, ki = SL > 1 ? tid - 256u : tid, vi = SL > 2 ? tid - 512u : 256u * SL - 1 - tid;
-    const uint32_t vcol = hb % groups * SL * 32 + vi;
+    const float *qs = conv, *ks = conv + d.dk_p, *vs = conv + 2 * d.dk_p;
+    const uint32_t n_conv = 2 * d.dk_p + 32 * SL, vcol = hb % groups * SL * 32;
+    constexpr int ROUNDS = (512 + 32 * SL + 256 * SL - 1) / (256 * SL);
     for (uint32_t t = 0; t < tokens; t++) {
         const uint32_t row = row0 + t, pos = pos0 + t;
         const float* lin = p.lin + (size_t)row * p.ld_lin;
-        float z[FINISH ? (SL + 1) / 2 : 1], nw[FINISH ? (SL + 1) / 2 : 1];
+        // the last wave forms the gates, the one before it what the finished output is multiplied by: neither has much of the
+        // convolutions to do
+        constexpr uint32_t GATES = 4 * SL - 1, LAST = 4 * SL - 2;
+        constexpr int E = (SL + 1) / 2;
+        float gate[E];
         if constexpr (FINISH) {
-            if (wave == 0) {
+            if (wave == LAST) {
 #pragma unroll
-                for (int e = 0; e < (SL + 1) / 2; e++) {
+                for (int e = 0; e < E; e++) {
                     const uint32_t i = min(lane + 64 * e, d.dv - 1);
-                    z[e] = lin[d.col_z + head * d.dv + i];
-                    nw[e] = p.norm_w[i];
+                    gate[e] = p.norm_w[i] * silu_of(lin[d.col_z + head * d.dv + i]);
                 }
             }
         }
-        float la, beta;
-        gates_of(p, row, head, &la, &beta);
-        const float a = expf(la);
-        if (qi < d.dk_p) qs[qi] = qi < d.dk ? conv_of(p, ring, row, t, pos, d.ch_q + qk * d.dk + qi) : 0.f;
-        if (ki < d.dk_p) ks[ki] = ki < d.dk ? conv_of(p, ring, row, t, pos, d.ch_k + qk * d.dk + ki) : 0.f;
-        if (vi < 32 * SL) vs[vi] = vcol < d.dv ? conv_of(p, ring, row, t, pos, d.ch_v + head * d.dv + vcol) : 0.f;
-        if (d.taps > 1 && t + d.taps > tokens) {   // inputs that later tokens convolve
-            float* keep = ring + (size_t)(pos & (d.ring - 1u)) * d.channels;
-            const float* x = lin + d.col_conv;
-            if (own_qk && qi < d.dk) keep[d.ch_q + qk * d.dk + qi] = x[d.ch_q + qk * d.dk + qi];
-            if (own_qk && ki < d.dk) keep[d.ch_k + qk * d.dk + ki] = x[d.ch_k + qk * d.dk + ki];
-            if (vi < 32 * SL && vcol < d.dv) keep[d.ch_v + head * d.dv + vcol] = x[d.ch_v + head * d.dv + vcol];
+        if (wave == GATES) {
+            float la, beta;
+            gates_of(p, row, head, &la, &beta);
+            if (lane == 0) gates[0] = expf(la), gates[1] = beta;
+        }
+#pragma unroll
+        for (int k = 0; k < ROUNDS; k++) {
+            const uint32_t it = tid + 256 * SL * k;
+            if (it >= n_conv) break;
+            const bool is_v = it >= 2 * d.dk_p, is_k = !is_v && it >= d.dk_p;
+            const uint32_t i = is_v ? it - 2 * d.dk_p + vcol : is_k ? it - d.dk_p : it, len = is_v ? d.dv : d.dk;
+            const uint32_t ch = (is_v ? d.ch_v + head * d.dv : (is_k ? d.ch_k : d.ch_q) + qk * d.dk) + i;
+            conv[it] = i < len ? conv_of(p, ring, row, t, pos, ch) : 0.f;
+            // inputs that later tokens convolve
+            if (d.taps > 1 && t + d.taps > tokens && i < len && (is_v || own_qk)) ring[(size_t)(pos & (d.ring - 1u)) * d.channels + ch] = lin[d.col_conv + ch];
+        }
+        if (t == 0) {
+#pragma unroll
+            for (int j = 0; j < RPT; j++)
+                if (!pos0) s[j] = (v4f){0.f, 0.f, 0.f, 0.f};
         }
         __syncthreads();
+        const float a = gates[0], beta = gates[1];
         float qq = 0.f, kk = 0.f, kq = 0.f;   // (every wave for itself)
         #pragma unroll 1
         for (uint32_t i = lane; i < d.dk_p; i += 64) {
@@ -139,18 +155,18 @@ __device__ __forceinline__ void recur_step(const OxbRecurParams& p, uint32_t n_t
         }
         if (FINISH || t + 1 < tokens) __syncthreads();
         if constexpr (FINISH) {
-            if (wave == 0) {
-                float y[(SL + 1) / 2], ss = 0.f;
+            if (wave == LAST) {
+                float y[E], ss = 0.f;
 #pragma unroll
-                for (int e = 0; e < (SL + 1) / 2; e++) {
+                for (int e = 0; e < E; e++) {
                     y[e] = lane + 64 * e < d.dv ? os[lane + 64 * e] : 0.f;
                     ss = fmaf(y[e], y[e], ss);
                 }
                 const float inv = d.out_scale / sqrtf(wave_sum_f32(ss) / (float)d.dv + d.eps);
                 T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ld_out + p.out_col;
 #pragma unroll
-                for (int e = 0; e < (SL + 1) / 2; e++)
-                    if (lane + 64 * e < d.dv) out[head * d.dv + lane + 64 * e] = (T)(y[e] * inv * nw[e] * silu_of(z[e]));
+                for (int e = 0; e < E; e++)
+                    if (lane + 64 * e < d.dv) out[head * d.dv + lane + 64 * e] = (T)(y[e] * inv * gate[e]);
                 if (head == 0)
                     for (uint32_t i = d.heads * d.dv + lane; i < p.out_fill; i += 64) out[i] = (T)0.f;
             }

@@ -59,7 +59,7 @@ struct OxbRecurParams {
     OxbRows rows;                      // rows of the whole launch (finish, step)
     const float* lin;                  // [rows.m][ld_lin] input product
     uint32_t ld_lin;
-    const float *conv_w, *conv_b;      // [channels][taps], last tap the current token's; [channels] or null
+    const float *conv_w, *conv_b;      // [taps][channels], last tap the current token's; [channels] or null
     const float *neg_a, *dt_bias;      // [heads]: -exp(A_log); bias
     const float* skip;                 // [heads] or null: o += skip v
     const float* norm_w;

@@ -5,7 +5,7 @@
 #include "recurrent_device.h"
 
 template <typename T, int RPT, int SL, bool FINISH, bool ONE>
-__global__ __launch_bounds__(256 * SL, ONE && RPT <= 4 ? (SL == 4 ? 8 : 7) : 4) void recur_step_kernel(OxbRecurParams p, uint32_t tokens) {   // grid (head x slice group, sequence)
+__global__ __launch_bounds__(256 * SL, ONE && RPT <= 4 ? (SL == 4 ? (RPT == 4 ? 4 : 8) : 7) : 4) void recur_step_kernel(OxbRecurParams p, uint32_t tokens) {   // grid (head x slice group, sequence)
     recur_step<T, RPT, SL, FINISH, ONE>(p, tokens, blockIdx.x, blockIdx.y);
 }
 
@@ -52,7 +52,7 @@ __global__ __launch_bounds__(256) void recur_prepare_kernel(OxbRecurParams p, ui
                 }
             }
 #pragma unroll
-            for (int t = 0; t < TAPS; t++) w[t][e] = p.conv_w[(size_t)c * TAPS + t];
+            for (int t = 0; t < TAPS; t++) w[t][e] = p.conv_w[(size_t)t * d.channels + c];
             bias[e] = p.conv_b ? p.conv_b[c] : 0.f;
         }
 #pragma unroll
