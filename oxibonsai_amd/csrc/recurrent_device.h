@@ -4,7 +4,8 @@
 #include "dense_device.h"
 #include "recurrent_kernels.h"
 
-__device__ __forceinline__ float silu_of(float z) { return z / (1.0f + expf(-z)); }
+// z / (1 + e^-z) on the hardware exponential and reciprocal (a few ulp where the result is not negligible beside z).
+__device__ __forceinline__ float silu_of(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.4426950408889634f)); }
 __device__ __forceinline__ float softplus_of(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ v4f load4(const float* p) { return *reinterpret_cast<const v4f*>(p); }
 

@@ -114,7 +114,7 @@ __device__ __forceinline__ v4f mfma16(v4f a, v4f b, v4f c) {   // 16 x 16 x 16, 
 // per wave), T_ij = -T_ii sum_k A_ik T_kj.
 // ---------------------------------------------------------------------------
 static constexpr uint32_t kLdT = 68;
-__global__ __launch_bounds__(256) void recur_chunk_kernel(OxbRecurParams p, uint32_t dv_p) {
+__global__ __launch_bounds__(256, 4) void recur_chunk_kernel(OxbRecurParams p, uint32_t dv_p) {
     const OxbRecurDims& d = p.d;
     __shared__ __attribute__((aligned(16))) float As[64][kLdT], Ts[64][kLdT];
     __shared__ double cum[64];
