@@ -327,35 +327,37 @@ __global__ __launch_bounds__(256, 1) void recur_scan_kernel(OxbRecurParams p, ui
 #pragma unroll
         for (int u = 0; u < DKU; u++) load_qw(q_at(i), w_at(i), i, u);
         load_u(i, i);
+        __builtin_amdgcn_sched_barrier(0);   // (the loop's order: its waits count requests)
     }
     load_pk(p_at(0), k_at(0), 0);
     load_pk(p_at(0), k_at(0), 1);
+    __builtin_amdgcn_sched_barrier(0);
     const float skip = p.skip ? p.skip[head] : 0.f;
     // Stores behind the end fall outside the buffer and are dropped: no branch, so the count of requests in flight stays known
     // and a chunk waits for its own operands alone.
     const uint32_t inner = d.heads * d.dv, o_bytes = p.n * inner * 4u;
     const __amdgpu_buffer_rsrc_t out = make_rsrc(p.o + (size_t)p.first * inner, o_bytes);
-    const uint32_t o_at = ((16 * w + 4 * g) * inner + head * d.dv + col) * 4u;
+    const uint32_t o_at = ((16 * w + 4 * g) * inner + head * d.dv + col) * 4u, o_rows = col < d.dv ? p.n : 0;
     auto step = [&](uint32_t ch, int set) {
         const bool live = ch < n_chunks;   // (the last group of NS chunks may run over the end)
         lds_barrier();
         v4f oq = {0.f, 0.f, 0.f, 0.f}, ws = oq;
         const float *qn = q_at(ch + NS), *wn = w_at(ch + NS), *pn = p_at(ch + 1), *kn = k_at(ch + 1);
         // an operand's successor is requested right behind its last product, so that the requests spread over the products
+        auto s_unit = [&](int u) { return join(load4(&Sx[c][32 * u + 4 * g]), load4(&Sx[c][32 * u + 16 + 4 * g])); };
+        v8f sb = s_unit(0);
 #pragma unroll
         for (int u = 0; u < DKU; u++) {
-            const v8f sb = join(load4(&Sx[c][32 * u + 4 * g]), load4(&Sx[c][32 * u + 16 + 4 * g]));
-            if constexpr (DELTA) ws = mfma32(wf[set][u], sb, ws);
-            oq = mfma32(qf[set][u], sb, oq);
+            const v8f next = s_unit(u + 1 < DKU ? u + 1 : u);
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                if constexpr (DELTA) ws = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[set][u][e], sb[e], ws, 0, 0, 0);
+                oq = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[set][u][e], sb[e], oq, 0, 0, 0);
+            }
             load_qw(qn, wn, set, u);
+            __builtin_amdgcn_sched_barrier(0);
+            sb = next;
         }
-#pragma unroll
-        for (int u = 0; u < DKU; u++) {
-            __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);                 // LDS read
-            __builtin_amdgcn_sched_group_barrier(0x008, DELTA ? 16 : 8, 0);    // matrix core
-            __builtin_amdgcn_sched_group_barrier(0x020, DELTA ? 4 : 2, 0);     // request
-        }
-        __builtin_amdgcn_sched_barrier(0);
         const v4f v = u0[set];
         v4f U = DELTA ? u0[set] - ws : u0[set] * beta[set];
         if (!live) U = (v4f){0.f, 0.f, 0.f, 0.f};
@@ -367,22 +369,23 @@ __global__ __launch_bounds__(256, 1) void recur_scan_kernel(OxbRecurParams p, ui
         for (int j = 0; j < TPW; j++) S[j] *= end;
         load_u(ch + NS, set);
         lds_barrier();
+        v8f ub[2], uf[2];
 #pragma unroll
         for (int u = 0; u < 2; u++) {
-            const v8f ub = join(load4(&Ux[c][32 * u + 4 * g]), load4(&Ux[c][32 * u + 16 + 4 * g]));
-            const v8f uf = join(load4(&Uf[c][32 * u + 4 * g]), load4(&Uf[c][32 * u + 16 + 4 * g]));
-            o = mfma32(pf[u], ub, o);
+            ub[u] = join(load4(&Ux[c][32 * u + 4 * g]), load4(&Ux[c][32 * u + 16 + 4 * g]));
+            uf[u] = join(load4(&Uf[c][32 * u + 4 * g]), load4(&Uf[c][32 * u + 16 + 4 * g]));
+        }
 #pragma unroll
-            for (int j = 0; j < TPW; j++) S[j] = mfma32(kf[j][u], uf, S[j]);
+        for (int u = 0; u < 2; u++) {
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(pf[u][e], ub[u][e], o, 0, 0, 0);
+#pragma unroll
+                for (int j = 0; j < TPW; j++) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[j][u][e], uf[u][e], S[j], 0, 0, 0);
+            }
             load_pk(pn, kn, u);
+            __builtin_amdgcn_sched_barrier(0);
         }
-#pragma unroll
-        for (int u = 0; u < 2; u++) {
-            __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
-            __builtin_amdgcn_sched_group_barrier(0x008, 8 * (1 + TPW), 0);
-            __builtin_amdgcn_sched_group_barrier(0x020, 2 * (1 + TPW), 0);
-        }
-        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int j = 0; j < TPW; j++) {
             const uint32_t r0 = 16 * (w + 4 * j) + 4 * g;
@@ -392,7 +395,7 @@ __global__ __launch_bounds__(256, 1) void recur_scan_kernel(OxbRecurParams p, ui
         for (int i = 0; i < 4; i++) {
             const uint32_t m = ch * 64 + 16 * w + 4 * g + i;
             __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(o[i] + (DELTA ? 0.f : skip * v[i])), out,
-                                                  (int)(m < p.n && col < d.dv ? o_at + (ch * 64 + i) * inner * 4u : OXB_OOB), 0, 0);
+                                                  (int)(m < o_rows ? o_at + (ch * 64 + i) * inner * 4u : OXB_OOB), 0, 0);
         }
     };
     for (uint32_t ch = 0; ch < n_chunks; ch += NS)
