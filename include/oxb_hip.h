@@ -301,10 +301,13 @@ int  oxb_hip_prefill_tokens(uint64_t model, uint64_t embedding, uint32_t seq, co
 /* ---- model designs described by a config.json (layer programs), and one loader for every kind of checkpoint.
  * A checkpoint is a GGUF file (as above) or a folder with config.json and model.safetensors; config.json's "architecture"
  * names the design in the library's registry (Fulirax: latent attention with sinks, dynamic-tanh norms, dense tanh-GELU
- * feed-forwards, a loop over a range of layers).  The model behind the handle is driven by the same calls as any other:
+ * feed-forwards, a loop over a range of layers; Muvonex: gated delta rule layers and layers of grouped attention beside a
+ * state space, parallel residual, gated feed-forwards).  The model behind the handle is driven by the same calls as any other:
  * oxb_hip_decode, oxb_hip_prefill[_tokens], oxb_hip_decode_tokens[_sampled], oxb_hip_forward_tokens, the paged-cache calls
- * and oxb_hip_model_reset / _destroy.  Its cache holds latent rows in the compute type: kv_dtype and window options, read_kv,
- * set_rope_rows, set_lm_head and decode_hidden do not apply and answer InvalidArgument. */
+ * and oxb_hip_model_reset / _destroy.  Its cache holds rows of its own kind in the compute type: kv_dtype and window options,
+ * read_kv, set_rope_rows, set_lm_head and decode_hidden do not apply and answer InvalidArgument.  Where layers are recurrent every
+ * sequence slot also keeps their state: a call's first position must be the one the slot stands at, or 0, which starts again
+ * from an empty state; anything else is InvalidArgument and changes nothing.  kv_release and reset free the slot. */
 enum { OXB_COMPUTE_BF16 = 0, OXB_COMPUTE_F32 = 1 };   /* F32: every product in 32 bits */
 typedef struct {
     char architecture[32];
