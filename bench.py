@@ -641,7 +641,7 @@ def main() -> int:
     ap.add_argument("--muvonex", action="store_true", help="the same for Muvonex")
     ap.add_argument("--design-layers", "--fulirax-layers", type=int, default=8)
     ap.add_argument("--design-shape", "--fulirax-shape", type=int, default=-1, help="one of the shapes alone")
-    ap.add_argument("--design-only", choices=["", "design", "qwen3"], default="", help="one of the two models alone (profiling)")
+    ap.add_argument("--design-only", "--fulirax-only", choices=["", "design", "fulirax", "muvonex", "qwen3"], default="", help="one of the two models alone (profiling)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build targets one GPU; run with --gpus 1 (multi-GPU sharding is design-only)",
@@ -662,7 +662,7 @@ def main() -> int:
         design = "fulirax" if args.fulirax else "muvonex"
         rows = design_leg(be, design, args.design_layers, 32768, args.decode_context, args.decode_tokens,
                           tuple(int(b) for b in args.decode_batches.split(",") if b), args.long_context,
-                          design if args.design_only == "design" else args.design_only, args.design_shape)
+                          args.design_only if args.design_only in ("", "qwen3") else design, args.design_shape)
         print(json.dumps({"metric": f"{design.capitalize()} prefill and decode", "n_gpus": 1, "dtype": "bf16", "data": "synthetic, random weights",
                           "prompt": args.decode_context, "steps": args.decode_tokens, "shapes": rows}), flush=True)
         return 0

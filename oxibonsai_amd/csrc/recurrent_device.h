@@ -39,10 +39,10 @@ __device__ __forceinline__ void gates_of(const OxbRecurParams& p, uint32_t row, 
 }
 
 // ---------------------------------------------------------------------------
-// Step.  Workgroup (hb, sb): head x slice group, sequence; 256 threads per slice of 32 columns: thread (rg, cl) = (tid / 8 % 32, tid % 8)
-// holds rows rg + 32 j and columns 4 cl .. + 3 of its slice of the state.  S^T k and S^T q come out of the state as it was, in
-// one pass: with the write k u^T, o = a (S^T q) + (k . q) u.  With every slice of a head in the workgroup (FINISH) the head's
-// output is gated and normed here as well.
+// Step.  Workgroup (hb, sb): head x slice group, sequence; 256 threads per slice of 32 columns.  Thread (rg, cl) = (tid / 8 %
+// 32, tid % 8) holds rows rg + 32 j and columns 4 cl .. + 3 of its slice of the state.  S^T k and S^T q come out of the state as
+// it was, in one pass: with the write k u^T, o = a (S^T q) + (k . q) u.  With every slice of a head in the workgroup (FINISH) the
+// head's output is gated and normed here as well.
 // ---------------------------------------------------------------------------
 template <typename T, int RPT, int SL, bool FINISH, bool ONE>
 __device__ __forceinline__ void recur_step(const OxbRecurParams& p, uint32_t n_tokens, uint32_t hb, uint32_t sb) {

@@ -4,8 +4,11 @@
 
 #include "recurrent_device.h"
 
-template <typename T, int RPT, int SL, bool FINISH, bool ONE>
-__global__ __launch_bounds__(256 * SL, ONE && RPT <= 4 ? (SL == 4 ? (RPT == 4 ? 4 : 8) : 7) : 4) void recur_step_kernel(OxbRecurParams p, uint32_t tokens) {   // grid (head x slice group, sequence)
+// Waves per SIMD that a step is compiled for: as many as its registers allow without spilling.
+constexpr int step_waves(int rpt, int sl, bool one) { return !one || rpt > 4 ? 4 : sl < 4 ? 7 : rpt < 4 ? 8 : 4; }
+
+template <typename T, int RPT, int SL, bool FINISH, bool ONE>   // grid (head x slice group, sequence)
+__global__ __launch_bounds__(256 * SL, step_waves(RPT, SL, ONE)) void recur_step_kernel(OxbRecurParams p, uint32_t tokens) {
     recur_step<T, RPT, SL, FINISH, ONE>(p, tokens, blockIdx.x, blockIdx.y);
 }
 
@@ -257,8 +260,8 @@ __global__ __launch_bounds__(256, 4) void recur_chunk_kernel(OxbRecurParams p, u
 }
 
 // ---------------------------------------------------------------------------
-// Scan.  Grid (head x 16 columns, the tiles of a head on one XCD: they share its L2), 4 waves: wave w takes token rows 16 w .. of every chunk and the state's row tiles w, w + 4,
-// ..; per chunk, with S the state at its start,
+// Scan.  Grid (head x 16 columns, the tiles of a head on one XCD: they share its L2), 4 waves: wave w takes token rows 16 w ..
+// of every chunk and the state's row tiles w, w + 4, ..; per chunk, with S the state at its start,
 //   U = U0 - W S        o = e^c (Q S) + P U        S <- e^(c_end) S + K^T diag(e^(c_end - c)) U
 // The operands of a later chunk are requested as soon as this chunk's have been used; the barriers order LDS alone.
 // ---------------------------------------------------------------------------

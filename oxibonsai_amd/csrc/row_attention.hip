@@ -437,7 +437,7 @@ hipError_t oxb_launch_row_decode(const OxbRowAttnParams& p, uint32_t head_tiles,
 }
 
 bool oxb_row_merge_ok(const OxbRowAttnParams& p, int dt) {
-    return rows_ok(p, dt) && p.part_o && p.part_ml && p.out && p.n_splits && p.n_splits <= OXB_MAX_SPLITS && p.out_col + p.heads * 16 * p.nt <= p.ld_out;
+    return rows_ok(p, dt) && p.nt <= 16 && p.part_o && p.part_ml && p.out && p.n_splits && p.n_splits <= OXB_MAX_SPLITS && p.out_col + p.heads * 16 * p.nt <= p.ld_out;
 }
 
 hipError_t oxb_launch_row_merge(const OxbRowAttnParams& p, int dt, hipStream_t st) {
@@ -470,7 +470,9 @@ template <typename T>
 static hipError_t raise_lds() {
     hipError_t e = hipSuccess;
 #define OXB_RAISE(H, K, N, D) \
-    if (e == hipSuccess) e = hipFuncSetAttribute((const void*)&row_decode_kernel<T, H, K, N, D>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)(kLdsMax - kDecodeStatic));
+    if (e == hipSuccess)                                                                                                       \
+        e = hipFuncSetAttribute((const void*)&row_decode_kernel<T, H, K, N, D>, hipFuncAttributeMaxDynamicSharedMemorySize,  \
+                                (int)(kLdsMax - kDecodeStatic));
     OXB_DECODE_SIZES(OXB_RAISE)
 #undef OXB_RAISE
     const void* prefill[] = {(const void*)&row_prefill_kernel<T, 2, 4, 8>, (const void*)&row_prefill_kernel<T, 1, 8, 16>};

@@ -68,7 +68,8 @@ template <typename T, int E, int ROWS> __device__ __forceinline__ void grouped_s
     }
 }
 
-// Merge of one head's splits - the sink joins the denominator here, once.  One workgroup of any size.
+// Merge of one head's splits - the sink joins the denominator here, once.  One workgroup of at least 256 threads (values have at
+// most 256 elements).
 template <typename T> __device__ __forceinline__ void row_merge(const OxbRowAttnParams& p, uint32_t head, uint32_t m) {
     __shared__ float wgt[OXB_MAX_SPLITS];
     const uint32_t tid = threadIdx.x, lane = tid & 63u;
@@ -98,18 +99,28 @@ template <typename T> __device__ __forceinline__ void row_merge(const OxbRowAttn
             if (lane + 64 * i < used) wgt[lane + 64 * i] = w[i] / L * p.out_scale;
     }
     __syncthreads();
+    // a thread per value element, the threads beyond take further shares of the splits
+    __shared__ float sums[1024];
+    const uint32_t shares = min(max(blockDim.x / dim, 1u), 8u), share = tid / dim;
     const float* po = p.part_o + (slot0 * 16 + col) * dim;
-    T* out = reinterpret_cast<T*>(p.out) + (size_t)m * p.ld_out + p.out_col + head * dim;
-    for (uint32_t i = tid; i < dim; i += blockDim.x) {
+    if (share < shares) {
+        const uint32_t i = tid % dim;
         float y = 0.f;
-        for (uint32_t s0 = 0; s0 < used; s0 += 8) {
+        for (uint32_t s0 = share; s0 < used; s0 += 8 * shares) {
             float v[8];
 #pragma unroll
-            for (int k = 0; k < 8; k++) v[k] = po[(size_t)min(s0 + k, used - 1) * 16 * dim + i];
+            for (int k = 0; k < 8; k++) v[k] = po[(size_t)min(s0 + k * shares, used - 1) * 16 * dim + i];
 #pragma unroll
             for (int k = 0; k < 8; k++)
-                if (s0 + k < used) y = fmaf(v[k], wgt[s0 + k], y);
+                if (s0 + k * shares < used) y = fmaf(v[k], wgt[s0 + k * shares], y);
         }
-        out[i] = (T)y;
+        sums[tid] = y;
+    }
+    __syncthreads();
+    T* out = reinterpret_cast<T*>(p.out) + (size_t)m * p.ld_out + p.out_col + head * dim;
+    if (tid < dim) {
+        float y = sums[tid];
+        for (uint32_t k = 1; k < shares; k++) y += sums[k * dim + tid];
+        out[tid] = (T)y;
     }
 }

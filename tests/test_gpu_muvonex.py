@@ -87,7 +87,7 @@ def test_gated_feed_forward_alone(make, dtype, ff, gain):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(3, 3, 16, 24), (8, 2, 64, 48), (20, 1, 34, 130), (2, 2, 256, 8), (4, 2, 6, 256)])
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(3, 3, 16, 24), (8, 2, 72, 40), (20, 1, 34, 130), (2, 2, 256, 8), (4, 2, 6, 256)])
 def test_grouped_attention_alone(make, dtype, heads, kv_heads, dim, vdim):
     cfg = mm.config(64, 40, [mm.parallel(mm.attention(heads, kv_heads, dim, vdim, scale=0.4), mm.space(1, 8, 8))])
     bits = mm.without(mm.weights(cfg, 5), "right.o")
